@@ -609,6 +609,138 @@ int ohara_phi_attn_bf16(const uint16_t* q, int ldq, const uint16_t* kcache, cons
                         const float* sin, int rot, int batch, int seq_len, int h, int dh, int t_max, int pos,
                         const int32_t* pos_dev, int n_split, void* workspace, uint16_t* out, void* stream);
 
+/* ---- hybrid decoders: attention with a distance bias beside recurrent layers -----------------------
+ * (no counterpart in the reference.)  Entry points ending in _bf16 keep activations, caches and weights
+ * in bfloat16, those ending in _f32 in 32-bit floats; the residual stream, every norm, score, softmax
+ * weight, decay and recurrent state is fp32 in both.  Vectors (norm, convolution, decay parameters)
+ * are fp32 in both.
+ *
+ * OharaSeq says which rows of a call belong to which sequence and where they sit: the call has
+ * batch * seq_len rows ordered (sequence, token); token s of sequence b sits at position start(b) + s with
+ * start(b) = pos, *pos_dev or pos_dev[b] (pos_stride 0 / 1).  lens: tokens of each sequence in this call
+ * (rows past them are padding: they change no cache or state and their results mean nothing); NULL: all
+ * have seq_len.  slots: cache row of each sequence; NULL: sequence b uses row b.  Two sequences of a call
+ * never share a cache row. */
+typedef struct OharaSeq {
+  int batch, seq_len, pos, pos_stride;
+  const int32_t* pos_dev;
+  const int32_t* lens;
+  const int32_t* slots;
+} OharaSeq;
+
+/* What the residual kernel puts into `out` after updating the residual row x. */
+#define OHARA_OUT_NONE 0
+#define OHARA_OUT_COPY 1 /* x */
+#define OHARA_OUT_CONV 2 /* x + causal depthwise convolution of x over time (seq_len 1; see conv_w / ring) */
+#define OHARA_OUT_NORM 3 /* group RMS norm of x times norm2_w */
+
+/* Residual update of a block with norms on the sublayer outputs, one launch:
+ *   ids != NULL:  x = table[id]              (table: activation type, vocab rows of d)
+ *   y != NULL:    x += norm_w * group_rms(y) (groups equal runs of the row, each over sqrt(mean square + eps))
+ * x: (rows, d) fp32, updated in place.  out (leading dimension ldo >= d, columns past d are set to zero)
+ * per out_mode.  OHARA_OUT_CONV: conv_w (taps, d) fp32 with the current token's row last, ring
+ * (cache rows, taps, d) fp32 holds the inputs of the last tokens at index position mod taps and is
+ * updated; inputs before position 0 count as zero, so a ring needs no clearing when its row is reused.
+ * OHARA_OUT_NORM takes norm2_w. */
+int ohara_residual_norm_bf16(float* x, int d, const int64_t* ids, const uint16_t* table, int vocab, const uint16_t* y,
+                             int ldy, const float* norm_w, int groups, float eps, int out_mode, uint16_t* out, int ldo,
+                             const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
+                             void* stream);
+int ohara_residual_norm_f32(float* x, int d, const int64_t* ids, const float* table, int vocab, const float* y, int ldy,
+                            const float* norm_w, int groups, float eps, int out_mode, float* out, int ldo,
+                            const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
+                            void* stream);
+/* out = x + causal depthwise convolution of x over time for any seq_len (the ring is only read: follow with
+ * ohara_conv_ring_store_f32), columns d .. ldo-1 of out are set to zero. */
+int ohara_input_conv_bf16(const float* x, int d, const float* conv_w, int taps, const float* ring, uint16_t* out, int ldo,
+                          const OharaSeq* seq, void* stream);
+int ohara_input_conv_f32(const float* x, int d, const float* conv_w, int taps, const float* ring, float* out, int ldo,
+                         const OharaSeq* seq, void* stream);
+/* The last taps - 1 input rows of each sequence (src: rows of `channels`, leading dimension ld) -> ring
+ * (cache rows, taps, channels) at index position mod taps. */
+int ohara_conv_ring_store_bf16(const uint16_t* src, int ld, int channels, int taps, uint16_t* ring, const OharaSeq* seq,
+                               void* stream);
+int ohara_conv_ring_store_f32(const float* src, int ld, int channels, int taps, float* ring, const OharaSeq* seq,
+                              void* stream);
+
+/* Plain fp32 product for models served in 32-bit: y = x W^T (+ bias), W (n, k) fp32 row-major, k % 4 == 0.
+ * w_up != NULL: y = silu(x W^T) * (x w_up^T).  cap > 0: y = cap * tanh(y / cap). */
+int ohara_gemm_f32(const float* x, int ldx, const float* w, const float* w_up, const float* bias, float cap, int n, int k,
+                   int rows, float* out, int ldo, void* stream);
+/* ohara_gemm_skinny_bf16 without a norm and with y = bf16(cap * tanh(fp32 sum / cap)) as the epilogue
+ * (vocabulary projections with soft-capped logits). */
+int ohara_gemm_softcap_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, float cap, int rows,
+                            uint16_t* out, int ldo, void* stream);
+
+/* Attention front end off one projection p with row layout [q (h*dh); k (h_kv*dh); v (h_kv*dv); ...]:
+ * q and k are each divided by the root mean square of ALL their elements of the row and multiplied by
+ * qn / kn; every value head is divided by its own root mean square.  q -> q_out (rows, h, dhp), keys and
+ * values -> caches (cache rows, t_max, h_kv, dhp) and (.., dvp) at the tokens' positions; dhp / dvp are
+ * dh / dv rounded up to multiples of 8, the columns past dh / dv are set to zero. */
+int ohara_qkv_norm_append_bf16(const uint16_t* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn,
+                               const float* kn, float eps, uint16_t* q_out, uint16_t* kcache, uint16_t* vcache, int t_max,
+                               const OharaSeq* seq, void* stream);
+int ohara_qkv_norm_append_f32(const float* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn, const float* kn,
+                              float eps, float* q_out, float* kcache, float* vcache, int t_max, const OharaSeq* seq,
+                              void* stream);
+/* Causal attention over the cache with a linear distance bias and a per-head output gate:
+ *   o[row, hd, :] = sigmoid(gate[row, hd]) * sum_j softmax_j(scale q . k_j - slopes[hd] (i - j)) v_j,  j <= i = position.
+ * Scores, softmax weights and sums are fp32 (the _bf16 prefill product carries every fp32 weight as three
+ * bfloat16 terms).  q / caches as written by ohara_qkv_norm_append; gate (leading dimension ldg, in the
+ * activation type; NULL: none); out rows of h*dv with leading dimension ldo, columns past h*dv are set to
+ * zero.  dh, dv <= 256.  n_split > 1 (seq_len 1): the context of a (sequence, KV head) is cut into that many chunks
+ * that meet in `workspace` (ohara_attn_bias_workspace_bytes, zero-filled once; calls sharing it must not
+ * overlap). */
+int64_t ohara_attn_bias_workspace_bytes(int rows, int h, int dv, int n_split);
+int ohara_attn_bias_bf16(const uint16_t* q, const uint16_t* kcache, const uint16_t* vcache, int h, int h_kv, int dh,
+                         int dv, int t_max, float scale, const float* slopes, const uint16_t* gate, int ldg, int n_split,
+                         void* workspace, uint16_t* out, int ldo, const OharaSeq* seq, void* stream);
+int ohara_attn_bias_f32(const float* q, const float* kcache, const float* vcache, int h, int h_kv, int dh, int dv,
+                        int t_max, float scale, const float* slopes, const float* gate, int ldg, int n_split,
+                        void* workspace, float* out, int ldo, const OharaSeq* seq, void* stream);
+
+/* Gated delta rule with one decay per head and key channel.  Per value head: S (dim x vdim) fp32,
+ *   S <- diag(exp(lg)) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q,
+ *   q, k, v: short causal convolution per channel (taps), silu; q, k over sqrt(sum of squares + 1e-6), q also times
+ *   dim^-1/2;  lg = neg_a[head] * softplus(W_a2 a1 + dt_bias);  beta = sigmoid(b);
+ *   out = o / rms(o) * norm_w * sigmoid(W_g2 g1).
+ * A projection row p holds [q (kv_heads*dim); k (kv_heads*dim); v (heads*vdim)] from column 0, the rank_a columns a1
+ * from off_a, the rank_g columns g1 from off_g (offsets and ranks multiples of 8) and the heads columns b from off_b.
+ * a2 (heads*dim, rank_a), g2 (heads*vdim, rank_g) row-major in the activation type; conv_w (taps, channels) fp32 with the
+ * current token's row last; state (cache rows, heads, dim, vdim rounded up to a multiple of 4) fp32; ring (cache rows,
+ * taps, channels) in the activation type.  A sequence whose first token sits at position 0 starts from zero
+ * whatever its state and ring hold.  dim, vdim <= 256. */
+typedef struct OharaDelta {
+  int heads, kv_heads, dim, vdim, taps, rank_a, rank_g, off_a, off_g, off_b;
+  float eps;
+  int reserved;
+  const float* conv_w;
+  const void* a2;
+  const void* g2;
+  const float* neg_a;
+  const float* dt_bias;
+  const float* norm_w;
+} OharaDelta;
+/* One token per sequence (seq_len 1): everything above in one launch; ring and state are updated. */
+int ohara_delta_step_bf16(const OharaDelta* d, const uint16_t* p, int ldp, float* state, uint16_t* ring, uint16_t* out,
+                          int ldo, const OharaSeq* seq, void* stream);
+int ohara_delta_step_f32(const OharaDelta* d, const float* p, int ldp, float* state, float* ring, float* out, int ldo,
+                         const OharaSeq* seq, void* stream);
+/* Any number of tokens per sequence, in chunks of 32 tokens: za (rows, heads*dim) = W_a2 a1 and zg (rows, heads*vdim)
+ * = W_g2 g1 come from the caller.  First the chunks are solved on their own in parallel, then the state walks
+ * over them on fp32 matrix products; state is updated, the ring is only read (follow with
+ * ohara_conv_ring_store over the first 2*kv_heads*dim + heads*vdim columns of p).  workspace:
+ * ohara_delta_workspace_bytes for the number of tokens per sequence worked on at a time (the call cuts
+ * longer sequences into segments that fit); o_tmp: (rows, heads*vdim) fp32. */
+int64_t ohara_delta_workspace_bytes(int heads, int dim, int vdim, int batch, int tokens);
+int ohara_delta_prefill_bf16(const OharaDelta* d, const uint16_t* p, int ldp, const uint16_t* za, int ldza,
+                             const uint16_t* zg, int ldzg, float* state, const uint16_t* ring, void* workspace,
+                             int64_t workspace_bytes, float* o_tmp, uint16_t* out, int ldo, const OharaSeq* seq,
+                             void* stream);
+int ohara_delta_prefill_f32(const OharaDelta* d, const float* p, int ldp, const float* za, int ldza, const float* zg,
+                            int ldzg, float* state, const float* ring, void* workspace, int64_t workspace_bytes,
+                            float* o_tmp, float* out, int ldo, const OharaSeq* seq, void* stream);
+
 /* ---- timing helpers (measurement only; no counterpart in the reference) -----------
  * Thin wrappers over hipEventCreate / hipEventDestroy / hipEventElapsedTime so that a
  * benchmark can time single launches on the stream they run on without another HIP

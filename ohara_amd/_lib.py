@@ -11,6 +11,8 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "lib", "libohara_decode.so")
+# fewer sources, the same entry points where present (ohara_amd.build.ensure); loaded if the full library is not built
+PARTIAL_LIB_PATH = os.path.join(_HERE, "lib", "libohara_serving.so")
 
 OK, EINVAL, ELAUNCH, ESIZE = 0, -1, -2, -3
 _ERR = {EINVAL: "invalid argument", ELAUNCH: "HIP launch failed", ESIZE: "size not supported"}
@@ -59,6 +61,19 @@ class OharaDecodeState(C.Structure):
     ]
 
 
+class OharaSeq(C.Structure):
+    _fields_ = [("batch", _i), ("seq_len", _i), ("pos", _i), ("pos_stride", _i), ("pos_dev", _p), ("lens", _p), ("slots", _p)]
+
+
+class OharaDelta(C.Structure):
+    _fields_ = [
+        ("heads", _i), ("kv_heads", _i), ("dim", _i), ("vdim", _i), ("taps", _i), ("rank_a", _i), ("rank_g", _i),
+        ("off_a", _i), ("off_g", _i), ("off_b", _i), ("eps", _f), ("reserved", _i),
+        ("conv_w", _p), ("a2", _p), ("g2", _p), ("neg_a", _p), ("dt_bias", _p), ("norm_w", _p),
+    ]
+
+
+OUT_NONE, OUT_COPY, OUT_CONV, OUT_NORM = 0, 1, 2, 3
 OHARA_LOGITS_NONE, OHARA_LOGITS_LAST, OHARA_LOGITS_ALL = 0, 1, 2
 
 _PROTOS = {
@@ -128,6 +143,20 @@ _PROTOS = {
     "ohara_bitnet_persistent_profile_offset": (_i64, [C.POINTER(OharaBitModel), _i, _i]),
     "ohara_bitnet_decode_persistent": (_i, [C.POINTER(OharaBitModel), C.POINTER(OharaDecodeState), _p, _i, _i, _i,
                                             C.c_uint, _p]),
+    **{f"ohara_{name}_{dt}": proto for dt in ("bf16", "f32") for name, proto in {
+        "residual_norm": (_i, [_p, _i, _p, _p, _i, _p, _i, _p, _i, _f, _i, _p, _i, _p, _p, _i, _p, C.POINTER(OharaSeq), _p]),
+        "input_conv": (_i, [_p, _i, _p, _i, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "conv_ring_store": (_i, [_p, _i, _i, _i, _p, C.POINTER(OharaSeq), _p]),
+        "qkv_norm_append": (_i, [_p, _i, _i, _i, _i, _i, _p, _p, _f, _p, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "attn_bias": (_i, [_p, _p, _p, _i, _i, _i, _i, _i, _f, _p, _p, _i, _i, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "delta_step": (_i, [C.POINTER(OharaDelta), _p, _i, _p, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "delta_prefill": (_i, [C.POINTER(OharaDelta), _p, _i, _p, _i, _p, _i, _p, _p, _p, _i64, _p, _p, _i,
+                               C.POINTER(OharaSeq), _p]),
+    }.items()},
+    "ohara_gemm_f32": (_i, [_p, _i, _p, _p, _p, _f, _i, _i, _i, _p, _i, _p]),
+    "ohara_gemm_softcap_bf16": (_i, [_p, _i, _p, _i, _i, _f, _i, _p, _i, _p]),
+    "ohara_attn_bias_workspace_bytes": (_i64, [_i, _i, _i, _i]),
+    "ohara_delta_workspace_bytes": (_i64, [_i, _i, _i, _i, _i]),
     "ohara_event_create": (_i, [C.POINTER(_p)]),
     "ohara_event_destroy": (_i, [_p]),
     "ohara_event_record": (_i, [_p, _p]),
@@ -141,13 +170,16 @@ def lib():
     """The loaded library; raises if it was never built."""
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
+        path = LIB_PATH if os.path.exists(LIB_PATH) else PARTIAL_LIB_PATH
+        if not os.path.exists(path):
             raise RuntimeError(
                 f"{LIB_PATH} is missing: build the HIP kernels first (python -m ohara_amd.build). "
                 "ohara_amd has no fallback path."
             )
-        handle = C.CDLL(LIB_PATH)
+        handle = C.CDLL(path)
         for name, (res, args) in _PROTOS.items():
+            if path == PARTIAL_LIB_PATH and not hasattr(handle, name):
+                continue  # an entry point of another kind of model: calling it raises
             fn = getattr(handle, name)
             fn.restype = res
             fn.argtypes = args

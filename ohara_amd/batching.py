@@ -14,7 +14,7 @@ from __future__ import annotations
 import torch
 
 from . import ops
-from .llama import BF16, Llama
+from .llama import Llama
 
 
 class ContinuousBatcher:
@@ -47,33 +47,112 @@ class ContinuousBatcher:
         return ops.sample_topk_topp(logits, self.sampling.temperature, self.sampling.top_k, self.sampling.top_p, u,
                                     valid_vocab=vv)
 
+    def _padded_forward(self, slots: list[int], tokens: list, last_only: bool) -> torch.Tensor:
+        """The given tokens of several slots in one call (models with ``supports_seq_lens``), each from its slot's own
+        position -> logits (rows, S or 1, V); rows shorter than the longest are padded."""
+        lens = [len(t) for t in tokens]
+        ids = torch.zeros(len(slots), max(lens), dtype=torch.int64)
+        for row, t in zip(ids, tokens):
+            row[: len(t)] = t
+        return self.model.forward(ids, self.cache, [self.lengths[b] for b in slots], last_only=last_only, seq_lens=lens,
+                                  slots=slots)
+
+    def _prefill(self, slots: list[int], prompts: list, last_only: bool = True) -> list[torch.Tensor]:
+        """Run prompts (1-D ids, on the host) into free slots -> the logits (1 or len, V) of each: one call for all where the
+        model takes prompts of different lengths, else one call per prompt over its slot's rows of the cache."""
+        for b in slots:
+            for c in self.cache:
+                c.lengths[b] = 0
+            self.lengths[b] = 0
+        if getattr(self.model, "supports_seq_lens", False):
+            logits = self._padded_forward(slots, prompts, last_only)
+            out = [row[: 1 if last_only else len(p)] for row, p in zip(logits, prompts)]
+        else:
+            out = []
+            for b, ids in zip(slots, prompts):
+                views = [c._row_view(b) for c in self.cache]
+                out.append(self.model.forward(ids.view(1, -1).to(self.model.device), views, 0, last_only=last_only)[0])
+        for b, ids in zip(slots, prompts):
+            self._book(b, len(ids))
+        return out
+
+    def _book(self, b: int, length: int) -> None:
+        """Slot b holds ``length`` tokens from now on."""
+        for c in self.cache:
+            c.lengths[b] = length
+            c.length = max(c.lengths)
+        self.lengths[b] = length
+        self.active[b] = True
+        self.seq_pos[b] = length
+        self.active_dev[b] = 1
+
+    def _host_ids(self, tokens, start: int = 0) -> torch.Tensor:
+        ids = torch.as_tensor(tokens, dtype=torch.int64).reshape(-1).cpu()
+        if ids.numel() < 1:
+            raise ValueError("input sequence cannot be empty")
+        if start + ids.numel() > self.model.config.max_sequence_length:
+            raise ValueError("input exceeds max_sequence_length")
+        return ids
+
     @torch.no_grad()
     def add(self, prompt_ids) -> tuple[int, int]:
         """Prefill a prompt (1-D ids) into a free slot -> (slot, first generated id)."""
+        return self.add_many([prompt_ids])[0]
+
+    @torch.no_grad()
+    def add_many(self, prompts) -> list[tuple[int, int]]:
+        """Prefill several prompts into free slots -> [(slot, first generated id)]."""
         free = self.free_slots()
-        if not free:
+        if len(free) < len(prompts):
             raise RuntimeError("no free slot")
-        ids = torch.as_tensor(prompt_ids, dtype=torch.int64).reshape(1, -1)
-        if ids.shape[1] < 1:
-            raise ValueError("input sequence cannot be empty")
-        if ids.shape[1] >= self.model.config.max_sequence_length:
-            raise ValueError("input exceeds max_sequence_length")
-        b = free[0]
-        for c in self.cache:
-            c.lengths[b] = 0
-        views = [c._row_view(b) for c in self.cache]
-        logits = self.model.forward(ids.to(self.model.device), views, 0, last_only=True)
-        tok = self._select(logits.view(1, -1))
-        n = ids.shape[1]
-        for c in self.cache:
-            c.lengths[b] = n
-            c.length = max(c.lengths)
-        self.lengths[b] = n
-        self.active[b] = True
-        self.last[b:b + 1] = tok
-        self.seq_pos[b] = n
-        self.active_dev[b] = 1
-        return b, int(tok.item())
+        prompts = [self._host_ids(p, start=1) for p in prompts]  # room for one generated token at least
+        slots = free[: len(prompts)]
+        out = []
+        for b, logits in zip(slots, self._prefill(slots, prompts)):
+            tok = self._select(logits.reshape(1, -1))
+            self.last[b:b + 1] = tok
+            out.append((b, int(tok.item())))
+        return out
+
+    @torch.no_grad()
+    def feed(self, entries) -> list[tuple[int, torch.Tensor]]:
+        """One step over GIVEN tokens instead of selected ones: ``entries`` holds (slot, ids), slot None for a sequence that
+        starts -> [(slot, logits (len(ids), V))] in the same order.  One id for each active slot runs the decode step of
+        ``step``; anything else runs the prompt path, all entries in one call where the model takes tokens of different
+        slots and lengths.  The next ``step`` continues from the last of the ids fed and the token after it is the
+        caller's to select."""
+        entries = [(b, self._host_ids(ids, 0 if b is None else self.lengths[b])) for b, ids in entries]
+        named = [b for b, _ in entries if b is not None]
+        if any(not self.active[b] for b in named) or len(set(named)) != len(named):
+            raise ValueError("entries must name distinct active slots")
+        free = iter(self.free_slots())
+        if len(entries) - len(named) > len(self.free_slots()):
+            raise RuntimeError("no free slot")
+        fresh = [b is None for b, _ in entries]
+        slots = [next(free) if b is None else b for b, _ in entries]
+        tokens = [ids for _, ids in entries]
+        if all(fresh):
+            out = self._prefill(slots, tokens, last_only=False)
+        elif not any(fresh) and all(len(t) == 1 for t in tokens) and sorted(slots) == [b for b in range(self.slots) if self.active[b]]:
+            for b, t in zip(slots, tokens):
+                self.last[b] = int(t)
+            logits = self._device_forward()
+            out = [logits[b] for b in slots]
+            for c in self.cache:
+                c.lengths = list(self.lengths)
+            for b in slots:
+                self._book(b, self.lengths[b] + 1)
+        elif getattr(self.model, "supports_seq_lens", False):
+            for b, new in zip(slots, fresh):
+                if new:
+                    self._book(b, 0)
+            logits = self._padded_forward(slots, tokens, False)
+            out = [row[: len(t)] for row, t in zip(logits, tokens)]
+            for b, t in zip(slots, tokens):
+                self._book(b, self.lengths[b] + len(t))
+        else:
+            raise ValueError("this model cannot mix prompts and continued sequences in one step")
+        return list(zip(slots, out))
 
     def remove(self, slot: int) -> None:
         self.active[slot] = False
@@ -84,11 +163,15 @@ class ContinuousBatcher:
         for c in self.cache:
             c.lengths[slot] = 0
 
+    def _device_forward(self) -> torch.Tensor:
+        """Logits (slots, 1, V) of the fed ids at the slots' own positions."""
+        return self.model.forward(self.last.view(self.slots, 1), self.cache, list(self.lengths), last_only=True,
+                                  seq_pos=self.seq_pos)
+
     def _device_step(self) -> None:
         """Everything of a step that runs on the device, with no host synchronisation: forward at
         the slots' own positions, selection, position advance, next inputs.  Capturable."""
-        logits = self.model.forward(self.last.view(self.slots, 1), self.cache, list(self.lengths), last_only=True,
-                                    seq_pos=self.seq_pos)
+        logits = self._device_forward()
         vv = self.valid_vocab or None
         if self.sampling is None:
             ops.argmax(logits.view(self.slots, -1), valid_vocab=vv, next_ids=self._toks)

@@ -18,6 +18,10 @@ INCLUDE = os.path.join(os.path.dirname(HERE), "include")
 LIB_DIR = os.path.join(HERE, "lib")
 OBJ_DIR = os.path.join(LIB_DIR, "obj")
 LIB_PATH = os.path.join(LIB_DIR, "libohara_decode.so")
+# A library of fewer sources for programs that serve one kind of model from a fresh checkout (``ensure``): the same
+# entry points, those of other models absent.
+PARTIAL_LIB_PATH = os.path.join(LIB_DIR, "libohara_serving.so")
+SERVING = ("attention_bias", "delta_rule", "gemm_f32", "gemm_skinny", "gemm_tile", "misc", "residual_norm", "sampler")
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = [
@@ -50,12 +54,16 @@ def _run(cmd: list[str]) -> str:
     return err
 
 
-def build_library(verbose: bool = False, incremental: bool = False, jobs: int = 8) -> str:
-    """One object per source (compiled in parallel), then one link."""
+def build_library(verbose: bool = False, incremental: bool = False, jobs: int = 8, only=None) -> str:
+    """One object per source (compiled in parallel), then one link.  ``only``: the names of the sources to build into
+    the partial library instead of all of them into the full one."""
     os.makedirs(OBJ_DIR, exist_ok=True)
     hdr = _headers_mtime()
     todo, objs = [], []
+    target = LIB_PATH if only is None else PARTIAL_LIB_PATH
     for src in sources():
+        if only is not None and os.path.basename(src)[:-4] not in only:
+            continue
         obj = os.path.join(OBJ_DIR, os.path.basename(src)[:-4] + ".o")
         objs.append(obj)
         fresh = (incremental and os.path.exists(obj) and os.path.getmtime(obj) >= os.path.getmtime(src)
@@ -64,12 +72,25 @@ def build_library(verbose: bool = False, incremental: bool = False, jobs: int = 
             todo.append((src, obj))
     with ThreadPoolExecutor(max_workers=max(1, jobs)) as pool:
         errs = list(pool.map(lambda so: _run([HIPCC, *FLAGS, "-c", so[0], "-o", so[1]]), todo))
-    errs.append(_run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", LIB_PATH]))
+    part = f"{target}.{os.getpid()}"
+    errs.append(_run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", part]))
+    os.replace(part, target)
     if verbose:
         for e in errs:
             if e.strip():
                 print(e, file=sys.stderr)
-    return LIB_PATH
+    return target
+
+
+def ensure(only) -> str:
+    """The full library if it is built, else the partial one with the sources ``only``, built now if it is missing or older than its sources."""
+    if os.path.exists(LIB_PATH):
+        return LIB_PATH
+    srcs = [s for s in sources() if os.path.basename(s)[:-4] in only]
+    newest = max(_headers_mtime(), *(os.path.getmtime(s) for s in srcs))
+    if not os.path.exists(PARTIAL_LIB_PATH) or os.path.getmtime(PARTIAL_LIB_PATH) < newest:
+        build_library(incremental=True, only=only)
+    return PARTIAL_LIB_PATH
 
 
 if __name__ == "__main__":

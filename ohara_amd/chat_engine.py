@@ -113,7 +113,7 @@ class ChatEngine:
             )
         if device is None:
             device = "cuda"
-        model = build_model(config, state, device=device)
+        model = build_model(config, state, device=device, dtype=dtype or torch.bfloat16)
         return cls(model, tokenizer, device=device, dtype=dtype, renderer=renderer, stop_ids=stop_ids)
 
     def metadata(self, checkpoint_path=None) -> dict[str, Any]:

@@ -124,9 +124,25 @@ def loop_moe_config(config: Config) -> Config:
     return replace(config, moe_grouped=True, moe_num_shared_experts=0, moe_normalize_weights=False)
 
 
+# Designs other than the reference's Llama, by the "architecture" of their config.json: module and names of the
+# config class (``from_dict``) and of the model class (config, state dict, device, dtype).
+ARCHITECTURES = {
+    "Povazen": ("povazen", "PovazenConfig", "Povazen"),
+}
+
+
+def _architecture(name: str):
+    from importlib import import_module
+
+    module, config_cls, model_cls = ARCHITECTURES[name]
+    module = import_module(f".{module}", __package__)
+    return getattr(module, config_cls), getattr(module, model_cls)
+
+
 def load_checkpoint(path, *, moe_experts_per_tok: int = 2, moe_gate_fn: str = "softmax",
-                    moe_normalize_weights: bool = True):
-    """-> (Config, state dict).  ``path`` is a ``.pt`` file holding a state dict (bare or under
+                    moe_normalize_weights: bool = True, max_sequence_length: int | None = None):
+    """-> (config, state dict).  A ``config.json`` that names an "architecture" (``ARCHITECTURES``) gives that design's
+    config, with caches of ``max_sequence_length`` tokens if given.  ``path`` is a ``.pt`` file holding a state dict (bare or under
     ``"model"``, chat_engine.py:307-308), a ``.safetensors`` file, or a directory with
     ``model.safetensors`` + ``config.json`` (export_safetensors.py:95-111)."""
     path = Path(path)
@@ -147,6 +163,8 @@ def load_checkpoint(path, *, moe_experts_per_tok: int = 2, moe_gate_fn: str = "s
         state = clean_state_dict(blob.get("model", blob))
     if cfg_json is not None and cfg_json.exists():
         payload = json.loads(cfg_json.read_text(encoding="utf-8"))
+        if payload.get("architecture") in ARCHITECTURES:
+            return _architecture(payload["architecture"])[0].from_dict(payload, max_sequence_length), state
         names = {f.name for f in fields(Config)}
         config = Config(**{k: v for k, v in payload.items() if k in names})
         if "vocab_proj.weight" not in state and config.weight_tying:  # the export drops aliases
@@ -157,8 +175,14 @@ def load_checkpoint(path, *, moe_experts_per_tok: int = 2, moe_gate_fn: str = "s
     return config, state
 
 
-def build_model(config: Config, state: Mapping[str, torch.Tensor], device="cuda"):
-    """The kernel-backed model for a config: dense ``Llama`` or ``MoeLlama``."""
+def build_model(config, state: Mapping[str, torch.Tensor], device="cuda", dtype=torch.bfloat16):
+    """The kernel-backed model for a config: dense ``Llama``, ``MoeLlama`` or a design of ``ARCHITECTURES``."""
+    for name in ARCHITECTURES:
+        config_cls, model_cls = _architecture(name)
+        if isinstance(config, config_cls):
+            return model_cls(config, dict(state), device=device, dtype=dtype)
+    if dtype != torch.bfloat16:
+        raise ValueError("ohara_amd runs the decode path in bfloat16 only")
     if config.moe_num_experts > 0:
         from .moe import MoeLlama
 

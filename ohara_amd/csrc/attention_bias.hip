@@ -1,0 +1,576 @@
+// Attention over the KV cache with a linear distance bias, norms over whole projections and a gate per head.
+//
+//   qkv_norm_append   q and k over the root mean square of the whole projection row, values over each head's,
+//                     keys and values into the cache: a workgroup per token
+//   attn_bias_kernel  one query token per workgroup (decode; any head width up to 256; bf16 or fp32)
+//   attn_bias_prefill many query tokens on bf16 MFMA
+//
+// Scores, softmax weights and sums are fp32.  In the MFMA kernel q and the cached rows are bf16 as stored, so
+// q.k is an fp32 sum of exact products; the second product keeps the fp32 weights by splitting each into
+// three bf16 terms (8 + 8 + 8 significant bits) that are multiplied one after another.
+#include "hybrid.h"
+
+namespace {
+
+// ---- front end -----------------------------------------------------------------------------
+template <typename T>
+struct FrontArgs {
+  const T* p;
+  const float* qn;
+  const float* kn;
+  T* q;
+  T* kc;
+  T* vc;
+  int ldp, H, G, D, V, Tmax;
+  float eps;
+  OharaSeq seq;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void qkv_norm_append_kernel(FrontArgs<T> a) {
+  __shared__ float red[2][4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int row = blockIdx.x, b = row / a.seq.seq_len, s = row - b * a.seq.seq_len;
+  const int pos = seq_start(a.seq, b) + s;
+  if (s >= seq_tokens(a.seq, b) || pos < 0 || pos >= a.Tmax) return;
+  const int nq = a.H * a.D, nk = a.G * a.D;
+  const int Dp = (a.D + 7) & ~7, Vp = (a.V + 7) & ~7;
+  const T* p = a.p + (size_t)row * a.ldp;
+  const bool vec = ((a.D | a.V | a.ldp) & 3) == 0;
+  float sq = 0.f, sk = 0.f;
+  if (vec) {
+    for (int i = tid * 4; i < nq + nk; i += 1024) {
+      float v[4];
+      ld4(p + i, v);
+      const float t = ((v[0] * v[0] + v[1] * v[1]) + v[2] * v[2]) + v[3] * v[3];
+      if (i < nq) sq += t;
+      else sk += t;
+    }
+  } else {
+    for (int i = tid; i < nq + nk; i += 256) {
+      const float v = ldv(p + i);
+      if (i < nq) sq += v * v;
+      else sk += v * v;
+    }
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if (lane == 0) {
+    red[0][wave] = sq;
+    red[1][wave] = sk;
+  }
+  __syncthreads();
+  const float iq = 1.0f / sqrtf((((red[0][0] + red[0][1]) + red[0][2]) + red[0][3]) / (float)nq + a.eps);
+  const float ik = 1.0f / sqrtf((((red[1][0] + red[1][1]) + red[1][2]) + red[1][3]) / (float)nk + a.eps);
+  T* qo = a.q + (size_t)row * a.H * Dp;
+  const size_t crow = (size_t)seq_slot(a.seq, b) * a.Tmax + pos;
+  T* ko = a.kc + crow * a.G * Dp;
+  T* vo = a.vc + crow * a.G * Vp;
+  if (vec) {
+    for (int i = tid * 4; i < nq + nk; i += 1024) {
+      const bool isq = i < nq;
+      const int j = isq ? i : i - nq, h = j / a.D, c = j - h * a.D;
+      float v[4], w[4];
+      ld4(p + i, v);
+      ld4((isq ? a.qn : a.kn) + j, w);
+      const float r = isq ? iq : ik;
+#pragma unroll
+      for (int u = 0; u < 4; ++u) v[u] = v[u] * r * w[u];
+      st4((isq ? qo : ko) + h * Dp + c, v);
+    }
+  } else {
+    for (int i = tid; i < nq + nk; i += 256) {
+      const bool isq = i < nq;
+      const int j = isq ? i : i - nq, h = j / a.D, c = j - h * a.D;
+      stv((isq ? qo : ko) + h * Dp + c, ldv(p + i) * (isq ? iq : ik) * (isq ? a.qn : a.kn)[j]);
+    }
+  }
+  if (Dp > a.D) {
+    const int pad = Dp - a.D;
+    for (int i = tid; i < (a.H + a.G) * pad; i += 256) {
+      const int h = i / pad, c = a.D + i - h * pad;
+      stv((h < a.H ? qo + h * Dp : ko + (h - a.H) * Dp) + c, 0.f);
+    }
+  }
+  const T* pv = p + nq + nk;
+  for (int g = wave; g < a.G; g += 4) {  // V <= 256: up to four values per lane
+    float v[4], sv = 0.f;
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int c = lane + 64 * u;
+      v[u] = c < a.V ? ldv(pv + g * a.V + c) : 0.f;
+      sv += v[u] * v[u];
+    }
+    const float iv = 1.0f / sqrtf(wave_sum(sv) / (float)a.V + a.eps);
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int c = lane + 64 * u;
+      if (c < Vp) stv(vo + g * Vp + c, v[u] * iv);
+    }
+  }
+}
+
+// ---- one query token per workgroup -----------------------------------------------------------
+template <typename T>
+struct AttnBiasArgs {
+  const T* q;
+  const T* kc;
+  const T* vc;
+  const T* gate;
+  const float* slopes;
+  T* out;
+  int H, G, D, V, Tmax, ldg, ldo;
+  int rb, nhb;     // query heads served together (at most RB) and such sets per KV head
+  int ns;
+  float scale;
+  float* ws;       // ns > 1: per (row, head, chunk) Vp + 2 floats {weighted sum, max, sum}
+  int* counters;   // ns > 1: per (row, KV head, head set) chunks finished; zero between calls
+  OharaSeq seq;
+};
+
+// LP lanes own one cached position (lane l elements 8l .. 8l+7 of key and value), so a workgroup walks 256 / LP
+// positions per round with an online softmax per lane group and query head; the groups are merged through LDS.
+// Scores are in log2 units.
+template <typename T, int LP, int RB>
+__global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
+  constexpr int NG = 256 / LP, W = 8 * LP;
+  __shared__ float gm[RB][NG], gl[RB][NG];
+  __shared__ float gacc[RB][NG][W];
+  __shared__ int is_last;
+  const int tid = threadIdx.x, l = tid % LP, grp = tid / LP;
+  const int Dp = (a.D + 7) & ~7, Vp = (a.V + 7) & ~7;
+  int w = blockIdx.x;
+  const int hb = w % a.nhb; w /= a.nhb;
+  const int g = w % a.G;
+  const int row = w / a.G;
+  const int b = row / a.seq.seq_len, s = row - b * a.seq.seq_len;
+  const int pq = seq_start(a.seq, b) + s;
+  if (hb == 0 && g == 0 && blockIdx.y == 0)
+    for (int i = a.H * a.V + tid; i < a.ldo; i += 256) stv(a.out + (size_t)row * a.ldo + i, 0.f);
+  if (s >= seq_tokens(a.seq, b) || pq < 0 || pq >= a.Tmax) return;  // the same for every chunk of the row
+  const int rep = a.H / a.G;
+  const int h0 = g * rep + hb * a.rb, nh = min(a.rb, rep - hb * a.rb);
+
+  const int e0 = 8 * l;
+  const bool ownk = e0 < Dp, ownv = e0 < Vp;
+  const float sl2 = a.scale * OHARA_LOG2E;
+  float qr[RB][8], slope[RB];
+#pragma unroll
+  for (int r = 0; r < RB; ++r) {
+    const int h = h0 + min(r, nh - 1);
+    slope[r] = a.slopes[h] * OHARA_LOG2E;
+    Raw8<T> v;
+    v.load(a.q + ((size_t)row * a.H + h) * Dp + (ownk ? e0 : 0));
+    v.get(qr[r]);
+#pragma unroll
+    for (int u = 0; u < 8; ++u) qr[r][u] = ownk ? qr[r][u] : 0.f;
+  }
+  float m[RB], lsum[RB], acc[RB][8];
+#pragma unroll
+  for (int r = 0; r < RB; ++r) {
+    m[r] = -INFINITY;
+    lsum[r] = 0.f;
+#pragma unroll
+    for (int u = 0; u < 8; ++u) acc[r][u] = 0.f;
+  }
+  // lanes past a row's end read its first elements: their products are zeroed (keys) or never stored (values)
+  const size_t kd = (size_t)a.G * Dp, vd = (size_t)a.G * Vp, base = (size_t)seq_slot(a.seq, b) * a.Tmax;
+  const T* kb = a.kc + base * kd + (size_t)g * Dp + (ownk ? e0 : 0);
+  const T* vb = a.vc + base * vd + (size_t)g * Vp + (ownv ? e0 : 0);
+  int t_lo = 0, t_hi = pq;
+  if (a.ns > 1) {
+    const int per = ((pq + a.ns) / a.ns + NG - 1) / NG * NG;  // ceil((pq + 1) / ns) in whole rounds
+    t_lo = blockIdx.y * per;
+    t_hi = min(pq, t_lo + per - 1);
+  }
+  constexpr int R = 2;  // positions a lane group has in flight
+  for (int t = t_lo + grp; t <= t_hi; t += NG * R) {
+    Raw8<T> kv[R], vv[R];
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+      const int tt = min(t + NG * i, t_hi);
+      kv[i].load(kb + (size_t)tt * kd);
+      vv[i].load(vb + (size_t)tt * vd);
+    }
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+      const int tt = t + NG * i;
+      if (tt > t_hi) break;  // uniform within the lane group
+      float k[8], v[8];
+      kv[i].get(k);
+      vv[i].get(v);
+      const float dist = (float)(pq - tt);
+#pragma unroll
+      for (int r = 0; r < RB; ++r) {
+        float dot = 0.f;
+#pragma unroll
+        for (int u = 0; u < 8; ++u) dot = __builtin_fmaf(k[u], qr[r][u], dot);
+        dot = lanes_sum<LP / 2, 1>(dot);
+        const float sc = dot * sl2 - slope[r] * dist;
+        const float mn = fmaxf(m[r], sc);
+        const float corr = __builtin_amdgcn_exp2f(m[r] - mn), p = __builtin_amdgcn_exp2f(sc - mn);
+        lsum[r] = lsum[r] * corr + p;
+#pragma unroll
+        for (int u = 0; u < 8; ++u) acc[r][u] = acc[r][u] * corr + p * v[u];
+        m[r] = mn;
+      }
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < RB; ++r) {
+    if (l == 0) {
+      gm[r][grp] = m[r];
+      gl[r][grp] = lsum[r];
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u) gacc[r][grp][e0 + u] = acc[r][u];
+  }
+  __syncthreads();
+  for (int i = tid; i < nh * a.V; i += 256) {
+    const int r = i / a.V, c = i - r * a.V, h = h0 + r;
+    float M = -INFINITY;
+    for (int n = 0; n < NG; ++n) M = fmaxf(M, gm[r][n]);
+    float num = 0.f, den = 0.f;
+    for (int n = 0; n < NG; ++n) {
+      if (gm[r][n] == -INFINITY) continue;  // a group that saw no position
+      const float wg = __builtin_amdgcn_exp2f(gm[r][n] - M);
+      num += wg * gacc[r][n][c];
+      den += wg * gl[r][n];
+    }
+    if (a.ns > 1) {
+      // write-through stores: the workgroup that merges may sit on another XCD
+      float* o = a.ws + (((size_t)row * a.H + h) * a.ns + blockIdx.y) * (Vp + 2);
+      st_coh4(o + c, __float_as_uint(num));
+      if (c == 0) {
+        st_coh4(o + Vp, __float_as_uint(M));  // -inf: this chunk lies past the query's position
+        st_coh4(o + Vp + 1, __float_as_uint(den));
+      }
+    } else {
+      const float gt = a.gate ? sigmoid_x(ldv(a.gate + (size_t)row * a.ldg + h)) : 1.0f;
+      stv(a.out + (size_t)row * a.ldo + h * a.V + c, num / den * gt);
+    }
+  }
+  if (a.ns == 1) return;
+  // the workgroup that finishes last merges the chunks in chunk order
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup");
+  wait_own_stores();
+  __syncthreads();
+  int* counter = a.counters + ((size_t)row * a.G + g) * a.nhb + hb;
+  if (tid == 0) {
+    const int old = __hip_atomic_fetch_add(counter, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    is_last = old == a.ns - 1;
+    if (is_last) __hip_atomic_store(counter, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // ready for the next call
+  }
+  __syncthreads();
+  if (!is_last) return;
+  // chunk maxima and sums into LDS (ns <= 64 = at most RB * 64 pairs)
+  float* cm = &gacc[0][0][0];  // RB * NG * W >= 2 * RB * 64 floats
+  float* cl = cm + RB * 64;
+  for (int i = tid; i < nh * a.ns; i += 256) {
+    const int r = i / a.ns, c = i - r * a.ns;
+    const float* o = a.ws + (((size_t)row * a.H + h0 + r) * a.ns + c) * (Vp + 2);
+    cm[r * 64 + c] = __uint_as_float(ld_coh4(o + Vp));
+    cl[r * 64 + c] = __uint_as_float(ld_coh4(o + Vp + 1));
+  }
+  __syncthreads();
+  for (int i = tid; i < nh * a.V; i += 256) {
+    const int r = i / a.V, c = i - r * a.V, h = h0 + r;
+    const float* o = a.ws + ((size_t)row * a.H + h) * a.ns * (Vp + 2) + c;
+    float M = -INFINITY;
+    for (int n = 0; n < a.ns; ++n) M = fmaxf(M, cm[r * 64 + n]);
+    float num = 0.f, den = 0.f;
+    for (int n0 = 0; n0 < a.ns; n0 += 16) {  // sixteen chunks' values in flight, every load unconditional
+      float av[16];
+#pragma unroll
+      for (int n = 0; n < 16; ++n) av[n] = __uint_as_float(ld_coh4(o + (size_t)min(n0 + n, a.ns - 1) * (Vp + 2)));
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int n = 0; n < 16; ++n) {
+        if (n0 + n >= a.ns || cm[r * 64 + n0 + n] == -INFINITY) continue;
+        const float wg = __builtin_amdgcn_exp2f(cm[r * 64 + n0 + n] - M);
+        num += wg * av[n];
+        den += wg * cl[r * 64 + n0 + n];
+      }
+    }
+    const float gt = a.gate ? sigmoid_x(ldv(a.gate + (size_t)row * a.ldg + h)) : 1.0f;
+    stv(a.out + (size_t)row * a.ldo + h * a.V + c, num / den * gt);
+  }
+}
+
+// ---- many query tokens: bf16 MFMA --------------------------------------------------------------
+// A workgroup (4 waves) owns 64 queries of one (sequence, head), a wave 16 of them; keys and values come
+// through LDS in tiles of 64 positions, the values transposed.  Both products are formed transposed,
+// S^T = K Q^T and O^T = V^T P^T, so a lane's scores belong to one query and its weights are, register for register,
+// the B operand of the second product (k-slot 8 g + i of window w <-> position 32 w + 4 g + i for i < 4,
+// 32 w + 16 + 4 g + i - 4 otherwise).
+template <int DP, int VP>
+__global__ __launch_bounds__(256, (DP + VP > 384 ? 1 : 2)) void attn_bias_prefill_kernel(AttnBiasArgs<bf16_t> a, int nqb) {
+  constexpr int KT = 64, NK = DP / 32, ND = VP / 16;
+  constexpr int LDK = DP + 8, LDV = KT + 4;
+  constexpr int CK = DP / 8, CV = VP / 8;            // 16-byte pieces per row
+  constexpr int NPK = KT * CK / 256, NPV = KT * CV / 256;
+  __shared__ __align__(16) bf16_t Ks[KT][LDK];
+  __shared__ __align__(16) bf16_t Vt[VP][LDV];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int m = lane & 15, g = lane >> 4;
+  const int qblk = nqb - 1 - (int)blockIdx.x;  // long contexts first
+  const int h = blockIdx.y, b = blockIdx.z;
+  const int len = seq_tokens(a.seq, b), pos0 = seq_start(a.seq, b);
+  const int q0 = qblk * 64;
+  // (padding: nothing but zeros in the columns past h*V, and those only matter for live rows)
+  if (q0 >= len || pos0 < 0 || pos0 + len > a.Tmax) return;
+  const int Dq = (a.D + 7) & ~7, Vq = (a.V + 7) & ~7;
+  const int kvh = h / (a.H / a.G);
+  const size_t kd = (size_t)a.G * Dq, vd = (size_t)a.G * Vq, base = (size_t)seq_slot(a.seq, b) * a.Tmax;
+  const bf16_t* kb = a.kc + base * kd + (size_t)kvh * Dq;
+  const bf16_t* vb = a.vc + base * vd + (size_t)kvh * Vq;
+  const int Lall = pos0 + len;
+  const int kv_end = min(pos0 + q0 + 64, Lall);
+  const int wq0 = q0 + wave * 16, qi = wq0 + m;
+  const int qpos = pos0 + min(qi, len - 1);   // lanes past the end repeat the last query and are not stored
+  const int wave_last = min(pos0 + wq0 + 15, Lall - 1);
+  const float sl2 = a.scale * OHARA_LOG2E, slope = a.slopes[h] * OHARA_LOG2E;
+  const size_t qrow = (size_t)b * a.seq.seq_len + min(qi, len - 1);
+
+  uint4 qf[NK];
+#pragma unroll
+  for (int j = 0; j < NK; ++j)
+    qf[j] = 32 * j + 8 * g < Dq ? ldg16(a.q + (qrow * a.H + h) * Dq + 32 * j + 8 * g) : make_uint4(0, 0, 0, 0);
+
+  f32x4 o[ND];
+#pragma unroll
+  for (int t = 0; t < ND; ++t) o[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float mrun = -INFINITY, lrun = 0.f;
+
+  uint4 kr[NPK], vr[NPV];
+  auto load_tile = [&](int t0) {
+#pragma unroll
+    for (int i = 0; i < NPK; ++i) {
+      const int idx = tid + 256 * i, p = idx / CK, c = idx % CK;
+      kr[i] = (t0 + p < Lall && 8 * c < Dq) ? ldg16(kb + (size_t)(t0 + p) * kd + 8 * c) : make_uint4(0, 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < NPV; ++i) {
+      // neighbouring threads take neighbouring positions of the same columns: the transposed writes spread over banks
+      const int idx = tid + 256 * i, p = idx % KT, c = idx / KT;
+      vr[i] = (t0 + p < Lall && 8 * c < Vq) ? ldg16(vb + (size_t)(t0 + p) * vd + 8 * c) : make_uint4(0, 0, 0, 0);
+    }
+  };
+  auto store_tile = [&]() {
+#pragma unroll
+    for (int i = 0; i < NPK; ++i) {
+      const int idx = tid + 256 * i;
+      *reinterpret_cast<uint4*>(&Ks[idx / CK][8 * (idx % CK)]) = kr[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NPV; ++i) {
+      const int idx = tid + 256 * i, p = idx % KT, c = 8 * (idx / KT);
+      const uint32_t w[4] = {vr[i].x, vr[i].y, vr[i].z, vr[i].w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        Vt[c + 2 * e][p] = (bf16_t)(w[e] & 0xffffu);
+        Vt[c + 2 * e + 1][p] = (bf16_t)(w[e] >> 16);
+      }
+    }
+  };
+
+  load_tile(0);
+  for (int t0 = 0; t0 < kv_end; t0 += KT) {
+    __syncthreads();  // everyone is done with the previous tile
+    store_tile();
+    __syncthreads();
+    if (t0 + KT < kv_end) load_tile(t0 + KT);  // in flight during the products
+    if (t0 > wave_last) continue;               // wholly masked for this wave (barriers stay uniform)
+    f32x4 s[4];
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk) {
+      s[kk] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < NK; ++j)
+        s[kk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(&Ks[kk * 16 + m][32 * j + 8 * g])),
+            __builtin_bit_cast(bf16x8, qf[j]), s[kk], 0, 0, 0);
+    }
+    float tmax = -INFINITY;
+    const float rel = (float)(t0 + 4 * g - qpos);  // -(distance) of the lane's first position
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        float v = s[kk][i] * sl2 + slope * (rel + (float)(16 * kk + i));
+        if (t0 + 16 * kk + 4 * g + i > qpos) v = -INFINITY;
+        s[kk][i] = v;
+        tmax = fmaxf(tmax, v);
+      }
+    tmax = lane_xor_max<32>(lane_xor_max<16>(tmax));
+    const float mn = fmaxf(mrun, tmax);  // finite: position 0 is visible to every query
+    const float corr = __builtin_amdgcn_exp2f(mrun - mn);
+    mrun = mn;
+    float ts = 0.f;
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        s[kk][i] = __builtin_amdgcn_exp2f(s[kk][i] - mn);
+        ts += s[kk][i];
+      }
+    lrun = lrun * corr + ts;  // this lane's share; the four lane groups are added at the end
+    if (__any(corr != 1.0f)) {
+#pragma unroll
+      for (int t = 0; t < ND; ++t)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[t][i] *= corr;
+    }
+#pragma unroll
+    for (int w = 0; w < 2; ++w) {
+      // three bf16 terms per weight: p = hi + mid + lo exactly
+      uint32_t hi[4], mid[4], lo[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float p0 = s[2 * w + (e >> 1)][2 * (e & 1)], p1 = s[2 * w + (e >> 1)][2 * (e & 1) + 1];
+        hi[e] = pack_bf(p0, p1);
+        const float r0 = p0 - lo_bf(hi[e]), r1 = p1 - hi_bf(hi[e]);
+        mid[e] = pack_bf(r0, r1);
+        lo[e] = pack_bf(r0 - lo_bf(mid[e]), r1 - hi_bf(mid[e]));
+      }
+      const bf16x8 ph = __builtin_bit_cast(bf16x8, make_uint4(hi[0], hi[1], hi[2], hi[3]));
+      const bf16x8 pm = __builtin_bit_cast(bf16x8, make_uint4(mid[0], mid[1], mid[2], mid[3]));
+      const bf16x8 pl = __builtin_bit_cast(bf16x8, make_uint4(lo[0], lo[1], lo[2], lo[3]));
+#pragma unroll
+      for (int t = 0; t < ND; ++t) {
+        const uint2 v0 = *reinterpret_cast<const uint2*>(&Vt[16 * t + m][32 * w + 4 * g]);
+        const uint2 v1 = *reinterpret_cast<const uint2*>(&Vt[16 * t + m][32 * w + 16 + 4 * g]);
+        const bf16x8 vf = __builtin_bit_cast(bf16x8, make_uint4(v0.x, v0.y, v1.x, v1.y));
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph, o[t], 0, 0, 0);
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pm, o[t], 0, 0, 0);
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, o[t], 0, 0, 0);
+      }
+    }
+  }
+  lrun = lane_xor_sum<32>(lane_xor_sum<16>(lrun));
+  if (qi >= len) return;
+  const float gt = a.gate ? sigmoid_x(ldv(a.gate + qrow * a.ldg + h)) : 1.0f;
+  const float inv = gt / lrun;
+  bf16_t* orow = a.out + qrow * a.ldo;
+#pragma unroll
+  for (int t = 0; t < ND; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int c = 16 * t + 4 * g + i;
+      if (c < a.V) orow[(size_t)h * a.V + c] = f2bf(o[t][i] * inv);
+    }
+  if (h == 0 && g == 0)
+    for (int i = a.H * a.V; i < a.ldo; ++i) orow[i] = 0;
+}
+
+template <int DP>
+int launch_prefill_v(const AttnBiasArgs<bf16_t>& a, dim3 grid, int nqb, hipStream_t st) {
+  if (a.V <= 32) hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, 32>), grid, dim3(256), 0, st, a, nqb);
+  else if (a.V <= 64) hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, 64>), grid, dim3(256), 0, st, a, nqb);
+  else if (a.V <= 128) hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, 128>), grid, dim3(256), 0, st, a, nqb);
+  else hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, 256>), grid, dim3(256), 0, st, a, nqb);
+  return ohara_launch_status();
+}
+
+int launch_prefill(const AttnBiasArgs<bf16_t>& a, hipStream_t st) {
+  const int nqb = (a.seq.seq_len + 63) / 64;
+  const dim3 grid((unsigned)nqb, (unsigned)a.H, (unsigned)a.seq.batch);
+  if (a.D <= 32) return launch_prefill_v<32>(a, grid, nqb, st);
+  if (a.D <= 64) return launch_prefill_v<64>(a, grid, nqb, st);
+  if (a.D <= 128) return launch_prefill_v<128>(a, grid, nqb, st);
+  return launch_prefill_v<256>(a, grid, nqb, st);
+}
+
+template <typename T>
+int launch_front(const FrontArgs<T>& a, hipStream_t st) {
+  if (!a.p || !a.qn || !a.kn || !a.q || !a.kc || !a.vc || !seq_ok(&a.seq)) return OHARA_EINVAL;
+  if (a.H < 1 || a.G < 1 || a.H % a.G || a.D < 1 || a.V < 1 || a.Tmax < 1) return OHARA_EINVAL;
+  if (a.D > 256 || a.V > 256) return OHARA_ESIZE;
+  if (a.ldp < a.H * a.D + a.G * (a.D + a.V)) return OHARA_EINVAL;
+  if (!a.seq.pos_dev && a.seq.pos + a.seq.seq_len > a.Tmax) return OHARA_EINVAL;
+  hipLaunchKernelGGL((qkv_norm_append_kernel<T>), dim3((unsigned)(a.seq.batch * a.seq.seq_len)), dim3(256), 0, st, a);
+  return ohara_launch_status();
+}
+
+template <typename T, int LP>
+int launch_bias_rb(AttnBiasArgs<T> a, hipStream_t st) {
+  const int rep = a.H / a.G;
+  a.rb = rep >= 4 ? 4 : (rep >= 2 ? 2 : 1);
+  a.nhb = (rep + a.rb - 1) / a.rb;
+  const int64_t gx = (int64_t)a.seq.batch * a.seq.seq_len * a.G * a.nhb;
+  if (gx > INT32_MAX) return OHARA_ESIZE;
+  const dim3 grid((unsigned)gx, (unsigned)a.ns);
+  if (a.rb == 4) hipLaunchKernelGGL((attn_bias_kernel<T, LP, 4>), grid, dim3(256), 0, st, a);
+  else if (a.rb == 2) hipLaunchKernelGGL((attn_bias_kernel<T, LP, 2>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((attn_bias_kernel<T, LP, 1>), grid, dim3(256), 0, st, a);
+  return ohara_launch_status();
+}
+
+template <typename T>
+int launch_bias(AttnBiasArgs<T> a, void* workspace, hipStream_t st) {
+  if (!a.q || !a.kc || !a.vc || !a.slopes || !a.out || !seq_ok(&a.seq)) return OHARA_EINVAL;
+  if (a.H < 1 || a.G < 1 || a.H % a.G || a.D < 1 || a.V < 1 || a.Tmax < 1) return OHARA_EINVAL;
+  if (a.D > 256 || a.V > 256) return OHARA_ESIZE;
+  if (a.ldo < a.H * a.V || (a.gate && a.ldg < 1)) return OHARA_EINVAL;
+  if (!a.seq.pos_dev && a.seq.pos + a.seq.seq_len > a.Tmax) return OHARA_EINVAL;
+  if (a.ns < 1 || a.ns > 64 || (a.ns > 1 && (!workspace || a.seq.seq_len != 1))) return OHARA_EINVAL;
+  const size_t cbytes = (((size_t)a.seq.batch * a.H * sizeof(int)) + 255) & ~(size_t)255;
+  a.counters = reinterpret_cast<int*>(workspace);
+  a.ws = reinterpret_cast<float*>(reinterpret_cast<char*>(workspace) + cbytes);
+  if constexpr (sizeof(T) == 2) {
+    if (a.seq.seq_len >= 16 && a.H <= 65535 && a.seq.batch <= 65535) return launch_prefill(a, st);
+  }
+  const int w = a.D > a.V ? a.D : a.V;
+  if (w <= 64) return launch_bias_rb<T, 8>(a, st);
+  if (w <= 128) return launch_bias_rb<T, 16>(a, st);
+  return launch_bias_rb<T, 32>(a, st);
+}
+
+}  // namespace
+
+extern "C" {
+
+int ohara_qkv_norm_append_bf16(const uint16_t* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn,
+                               const float* kn, float eps, uint16_t* q_out, uint16_t* kcache, uint16_t* vcache, int t_max,
+                               const OharaSeq* seq, void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  return launch_front<bf16_t>(FrontArgs<bf16_t>{p, qn, kn, q_out, kcache, vcache, ldp, h, h_kv, dh, dv, t_max, eps, *seq},
+                              (hipStream_t)stream);
+}
+int ohara_qkv_norm_append_f32(const float* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn, const float* kn,
+                              float eps, float* q_out, float* kcache, float* vcache, int t_max, const OharaSeq* seq,
+                              void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  return launch_front<float>(FrontArgs<float>{p, qn, kn, q_out, kcache, vcache, ldp, h, h_kv, dh, dv, t_max, eps, *seq},
+                             (hipStream_t)stream);
+}
+
+int64_t ohara_attn_bias_workspace_bytes(int rows, int h, int dv, int n_split) {
+  if (rows < 1 || h < 1 || dv < 1 || n_split < 1) return OHARA_EINVAL;
+  const int64_t counters = ((int64_t)rows * h * (int64_t)sizeof(int) + 255) & ~(int64_t)255;
+  return counters + (int64_t)rows * h * n_split * (((dv + 7) & ~7) + 2) * (int64_t)sizeof(float);
+}
+
+int ohara_attn_bias_bf16(const uint16_t* q, const uint16_t* kcache, const uint16_t* vcache, int h, int h_kv, int dh,
+                         int dv, int t_max, float scale, const float* slopes, const uint16_t* gate, int ldg, int n_split,
+                         void* workspace, uint16_t* out, int ldo, const OharaSeq* seq, void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  AttnBiasArgs<bf16_t> a{};
+  a.q = q; a.kc = kcache; a.vc = vcache; a.gate = gate; a.slopes = slopes; a.out = out;
+  a.H = h; a.G = h_kv; a.D = dh; a.V = dv; a.Tmax = t_max; a.ldg = ldg; a.ldo = ldo; a.ns = n_split; a.scale = scale;
+  a.seq = *seq;
+  return launch_bias<bf16_t>(a, workspace, (hipStream_t)stream);
+}
+int ohara_attn_bias_f32(const float* q, const float* kcache, const float* vcache, int h, int h_kv, int dh, int dv,
+                        int t_max, float scale, const float* slopes, const float* gate, int ldg, int n_split,
+                        void* workspace, float* out, int ldo, const OharaSeq* seq, void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  AttnBiasArgs<float> a{};
+  a.q = q; a.kc = kcache; a.vc = vcache; a.gate = gate; a.slopes = slopes; a.out = out;
+  a.H = h; a.G = h_kv; a.D = dh; a.V = dv; a.Tmax = t_max; a.ldg = ldg; a.ldo = ldo; a.ns = n_split; a.scale = scale;
+  a.seq = *seq;
+  return launch_bias<float>(a, workspace, (hipStream_t)stream);
+}
+
+}  // extern "C"

@@ -1,0 +1,574 @@
+// Gated delta rule with one decay per head and key channel, with its short convolutions, unit norms, step sizes and
+// gated output norm.  Per value head, S (dim x vdim, fp32) from zero:
+//   S <- diag(exp(lg)) S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q.
+//
+// delta_step_kernel: one token per sequence, everything in one launch, a workgroup per (sequence, value head).  The
+// state's slice is requested before anything else, so its latency runs under the convolutions and the
+// low-rank products.  o = S_new^T q is formed as (diag(exp(lg)) S)^T q + (q . k) u, so both products with
+// the state share one pass over it.
+//
+// Prompts: tokens in chunks of C = 32.  With G the running sum of lg inside a chunk (inclusive) and S0 the state before it,
+//   A_ij = beta_i sum_d k_id k_jd exp(G_id - G_jd)  (j < i)          B_ij = sum_d q_id k_jd exp(G_id - G_jd)  (j <= i)
+//   (I + A) u = beta (v - (k exp(G)) S0)  =>  u = U - W S0,  (I + A) U = beta v,  (I + A) W = beta k exp(G)
+//   o = (q exp(G)) S0 + B u               S1 = diag(exp(G_C)) S0 + (k exp(G_C - G))^T u
+// chunk_solve_kernel forms U, W, B and the scaled q, k of every chunk on its own (all chunks in parallel); every
+// exponent there is a sum of logarithms of decays of tokens between j and i, never positive, however strong the decay.
+// chunk_walk_kernel carries the state over the chunks: a workgroup per (sequence, head, 16 value
+// columns), all products on fp32 MFMA with the state in accumulators.
+#include "hybrid.h"
+
+namespace {
+
+constexpr int C = 32;        // tokens per chunk
+constexpr float UNIT_EPS = 1e-6f;
+
+template <typename T>
+struct DeltaArgs {
+  OharaDelta d;
+  const T* p;
+  const T* za;
+  const T* zg;
+  float* state;
+  T* ring;
+  float* ws;
+  float* o;
+  T* out;
+  int ldp, ldza, ldzg, ldo;
+  int chunk0, nchunks;  // chunks of this segment
+  OharaSeq seq;
+};
+
+__host__ __device__ __forceinline__ int up(int v, int m) { return (v + m - 1) / m * m; }
+
+// ---- one token -------------------------------------------------------------------------------
+constexpr int STEP_ROWS = 16;  // state rows a thread holds
+
+template <typename T, int NT>
+__global__ __launch_bounds__(NT) void delta_step_kernel(DeltaArgs<T> a) {
+  constexpr int NW = NT / 64;
+  __shared__ __align__(16) float qs[256], ks[256], gs[256], vs[256], us[256], gate[256];
+  __shared__ __align__(16) float rk[NT * 4], rq[NT * 4];
+  __shared__ float red[NW];
+  const OharaDelta& dd = a.d;
+  const int H = dd.heads, D = dd.dim, V = dd.vdim;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int b = blockIdx.x / H, h = blockIdx.x - b * H;
+  const int rep = H / dd.kv_heads, kvh = h / rep;
+  T* orow = a.out + (size_t)b * a.ldo;
+  if (h == 0)
+    for (int i = H * V + tid; i < a.ldo; i += NT) stv(orow + i, 0.f);
+  const int pos = seq_start(a.seq, b);
+  if (seq_tokens(a.seq, b) < 1 || pos < 0) return;
+  const int slot = seq_slot(a.seq, b);
+
+  // this thread's slice of the state: four columns, rows grp, grp + ngrp, ...
+  const int Vp = up(V, 4), c4 = Vp / 4, ngrp = NT / c4;
+  const int grp = tid / c4, col = 4 * (tid - grp * c4);
+  float* S = a.state + ((size_t)slot * H + h) * D * Vp + col;
+  float4 st[STEP_ROWS];
+#pragma unroll
+  for (int i = 0; i < STEP_ROWS; ++i) {
+    const int r = grp + i * ngrp;
+    st[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (grp < ngrp && r < D && pos > 0) st[i] = *reinterpret_cast<const float4*>(S + (size_t)r * Vp);
+  }
+
+  // short convolutions of this head's q, k, v channels
+  const T* p = a.p + (size_t)b * a.ldp;
+  const int nqk = dd.kv_heads * D, channels = 2 * nqk + H * V, taps = dd.taps;
+  T* ring = a.ring + (size_t)slot * taps * channels;
+  for (int i = tid; i < 2 * D + V; i += NT) {
+    const int ch = i < D ? kvh * D + i : (i < 2 * D ? nqk + kvh * D + (i - D) : 2 * nqk + h * V + (i - 2 * D));
+    const float cur = ldv(p + ch);
+    float c = dd.conv_w[(size_t)(taps - 1) * channels + ch] * cur;
+    for (int lag = 1; lag < taps; ++lag)
+      if (pos >= lag) c += dd.conv_w[(size_t)(taps - 1 - lag) * channels + ch] * ldv(ring + (size_t)((pos - lag) % taps) * channels + ch);
+    // the slot written belongs to the token `taps` back, which no workgroup of this launch reads
+    if (i >= 2 * D || h == kvh * rep) ring[(size_t)(pos % taps) * channels + ch] = p[ch];
+    const float y = silu_x(c);
+    if (i < D) qs[i] = y;
+    else if (i < 2 * D) ks[i - D] = y;
+    else vs[i - 2 * D] = y;
+  }
+  // decays and output gates: eight lanes per row of a2 / g2
+  {
+    const int l8 = tid & 7;
+    const float na = dd.neg_a[h];
+    const T* a1 = p + dd.off_a;
+    const T* g1 = p + dd.off_g;
+    for (int r0 = 0; r0 < D + V; r0 += NT / 8) {
+      const int r = r0 + (tid >> 3);
+      const bool live = r < D + V, isa = r < D;
+      const int n = isa ? dd.rank_a : dd.rank_g;
+      const T* wrow = isa ? (const T*)dd.a2 + ((size_t)h * D + r) * n : (const T*)dd.g2 + ((size_t)h * V + (r - D)) * n;
+      const T* xr = isa ? a1 : g1;
+      float s = 0.f;
+      if (live)
+        for (int i = 8 * l8; i < n; i += 64) {
+          Raw8<T> wv, xv;
+          wv.load(wrow + i);
+          xv.load(xr + i);
+          float wf[8], xf[8];
+          wv.get(wf);
+          xv.get(xf);
+#pragma unroll
+          for (int u = 0; u < 8; ++u) s = __builtin_fmaf(wf[u], xf[u], s);
+        }
+      s = lanes_sum<4, 1>(s);
+      if (live && l8 == 0) {
+        if (isa) gs[r] = expf(na * softplus_x(s + dd.dt_bias[(size_t)h * D + r]));
+        else gate[r - D] = sigmoid_x(s);
+      }
+    }
+  }
+  __syncthreads();
+  // every wave forms the sums over q and k for itself
+  float sq = 0.f, sk = 0.f, qk = 0.f;
+  for (int i = lane; i < D; i += 64) {
+    const float q = qs[i], k = ks[i];
+    sq += q * q;
+    sk += k * k;
+    qk += q * k;
+  }
+  const float iq = (1.0f / sqrtf(wave_sum(sq) + UNIT_EPS)) * (1.0f / sqrtf((float)D));
+  const float ik = 1.0f / sqrtf(wave_sum(sk) + UNIT_EPS);
+  qk = wave_sum(qk) * iq * ik;
+  const float beta = sigmoid_x(ldv(p + dd.off_b + h));
+
+  // decayed state against k and q
+  float4 pk = make_float4(0.f, 0.f, 0.f, 0.f), pq = pk;
+#pragma unroll
+  for (int i = 0; i < STEP_ROWS; ++i) {
+    const int r = grp + i * ngrp;
+    if (r < D) {
+      const float g = gs[r], kk = ks[r] * ik, qq = qs[r] * iq;
+      st[i].x *= g; st[i].y *= g; st[i].z *= g; st[i].w *= g;
+      pk.x += st[i].x * kk; pk.y += st[i].y * kk; pk.z += st[i].z * kk; pk.w += st[i].w * kk;
+      pq.x += st[i].x * qq; pq.y += st[i].y * qq; pq.z += st[i].z * qq; pq.w += st[i].w * qq;
+    }
+  }
+  if (grp < ngrp) {
+    *reinterpret_cast<float4*>(rk + (size_t)grp * Vp + col) = pk;
+    *reinterpret_cast<float4*>(rq + (size_t)grp * Vp + col) = pq;
+  }
+  __syncthreads();
+  float o = 0.f;
+  if (tid < V) {
+    float sk_ = 0.f, sq_ = 0.f;
+    for (int i = 0; i < ngrp; ++i) {
+      sk_ += rk[i * Vp + tid];
+      sq_ += rq[i * Vp + tid];
+    }
+    const float u = beta * (vs[tid] - sk_);
+    us[tid] = u;
+    o = sq_ + qk * u;
+  } else if (tid < Vp) {
+    us[tid] = 0.f;
+  }
+  const float so = wave_sum(o * o);
+  if (lane == 0) red[wave] = so;
+  __syncthreads();
+  if (grp < ngrp) {
+    const float4 u = *reinterpret_cast<const float4*>(us + col);
+#pragma unroll
+    for (int i = 0; i < STEP_ROWS; ++i) {
+      const int r = grp + i * ngrp;
+      if (r < D) {
+        const float kk = ks[r] * ik;
+        *reinterpret_cast<float4*>(S + (size_t)r * Vp) =
+            make_float4(st[i].x + kk * u.x, st[i].y + kk * u.y, st[i].z + kk * u.z, st[i].w + kk * u.w);
+      }
+    }
+  }
+  if (tid < V) {
+    float tot = 0.f;
+#pragma unroll
+    for (int w = 0; w < (NW < 4 ? NW : 4); ++w) tot += red[w];  // V <= 256: the first four waves
+    const float inv = 1.0f / sqrtf(tot / (float)V + dd.eps);
+    stv(orow + h * V + tid, o * inv * dd.norm_w[tid] * gate[tid]);
+  }
+}
+
+// ---- prompts: workspace ------------------------------------------------------------------------
+// Per (sequence, head, chunk), floats: W [C][Dp] | q exp(G) [C][Dp] | (k exp(G_C - G))^T [Dp][C] | U [C][Vq] | B [C][C] | exp(G_C) [Dp]
+// with Dp = dim rounded up to 32 / 64 / 128 / 256 and Vq = vdim rounded up to 16; padding is zero.
+__host__ __device__ __forceinline__ int dim_padded(int d) { return d <= 32 ? 32 : (d <= 64 ? 64 : (d <= 128 ? 128 : 256)); }
+__host__ __device__ __forceinline__ size_t chunk_floats(int D, int V) {
+  const int Dp = dim_padded(D), Vq = up(V, 16);
+  return (size_t)3 * C * Dp + (size_t)C * Vq + C * C + Dp;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void chunk_solve_kernel(DeltaArgs<T> a) {
+  extern __shared__ __align__(16) float sm[];
+  const OharaDelta& dd = a.d;
+  const int H = dd.heads, D = dd.dim, V = dd.vdim;
+  const int Dp = dim_padded(D), Vq = up(V, 16), LD = Dp + 4;
+  float* Q = sm;               // [C][LD]
+  float* K = Q + C * LD;
+  float* G = K + C * LD;       // running sum of the decays' logarithms
+  float* X = G + C * LD;       // v: [C][Vq]
+  float* A = X + C * Vq;       // [C][C + 4]
+  float* B = A + C * (C + 4);
+  float* beta = B + C * (C + 4);  // [C]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int ci = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int len = seq_tokens(a.seq, b);
+  const int s0 = (a.chunk0 + ci) * C;
+  if (s0 >= len) return;
+  const int n = min(C, len - s0);  // tokens of this chunk
+  const int pos0 = seq_start(a.seq, b), slot = seq_slot(a.seq, b);
+  const int rep = H / dd.kv_heads, kvh = h / rep;
+  const int nqk = dd.kv_heads * D, channels = 2 * nqk + H * V, taps = dd.taps;
+  const T* ring = a.ring + (size_t)slot * taps * channels;
+  const T* prow = a.p + (size_t)b * a.seq.seq_len * a.ldp;  // row of the sequence's first token in this call
+  // convolution + silu of channel ch at token s of this call
+  auto conv = [&](int s, int ch) {
+    float c = 0.f;
+    for (int lag = 0; lag < taps; ++lag) {
+      float x;
+      if (lag <= s) x = ldv(prow + (size_t)(s - lag) * a.ldp + ch);
+      else if (pos0 + s >= lag) x = ldv(ring + (size_t)((pos0 + s - lag) % taps) * channels + ch);
+      else break;
+      c += dd.conv_w[(size_t)(taps - 1 - lag) * channels + ch] * x;
+    }
+    return silu_x(c);
+  };
+  for (int i = tid; i < C * Dp; i += 256) {
+    const int t = i / Dp, c = i - t * Dp;
+    const bool in = t < n && c < D;
+    Q[t * LD + c] = in ? conv(s0 + t, kvh * D + c) : 0.f;
+    K[t * LD + c] = in ? conv(s0 + t, nqk + kvh * D + c) : 0.f;
+    float lg = 0.f;
+    if (in) {
+      const size_t row = (size_t)b * a.seq.seq_len + s0 + t;
+      lg = dd.neg_a[h] * softplus_x(ldv(a.za + row * a.ldza + (size_t)h * D + c) + dd.dt_bias[(size_t)h * D + c]);
+    }
+    G[t * LD + c] = lg;
+  }
+  for (int i = tid; i < C * Vq; i += 256) {
+    const int t = i / Vq, c = i - t * Vq;
+    X[i] = t < n && c < V ? conv(s0 + t, 2 * nqk + h * V + c) : 0.f;
+  }
+  if (tid < C) beta[tid] = tid < n ? sigmoid_x(ldv(prow + (size_t)(s0 + tid) * a.ldp + dd.off_b + h)) : 0.f;
+  __syncthreads();
+  // unit q and k; running sums
+  for (int r = wave; r < 2 * C; r += 4) {
+    float* x = (r < C ? Q + r * LD : K + (r - C) * LD);
+    float s = 0.f;
+    for (int i = lane; i < D; i += 64) s += x[i] * x[i];
+    s = 1.0f / sqrtf(wave_sum(s) + UNIT_EPS);
+    if (r < C) s *= 1.0f / sqrtf((float)D);
+    for (int i = lane; i < D; i += 64) x[i] *= s;
+  }
+  for (int c = tid; c < Dp; c += 256) {
+    float s = 0.f;
+    for (int t = 0; t < C; ++t) {
+      s += G[t * LD + c];
+      G[t * LD + c] = s;
+    }
+  }
+  __syncthreads();
+  // A and B, one (i, j) pair per thread and round: the two diagonal 16 x 16 blocks and the one below
+  for (int blk = 0; blk < 4; ++blk) {
+    const int i = (blk >> 1) * 16 + (tid & 15), j = (blk & 1) * 16 + (tid >> 4);
+    float sa = 0.f, sb = 0.f;
+    if (blk != 1) {
+      const float *ki = K + i * LD, *qi = Q + i * LD, *gi = G + i * LD, *kj = K + j * LD, *gj = G + j * LD;
+      if (j <= i) {
+        for (int c = 0; c < D; c += 4) {  // columns past D are zero
+          const float4 k1 = *reinterpret_cast<const float4*>(ki + c), q1 = *reinterpret_cast<const float4*>(qi + c);
+          const float4 g1 = *reinterpret_cast<const float4*>(gi + c), k2 = *reinterpret_cast<const float4*>(kj + c);
+          const float4 g2 = *reinterpret_cast<const float4*>(gj + c);
+          const float e0 = k2.x * __expf(g1.x - g2.x), e1 = k2.y * __expf(g1.y - g2.y);
+          const float e2 = k2.z * __expf(g1.z - g2.z), e3 = k2.w * __expf(g1.w - g2.w);
+          sa += k1.x * e0; sa += k1.y * e1; sa += k1.z * e2; sa += k1.w * e3;
+          sb += q1.x * e0; sb += q1.y * e1; sb += q1.z * e2; sb += q1.w * e3;
+        }
+      }
+    }
+    A[i * (C + 4) + j] = j < i ? sa * beta[i] : 0.f;
+    B[i * (C + 4) + j] = sb;
+  }
+  __syncthreads();
+  float* w = a.ws + (((size_t)b * H + h) * a.nchunks + ci) * chunk_floats(D, V);
+  float* wW = w;
+  float* wQ = wW + C * Dp;
+  float* wK = wQ + C * Dp;
+  float* wU = wK + C * Dp;
+  float* wB = wU + C * Vq;
+  float* wG = wB + C * C;
+  // forward substitution, a column per thread: rows of A are read by all lanes at once
+  for (int c = tid; c < Dp + Vq; c += 256) {
+    float x[C];
+    const bool isw = c < Dp;
+    const int vc = c - Dp;
+#pragma unroll
+    for (int t = 0; t < C; ++t) x[t] = beta[t] * (isw ? K[t * LD + c] * expf(G[t * LD + c]) : X[t * Vq + vc]);
+    float* dst = isw ? wW + c : wU + vc;
+    const int ld = isw ? Dp : Vq;
+    dst[0] = x[0];
+#pragma unroll
+    for (int t = 1; t < C; ++t) {
+      const float* ar = A + t * (C + 4);
+      float s = x[t];
+#pragma unroll
+      for (int j = 0; j < t; ++j) s -= ar[j] * x[j];
+      x[t] = s;
+      dst[(size_t)t * ld] = s;
+      __builtin_amdgcn_sched_barrier(0);  // row by row: hoisting the reads of all of A would spill
+    }
+  }
+  for (int i = tid; i < C * Dp; i += 256) {
+    const int t = i / Dp, c = i - t * Dp;
+    wQ[i] = Q[t * LD + c] * expf(G[t * LD + c]);
+  }
+  for (int i = tid; i < C * Dp; i += 256) {
+    const int c = i / C, t = i - c * C;
+    wK[i] = K[t * LD + c] * expf(G[(C - 1) * LD + c] - G[t * LD + c]);
+  }
+  for (int i = tid; i < C * C; i += 256) wB[i] = B[(i / C) * (C + 4) + (i % C)];
+  for (int c = tid; c < Dp; c += 256) wG[c] = expf(G[(C - 1) * LD + c]);
+}
+
+// The state over the chunks.  v_mfma_f32_16x16x4_f32: A lane (row = lane & 15, k = lane >> 4), B lane (k = lane >> 4,
+// column = lane & 15), result row 4 (lane >> 4) + r, column lane & 15.  A step of 16 k's takes four products whose k-slot g
+// of product j stands for k = 4 g + j, so a lane fetches the four A elements it needs as one float4.
+template <typename T, int DPT>  // Dp / 16
+__global__ __launch_bounds__(256) void chunk_walk_kernel(DeltaArgs<T> a) {
+  constexpr int Dp = 16 * DPT, MT = (DPT + 3) / 4, LS = 17;
+  __shared__ float Sl[Dp * LS];
+  __shared__ float Un[C * LS];
+  const OharaDelta& dd = a.d;
+  const int H = dd.heads, D = dd.dim, V = dd.vdim, Vp = up(V, 4), Vq = up(V, 16);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 15, g = lane >> 4;
+  const int v0 = blockIdx.x * 16, h = blockIdx.y, b = blockIdx.z;
+  const int len = seq_tokens(a.seq, b);
+  const int nch = min(a.nchunks, (len + C - 1) / C - a.chunk0);
+  if (nch < 1) return;
+  const int pos0 = seq_start(a.seq, b);
+  float* S = a.state + ((size_t)seq_slot(a.seq, b) * H + h) * D * Vp;
+  const bool fresh = a.chunk0 == 0 && pos0 == 0;
+  f32x4 acc[MT];
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const int tile = wave + 4 * i;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = 16 * tile + 4 * g + r;
+      acc[i][r] = (!fresh && tile < DPT && d < D && v0 + m < V) ? S[(size_t)d * Vp + v0 + m] : 0.f;
+      if (tile < DPT) Sl[d * LS + m] = acc[i][r];
+    }
+  }
+  const size_t cf = chunk_floats(D, V);
+  const float* w = a.ws + ((size_t)b * H + h) * a.nchunks * cf;
+  const bool left = wave < 2;           // waves 0, 1: u; waves 2, 3: o
+  const int mrow = 16 * (wave & 1);     // this wave's token rows
+  // operands of a chunk, fetched one chunk ahead
+  float4 fa[DPT], fk[MT][2], fg[MT], fb[2];
+  float fu[4];
+  auto fetch = [&](const float* x) {
+    const float* ap = x + (left ? 0 : C * Dp) + (size_t)(mrow + m) * Dp + 4 * g;
+#pragma unroll
+    for (int i = 0; i < DPT; ++i) fa[i] = *reinterpret_cast<const float4*>(ap + 16 * i);
+    const float* kp = x + 2 * C * Dp;
+    const float* up_ = kp + C * Dp;
+    const float* bp = up_ + C * Vq;
+    const float* gp = bp + C * C;
+#pragma unroll
+    for (int i = 0; i < MT; ++i) {
+      const int tile = wave + 4 * i;
+      if (tile < DPT) {
+#pragma unroll
+        for (int j = 0; j < 2; ++j) fk[i][j] = *reinterpret_cast<const float4*>(kp + (size_t)(16 * tile + m) * C + 16 * j + 4 * g);
+        fg[i] = *reinterpret_cast<const float4*>(gp + 16 * tile + 4 * g);
+      }
+    }
+    if (left) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) fu[r] = up_[(size_t)(mrow + 4 * g + r) * Vq + v0 + m];
+    } else {
+#pragma unroll
+      for (int j = 0; j < 2; ++j) fb[j] = *reinterpret_cast<const float4*>(bp + (size_t)(mrow + m) * C + 16 * j + 4 * g);
+    }
+  };
+  auto mul4 = [&](float4 av, const float* bcol, f32x4 c) {  // bcol: row 4 g of the step's B rows, column m
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.x, bcol[0], c, 0, 0, 0);
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.y, bcol[LS], c, 0, 0, 0);
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.z, bcol[2 * LS], c, 0, 0, 0);
+    return __builtin_amdgcn_mfma_f32_16x16x4f32(av.w, bcol[3 * LS], c, 0, 0, 0);
+  };
+  fetch(w);
+  __syncthreads();
+  for (int ci = 0; ci < nch; ++ci) {
+    f32x4 x = (f32x4){0.f, 0.f, 0.f, 0.f}, x2 = x;
+#pragma unroll
+    for (int i = 0; i < DPT; i += 2) {
+      x = mul4(fa[i], Sl + (16 * i + 4 * g) * LS + m, x);
+      x2 = mul4(fa[i + 1], Sl + (16 * (i + 1) + 4 * g) * LS + m, x2);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) x[r] += x2[r];
+    if (left) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) Un[(mrow + 4 * g + r) * LS + m] = fu[r] - x[r];
+    }
+    __syncthreads();  // u is complete; the state in LDS has been read
+    if (!left) {
+#pragma unroll
+      for (int j = 0; j < 2; ++j) x = mul4(fb[j], Un + (16 * j + 4 * g) * LS + m, x);
+      const int s = (a.chunk0 + ci) * C + mrow + 4 * g;
+      float* op = a.o + ((size_t)b * a.seq.seq_len + s) * H * V + (size_t)h * V + v0 + m;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (s + r < len && v0 + m < V) op[(size_t)r * H * V] = x[r];
+    }
+#pragma unroll
+    for (int i = 0; i < MT; ++i) {
+      const int tile = wave + 4 * i;
+      if (tile < DPT) {
+        acc[i][0] *= fg[i].x; acc[i][1] *= fg[i].y; acc[i][2] *= fg[i].z; acc[i][3] *= fg[i].w;
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i] = mul4(fk[i][j], Un + (16 * j + 4 * g) * LS + m, acc[i]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) Sl[(16 * tile + 4 * g + r) * LS + m] = acc[i][r];
+      }
+    }
+    if (ci + 1 < nch) fetch(w + (size_t)(ci + 1) * cf);
+    __syncthreads();  // the new state is in LDS; u has been read
+  }
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const int tile = wave + 4 * i;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = 16 * tile + 4 * g + r;
+      if (tile < DPT && d < D && v0 + m < V) S[(size_t)d * Vp + v0 + m] = acc[i][r];
+    }
+  }
+}
+
+// out = o / rms(o) * norm_w * sigmoid(zg): a wave per (row, head)
+template <typename T>
+__global__ __launch_bounds__(256) void delta_out_kernel(DeltaArgs<T> a) {
+  const OharaDelta& dd = a.d;
+  const int H = dd.heads, V = dd.vdim;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int row = blockIdx.x, b = row / a.seq.seq_len, s = row - b * a.seq.seq_len;
+  T* orow = a.out + (size_t)row * a.ldo;
+  for (int i = H * V + threadIdx.x; i < a.ldo; i += 256) stv(orow + i, 0.f);
+  if (s >= seq_tokens(a.seq, b)) return;
+  for (int h = blockIdx.y * 4 + wave; h < H; h += 4 * gridDim.y) {
+    const float* o = a.o + ((size_t)row * H + h) * V;
+    float v[4], z[4], ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int c = lane + 64 * u;
+      v[u] = c < V ? o[c] : 0.f;
+      z[u] = c < V ? ldv(a.zg + (size_t)row * a.ldzg + (size_t)h * V + c) : 0.f;
+      ss += v[u] * v[u];
+    }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)V + dd.eps);
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int c = lane + 64 * u;
+      if (c < V) stv(orow + h * V + c, v[u] * inv * dd.norm_w[c] * sigmoid_x(z[u]));
+    }
+  }
+}
+
+bool delta_ok(const OharaDelta* d, int ldp) {
+  if (!d || !d->conv_w || !d->a2 || !d->g2 || !d->neg_a || !d->dt_bias || !d->norm_w) return false;
+  if (d->heads < 1 || d->kv_heads < 1 || d->heads % d->kv_heads || d->dim < 1 || d->vdim < 1 || d->taps < 1) return false;
+  const int channels = 2 * d->kv_heads * d->dim + d->heads * d->vdim;
+  if (d->rank_a < 8 || d->rank_g < 8 || ((d->rank_a | d->rank_g | d->off_a | d->off_g | ldp) & 7)) return false;
+  return ldp >= channels && d->off_a >= channels && d->off_a + d->rank_a <= ldp && d->off_g >= channels &&
+         d->off_g + d->rank_g <= ldp && d->off_b >= channels && d->off_b + d->heads <= ldp;
+}
+
+template <typename T>
+int delta_step(const OharaDelta* d, const T* p, int ldp, float* state, T* ring, T* out, int ldo, const OharaSeq* seq,
+               hipStream_t st) {
+  if (!delta_ok(d, ldp) || !p || !state || !ring || !out || !seq_ok(seq) || seq->seq_len != 1) return OHARA_EINVAL;
+  if (ldo < d->heads * d->vdim) return OHARA_EINVAL;
+  if (d->dim > 256 || d->vdim > 256) return OHARA_ESIZE;
+  if ((int64_t)seq->batch * d->heads > INT32_MAX) return OHARA_ESIZE;
+  DeltaArgs<T> a{};
+  a.d = *d; a.p = p; a.ldp = ldp; a.state = state; a.ring = ring; a.out = out; a.ldo = ldo; a.seq = *seq;
+  const dim3 grid((unsigned)(seq->batch * d->heads));
+  const int c4 = up(d->vdim, 4) / 4;
+  // enough threads that no one holds more than STEP_ROWS rows of the state
+  if ((256 / c4) * STEP_ROWS >= d->dim) hipLaunchKernelGGL((delta_step_kernel<T, 256>), grid, dim3(256), 0, st, a);
+  else if ((512 / c4) * STEP_ROWS >= d->dim) hipLaunchKernelGGL((delta_step_kernel<T, 512>), grid, dim3(512), 0, st, a);
+  else hipLaunchKernelGGL((delta_step_kernel<T, 1024>), grid, dim3(1024), 0, st, a);
+  return ohara_launch_status();
+}
+
+template <typename T>
+int delta_prefill(const OharaDelta* d, const T* p, int ldp, const T* za, int ldza, const T* zg, int ldzg, float* state,
+                  const T* ring, void* ws, int64_t ws_bytes, float* o, T* out, int ldo, const OharaSeq* seq, hipStream_t st) {
+  if (!delta_ok(d, ldp) || !p || !za || !zg || !state || !ring || !ws || !o || !out || !seq_ok(seq)) return OHARA_EINVAL;
+  if (ldo < d->heads * d->vdim || ldza < d->heads * d->dim || ldzg < d->heads * d->vdim) return OHARA_EINVAL;
+  if (d->dim > 256 || d->vdim > 256 || d->heads > 65535 || seq->batch > 65535) return OHARA_ESIZE;
+  DeltaArgs<T> a{};
+  a.d = *d; a.p = p; a.ldp = ldp; a.za = za; a.ldza = ldza; a.zg = zg; a.ldzg = ldzg; a.state = state;
+  a.ring = const_cast<T*>(ring); a.ws = reinterpret_cast<float*>(ws); a.o = o; a.out = out; a.ldo = ldo; a.seq = *seq;
+  const int Dp = dim_padded(d->dim);
+  const int64_t per_chunk = (int64_t)chunk_floats(d->dim, d->vdim) * sizeof(float) * d->heads * seq->batch;
+  const int all = (seq->seq_len + C - 1) / C;
+  int fit = (int)(ws_bytes / per_chunk < all ? ws_bytes / per_chunk : all);
+  if (fit < 1) return OHARA_EINVAL;
+  const size_t smem = ((size_t)3 * C * (Dp + 4) + (size_t)C * up(d->vdim, 16) + 2 * C * (C + 4) + C) * sizeof(float);
+  if (smem > 64 * 1024)
+    (void)hipFuncSetAttribute((const void*)chunk_solve_kernel<T>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+  const dim3 wgrid((unsigned)((d->vdim + 15) / 16), (unsigned)d->heads, (unsigned)seq->batch);
+  for (int c0 = 0; c0 < all; c0 += fit) {
+    a.chunk0 = c0;
+    a.nchunks = all - c0 < fit ? all - c0 : fit;
+    hipLaunchKernelGGL((chunk_solve_kernel<T>), dim3((unsigned)a.nchunks, (unsigned)d->heads, (unsigned)seq->batch), dim3(256),
+                       smem, st, a);
+    switch (Dp) {
+      case 32: hipLaunchKernelGGL((chunk_walk_kernel<T, 2>), wgrid, dim3(256), 0, st, a); break;
+      case 64: hipLaunchKernelGGL((chunk_walk_kernel<T, 4>), wgrid, dim3(256), 0, st, a); break;
+      case 128: hipLaunchKernelGGL((chunk_walk_kernel<T, 8>), wgrid, dim3(256), 0, st, a); break;
+      default: hipLaunchKernelGGL((chunk_walk_kernel<T, 16>), wgrid, dim3(256), 0, st, a); break;
+    }
+  }
+  const int rows = seq->batch * seq->seq_len;
+  hipLaunchKernelGGL((delta_out_kernel<T>), dim3((unsigned)rows, (unsigned)((d->heads + 3) / 4)), dim3(256), 0, st, a);
+  return ohara_launch_status();
+}
+
+}  // namespace
+
+extern "C" {
+
+int ohara_delta_step_bf16(const OharaDelta* d, const uint16_t* p, int ldp, float* state, uint16_t* ring, uint16_t* out,
+                          int ldo, const OharaSeq* seq, void* stream) {
+  return delta_step<bf16_t>(d, p, ldp, state, ring, out, ldo, seq, (hipStream_t)stream);
+}
+int ohara_delta_step_f32(const OharaDelta* d, const float* p, int ldp, float* state, float* ring, float* out, int ldo,
+                         const OharaSeq* seq, void* stream) {
+  return delta_step<float>(d, p, ldp, state, ring, out, ldo, seq, (hipStream_t)stream);
+}
+
+int64_t ohara_delta_workspace_bytes(int heads, int dim, int vdim, int batch, int tokens) {
+  if (heads < 1 || dim < 1 || dim > 256 || vdim < 1 || vdim > 256 || batch < 1 || tokens < 1) return OHARA_EINVAL;
+  return (int64_t)chunk_floats(dim, vdim) * (int64_t)sizeof(float) * heads * batch * ((tokens + C - 1) / C);
+}
+
+int ohara_delta_prefill_bf16(const OharaDelta* d, const uint16_t* p, int ldp, const uint16_t* za, int ldza,
+                             const uint16_t* zg, int ldzg, float* state, const uint16_t* ring, void* workspace,
+                             int64_t workspace_bytes, float* o_tmp, uint16_t* out, int ldo, const OharaSeq* seq,
+                             void* stream) {
+  return delta_prefill<bf16_t>(d, p, ldp, za, ldza, zg, ldzg, state, ring, workspace, workspace_bytes, o_tmp, out, ldo, seq,
+                               (hipStream_t)stream);
+}
+int ohara_delta_prefill_f32(const OharaDelta* d, const float* p, int ldp, const float* za, int ldza, const float* zg,
+                            int ldzg, float* state, const float* ring, void* workspace, int64_t workspace_bytes,
+                            float* o_tmp, float* out, int ldo, const OharaSeq* seq, void* stream) {
+  return delta_prefill<float>(d, p, ldp, za, ldza, zg, ldzg, state, ring, workspace, workspace_bytes, o_tmp, out, ldo, seq,
+                              (hipStream_t)stream);
+}
+
+}  // extern "C"

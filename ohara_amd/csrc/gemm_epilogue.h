@@ -4,10 +4,11 @@
 //   SwiGLU             ohara/modules/mlp.py:152
 //   rotary + KV append ohara/embeddings_pos/rotary.py:55-93, ohara/modules/kv_cache.py:104-105
 //   bias / new_gelu / parallel-block sum of Phi   ohara/models/phi.py:37-52, :147-151
+//   soft cap of the fp32 sum (vocabulary projections with capped logits)
 #pragma once
 #include "common.h"
 
-enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3, EPI_BIAS = 4, EPI_BIAS_GELU = 5, EPI_BIAS_ADD2 = 6, EPI_PHI_IN = 7 };
+enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3, EPI_BIAS = 4, EPI_BIAS_GELU = 5, EPI_BIAS_ADD2 = 6, EPI_PHI_IN = 7, EPI_SOFTCAP = 8 };
 
 struct GemmArgs {
   const uint4* wp;
@@ -43,6 +44,7 @@ struct GemmArgs {
   int split_n;
   bf16_t* out2;
   int ldo2;
+  float cap;  // EPI_SOFTCAP: cap * tanh(acc / cap)
 };
 
 // gemm_tile.hip: the tiled kernel for calls with many rows (a.B rows, no fused norm).
@@ -89,6 +91,20 @@ __device__ __forceinline__ void gemm_epilogue_fetch(const GemmArgs& a, int b, in
 template <int EPI, bool PRE = false>  // PRE: the operands were fetched ahead into `p`
 __device__ __forceinline__ void gemm_epilogue(const GemmArgs& a, int b, int strip, int g, f32x4 acc, const EpiPre& p = EpiPre{}) {
   const int r0 = strip * 16 + 4 * g;
+  if (EPI == EPI_SOFTCAP) {
+    bf16_t* o = a.out + (size_t)b * a.ldo + r0;
+    float v[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = a.cap * tanhf(acc[i] / a.cap);
+    if (r0 + 3 < a.N && ((a.ldo & 3) == 0)) {
+      *reinterpret_cast<uint2*>(o) = make_uint2(pack_bf(v[0], v[1]), pack_bf(v[2], v[3]));
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (r0 + i < a.N) o[i] = f2bf(v[i]);
+    }
+    return;
+  }
   const float y0 = rbf(acc[0]), y1 = rbf(acc[1]), y2 = rbf(acc[2]), y3 = rbf(acc[3]);
   if (EPI == EPI_STORE || EPI == EPI_RESIDUAL) {
     float v[4] = {y0, y1, y2, y3};

@@ -1,0 +1,109 @@
+// fp32 matrix product for models served in 32-bit: y = x W^T with bias, SwiGLU or soft-cap epilogues, on
+// v_mfma_f32_16x16x4_f32 (true fp32 products and sums).  A workgroup owns 64 rows x 64 weight rows, a wave a
+// 32 x 32 quarter; 16 columns of both operands per step go through LDS, the next step's loads are in flight
+// during the products.
+#include "hybrid.h"
+
+namespace {
+
+struct GemmF32Args {
+  const float* x;
+  const float* w;
+  const float* w2;  // SwiGLU: the up projection
+  const float* bias;
+  float* out;
+  int ldx, ldo, n, k, rows;
+  float cap;
+};
+
+constexpr int GT = 64, GK = 16, GL = GK + 4;
+
+template <bool SWIGLU>
+__global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32Args a) {
+  constexpr int NB = SWIGLU ? 2 : 1;
+  __shared__ __align__(16) float xs[GT * GL];
+  __shared__ __align__(16) float ws[NB][GT * GL];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 15, g = lane >> 4;
+  const int r0 = blockIdx.y * GT, c0 = blockIdx.x * GT;
+  const int wr = (wave & 1) * 32, wc = (wave >> 1) * 32;
+  const int lr = tid >> 2, lc = (tid & 3) * 4;  // loader: one float4 per thread and operand
+  f32x4 acc[NB][2][2];
+#pragma unroll
+  for (int u = 0; u < NB; ++u)
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int j = 0; j < 2; ++j) acc[u][i][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  const uint4 zero = make_uint4(0, 0, 0, 0);
+  uint4 xv, wv[NB];
+  auto load = [&](int k0) {
+    const int k = k0 + lc;
+    const bool ink = k < a.k;  // k is a multiple of 4
+    xv = (ink && r0 + lr < a.rows) ? ldg16(a.x + (size_t)(r0 + lr) * a.ldx + k) : zero;
+#pragma unroll
+    for (int u = 0; u < NB; ++u)
+      wv[u] = (ink && c0 + lr < a.n) ? ldg16((u ? a.w2 : a.w) + (size_t)(c0 + lr) * a.k + k) : zero;
+  };
+  load(0);
+  for (int k0 = 0; k0 < a.k; k0 += GK) {
+    __syncthreads();
+    *reinterpret_cast<uint4*>(xs + lr * GL + lc) = xv;
+#pragma unroll
+    for (int u = 0; u < NB; ++u) *reinterpret_cast<uint4*>(ws[u] + lr * GL + lc) = wv[u];
+    __syncthreads();
+    if (k0 + GK < a.k) load(k0 + GK);
+    // k-slot g of product j stands for k = 4 g + j
+    float4 xf[2], wf[NB][2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      xf[i] = *reinterpret_cast<const float4*>(xs + (wr + 16 * i + m) * GL + 4 * g);
+#pragma unroll
+      for (int u = 0; u < NB; ++u) wf[u][i] = *reinterpret_cast<const float4*>(ws[u] + (wc + 16 * i + m) * GL + 4 * g);
+    }
+#pragma unroll
+    for (int u = 0; u < NB; ++u)
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+          f32x4 c = acc[u][i][j];
+          c = __builtin_amdgcn_mfma_f32_16x16x4f32(xf[i].x, wf[u][j].x, c, 0, 0, 0);
+          c = __builtin_amdgcn_mfma_f32_16x16x4f32(xf[i].y, wf[u][j].y, c, 0, 0, 0);
+          c = __builtin_amdgcn_mfma_f32_16x16x4f32(xf[i].z, wf[u][j].z, c, 0, 0, 0);
+          acc[u][i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(xf[i].w, wf[u][j].w, c, 0, 0, 0);
+        }
+  }
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int c = c0 + wc + 16 * j + m;
+      if (c >= a.n) continue;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = r0 + wr + 16 * i + 4 * g + r;
+        if (row >= a.rows) continue;
+        float v = acc[0][i][j][r];
+        if (SWIGLU) v = silu_x(v) * acc[NB - 1][i][j][r];
+        if (a.bias) v += a.bias[c];
+        if (a.cap > 0.f) v = a.cap * tanhf(v / a.cap);
+        a.out[(size_t)row * a.ldo + c] = v;
+      }
+    }
+}
+
+}  // namespace
+
+extern "C" int ohara_gemm_f32(const float* x, int ldx, const float* w, const float* w_up, const float* bias, float cap,
+                              int n, int k, int rows, float* out, int ldo, void* stream) {
+  if (!x || !w || !out || n < 1 || k < 1 || rows < 1) return OHARA_EINVAL;
+  if ((k & 3) || (ldx & 3) || ldx < k || ldo < n) return OHARA_EINVAL;  // 16-byte loads
+  if (w_up && (bias || cap > 0.f)) return OHARA_EINVAL;
+  const int64_t ny = ((int64_t)rows + GT - 1) / GT;
+  if (ny > 65535) return OHARA_ESIZE;
+  const GemmF32Args a{x, w, w_up, bias, out, ldx, ldo, n, k, rows, cap};
+  const dim3 grid((unsigned)((n + GT - 1) / GT), (unsigned)ny);
+  if (w_up) hipLaunchKernelGGL((gemm_f32_kernel<true>), grid, dim3(256), 0, (hipStream_t)stream, a);
+  else hipLaunchKernelGGL((gemm_f32_kernel<false>), grid, dim3(256), 0, (hipStream_t)stream, a);
+  return ohara_launch_status();
+}

@@ -96,7 +96,7 @@ __global__ __launch_bounds__(NW * 64) void skinny_kernel(GemmArgs a) {
   // the weights of the whole share in one go - the rows arrive first (loads return in order), the norm's sums run
   // while the weights are still on their way, and the rows are not fetched a second time.
   constexpr int SP = 8;
-  const bool pre_ok = ((a.N | a.ldo | a.ldr | a.ldr2) & 3) == 0 && EPI != EPI_STORE && EPI != EPI_SWIGLU;
+  const bool pre_ok = ((a.N | a.ldo | a.ldr | a.ldr2) & 3) == 0 && EPI != EPI_STORE && EPI != EPI_SWIGLU && EPI != EPI_SOFTCAP;
   EpiPre ep[BT];
   if (wave == 0 && pre_ok) {
 #pragma unroll
@@ -413,6 +413,8 @@ int launch_wide_bt(const GemmArgs& a, int epi, hipStream_t st) {
   if (epi == EPI_STORE) {
     if (a.norm_w) OHARA_WIDE(true, EPI_STORE);
     else OHARA_WIDE(false, EPI_STORE);
+  } else if (epi == EPI_SOFTCAP) {
+    OHARA_WIDE(false, EPI_SOFTCAP);
   } else {
     return OHARA_EINVAL;
   }
@@ -420,11 +422,11 @@ int launch_wide_bt(const GemmArgs& a, int epi, hipStream_t st) {
   return ohara_launch_status();
 }
 
-// The wide kernel serves plain stores of many strips whose rows fit LDS.
+// The wide kernel serves plain and soft-capped stores of many strips whose rows fit LDS.
 bool wide_applies(const GemmArgs& a, int epi, int strips) {
   const int KS = (a.K + 31) >> 5;
   const int bt = (a.B + 15) / 16;
-  return epi == EPI_STORE && strips >= 1024 && a.B <= 64 && (size_t)16 * bt * (KS * 32 + 8) * 2 <= 160 * 1024;
+  return (epi == EPI_STORE || epi == EPI_SOFTCAP) && strips >= 1024 && a.B <= 64 && (size_t)16 * bt * (KS * 32 + 8) * 2 <= 160 * 1024;
 }
 
 int launch_wide(const GemmArgs& a0, int epi, int strips, hipStream_t st) {
@@ -443,7 +445,7 @@ int launch_epi(const GemmArgs& a, int epi, int strips, hipStream_t st) {
   dim3 grid((unsigned)((strips + 7) / 8 * 8 * a.ny)), block(256);
   // Linear-with-bias calls with a long K (2048 and up): 16 waves per workgroup.  (For the d12 Llama
   // projections, K 768 / 2048 with 48 - 256 strips, 16 waves measured no faster than 4.)
-  if (!NORM && epi >= EPI_BIAS && a.K >= 2048) {
+  if (!NORM && epi >= EPI_BIAS && epi <= EPI_BIAS_ADD2 && a.K >= 2048) {
     if (strips * a.ny >= 400) {  // enough workgroups for four per CU: 8 waves each measured 5-9 % faster
       dim3 mid(512);
       switch (epi) {
@@ -468,6 +470,7 @@ int launch_epi(const GemmArgs& a, int epi, int strips, hipStream_t st) {
     case EPI_RESIDUAL: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_RESIDUAL>), grid, block, 0, st, a); break;
     case EPI_SWIGLU: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_SWIGLU>), grid, block, 0, st, a); break;
     case EPI_ROPE: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_ROPE>), grid, block, 0, st, a); break;
+    case EPI_SOFTCAP: hipLaunchKernelGGL((skinny_kernel<BT, false, EPI_SOFTCAP>), grid, block, 0, st, a); break;  // never with a norm
     case EPI_BIAS: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS>), grid, block, 0, st, a); break;
     case EPI_BIAS_GELU: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS_GELU>), grid, block, 0, st, a); break;
     case EPI_BIAS_ADD2: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS_ADD2>), grid, block, 0, st, a); break;
@@ -621,6 +624,17 @@ int ohara_phi_block_in_bf16(const uint16_t* x, int ldx, const uint16_t* ln_w, co
   a.S = seq_len; a.Tmax = t_max; a.pos = pos; a.pos_dev = pos_dev; a.kcache = kcache; a.vcache = vcache;
   if (a.B > 128 && !ln_w) return ohara_launch_gemm_tile(a, EPI_PHI_IN, (a.N + 15) / 16 * 16, (hipStream_t)stream);  // prefill
   return launch_skinny(a, EPI_PHI_IN, (a.N + 15) / 16 * 16, (hipStream_t)stream);
+}
+
+int ohara_gemm_softcap_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, float cap, int rows,
+                            uint16_t* out, int ldo, void* stream) {
+  if (!x || !wp || !out || n < 1 || k < 1 || rows < 1 || !(cap > 0.f)) return OHARA_EINVAL;
+  if ((k & 7) || (ldx & 7) || ldx < k || ldo < n) return OHARA_EINVAL;
+  GemmArgs a{};
+  a.wp = reinterpret_cast<const uint4*>(wp);
+  a.x = x; a.ldx = ldx; a.B = rows; a.N = n; a.K = k; a.out = out; a.ldo = ldo; a.cap = cap;
+  if (rows > 64) return ohara_launch_gemm_tile(a, EPI_SOFTCAP, (n + 15) / 16 * 16, (hipStream_t)stream);
+  return launch_skinny(a, EPI_SOFTCAP, (n + 15) / 16 * 16, (hipStream_t)stream);
 }
 
 int ohara_gemm_skinny_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, const uint16_t* norm_w,

@@ -1,0 +1,293 @@
+// Residual stream of blocks whose norm sits on the sublayer output, and the causal depthwise convolution in
+// front of a mixer.  The residual is fp32 throughout.
+//
+// Decode (one token per sequence): embedding or residual update, group norm, input convolution and its ring
+// update are ONE launch, a workgroup per row.  Prompts: the residual update is a workgroup per row, the
+// convolution a second launch (it reads the neighbouring rows).
+#include "hybrid.h"
+
+namespace {
+
+template <typename T>
+struct ResidualArgs {
+  float* x;
+  const int64_t* ids;
+  const T* table;
+  const T* y;
+  const float* norm_w;
+  T* out;
+  const float* norm2_w;
+  const float* conv_w;
+  float* ring;
+  int d, vocab, ldy, groups, ldo, mode, taps;
+  float eps;
+  OharaSeq seq;
+};
+
+// inv[g] = 1 / sqrt(mean square of group g + eps) for a row in LDS.  Ends with a barrier.
+__device__ __forceinline__ void group_inverse(const float* row, int d, int groups, float eps, float* inv, float* red) {
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int gs = d / groups;
+  if (groups >= 4) {  // a wave per group
+    for (int g = wave; g < groups; g += 4) {
+      float s = 0.f;
+      for (int i = lane; i < gs; i += 64) {
+        const float v = row[g * gs + i];
+        s += v * v;
+      }
+      s = wave_sum(s);
+      if (lane == 0) inv[g] = 1.0f / sqrtf(s / (float)gs + eps);
+    }
+    __syncthreads();
+    return;
+  }
+  for (int g = 0; g < groups; ++g) {
+    float s = 0.f;
+    for (int i = tid; i < gs; i += 256) {
+      const float v = row[g * gs + i];
+      s += v * v;
+    }
+    s = wave_sum(s);
+    if (lane == 0) red[4 * g + wave] = s;
+  }
+  __syncthreads();
+  if (tid < groups) {
+    const float* r = red + 4 * tid;
+    inv[tid] = 1.0f / sqrtf((((r[0] + r[1]) + r[2]) + r[3]) / (float)gs + eps);
+  }
+  __syncthreads();
+}
+
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void residual_norm_kernel(ResidualArgs<T> a) {
+  extern __shared__ __align__(16) float smem[];
+  const int tid = threadIdx.x, row = blockIdx.x, d = a.d;
+  float* ys = smem;                 // the sublayer's output, then the new residual
+  float* inv = ys + ((d + 3) & ~3); // one per group
+  float* red = inv + a.groups;      // 16 partial sums
+  float* xr = a.x + (size_t)row * d;
+  const int gs = d / a.groups;
+  if (a.ids) {
+    int64_t id = a.ids[row];
+    if (id < 0 || id >= a.vocab) id = 0;  // the host validates ids; never read out of bounds
+    const T* src = a.table + (size_t)id * d;
+    for (int i = tid; i < d; i += 256) {
+      const float v = ldv(src + i);
+      ys[i] = v;
+      xr[i] = v;
+    }
+    __syncthreads();
+  } else if (a.y) {
+    const T* yr = a.y + (size_t)row * a.ldy;
+    if (VEC) {
+      for (int i = tid * 4; i < d; i += 1024) {
+        float v[4];
+        ld4(yr + i, v);
+        *reinterpret_cast<float4*>(ys + i) = make_float4(v[0], v[1], v[2], v[3]);
+      }
+    } else {
+      for (int i = tid; i < d; i += 256) ys[i] = ldv(yr + i);
+    }
+    __syncthreads();
+    group_inverse(ys, d, a.groups, a.eps, inv, red);
+    if (VEC) {
+      for (int i = tid * 4; i < d; i += 1024) {
+        float v[4], w[4];
+        ld4(xr + i, v);
+        ld4(a.norm_w + i, w);
+        const float4 s = *reinterpret_cast<const float4*>(ys + i);
+        const float r = inv[i / gs];
+        v[0] += s.x * r * w[0]; v[1] += s.y * r * w[1]; v[2] += s.z * r * w[2]; v[3] += s.w * r * w[3];
+        st4(xr + i, v);
+        *reinterpret_cast<float4*>(ys + i) = make_float4(v[0], v[1], v[2], v[3]);
+      }
+    } else {
+      for (int i = tid; i < d; i += 256) {
+        const float v = xr[i] + ys[i] * inv[i / gs] * a.norm_w[i];
+        xr[i] = v;
+        ys[i] = v;
+      }
+    }
+    __syncthreads();
+  } else {
+    for (int i = tid; i < d; i += 256) ys[i] = xr[i];
+    __syncthreads();
+  }
+  if (a.mode == OHARA_OUT_NONE) return;
+  T* o = a.out + (size_t)row * a.ldo;
+  for (int i = d + tid; i < a.ldo; i += 256) stv(o + i, 0.f);
+  if (a.mode == OHARA_OUT_NORM) {
+    group_inverse(ys, d, a.groups, a.eps, inv, red);
+    for (int i = tid; i < d; i += 256) stv(o + i, ys[i] * inv[i / gs] * a.norm2_w[i]);
+  } else if (a.mode == OHARA_OUT_COPY) {
+    if (VEC) {
+      for (int i = tid * 4; i < d; i += 1024) {
+        const float4 s = *reinterpret_cast<const float4*>(ys + i);
+        const float v[4] = {s.x, s.y, s.z, s.w};
+        st4(o + i, v);
+      }
+    } else {
+      for (int i = tid; i < d; i += 256) stv(o + i, ys[i]);
+    }
+  } else {  // one token per sequence: row = sequence
+    const int pos = seq_start(a.seq, row);
+    float* ring = a.ring + (size_t)seq_slot(a.seq, row) * a.taps * d;
+    const bool live = seq_tokens(a.seq, row) > 0 && pos >= 0;
+    for (int i = tid; i < d; i += 256) {
+      const float cur = ys[i];
+      float c = a.conv_w[(size_t)(a.taps - 1) * d + i] * cur;
+      for (int lag = 1; lag < a.taps; ++lag)
+        if (pos >= lag) c += a.conv_w[(size_t)(a.taps - 1 - lag) * d + i] * ring[(size_t)((pos - lag) % a.taps) * d + i];
+      if (live) ring[(size_t)(pos % a.taps) * d + i] = cur;
+      stv(o + i, cur + c);
+    }
+  }
+}
+
+// out = x + conv(x): a workgroup per (row, 1024 columns), four columns per thread
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void input_conv_kernel(const float* x, int d, const float* w, int taps, const float* ring,
+                                                         T* out, int ldo, OharaSeq q) {
+  const int row = blockIdx.x, b = row / q.seq_len, s = row - b * q.seq_len;
+  const int pos = seq_start(q, b);
+  const float* rg = ring + (size_t)seq_slot(q, b) * taps * d;
+  const float* xr = x + (size_t)row * d;
+  T* o = out + (size_t)row * ldo;
+  const int c0 = blockIdx.y * 1024;
+  if (VEC) {
+    const int i = c0 + threadIdx.x * 4;
+    if (i < d) {
+      float v[4], r[4];
+      ld4(xr + i, v);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) r[u] = v[u];
+      for (int lag = 0; lag < taps; ++lag) {
+        float t[4] = {v[0], v[1], v[2], v[3]}, k[4];
+        if (lag > s) {
+          if (pos + s < lag) break;
+          ld4(rg + (size_t)((pos + s - lag) % taps) * d + i, t);
+        } else if (lag > 0) {
+          ld4(xr - (size_t)lag * d + i, t);
+        }
+        ld4(w + (size_t)(taps - 1 - lag) * d + i, k);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) r[u] += k[u] * t[u];
+      }
+      st4(o + i, r);
+    } else if (i < ldo) {
+      const float z[4] = {0.f, 0.f, 0.f, 0.f};
+      st4(o + i, z);  // d, ldo are multiples of 4 here
+    }
+    return;
+  }
+  for (int i = c0 + threadIdx.x; i < min(ldo, c0 + 1024); i += 256) {
+    if (i >= d) {
+      stv(o + i, 0.f);
+      continue;
+    }
+    float r = xr[i];
+    for (int lag = 0; lag < taps; ++lag) {
+      float t;
+      if (lag > s) {
+        if (pos + s < lag) break;
+        t = rg[(size_t)((pos + s - lag) % taps) * d + i];
+      } else {
+        t = xr[i - (ptrdiff_t)lag * d];
+      }
+      r += w[(size_t)(taps - 1 - lag) * d + i] * t;
+    }
+    stv(o + i, r);
+  }
+}
+
+// the last inputs of every sequence -> ring; blockIdx.y = how many tokens before the last
+template <typename T>
+__global__ __launch_bounds__(256) void ring_store_kernel(const T* src, int ld, int channels, int taps, T* ring, OharaSeq q) {
+  const int b = blockIdx.z, back = blockIdx.y;
+  const int len = seq_tokens(q, b), pos = seq_start(q, b) + len - 1 - back;
+  if (back >= len || pos < 0) return;  // older inputs are in the ring already
+  const T* s = src + ((size_t)b * q.seq_len + (len - 1 - back)) * ld;
+  T* r = ring + ((size_t)seq_slot(q, b) * taps + pos % taps) * channels;
+  for (int i = blockIdx.x * 256 + threadIdx.x; i < channels; i += gridDim.x * 256) r[i] = s[i];
+}
+
+template <typename T>
+int launch_residual(ResidualArgs<T> a, const OharaSeq* seq, hipStream_t st) {
+  if (!a.x || a.d < 1 || a.groups < 1 || a.d % a.groups || !seq_ok(seq)) return OHARA_EINVAL;
+  if (a.ids && (!a.table || a.vocab < 1)) return OHARA_EINVAL;
+  if (!a.ids && a.y && (!a.norm_w || a.ldy < a.d)) return OHARA_EINVAL;
+  if (a.mode < OHARA_OUT_NONE || a.mode > OHARA_OUT_NORM) return OHARA_EINVAL;
+  if (a.mode != OHARA_OUT_NONE && (!a.out || a.ldo < a.d)) return OHARA_EINVAL;
+  if (a.mode == OHARA_OUT_NORM && !a.norm2_w) return OHARA_EINVAL;
+  if (a.mode == OHARA_OUT_CONV && (!a.conv_w || !a.ring || a.taps < 1 || seq->seq_len != 1)) return OHARA_EINVAL;
+  a.seq = *seq;
+  const size_t smem = (((size_t)a.d + 3) / 4 * 4 + a.groups + 16) * sizeof(float);
+  if (smem > 64 * 1024) return OHARA_ESIZE;
+  const dim3 grid((unsigned)(seq->batch * seq->seq_len));
+  const bool vec = (a.d & 3) == 0 && ((a.d / a.groups) & 3) == 0 && (a.ldy & 3) == 0 && (a.ldo & 3) == 0;
+  if (vec) hipLaunchKernelGGL((residual_norm_kernel<T, true>), grid, dim3(256), smem, st, a);
+  else hipLaunchKernelGGL((residual_norm_kernel<T, false>), grid, dim3(256), smem, st, a);
+  return ohara_launch_status();
+}
+
+template <typename T>
+int launch_input_conv(const float* x, int d, const float* w, int taps, const float* ring, T* out, int ldo, const OharaSeq* seq,
+                      hipStream_t st) {
+  if (!x || !w || !ring || !out || d < 1 || taps < 1 || ldo < d || !seq_ok(seq)) return OHARA_EINVAL;
+  const dim3 grid((unsigned)(seq->batch * seq->seq_len), (unsigned)((ldo + 1023) / 1024));
+  if (((d | ldo) & 3) == 0)
+    hipLaunchKernelGGL((input_conv_kernel<T, true>), grid, dim3(256), 0, st, x, d, w, taps, ring, out, ldo, *seq);
+  else
+    hipLaunchKernelGGL((input_conv_kernel<T, false>), grid, dim3(256), 0, st, x, d, w, taps, ring, out, ldo, *seq);
+  return ohara_launch_status();
+}
+
+template <typename T>
+int launch_ring_store(const T* src, int ld, int channels, int taps, T* ring, const OharaSeq* seq, hipStream_t st) {
+  if (!src || !ring || channels < 1 || ld < channels || taps < 1 || !seq_ok(seq)) return OHARA_EINVAL;
+  if (taps == 1) return OHARA_OK;  // nothing is remembered
+  if (taps > 65535 || seq->batch > 65535) return OHARA_ESIZE;
+  const int bx = (channels + 255) / 256 < 64 ? (channels + 255) / 256 : 64;
+  hipLaunchKernelGGL((ring_store_kernel<T>), dim3((unsigned)bx, (unsigned)(taps - 1), (unsigned)seq->batch), dim3(256), 0, st, src,
+                     ld, channels, taps, ring, *seq);
+  return ohara_launch_status();
+}
+
+}  // namespace
+
+extern "C" {
+
+int ohara_residual_norm_bf16(float* x, int d, const int64_t* ids, const uint16_t* table, int vocab, const uint16_t* y,
+                             int ldy, const float* norm_w, int groups, float eps, int out_mode, uint16_t* out, int ldo,
+                             const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
+                             void* stream) {
+  return launch_residual<bf16_t>(ResidualArgs<bf16_t>{x, ids, table, y, norm_w, out, norm2_w, conv_w, ring, d, vocab, ldy,
+                                                      groups, ldo, out_mode, taps, eps, {}}, seq, (hipStream_t)stream);
+}
+int ohara_residual_norm_f32(float* x, int d, const int64_t* ids, const float* table, int vocab, const float* y, int ldy,
+                            const float* norm_w, int groups, float eps, int out_mode, float* out, int ldo,
+                            const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
+                            void* stream) {
+  return launch_residual<float>(ResidualArgs<float>{x, ids, table, y, norm_w, out, norm2_w, conv_w, ring, d, vocab, ldy, groups,
+                                                    ldo, out_mode, taps, eps, {}}, seq, (hipStream_t)stream);
+}
+
+int ohara_input_conv_bf16(const float* x, int d, const float* conv_w, int taps, const float* ring, uint16_t* out, int ldo,
+                          const OharaSeq* seq, void* stream) {
+  return launch_input_conv<bf16_t>(x, d, conv_w, taps, ring, out, ldo, seq, (hipStream_t)stream);
+}
+int ohara_input_conv_f32(const float* x, int d, const float* conv_w, int taps, const float* ring, float* out, int ldo,
+                         const OharaSeq* seq, void* stream) {
+  return launch_input_conv<float>(x, d, conv_w, taps, ring, out, ldo, seq, (hipStream_t)stream);
+}
+
+int ohara_conv_ring_store_bf16(const uint16_t* src, int ld, int channels, int taps, uint16_t* ring, const OharaSeq* seq,
+                               void* stream) {
+  return launch_ring_store<bf16_t>(src, ld, channels, taps, ring, seq, (hipStream_t)stream);
+}
+int ohara_conv_ring_store_f32(const float* src, int ld, int channels, int taps, float* ring, const OharaSeq* seq,
+                              void* stream) {
+  return launch_ring_store<float>(src, ld, channels, taps, ring, seq, (hipStream_t)stream);
+}
+
+}  // extern "C"

@@ -21,6 +21,7 @@ import torch
 
 from . import _lib, ops
 from ._lib import OharaDecodeState, OharaLayer, OharaModel, check, lib
+from .state_cache import SequenceBook
 
 BF16 = torch.bfloat16
 
@@ -73,19 +74,15 @@ def _validate_config(cfg: Config, allow_bias: bool = False) -> None:
         raise ValueError("ohara_amd: Linear biases are served for dense feed-forwards only, by BiasLlama")
 
 
-class KVCache:
+class KVCache(SequenceBook):
     """ohara/modules/kv_cache.py:35-118 (bf16 storage): (batch, T_max, H_kv, D) key and
     value tensors written sequentially.  ``forward`` keeps the reference's semantics
     and error messages for external callers; the model's own path appends inside the
     fused projection kernel and only does the bookkeeping here (``_reserve``)."""
 
     def __init__(self, shape, max_seq_length, idx=None, device=None, dtype=None, int8=False):
-        self.idx = idx
+        super().__init__(shape[0], max_seq_length, idx)
         self.int8 = bool(int8)
-        self.max_seq_length = max_seq_length
-        self.length = 0
-        self.batch_size = None
-        self.lengths = None  # per-sequence lengths, once sequences have advanced by different amounts
         self.dtype = dtype
         storage = torch.int8 if self.int8 else dtype
         self.key = torch.zeros(shape, device=device, dtype=storage)
@@ -100,60 +97,17 @@ class KVCache:
             self.key_scale, self.key_min, self.value_scale, self.value_min = (
                 self.stats[..., i:i + 1].permute(0, 2, 1, 3) for i in range(4))
 
-    def _reserve(self, bsz: int, seq_len: int, start_pos: int) -> int:
-        # ohara/modules/kv_cache.py:80-90, same order
-        if bsz > self.key.size(0):
-            raise ValueError("KV cache batch size is smaller than the input batch")
-        if self.batch_size is not None and bsz != self.batch_size:
-            raise ValueError("KV cache batch size cannot change during decoding")
-        if self.lengths is not None and any(n != self.lengths[0] for n in self.lengths[:bsz]):
-            raise ValueError("KV cache writes must be sequential: the sequences have different lengths, "
-                             "pass one position per sequence")
-        if start_pos != self.length:
-            raise ValueError(
-                f"KV cache writes must be sequential: expected position {self.length}, got {start_pos}"
-            )
-        if start_pos < 0 or start_pos + seq_len > self.max_seq_length:
-            raise ValueError("KV cache position exceeds max_sequence_length")
-        return start_pos + seq_len
-
-    def _commit(self, bsz: int, end: int) -> None:
-        self.length = end
-        self.batch_size = bsz
-        self.lengths = None
-
-    # One position per sequence (no counterpart in the reference, whose cache has a single length):
-    # the same checks as above, sequence by sequence.
-    def _reserve_ragged(self, bsz: int, seq_len: int, starts) -> list:
-        if bsz > self.key.size(0):
-            raise ValueError("KV cache batch size is smaller than the input batch")
-        if self.batch_size is not None and bsz != self.batch_size:
-            raise ValueError("KV cache batch size cannot change during decoding")
-        have = self.lengths if self.lengths is not None else [self.length] * bsz
-        for b, (start, n) in enumerate(zip(starts, have)):
-            if start != n:
-                raise ValueError(f"KV cache writes must be sequential: expected position {n}, got {start} "
-                                 f"(sequence {b})")
-            if start < 0 or start + seq_len > self.max_seq_length:
-                raise ValueError("KV cache position exceeds max_sequence_length")
-        return [start + seq_len for start in starts]
-
-    def _commit_ragged(self, bsz: int, ends) -> None:
-        self.lengths = list(ends)
-        self.length = max(ends)
-        self.batch_size = bsz
-
     def _row_view(self, b: int) -> "KVCache":
         """The cache of sequence b alone, sharing storage."""
         v = KVCache.__new__(KVCache)
-        v.idx, v.int8, v.max_seq_length, v.dtype = self.idx, self.int8, self.max_seq_length, self.dtype
+        SequenceBook.__init__(v, 1, self.max_seq_length, self.idx)
+        v.int8, v.dtype = self.int8, self.dtype
         v.key, v.value = self.key[b:b + 1], self.value[b:b + 1]
         if self.int8:
             v.stats = self.stats[b:b + 1]
             v.key_scale, v.key_min, v.value_scale, v.value_min = (
                 v.stats[..., i:i + 1].permute(0, 2, 1, 3) for i in range(4))
         v.length = (self.lengths[b] if self.lengths is not None else self.length)
-        v.batch_size, v.lengths = None, None
         return v
 
     def forward(self, keys, values, start_pos):

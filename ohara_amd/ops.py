@@ -322,11 +322,20 @@ def advance_ragged(seq_pos: torch.Tensor, active: torch.Tensor | None, new_ids: 
                                      _stream()), "advance_ragged")
 
 
+_zero_draws: dict = {}  # (rows, device) -> fp32 zeros
+
+
 def argmax(logits: torch.Tensor, valid_vocab: int | None = None, next_ids=None, history=None, step_state=None):
-    _need(logits, BF16, "logits")
     b, v = logits.shape
     if next_ids is None:
         next_ids = torch.empty(b, dtype=torch.int64, device=logits.device)
+    if logits.dtype == torch.float32:
+        # the candidates of top-k 1 are the ids tied at the maximum; a draw of 0 takes the lowest of them
+        u = _zero_draws.get((b, logits.device))
+        if u is None:
+            u = _zero_draws[(b, logits.device)] = torch.zeros(b, dtype=torch.float32, device=logits.device)
+        return sample_topk_topp(logits, 1.0, 1, 1.0, u, valid_vocab, out=next_ids, history=history, step_state=step_state)
+    _need(logits, BF16, "logits")
     check(
         lib().ohara_argmax_bf16(
             _ptr(logits), logits.stride(0), b, v, v if valid_vocab is None else valid_vocab, _ptr(next_ids),
@@ -577,4 +586,164 @@ def phi_attn(q, kcache, vcache, cos, sin, rot, batch, seq_len, h, dh, pos, pos_d
     check(lib().ohara_phi_attn_bf16(_ptr(q), q.stride(0), _ptr(kcache), _ptr(vcache), _ptr(cos), _ptr(sin), rot, batch,
                                     seq_len, h, dh, kcache.shape[1], pos, _ptr(pos_dev), n_split, _ptr(workspace), _ptr(out),
                                     _stream()), "phi_attn")
+    return out
+
+
+# ---- hybrid decoders: attention with a distance bias beside recurrent layers -------------------------
+# bf16 or fp32 activations: the entry point follows the dtype of the activations.
+
+F32 = torch.float32
+
+
+def _typed(name: str, dtype):
+    return getattr(lib(), f"ohara_{name}_{'f32' if dtype == F32 else 'bf16'}")
+
+
+def round8(n: int) -> int:
+    return (n + 7) // 8 * 8
+
+
+class Seq:
+    """Which rows of a call belong to which sequence and where they sit (OharaSeq).  ``pos_dev`` (int32): one
+    position for all sequences, or one per sequence with ``per_sequence``; ``lens`` / ``slots`` (int32, one entry per
+    sequence): tokens of each sequence in the call, cache row of each sequence."""
+
+    __slots__ = ("c", "batch", "seq_len", "lens", "_keep")
+
+    def __init__(self, batch: int, seq_len: int, pos: int = 0, pos_dev=None, per_sequence: bool = False, lens=None, slots=None):
+        for name, t in (("pos_dev", pos_dev), ("lens", lens), ("slots", slots)):
+            if t is not None:
+                _need(t, torch.int32, name)
+                if t.numel() < (1 if name == "pos_dev" and not per_sequence else batch):
+                    raise ValueError(f"{name}: one entry per sequence is required")
+        self.batch, self.seq_len, self.lens = batch, seq_len, lens
+        self._keep = (pos_dev, lens, slots)
+        self.c = _lib.OharaSeq(batch, seq_len, int(pos), int(per_sequence), _ptr(pos_dev), _ptr(lens), _ptr(slots))
+
+    @property
+    def rows(self) -> int:
+        return self.batch * self.seq_len
+
+    @property
+    def ref(self):
+        return C.byref(self.c)
+
+
+def residual_norm(x, seq: Seq, dtype, *, ids=None, table=None, y=None, norm_w=None, groups=1, eps=0.0, mode="none",
+                  norm2_w=None, conv_w=None, ring=None):
+    """x (rows, d) fp32 <- table[ids], or x + norm_w * group_rms(y), in place; returns what ``mode`` asks for as
+    (rows, d rounded up to 8) in ``dtype``: "copy" of x, "conv" (x + causal depthwise convolution over time, one token per
+    sequence, ring updated), "norm" (group RMS norm of x times norm2_w), or None."""
+    _need(x, F32, "x")
+    rows, d = x.shape
+    m = {"none": _lib.OUT_NONE, "copy": _lib.OUT_COPY, "conv": _lib.OUT_CONV, "norm": _lib.OUT_NORM}[mode]
+    if rows != seq.rows:
+        raise ValueError("x has one row per token of the call")
+    for t, name in ((y, "y"), (table, "table")):
+        if t is not None:
+            _need(t, dtype, name)
+    out = torch.empty(rows, round8(d), dtype=dtype, device=x.device) if mode != "none" else None
+    check(_typed("residual_norm", dtype)(
+        _ptr(x), d, _ptr(ids), _ptr(table), 0 if table is None else table.shape[0], _ptr(y), 0 if y is None else y.stride(0),
+        _ptr(norm_w), groups, eps, m, _ptr(out), 0 if out is None else out.stride(0), _ptr(norm2_w), _ptr(conv_w),
+        0 if conv_w is None else conv_w.shape[0], _ptr(ring), seq.ref, _stream()), "residual_norm")
+    return out
+
+
+def input_conv(x, conv_w, ring, seq: Seq, dtype):
+    """x (rows, d) fp32 -> x + causal depthwise convolution over time, (rows, d rounded up to 8) in ``dtype``; then the
+    last inputs of every sequence go into the ring."""
+    _need(x, F32, "x")
+    rows, d = x.shape
+    taps = conv_w.shape[0]
+    out = torch.empty(rows, round8(d), dtype=dtype, device=x.device)
+    check(_typed("input_conv", dtype)(_ptr(x), d, _ptr(conv_w), taps, _ptr(ring), _ptr(out), out.stride(0), seq.ref, _stream()),
+          "input_conv")
+    conv_ring_store(x, d, ring, seq)
+    return out
+
+
+def conv_ring_store(src, channels: int, ring, seq: Seq) -> None:
+    """The last inputs of every sequence (the first ``channels`` columns of src) -> ring (cache rows, taps, channels)."""
+    if ring.shape[2] != channels or ring.dtype != src.dtype or src.shape[0] != seq.rows:
+        raise ValueError("ring does not fit the inputs")
+    check(_typed("conv_ring_store", src.dtype)(_ptr(src), src.stride(0), channels, ring.shape[1], _ptr(ring), seq.ref, _stream()),
+          "conv_ring_store")
+
+
+def gemm_f32(x, w, bias=None, w_up=None, cap: float = 0.0, out=None):
+    """fp32 y = x W^T (+ bias, cap * tanh(y / cap)), or silu(x W^T) * (x w_up^T).  x: (rows, K), any row stride."""
+    if x.dtype != F32 or not x.is_cuda or x.stride(1) != 1 or x.shape[1] != w.shape[1]:
+        raise ValueError("x must be an fp32 device matrix with unit column stride and W's columns")
+    rows, n = x.shape[0], w.shape[0]
+    if out is None:
+        out = torch.empty(rows, n, dtype=F32, device=x.device)
+    check(lib().ohara_gemm_f32(_ptr(x), x.stride(0), _ptr(w), _ptr(w_up), _ptr(bias), cap, n, w.shape[1], rows, _ptr(out),
+                               out.stride(0), _stream()), "gemm_f32")
+    return out
+
+
+def gemm_softcap(x, w: PackedLinear, cap: float, out=None):
+    """bf16(cap * tanh(x W^T / cap)) on a packed weight."""
+    _need(x, BF16, "x")
+    rows, k = x.shape
+    if k != w.k:
+        raise ValueError(f"x has {k} columns, weight expects {w.k}")
+    if out is None:
+        out = torch.empty(rows, w.n, dtype=BF16, device=x.device)
+    check(lib().ohara_gemm_softcap_bf16(_ptr(x), x.stride(0), _ptr(w.data), w.n, w.k, cap, rows, _ptr(out), out.stride(0),
+                                        _stream()), "gemm_softcap")
+    return out
+
+
+def qkv_norm_append(p, h, h_kv, dh, dv, qn, kn, eps, kcache, vcache, seq: Seq):
+    """p rows [q; k; v; ...] -> normalised q (rows, h * round8(dh)); keys and values into the caches."""
+    q = torch.empty(p.shape[0], h * round8(dh), dtype=p.dtype, device=p.device)
+    check(_typed("qkv_norm_append", p.dtype)(_ptr(p), p.stride(0), h, h_kv, dh, dv, _ptr(qn), _ptr(kn), eps, _ptr(q), _ptr(kcache),
+                                             _ptr(vcache), kcache.shape[1], seq.ref, _stream()), "qkv_norm_append")
+    return q
+
+
+def attn_bias_workspace(rows, h, dv, n_split, device) -> torch.Tensor:
+    n = lib().ohara_attn_bias_workspace_bytes(rows, h, dv, n_split)
+    if n < 0:
+        raise ValueError("bad attention workspace shape")
+    return torch.zeros(n, dtype=torch.uint8, device=device)  # the chunk counters start at zero
+
+
+def attn_bias(q, kcache, vcache, h, h_kv, dh, dv, scale, slopes, gate, seq: Seq, n_split=1, workspace=None):
+    """Causal attention with the bias -slopes[head] * distance, head outputs times sigmoid(gate) -> (rows, round8(h * dv)).
+    gate: a (rows, h) column slice of the projection (or None)."""
+    out = torch.empty(q.shape[0], round8(h * dv), dtype=q.dtype, device=q.device)
+    check(_typed("attn_bias", q.dtype)(
+        _ptr(q), _ptr(kcache), _ptr(vcache), h, h_kv, dh, dv, kcache.shape[1], scale, _ptr(slopes), _ptr(gate),
+        0 if gate is None else gate.stride(0), n_split, _ptr(workspace), _ptr(out), out.stride(0), seq.ref, _stream()),
+        "attn_bias")
+    return out
+
+
+def delta_step(d: "_lib.OharaDelta", p, state, ring, seq: Seq):
+    """One token per sequence of the gated delta rule -> (rows, round8(heads * vdim)); state and ring updated."""
+    out = torch.empty(p.shape[0], round8(d.heads * d.vdim), dtype=p.dtype, device=p.device)
+    check(_typed("delta_step", p.dtype)(C.byref(d), _ptr(p), p.stride(0), _ptr(state), _ptr(ring), _ptr(out), out.stride(0),
+                                        seq.ref, _stream()), "delta_step")
+    return out
+
+
+def delta_workspace_bytes(heads, dim, vdim, batch, tokens) -> int:
+    n = lib().ohara_delta_workspace_bytes(heads, dim, vdim, batch, tokens)
+    if n < 0:
+        raise ValueError("bad delta rule shape")
+    return n
+
+
+def delta_prefill(d: "_lib.OharaDelta", p, za, zg, state, ring, workspace, seq: Seq):
+    """Any number of tokens per sequence of the gated delta rule; the ring is updated after the call's convolutions."""
+    rows = p.shape[0]
+    out = torch.empty(rows, round8(d.heads * d.vdim), dtype=p.dtype, device=p.device)
+    o_tmp = torch.empty(rows, d.heads * d.vdim, dtype=F32, device=p.device)
+    check(_typed("delta_prefill", p.dtype)(
+        C.byref(d), _ptr(p), p.stride(0), _ptr(za), za.stride(0), _ptr(zg), zg.stride(0), _ptr(state), _ptr(ring),
+        _ptr(workspace), workspace.numel(), _ptr(o_tmp), _ptr(out), out.stride(0), seq.ref, _stream()), "delta_prefill")
+    conv_ring_store(p, 2 * d.kv_heads * d.dim + d.heads * d.vdim, ring, seq)
     return out

@@ -1,0 +1,112 @@
+"""Per-layer sequence state: the bookkeeping every layer cache shares, and the cache of a layer whose
+state is more than keys and values.
+
+``SequenceBook`` keeps how many tokens each row of a cache holds and checks that writes are sequential
+(ohara/modules/kv_cache.py:80-90).  ``ohara_amd.llama.KVCache`` adds keys and values to it, ``LayerState``
+any set of tensors whose first dimension is the row: keys and values, recurrent state, rings of past inputs.
+"""
+
+from __future__ import annotations
+
+
+class SequenceBook:
+    def __init__(self, capacity: int, max_seq_length: int, idx=None):
+        self.idx = idx
+        self.capacity = capacity
+        self.max_seq_length = max_seq_length
+        self.length = 0
+        self.batch_size = None
+        self.lengths = None  # per-sequence lengths, once sequences have advanced by different amounts
+
+    def _reserve(self, bsz: int, seq_len: int, start_pos: int) -> int:
+        # ohara/modules/kv_cache.py:80-90, same order
+        if bsz > self.capacity:
+            raise ValueError("KV cache batch size is smaller than the input batch")
+        if self.batch_size is not None and bsz != self.batch_size:
+            raise ValueError("KV cache batch size cannot change during decoding")
+        if self.lengths is not None and any(n != self.lengths[0] for n in self.lengths[:bsz]):
+            raise ValueError("KV cache writes must be sequential: the sequences have different lengths, "
+                             "pass one position per sequence")
+        if start_pos != self.length:
+            raise ValueError(
+                f"KV cache writes must be sequential: expected position {self.length}, got {start_pos}"
+            )
+        if start_pos < 0 or start_pos + seq_len > self.max_seq_length:
+            raise ValueError("KV cache position exceeds max_sequence_length")
+        return start_pos + seq_len
+
+    def _commit(self, bsz: int, end: int) -> None:
+        self.length = end
+        self.batch_size = bsz
+        self.lengths = None
+
+    # One position per sequence (no counterpart in the reference, whose cache has a single length):
+    # the same checks as above, sequence by sequence.
+    def _reserve_ragged(self, bsz: int, seq_len, starts) -> list:
+        """``seq_len``: the tokens of every sequence, or a list with one count per sequence."""
+        if bsz > self.capacity:
+            raise ValueError("KV cache batch size is smaller than the input batch")
+        if self.batch_size is not None and bsz != self.batch_size:
+            raise ValueError("KV cache batch size cannot change during decoding")
+        have = self.lengths if self.lengths is not None else [self.length] * bsz
+        counts = seq_len if isinstance(seq_len, (list, tuple)) else [seq_len] * bsz
+        for b, (start, n, count) in enumerate(zip(starts, have, counts)):
+            self._check_row(start, n, count, b)
+        return [start + count for start, count in zip(starts, counts)]
+
+    def _check_row(self, start: int, have: int, count: int, b: int) -> None:
+        if start != have:
+            raise ValueError(f"KV cache writes must be sequential: expected position {have}, got {start} "
+                             f"(sequence {b})")
+        if start < 0 or start + count > self.max_seq_length:
+            raise ValueError("KV cache position exceeds max_sequence_length")
+
+    def _commit_ragged(self, bsz: int, ends) -> None:
+        self.lengths = list(ends)
+        self.length = max(ends)
+        self.batch_size = bsz
+
+    # Some rows of the cache only (``slots``: the row of each sequence of the call).
+    def _reserve_rows(self, slots, counts, starts) -> list:
+        if len(set(slots)) != len(slots) or min(slots) < 0 or max(slots) >= self.capacity:
+            raise ValueError("slots must be distinct rows of the cache")
+        for b, (slot, start, count) in enumerate(zip(slots, starts, counts)):
+            self._check_row(start, self.row_length(slot), count, b)
+        return [start + count for start, count in zip(starts, counts)]
+
+    def _commit_rows(self, slots, ends) -> None:
+        lengths = [self.row_length(b) for b in range(self.capacity)]
+        for slot, end in zip(slots, ends):
+            lengths[slot] = end
+        self._commit_ragged(self.capacity, lengths)
+
+    def row_length(self, b: int) -> int:
+        if self.lengths is not None:
+            return self.lengths[b]
+        return self.length if self.batch_size is not None and b < self.batch_size else 0
+
+
+class LayerState(SequenceBook):
+    """Named tensors of one layer, (rows, ...) each, readable as attributes.  They need no clearing when a
+    row is taken by another sequence: what lies before a sequence's start is never read."""
+
+    int8 = False
+
+    def __init__(self, max_seq_length: int, tensors: dict, idx=None):
+        super().__init__(next(iter(tensors.values())).shape[0], max_seq_length, idx)
+        self.tensors = dict(tensors)
+
+    def __getattr__(self, name):
+        tensors = self.__dict__.get("tensors", {})
+        if name in tensors:
+            return tensors[name]
+        raise AttributeError(name)
+
+    def _row_view(self, b: int) -> "LayerState":
+        """The state of sequence b alone, sharing storage."""
+        v = LayerState(self.max_seq_length, {k: t[b:b + 1] for k, t in self.tensors.items()}, self.idx)
+        v.length = self.row_length(b)
+        return v
+
+    def nbytes(self) -> int:
+        return sum(t.numel() * t.element_size() for t in self.tensors.values())
