@@ -702,6 +702,212 @@ def bitnet_phase_timeline(dev, batch=1, steps=16):
     return out
 
 
+def povazen_size(name):
+    """(config dict of the hybrid model, Config keywords of a Llama of the same width, depth, heads and feed-forward)."""
+    d, n, H, G, dh, ff = {"d1024": (1024, 8, 8, 4, 128, 2816), "d2048": (2048, 8, 16, 4, 128, 5632)}[name]
+    mlp = {"kind": "dense", "ff": ff}
+    delta = {"type": "channel_delta", "mixer": {"heads": H, "kv_heads": H, "dim": dh, "vdim": dh, "conv": 4}, "mlp": mlp}
+    att = {"type": "attention", "mixer": {"heads": H, "kv_heads": G, "dim": dh, "vdim": dh, "scale": dh ** -0.5}, "mlp": mlp}
+    cfg = {"width": d, "vocab": 32000, "canon": {"taps": 4}, "norm": {"eps": 1e-6, "groups": 1}, "logit_softcap": 30.0,
+           "layers": ([delta] * 3 + [att]) * (n // 4)}
+    llama = dict(vocab_size=32000, hidden_size=d, intermediate_size=ff, num_attention_heads=H, num_key_value_heads=G,
+                 num_hidden_layers=n, dropout=0.0)
+    return cfg, llama
+
+
+def povazen_state(cfg, dev, rank=128, seed=5):
+    """Random weights of a hybrid config: matrices N(0, 1/columns), unit norms, decays of some tens of tokens."""
+    g = torch.Generator(device=dev).manual_seed(seed)
+    n = lambda *shape, s=1.0: (torch.randn(*shape, generator=g, device=dev) * s).to(torch.bfloat16)  # noqa: E731
+    lin = lambda o, i: n(o, i, s=i ** -0.5)  # noqa: E731
+    one = lambda k: torch.ones(k, device=dev, dtype=torch.bfloat16)  # noqa: E731
+    d = cfg["width"]
+    st = {"embed": n(cfg["vocab"], d), "head": lin(cfg["vocab"], d), "final.norm": one(d)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, ff = f"l{i}.", layer["mixer"], layer["mlp"]["ff"]
+        H, K, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        st.update({p + "norm1": one(d), p + "norm2": one(d), p + "canon1": n(d, cfg["canon"]["taps"], s=0.2),
+                   p + "mlp.gate": lin(ff, d), p + "mlp.up": lin(ff, d), p + "mlp.down": lin(d, ff)})
+        p += "mix."
+        st.update({p + "k": lin(K * D, d), p + "o": lin(d, H * V)})
+        if layer["type"] == "attention":
+            st.update({p + "q": lin(H * D, d), p + "v": lin(K * V, d), p + "q.b": n(H * D, s=0.1), p + "k.b": n(K * D, s=0.1),
+                       p + "v.b": n(K * V, s=0.1), p + "q.norm": one(H * D), p + "k.norm": one(K * D), p + "g": lin(H, d)})
+        else:
+            st.update({p + "q": lin(K * D, d), p + "v": lin(H * V, d), p + "b": lin(H, d), p + "norm": one(V),
+                       p + "A_log": torch.zeros(H, device=dev, dtype=torch.bfloat16), p + "dt_bias": n(H * D) - 3.0,
+                       p + "a1": lin(rank, d), p + "a2": lin(H * D, rank), p + "g1": lin(rank, d), p + "g2": lin(H * V, rank)})
+            for c, k in (("q", K * D), ("k", K * D), ("v", H * V)):
+                st[p + c + ".conv"] = n(k, m["conv"], s=0.5)
+    return st
+
+
+def _time_model_prefill(model, B, S, dev, reps=3):
+    ids = torch.randint(0, model.config.vocab_size, (B, S), device=dev)
+    cache = model.build_kv_cache(B)
+    best = None
+    for _ in range(reps + 1):
+        for c in cache:
+            c.length, c.batch_size, c.lengths = 0, None, None
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        model(ids, cache, 0, last_only=True)
+        torch.cuda.synchronize()
+        dt = time.perf_counter() - t0
+        best = dt if best is None else min(best, dt)
+    return {"ms": round(best * 1e3, 3), "tokens_per_s": round(B * S / best, 1)}
+
+
+def _time_model_decode(model, B, context, steps=64):
+    sess = model.session(B, steps + 32)
+    sess.prefill(torch.randint(0, model.config.vocab_size, (B, context)))
+    sess.capture()
+    sess.run(8)
+    torch.cuda.synchronize()
+    best = None
+    for _ in range(2):
+        t0 = time.perf_counter()
+        sess.run(steps // 4)
+        torch.cuda.synchronize()
+        dt = (time.perf_counter() - t0) / (steps // 4)
+        best = dt if best is None else min(best, dt)
+    sess.check_error()
+    return {"ms_per_step": round(best * 1e3, 4), "tokens_per_s": round(B / best, 1)}
+
+
+FP32_MFMA_PEAK_TFLOPS = 157.3
+
+
+def _hbm(t, by):
+    return {"us": round(t * 1e6, 1), "GBs": round(by / t / 1e9, 1), "frac_of_hbm_peak": round(by / t / 1e9 / HBM_PEAK_GBS, 4)}
+
+
+def _flops(t, fl, peak):
+    return {"us": round(t * 1e6, 1), "TFLOPs": round(fl / t / 1e12, 1), "frac_of_peak": round(fl / t / 1e12 / peak, 4)}
+
+
+def bench_povazen_kernels(cfg, dev):
+    """The hybrid model's own kernels beside the like kernels of Llama at one layer's sizes."""
+    from ohara_amd import ops
+    from ohara_amd.hybrid import distance_slopes
+    from ohara_amd.povazen import Povazen, PovazenConfig
+
+    bf = torch.bfloat16
+    model = Povazen(PovazenConfig.from_dict({**cfg, "layers": cfg["layers"][2:4]}, 4096),
+                    {k.replace("l2.", "l0.").replace("l3.", "l1."): v for k, v in povazen_state(cfg, dev).items()
+                     if not k.startswith(("l0.", "l1."))}, device=dev)
+    delta, att = (b["mixer"] for b in model.layers)
+    H, G, D, V, d = att.heads, att.kv_heads, att.dim, att.vdim, cfg["width"]
+    slopes = distance_slopes(H).to(dev)
+    rnd = lambda *shape, dt=bf: torch.randn(*shape, device=dev).to(dt)  # noqa: E731
+    rows = []
+
+    def timed(fn, n=8):  # n calls per graph: what a single-launch graph costs to start would swamp the small kernels
+        return graph_time(lambda: [fn() for _ in range(n)], iters=20) / n
+
+    for B, L in ((1, 4096), (8, 4096), (32, 2048)):
+        q, k, v = rnd(B, H * D), rnd(B, L, G, D), rnd(B, L, G, V)
+        ns = att.n_split(B, L)
+        ws = ops.attn_bias_workspace(B, H, V, ns, dev)
+        gate = rnd(B, H)
+        seq = ops.Seq(B, 1, L - 1)
+        by = 2.0 * G * (D + V) * B * L
+        row = {"kernel": "decode attention", "batch": B, "context": L,
+               "attn_bias_kernel": _hbm(timed(lambda: ops.attn_bias(q, k, v, H, G, D, V, 0.1, slopes, gate, seq, ns, ws)), by)}
+        n2 = max(1, min(1024 // (B * G), L // 128, 64))
+        ws2 = ops.attn_workspace(B, H, G, D, n2, dev)
+        row["llama attn_decode_kernel"] = _hbm(timed(lambda: ops.attn_decode(q, k, v, H, G, D, L, n2, ws2)), by)
+        rows.append(row)
+    for B, S in ((1, 4096), (8, 1024)):
+        q, k, v = rnd(B * S, H * D), rnd(B, S, G, D), rnd(B, S, G, V)
+        gate = rnd(B * S, H)
+        seq = ops.Seq(B, S, 0)
+        fl = 2.0 * B * H * (D + V) * S * (S + 1) / 2
+        rows.append({"kernel": "prompt attention", "batch": B, "tokens": S,
+                     "attn_bias_prefill_kernel": _flops(timed(lambda: ops.attn_bias(q, k, v, H, G, D, V, 0.1, slopes, gate, seq)),
+                                                        fl, MFMA_BF16_PEAK_TFLOPS),
+                     "llama attn_prefill_kernel": _flops(timed(lambda: ops.attn_prefill(q, k, v, H, G, D, 0, S)), fl,
+                                                         MFMA_BF16_PEAK_TFLOPS)})
+    x = rnd(1, 2048)
+    wn = torch.ones(2048, device=dev, dtype=bf)
+    base = _hbm(timed(lambda: ops.rmsnorm(x, wn)), 2.0 * 2 * 2048)
+    for B in (1, 8, 32):
+        st = delta.state(B, 4096)
+        p = rnd(B, delta.proj.n)
+        seq = ops.Seq(B, 1, 100)
+        h = delta.heads
+        by = 2.0 * 4 * B * h * delta.dim * delta.vdim + 2.0 * (delta.a2.numel() + delta.g2.numel())
+        row = {"kernel": "delta rule, one token", "batch": B,
+               "delta_step_kernel": _hbm(timed(lambda: ops.delta_step(delta._c, p, st["delta"], st["ring"], seq)), by)}
+        xf, y = rnd(B, d, dt=torch.float32), rnd(B, d)
+        blk = model.layers[0]
+        ring = blk["conv"].state(B)
+        row["residual_norm_kernel (norm, residual, convolution)"] = _hbm(timed(lambda: ops.residual_norm(
+            xf, seq, bf, y=y, norm_w=blk["norm1"].w, groups=1, eps=1e-6, mode="conv", conv_w=blk["conv"].w, ring=ring)),
+            B * d * (8.0 + 2 + 2 + 4 * 4 + 4))
+        row["llama rmsnorm_kernel, one row"] = base
+        rows.append(row)
+    for B, S in ((1, 4096), (8, 1024)):
+        st = delta.state(B, 4096)
+        p = rnd(B * S, delta.proj.n)
+        za, zg = rnd(B * S, delta.heads * delta.dim) - 3.0, rnd(B * S, delta.heads * delta.vdim)
+        ws = delta._workspace(B, S)
+        seq = ops.Seq(B, S, 0)
+        t = timed(lambda: ops.delta_prefill(delta._c, p, za, zg, st["delta"], st["ring"], ws, seq))
+        # the recurrence's own work: decay, two products with the state and the write, per token and head
+        fl = 7.0 * B * S * delta.heads * delta.dim * delta.vdim
+        xf, y = rnd(B * S, d, dt=torch.float32), rnd(B * S, d)
+        blk = model.layers[0]
+        ring = blk["conv"].state(B)
+        tn = timed(lambda: ops.residual_norm(xf, seq, bf, y=y, norm_w=blk["norm1"].w, groups=1, eps=1e-6, mode="none"))
+        tc = timed(lambda: ops.input_conv(xf, blk["conv"].w, ring, seq, bf))
+        tr = timed(lambda: ops.rmsnorm(y, blk["norm1"].w.to(bf)))
+        big = rnd(B * S, att.proj.n)
+        kc, vc = rnd(B, S, G, D), rnd(B, S, G, V)
+        tq = timed(lambda: ops.qkv_norm_append(big, H, G, D, V, att.q_norm, att.k_norm, 1e-6, kc, vc, seq))
+        rows.append({"kernel": "delta rule, prompt", "batch": B, "tokens": S, "delta_prefill (3 kernels)": _flops(t, fl, FP32_MFMA_PEAK_TFLOPS),
+                     "residual_norm_kernel": _hbm(tn, B * S * d * 10.0), "input_conv_kernel + ring": _hbm(tc, B * S * d * 6.0),
+                     "qkv_norm_append_kernel": _hbm(tq, 4.0 * B * S * (H * D + G * (D + V))),
+                     "llama rmsnorm_kernel": _hbm(tr, B * S * d * 4.0)})
+    return rows
+
+
+def bench_povazen(dev, sizes=("d1024", "d2048"), kernels=True):
+    """Prefill and decode of the hybrid model (three delta-rule layers to one attention layer, SwiGLU everywhere, random
+    weights) beside Llama at the same width, depth, heads and feed-forward."""
+    from ohara_amd.llama import Config, Llama
+    from ohara_amd.povazen import Povazen, PovazenConfig
+
+    out = {}
+    for name in sizes:
+        cfg, kw = povazen_size(name)
+        res = {"layers": len(cfg["layers"]), "width": cfg["width"]}
+        lcfg = Config(**kw, max_sequence_length=4608)
+        g = torch.Generator(device=dev).manual_seed(0)
+        d, f, kvw = lcfg.hidden_size, lcfg.intermediate_size, lcfg.num_key_value_heads * (lcfg.hidden_size // lcfg.num_attention_heads)
+        n = lambda *shape: (torch.randn(*shape, generator=g, device=dev) * 0.02).to(torch.bfloat16)  # noqa: E731
+        one = torch.ones(d, dtype=torch.bfloat16, device=dev)
+        st = {"token_emb.weight": n(32000, d), "vocab_proj.weight": n(32000, d), "norm.weight": one}
+        for i in range(lcfg.num_hidden_layers):
+            p = f"layers.{i}."
+            st.update({p + "attn.query.weight": n(d, d), p + "attn.key.weight": n(kvw, d), p + "attn.value.weight": n(kvw, d),
+                       p + "attn.proj.weight": n(d, d), p + "ff.up.weight": n(f, d), p + "ff.gate.weight": n(f, d),
+                       p + "ff.down.weight": n(d, f), p + "norm1.weight": one, p + "norm2.weight": one})
+        for label, make in (("povazen", lambda: Povazen(PovazenConfig.from_dict(cfg, 4608), povazen_state(cfg, dev), device=dev)),
+                            ("llama", lambda: Llama(lcfg, st, device=dev))):
+            model = make()
+            res[label] = {"parameters": sum(t.numel() for t in model.parameters()),
+                          "prefill": {f"{B}x{S}": _time_model_prefill(model, B, S, dev) for B, S in ((1, 512), (1, 4096), (8, 1024))},
+                          "decode": {f"batch {B}, context {L}": _time_model_decode(model, B, L)
+                                     for B, L in ((1, 1024), (1, 4096), (8, 4096), (32, 2048))}}
+            del model
+            torch.cuda.empty_cache()
+        if kernels:
+            res["kernels"] = bench_povazen_kernels(cfg, dev)
+        out[name] = res
+    return out
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -731,6 +937,8 @@ def main():
                     help="run the d12 prefill figures (tiled MFMA GEMMs, prefill attention) alone and exit")
     ap.add_argument("--attention-only", action="store_true",
                     help="run the GQA decode-attention figures (bf16 and int8 cache) alone and exit")
+    ap.add_argument("--povazen-only", type=str, nargs="?", const="d1024,d2048", default="", metavar="SIZES",
+                    help="run the Povazen prefill, decode and kernel figures beside Llama at equal sizes alone and exit")
     ap.add_argument("--phi-decode-only", type=int, default=0, metavar="B",
                     help="run 12 eager Phi-2 decode steps of B sequences at context 1024 and exit (profiling workload)")
     args = ap.parse_args()
@@ -752,6 +960,9 @@ def main():
             dst.copy_(src)
         torch.cuda.synchronize()
         del src, dst
+    if args.povazen_only:
+        print(json.dumps(bench_povazen(dev, tuple(args.povazen_only.split(","))), indent=1))
+        return
     if args.phi_decode_only:
         print(json.dumps(phi_decode_only(dev, args.phi_decode_only)))
         return

@@ -299,26 +299,30 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
 }
 
 // ---- many query tokens: bf16 MFMA --------------------------------------------------------------
-// A workgroup (4 waves) owns 64 queries of one (sequence, head), a wave 16 of them; keys and values come
+// A workgroup (4 waves) owns 64 * QW queries of one (sequence, head), a wave 16 * QW of them; keys and values come
 // through LDS in tiles of 64 positions, the values transposed.  Both products are formed transposed,
 // S^T = K Q^T and O^T = V^T P^T, so a lane's scores belong to one query and its weights are, register for register,
 // the B operand of the second product (k-slot 8 g + i of window w <-> position 32 w + 4 g + i for i < 4,
-// 32 w + 16 + 4 g + i - 4 otherwise).
-template <int DP, int VP>
-__global__ __launch_bounds__(256, (DP + VP > 384 ? 1 : 2)) void attn_bias_prefill_kernel(AttnBiasArgs<bf16_t> a, int nqb) {
+// 32 w + 16 + 4 g + i - 4 otherwise).  The running maximum is kept as an integer in log2 units, so most tiles leave it
+// alone and the accumulators need no rescaling.
+template <int DP, int VP, int QW>
+__global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias_prefill_kernel(AttnBiasArgs<bf16_t> a, int nqb) {
   constexpr int KT = 64, NK = DP / 32, ND = VP / 16;
   constexpr int LDK = DP + 8, LDV = KT + 4;
   constexpr int CK = DP / 8, CV = VP / 8;            // 16-byte pieces per row
   constexpr int NPK = KT * CK / 256, NPV = KT * CV / 256;
+  constexpr int GP = NPV >= 4 ? 4 : NPV;             // positions a thread transposes together
   __shared__ __align__(16) bf16_t Ks[KT][LDK];
   __shared__ __align__(16) bf16_t Vt[VP][LDV];
+  // A column's positions are rotated by four per group of eight columns: the threads that transpose one position group
+  // write columns eight apart, which would land on two banks.
+  auto vt_off = [](int col, int p) { return GP == 4 ? ((p + 4 * (col >> 3)) & (KT - 1)) : p; };
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int m = lane & 15, g = lane >> 4;
   const int qblk = nqb - 1 - (int)blockIdx.x;  // long contexts first
   const int h = blockIdx.y, b = blockIdx.z;
   const int len = seq_tokens(a.seq, b), pos0 = seq_start(a.seq, b);
-  const int q0 = qblk * 64;
-  // (padding: nothing but zeros in the columns past h*V, and those only matter for live rows)
+  const int q0 = qblk * 64 * QW;
   if (q0 >= len || pos0 < 0 || pos0 + len > a.Tmax) return;
   const int Dq = (a.D + 7) & ~7, Vq = (a.V + 7) & ~7;
   const int kvh = h / (a.H / a.G);
@@ -326,24 +330,35 @@ __global__ __launch_bounds__(256, (DP + VP > 384 ? 1 : 2)) void attn_bias_prefil
   const bf16_t* kb = a.kc + base * kd + (size_t)kvh * Dq;
   const bf16_t* vb = a.vc + base * vd + (size_t)kvh * Vq;
   const int Lall = pos0 + len;
-  const int kv_end = min(pos0 + q0 + 64, Lall);
-  const int wq0 = q0 + wave * 16, qi = wq0 + m;
-  const int qpos = pos0 + min(qi, len - 1);   // lanes past the end repeat the last query and are not stored
-  const int wave_last = min(pos0 + wq0 + 15, Lall - 1);
+  const int kv_end = min(pos0 + q0 + 64 * QW, Lall);
+  const int wq0 = q0 + wave * 16 * QW;
+  const int wave_last = min(pos0 + wq0 + 16 * QW - 1, Lall - 1);
   const float sl2 = a.scale * OHARA_LOG2E, slope = a.slopes[h] * OHARA_LOG2E;
-  const size_t qrow = (size_t)b * a.seq.seq_len + min(qi, len - 1);
 
-  uint4 qf[NK];
+  uint4 qf[QW][NK];
+  int qpos[QW];
+  size_t qrow[QW];
 #pragma unroll
-  for (int j = 0; j < NK; ++j)
-    qf[j] = 32 * j + 8 * g < Dq ? ldg16(a.q + (qrow * a.H + h) * Dq + 32 * j + 8 * g) : make_uint4(0, 0, 0, 0);
-
-  f32x4 o[ND];
+  for (int u = 0; u < QW; ++u) {
+    const int qi = min(wq0 + 16 * u + m, len - 1);  // lanes past the end repeat the last query and are not stored
+    qpos[u] = pos0 + qi;
+    qrow[u] = (size_t)b * a.seq.seq_len + qi;
 #pragma unroll
-  for (int t = 0; t < ND; ++t) o[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  float mrun = -INFINITY, lrun = 0.f;
+    for (int j = 0; j < NK; ++j)
+      qf[u][j] = 32 * j + 8 * g < Dq ? ldg16(a.q + (qrow[u] * a.H + h) * Dq + 32 * j + 8 * g) : make_uint4(0, 0, 0, 0);
+  }
+  f32x4 o[QW][ND];
+  float mrun[QW], lrun[QW];
+#pragma unroll
+  for (int u = 0; u < QW; ++u) {
+    mrun[u] = -INFINITY;
+    lrun[u] = 0.f;
+#pragma unroll
+    for (int t = 0; t < ND; ++t) o[u][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  }
 
   uint4 kr[NPK], vr[NPV];
+  const int vrow = tid / CV, vcol = 8 * (tid % CV);
   auto load_tile = [&](int t0) {
 #pragma unroll
     for (int i = 0; i < NPK; ++i) {
@@ -351,10 +366,9 @@ __global__ __launch_bounds__(256, (DP + VP > 384 ? 1 : 2)) void attn_bias_prefil
       kr[i] = (t0 + p < Lall && 8 * c < Dq) ? ldg16(kb + (size_t)(t0 + p) * kd + 8 * c) : make_uint4(0, 0, 0, 0);
     }
 #pragma unroll
-    for (int i = 0; i < NPV; ++i) {
-      // neighbouring threads take neighbouring positions of the same columns: the transposed writes spread over banks
-      const int idx = tid + 256 * i, p = idx % KT, c = idx / KT;
-      vr[i] = (t0 + p < Lall && 8 * c < Vq) ? ldg16(vb + (size_t)(t0 + p) * vd + 8 * c) : make_uint4(0, 0, 0, 0);
+    for (int i = 0; i < NPV; ++i) {  // GP consecutive positions per thread and group: the transposed write is wide
+      const int p = GP * (vrow + (i / GP) * (256 / CV)) + i % GP;
+      vr[i] = (t0 + p < Lall && vcol < Vq) ? ldg16(vb + (size_t)(t0 + p) * vd + vcol) : make_uint4(0, 0, 0, 0);
     }
   };
   auto store_tile = [&]() {
@@ -364,13 +378,34 @@ __global__ __launch_bounds__(256, (DP + VP > 384 ? 1 : 2)) void attn_bias_prefil
       *reinterpret_cast<uint4*>(&Ks[idx / CK][8 * (idx % CK)]) = kr[i];
     }
 #pragma unroll
-    for (int i = 0; i < NPV; ++i) {
-      const int idx = tid + 256 * i, p = idx % KT, c = 8 * (idx / KT);
-      const uint32_t w[4] = {vr[i].x, vr[i].y, vr[i].z, vr[i].w};
+    for (int grp = 0; grp < NPV / GP; ++grp) {
+      const int p0 = GP * (vrow + grp * (256 / CV));
+      uint32_t w[GP][4];
+#pragma unroll
+      for (int r = 0; r < GP; ++r) {
+        w[r][0] = vr[GP * grp + r].x; w[r][1] = vr[GP * grp + r].y;
+        w[r][2] = vr[GP * grp + r].z; w[r][3] = vr[GP * grp + r].w;
+      }
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        Vt[c + 2 * e][p] = (bf16_t)(w[e] & 0xffffu);
-        Vt[c + 2 * e + 1][p] = (bf16_t)(w[e] >> 16);
+        bf16_t* c0 = &Vt[vcol + 2 * e][vt_off(vcol + 2 * e, p0)];
+        bf16_t* c1 = &Vt[vcol + 2 * e + 1][vt_off(vcol + 2 * e + 1, p0)];
+        if constexpr (GP == 1) {
+          *c0 = (bf16_t)(w[0][e] & 0xffffu);
+          *c1 = (bf16_t)(w[0][e] >> 16);
+        } else {
+          const uint32_t lo01 = (w[0][e] & 0xffffu) | (w[1][e] << 16);
+          const uint32_t hi01 = (w[0][e] >> 16) | (w[1][e] & 0xffff0000u);
+          if constexpr (GP == 4) {
+            const uint32_t lo23 = (w[2][e] & 0xffffu) | (w[3][e] << 16);
+            const uint32_t hi23 = (w[2][e] >> 16) | (w[3][e] & 0xffff0000u);
+            *reinterpret_cast<uint2*>(c0) = make_uint2(lo01, lo23);
+            *reinterpret_cast<uint2*>(c1) = make_uint2(hi01, hi23);
+          } else {
+            *reinterpret_cast<uint32_t*>(c0) = lo01;
+            *reinterpret_cast<uint32_t*>(c1) = hi01;
+          }
+        }
       }
     }
   };
@@ -382,104 +417,155 @@ __global__ __launch_bounds__(256, (DP + VP > 384 ? 1 : 2)) void attn_bias_prefil
     __syncthreads();
     if (t0 + KT < kv_end) load_tile(t0 + KT);  // in flight during the products
     if (t0 > wave_last) continue;               // wholly masked for this wave (barriers stay uniform)
-    f32x4 s[4];
+    f32x4 s[4][QW];
 #pragma unroll
     for (int kk = 0; kk < 4; ++kk) {
-      s[kk] = (f32x4){0.f, 0.f, 0.f, 0.f};
+      uint4 kf[NK];  // read before the first product, not one by one between them
+#pragma unroll
+      for (int j = 0; j < NK; ++j) kf[j] = *reinterpret_cast<const uint4*>(&Ks[kk * 16 + m][32 * j + 8 * g]);
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int u = 0; u < QW; ++u) s[kk][u] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int j = 0; j < NK; ++j)
-        s[kk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-            __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(&Ks[kk * 16 + m][32 * j + 8 * g])),
-            __builtin_bit_cast(bf16x8, qf[j]), s[kk], 0, 0, 0);
+#pragma unroll
+        for (int u = 0; u < QW; ++u)
+          s[kk][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kf[j]), __builtin_bit_cast(bf16x8, qf[u][j]),
+                                                             s[kk][u], 0, 0, 0);
     }
-    float tmax = -INFINITY;
-    const float rel = (float)(t0 + 4 * g - qpos);  // -(distance) of the lane's first position
+    const bool edge = t0 + KT - 1 > pos0 + wq0;  // (wave-uniform) the tile reaches past the wave's first query
 #pragma unroll
-    for (int kk = 0; kk < 4; ++kk)
+    for (int u = 0; u < QW; ++u) {
+      float tmax = -INFINITY;
+      const float b0 = slope * (float)(t0 + 4 * g - qpos[u]);  // minus the distance of the lane's first position
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        float v = s[kk][i] * sl2 + slope * (rel + (float)(16 * kk + i));
-        if (t0 + 16 * kk + 4 * g + i > qpos) v = -INFINITY;
-        s[kk][i] = v;
-        tmax = fmaxf(tmax, v);
+      for (int kk = 0; kk < 4; ++kk)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          float v = __builtin_fmaf(s[kk][u][i], sl2, __builtin_fmaf(slope, (float)(16 * kk + i), b0));
+          if (edge && t0 + 16 * kk + 4 * g + i > qpos[u]) v = -INFINITY;
+          s[kk][u][i] = v;
+          tmax = fmaxf(tmax, v);
+        }
+      tmax = lane_xor_max<32>(lane_xor_max<16>(tmax));
+      const float mn = fmaxf(mrun[u], ceilf(tmax));  // finite: position 0 is visible to every query
+      const float corr = __builtin_amdgcn_exp2f(mrun[u] - mn);
+      mrun[u] = mn;
+      float ts = 0.f;
+#pragma unroll
+      for (int kk = 0; kk < 4; ++kk)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          s[kk][u][i] = __builtin_amdgcn_exp2f(s[kk][u][i] - mn);
+          ts += s[kk][u][i];
+        }
+      lrun[u] = lrun[u] * corr + ts;  // this lane's share; the four lane groups are added at the end
+      if (__any(corr != 1.0f)) {
+#pragma unroll
+        for (int t = 0; t < ND; ++t)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) o[u][t][i] *= corr;
       }
-    tmax = lane_xor_max<32>(lane_xor_max<16>(tmax));
-    const float mn = fmaxf(mrun, tmax);  // finite: position 0 is visible to every query
-    const float corr = __builtin_amdgcn_exp2f(mrun - mn);
-    mrun = mn;
-    float ts = 0.f;
-#pragma unroll
-    for (int kk = 0; kk < 4; ++kk)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        s[kk][i] = __builtin_amdgcn_exp2f(s[kk][i] - mn);
-        ts += s[kk][i];
-      }
-    lrun = lrun * corr + ts;  // this lane's share; the four lane groups are added at the end
-    if (__any(corr != 1.0f)) {
-#pragma unroll
-      for (int t = 0; t < ND; ++t)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) o[t][i] *= corr;
     }
 #pragma unroll
     for (int w = 0; w < 2; ++w) {
       // three bf16 terms per weight: p = hi + mid + lo exactly
-      uint32_t hi[4], mid[4], lo[4];
+      uint4 pt[QW][3];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const float p0 = s[2 * w + (e >> 1)][2 * (e & 1)], p1 = s[2 * w + (e >> 1)][2 * (e & 1) + 1];
-        hi[e] = pack_bf(p0, p1);
-        const float r0 = p0 - lo_bf(hi[e]), r1 = p1 - hi_bf(hi[e]);
-        mid[e] = pack_bf(r0, r1);
-        lo[e] = pack_bf(r0 - lo_bf(mid[e]), r1 - hi_bf(mid[e]));
+      for (int u = 0; u < QW; ++u) {
+        uint32_t hi[4], mid[4], lo[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float p0 = s[2 * w + (e >> 1)][u][2 * (e & 1)], p1 = s[2 * w + (e >> 1)][u][2 * (e & 1) + 1];
+          hi[e] = pack_bf(p0, p1);
+          const float r0 = p0 - lo_bf(hi[e]), r1 = p1 - hi_bf(hi[e]);
+          mid[e] = pack_bf(r0, r1);
+          lo[e] = pack_bf(r0 - lo_bf(mid[e]), r1 - hi_bf(mid[e]));
+        }
+        pt[u][0] = make_uint4(hi[0], hi[1], hi[2], hi[3]);
+        pt[u][1] = make_uint4(mid[0], mid[1], mid[2], mid[3]);
+        pt[u][2] = make_uint4(lo[0], lo[1], lo[2], lo[3]);
       }
-      const bf16x8 ph = __builtin_bit_cast(bf16x8, make_uint4(hi[0], hi[1], hi[2], hi[3]));
-      const bf16x8 pm = __builtin_bit_cast(bf16x8, make_uint4(mid[0], mid[1], mid[2], mid[3]));
-      const bf16x8 pl = __builtin_bit_cast(bf16x8, make_uint4(lo[0], lo[1], lo[2], lo[3]));
+      constexpr int NB = ND < 4 || QW == 2 ? 2 : 4;  // 16-column blocks whose fragments are read together
 #pragma unroll
-      for (int t = 0; t < ND; ++t) {
-        const uint2 v0 = *reinterpret_cast<const uint2*>(&Vt[16 * t + m][32 * w + 4 * g]);
-        const uint2 v1 = *reinterpret_cast<const uint2*>(&Vt[16 * t + m][32 * w + 16 + 4 * g]);
-        const bf16x8 vf = __builtin_bit_cast(bf16x8, make_uint4(v0.x, v0.y, v1.x, v1.y));
-        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph, o[t], 0, 0, 0);
-        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pm, o[t], 0, 0, 0);
-        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, o[t], 0, 0, 0);
+      for (int t1 = 0; t1 < ND; t1 += NB) {
+        uint4 vf[NB];
+#pragma unroll
+        for (int t = 0; t < NB; ++t) {
+          const int col = 16 * (t1 + t) + m;
+          const uint2 v0 = *reinterpret_cast<const uint2*>(&Vt[col][vt_off(col, 32 * w + 4 * g)]);
+          const uint2 v1 = *reinterpret_cast<const uint2*>(&Vt[col][vt_off(col, 32 * w + 16 + 4 * g)]);
+          vf[t] = make_uint4(v0.x, v0.y, v1.x, v1.y);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int k = 0; k < 3; ++k)
+#pragma unroll
+          for (int t = 0; t < NB; ++t)
+#pragma unroll
+            for (int u = 0; u < QW; ++u)
+              o[u][t1 + t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, vf[t]),
+                                                                     __builtin_bit_cast(bf16x8, pt[u][k]), o[u][t1 + t], 0, 0, 0);
       }
     }
   }
-  lrun = lane_xor_sum<32>(lane_xor_sum<16>(lrun));
-  if (qi >= len) return;
-  const float gt = a.gate ? sigmoid_x(ldv(a.gate + qrow * a.ldg + h)) : 1.0f;
-  const float inv = gt / lrun;
-  bf16_t* orow = a.out + qrow * a.ldo;
 #pragma unroll
-  for (int t = 0; t < ND; ++t)
+  for (int u = 0; u < QW; ++u) {
+    const float l = lane_xor_sum<32>(lane_xor_sum<16>(lrun[u]));
+    if (wq0 + 16 * u + m >= len) continue;
+    const float inv = (a.gate ? sigmoid_x(ldv(a.gate + qrow[u] * a.ldg + h)) : 1.0f) / l;
+    bf16_t* orow = a.out + qrow[u] * a.ldo;
+    const bool wide = ((a.V | a.ldo) & 3) == 0;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int c = 16 * t + 4 * g + i;
-      if (c < a.V) orow[(size_t)h * a.V + c] = f2bf(o[t][i] * inv);
+    for (int t = 0; t < ND; ++t) {
+      const int c = 16 * t + 4 * g;
+      if (wide) {
+        const float v[4] = {o[u][t][0] * inv, o[u][t][1] * inv, o[u][t][2] * inv, o[u][t][3] * inv};
+        if (c < a.V) st4(orow + (size_t)h * a.V + c, v);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (c + i < a.V) orow[(size_t)h * a.V + c + i] = f2bf(o[u][t][i] * inv);
+      }
     }
-  if (h == 0 && g == 0)
-    for (int i = a.H * a.V; i < a.ldo; ++i) orow[i] = 0;
+    if (h == 0 && g == 0)
+      for (int i = a.H * a.V; i < a.ldo; ++i) orow[i] = 0;
+  }
 }
 
-template <int DP>
-int launch_prefill_v(const AttnBiasArgs<bf16_t>& a, dim3 grid, int nqb, hipStream_t st) {
-  if (a.V <= 32) hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, 32>), grid, dim3(256), 0, st, a, nqb);
-  else if (a.V <= 64) hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, 64>), grid, dim3(256), 0, st, a, nqb);
-  else if (a.V <= 128) hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, 128>), grid, dim3(256), 0, st, a, nqb);
-  else hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, 256>), grid, dim3(256), 0, st, a, nqb);
+template <int DP, int VP>
+int launch_prefill_dv(const AttnBiasArgs<bf16_t>& a, hipStream_t st) {
+  // 32 queries per wave where there are enough workgroups for it: half the LDS reads per product
+  constexpr int QW = DP + VP <= 256 ? 2 : 1;
+  static int cus = 0;
+  if (!cus) {
+    int dev = 0;
+    if (hipGetDevice(&dev) != hipSuccess || hipDeviceGetAttribute(&cus, hipDeviceAttributeMultiprocessorCount, dev) != hipSuccess)
+      cus = 256;
+  }
+  const int n2 = (a.seq.seq_len + 64 * QW - 1) / (64 * QW), n1 = (a.seq.seq_len + 63) / 64;
+  if (QW > 1 && (int64_t)n2 * a.H * a.seq.batch >= 2 * (int64_t)cus)
+    hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, VP, QW>), dim3((unsigned)n2, (unsigned)a.H, (unsigned)a.seq.batch), dim3(256),
+                       0, st, a, n2);
+  else
+    hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, VP, 1>), dim3((unsigned)n1, (unsigned)a.H, (unsigned)a.seq.batch), dim3(256),
+                       0, st, a, n1);
   return ohara_launch_status();
 }
 
+template <int DP>
+int launch_prefill_v(const AttnBiasArgs<bf16_t>& a, hipStream_t st) {
+  if (a.V <= 32) return launch_prefill_dv<DP, 32>(a, st);
+  if (a.V <= 64) return launch_prefill_dv<DP, 64>(a, st);
+  if (a.V <= 128) return launch_prefill_dv<DP, 128>(a, st);
+  return launch_prefill_dv<DP, 256>(a, st);
+}
+
 int launch_prefill(const AttnBiasArgs<bf16_t>& a, hipStream_t st) {
-  const int nqb = (a.seq.seq_len + 63) / 64;
-  const dim3 grid((unsigned)nqb, (unsigned)a.H, (unsigned)a.seq.batch);
-  if (a.D <= 32) return launch_prefill_v<32>(a, grid, nqb, st);
-  if (a.D <= 64) return launch_prefill_v<64>(a, grid, nqb, st);
-  if (a.D <= 128) return launch_prefill_v<128>(a, grid, nqb, st);
-  return launch_prefill_v<256>(a, grid, nqb, st);
+  if (a.D <= 32) return launch_prefill_v<32>(a, st);
+  if (a.D <= 64) return launch_prefill_v<64>(a, st);
+  if (a.D <= 128) return launch_prefill_v<128>(a, st);
+  return launch_prefill_v<256>(a, st);
 }
 
 template <typename T>

@@ -41,9 +41,7 @@ struct DeltaArgs {
 __host__ __device__ __forceinline__ int up(int v, int m) { return (v + m - 1) / m * m; }
 
 // ---- one token -------------------------------------------------------------------------------
-constexpr int STEP_ROWS = 16;  // state rows a thread holds
-
-template <typename T, int NT>
+template <typename T, int NT, int STEP_ROWS>  // threads; state rows a thread holds at most
 __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaArgs<T> a) {
   constexpr int NW = NT / 64;
   __shared__ __align__(16) float qs[256], ks[256], gs[256], vs[256], us[256], gate[256];
@@ -90,34 +88,54 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaArgs<T> a) {
     else if (i < 2 * D) ks[i - D] = y;
     else vs[i - 2 * D] = y;
   }
-  // decays and output gates: eight lanes per row of a2 / g2
+  // decays and output gates: eight lanes per row of a2 / g2, two rows and 128 columns in flight
   {
     const int l8 = tid & 7;
     const float na = dd.neg_a[h];
-    const T* a1 = p + dd.off_a;
-    const T* g1 = p + dd.off_g;
-    for (int r0 = 0; r0 < D + V; r0 += NT / 8) {
-      const int r = r0 + (tid >> 3);
-      const bool live = r < D + V, isa = r < D;
-      const int n = isa ? dd.rank_a : dd.rank_g;
-      const T* wrow = isa ? (const T*)dd.a2 + ((size_t)h * D + r) * n : (const T*)dd.g2 + ((size_t)h * V + (r - D)) * n;
-      const T* xr = isa ? a1 : g1;
-      float s = 0.f;
-      if (live)
-        for (int i = 8 * l8; i < n; i += 64) {
-          Raw8<T> wv, xv;
-          wv.load(wrow + i);
-          xv.load(xr + i);
-          float wf[8], xf[8];
-          wv.get(wf);
-          xv.get(xf);
+    constexpr int RP = NT / 8;  // rows per pass
+    for (int r0 = 0; r0 < D + V; r0 += 2 * RP) {
+      float s[2] = {0.f, 0.f};
+      const int nmax = max(dd.rank_a, dd.rank_g);
+      for (int i0 = 0; i0 < nmax; i0 += 128) {
+        Raw8<T> wv[2][2], xv[2][2];
 #pragma unroll
-          for (int u = 0; u < 8; ++u) s = __builtin_fmaf(wf[u], xf[u], s);
+        for (int u = 0; u < 2; ++u) {
+          const int r = r0 + u * RP + (tid >> 3);
+          const bool isa = r < D;
+          const int n = isa ? dd.rank_a : dd.rank_g;
+          const T* wrow = isa ? (const T*)dd.a2 + ((size_t)h * D + r) * n : (const T*)dd.g2 + ((size_t)h * V + (r - D)) * n;
+          const T* xr = p + (isa ? dd.off_a : dd.off_g);
+#pragma unroll
+          for (int e = 0; e < 2; ++e) {
+            const int i = i0 + 64 * e + 8 * l8;
+            if (r < D + V && i < n) {
+              wv[u][e].load(wrow + i);
+              xv[u][e].load(xr + i);
+            } else {
+              wv[u][e].zero();
+              xv[u][e].zero();
+            }
+          }
         }
-      s = lanes_sum<4, 1>(s);
-      if (live && l8 == 0) {
-        if (isa) gs[r] = expf(na * softplus_x(s + dd.dt_bias[(size_t)h * D + r]));
-        else gate[r - D] = sigmoid_x(s);
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+          for (int e = 0; e < 2; ++e) {
+            float wf[8], xf[8];
+            wv[u][e].get(wf);
+            xv[u][e].get(xf);
+#pragma unroll
+            for (int c = 0; c < 8; ++c) s[u] = __builtin_fmaf(wf[c], xf[c], s[u]);
+          }
+      }
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        const int r = r0 + u * RP + (tid >> 3);
+        const float z = lanes_sum<4, 1>(s[u]);
+        if (r < D + V && l8 == 0) {
+          if (r < D) gs[r] = expf(na * softplus_x(z + dd.dt_bias[(size_t)h * D + r]));
+          else gate[r - D] = sigmoid_x(z);
+        }
       }
     }
   }
@@ -198,8 +216,47 @@ __host__ __device__ __forceinline__ size_t chunk_floats(int D, int V) {
   return (size_t)3 * C * Dp + (size_t)C * Vq + C * C + Dp;
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void chunk_solve_kernel(DeltaArgs<T> a) {
+// Convolution + silu of the 8 channels ch .. ch+7 at the four tokens t .. t+3 of this call (TAPS at compile time: the
+// rows' loads are issued together); tokens from len on give zero.
+template <typename T, int TAPS>
+__device__ __forceinline__ void conv8x4(const DeltaArgs<T>& a, const T* prow, const T* ring, int channels, int pos0, int len,
+                                        int t, int ch, float (&y)[4][8]) {
+  constexpr int NR = 4 + TAPS - 1;
+  Raw8<T> raw[NR];
+#pragma unroll
+  for (int j = 0; j < NR; ++j) {
+    const int s = t - (TAPS - 1) + j;
+    if (s >= 0 && s < len) raw[j].load(prow + (size_t)s * a.ldp + ch);
+    else if (s < 0 && pos0 + s >= 0) raw[j].load(ring + (size_t)((pos0 + s) % TAPS) * channels + ch);
+    else raw[j].zero();
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int c = 0; c < 8; ++c) y[i][c] = 0.f;
+#pragma unroll
+  for (int k = 0; k < TAPS; ++k) {
+    float w[8];
+    const float* wp = a.d.conv_w + (size_t)k * channels + ch;
+    ld4(wp, w);
+    ld4(wp + 4, w + 4);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float x[8];
+      raw[i + k].get(x);
+#pragma unroll
+      for (int c = 0; c < 8; ++c) y[i][c] = __builtin_fmaf(w[c], x[c], y[i][c]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int c = 0; c < 8; ++c) y[i][c] = t + i < len ? silu_x(y[i][c]) : 0.f;
+}
+
+// TAPS > 0: that many taps and head sizes that are multiples of 8 (16-byte loads); 0: any.
+template <typename T, int TAPS>
+__global__ __launch_bounds__(256, 2) void chunk_solve_kernel(DeltaArgs<T> a) {
   extern __shared__ __align__(16) float sm[];
   const OharaDelta& dd = a.d;
   const int H = dd.heads, D = dd.dim, V = dd.vdim;
@@ -222,73 +279,168 @@ __global__ __launch_bounds__(256) void chunk_solve_kernel(DeltaArgs<T> a) {
   const int nqk = dd.kv_heads * D, channels = 2 * nqk + H * V, taps = dd.taps;
   const T* ring = a.ring + (size_t)slot * taps * channels;
   const T* prow = a.p + (size_t)b * a.seq.seq_len * a.ldp;  // row of the sequence's first token in this call
-  // convolution + silu of channel ch at token s of this call
-  auto conv = [&](int s, int ch) {
-    float c = 0.f;
-    for (int lag = 0; lag < taps; ++lag) {
-      float x;
-      if (lag <= s) x = ldv(prow + (size_t)(s - lag) * a.ldp + ch);
-      else if (pos0 + s >= lag) x = ldv(ring + (size_t)((pos0 + s - lag) % taps) * channels + ch);
-      else break;
-      c += dd.conv_w[(size_t)(taps - 1 - lag) * channels + ch] * x;
-    }
-    return silu_x(c);
-  };
-  for (int i = tid; i < C * Dp; i += 256) {
-    const int t = i / Dp, c = i - t * Dp;
-    const bool in = t < n && c < D;
-    Q[t * LD + c] = in ? conv(s0 + t, kvh * D + c) : 0.f;
-    K[t * LD + c] = in ? conv(s0 + t, nqk + kvh * D + c) : 0.f;
-    float lg = 0.f;
-    if (in) {
-      const size_t row = (size_t)b * a.seq.seq_len + s0 + t;
-      lg = dd.neg_a[h] * softplus_x(ldv(a.za + row * a.ldza + (size_t)h * D + c) + dd.dt_bias[(size_t)h * D + c]);
-    }
-    G[t * LD + c] = lg;
-  }
-  for (int i = tid; i < C * Vq; i += 256) {
-    const int t = i / Vq, c = i - t * Vq;
-    X[i] = t < n && c < V ? conv(s0 + t, 2 * nqk + h * V + c) : 0.f;
-  }
+  const T* zrow = a.za + (size_t)b * a.seq.seq_len * a.ldza + (size_t)h * D;
+  const float na = dd.neg_a[h];
   if (tid < C) beta[tid] = tid < n ? sigmoid_x(ldv(prow + (size_t)(s0 + tid) * a.ldp + dd.off_b + h)) : 0.f;
-  __syncthreads();
-  // unit q and k; running sums
-  for (int r = wave; r < 2 * C; r += 4) {
-    float* x = (r < C ? Q + r * LD : K + (r - C) * LD);
-    float s = 0.f;
-    for (int i = lane; i < D; i += 64) s += x[i] * x[i];
-    s = 1.0f / sqrtf(wave_sum(s) + UNIT_EPS);
-    if (r < C) s *= 1.0f / sqrtf((float)D);
-    for (int i = lane; i < D; i += 64) x[i] *= s;
-  }
-  for (int c = tid; c < Dp; c += 256) {
-    float s = 0.f;
-    for (int t = 0; t < C; ++t) {
-      s += G[t * LD + c];
-      G[t * LD + c] = s;
-    }
-  }
-  __syncthreads();
-  // A and B, one (i, j) pair per thread and round: the two diagonal 16 x 16 blocks and the one below
-  for (int blk = 0; blk < 4; ++blk) {
-    const int i = (blk >> 1) * 16 + (tid & 15), j = (blk & 1) * 16 + (tid >> 4);
-    float sa = 0.f, sb = 0.f;
-    if (blk != 1) {
-      const float *ki = K + i * LD, *qi = Q + i * LD, *gi = G + i * LD, *kj = K + j * LD, *gj = G + j * LD;
-      if (j <= i) {
-        for (int c = 0; c < D; c += 4) {  // columns past D are zero
-          const float4 k1 = *reinterpret_cast<const float4*>(ki + c), q1 = *reinterpret_cast<const float4*>(qi + c);
-          const float4 g1 = *reinterpret_cast<const float4*>(gi + c), k2 = *reinterpret_cast<const float4*>(kj + c);
-          const float4 g2 = *reinterpret_cast<const float4*>(gj + c);
-          const float e0 = k2.x * __expf(g1.x - g2.x), e1 = k2.y * __expf(g1.y - g2.y);
-          const float e2 = k2.z * __expf(g1.z - g2.z), e3 = k2.w * __expf(g1.w - g2.w);
-          sa += k1.x * e0; sa += k1.y * e1; sa += k1.z * e2; sa += k1.w * e3;
-          sb += q1.x * e0; sb += q1.y * e1; sb += q1.z * e2; sb += q1.w * e3;
-        }
+  if constexpr (TAPS > 0) {
+    const int d8 = D / 8, v8 = V / 8;
+    for (int it = tid; it < (2 * d8 + v8) * (C / 4); it += 256) {
+      const int t = 4 * (it / (2 * d8 + v8)), c8 = it % (2 * d8 + v8);
+      const int ch = c8 < d8 ? kvh * D + 8 * c8
+                             : (c8 < 2 * d8 ? nqk + kvh * D + 8 * (c8 - d8) : 2 * nqk + h * V + 8 * (c8 - 2 * d8));
+      float y[4][8];
+      conv8x4<T, TAPS>(a, prow, ring, channels, pos0, len, s0 + t, ch, y);
+      float* dst = c8 < d8 ? Q + t * LD + 8 * c8 : (c8 < 2 * d8 ? K + t * LD + 8 * (c8 - d8) : X + t * Vq + 8 * (c8 - 2 * d8));
+      const int ld = c8 < 2 * d8 ? LD : Vq;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        *reinterpret_cast<float4*>(dst + i * ld) = make_float4(y[i][0], y[i][1], y[i][2], y[i][3]);
+        *reinterpret_cast<float4*>(dst + i * ld + 4) = make_float4(y[i][4], y[i][5], y[i][6], y[i][7]);
       }
     }
-    A[i * (C + 4) + j] = j < i ? sa * beta[i] : 0.f;
+    // decays: 8 channels of two tokens per thread and round
+    for (int it = tid; it < d8 * (C / 2); it += 256) {
+      const int t = it / d8, c = 8 * (it % d8);
+      Raw8<T> z[2];
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        if (t + 16 * i < n) z[i].load(zrow + (size_t)(s0 + t + 16 * i) * a.ldza + c);
+        else z[i].zero();
+      }
+      float bias[8];
+      ld4(dd.dt_bias + (size_t)h * D + c, bias);
+      ld4(dd.dt_bias + (size_t)h * D + c + 4, bias + 4);
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        float x[8];
+        z[i].get(x);
+#pragma unroll
+        for (int u = 0; u < 8; ++u) x[u] = t + 16 * i < n ? na * softplus_x(x[u] + bias[u]) : 0.f;
+        float* dst = G + (t + 16 * i) * LD + c;
+        *reinterpret_cast<float4*>(dst) = make_float4(x[0], x[1], x[2], x[3]);
+        *reinterpret_cast<float4*>(dst + 4) = make_float4(x[4], x[5], x[6], x[7]);
+      }
+    }
+    for (int i = tid; i < C * (Dp - D); i += 256) {
+      const int t = i / (Dp - D), c = D + i % (Dp - D);
+      Q[t * LD + c] = K[t * LD + c] = G[t * LD + c] = 0.f;
+    }
+    for (int i = tid; i < C * (Vq - V); i += 256) X[(i / (Vq - V)) * Vq + V + i % (Vq - V)] = 0.f;
+  } else {
+    auto conv = [&](int s, int ch) {
+      float c = 0.f;
+      for (int lag = 0; lag < taps; ++lag) {
+        float x;
+        if (lag <= s) x = ldv(prow + (size_t)(s - lag) * a.ldp + ch);
+        else if (pos0 + s >= lag) x = ldv(ring + (size_t)((pos0 + s - lag) % taps) * channels + ch);
+        else break;
+        c += dd.conv_w[(size_t)(taps - 1 - lag) * channels + ch] * x;
+      }
+      return silu_x(c);
+    };
+    for (int i = tid; i < C * Dp; i += 256) {
+      const int t = i / Dp, c = i - t * Dp;
+      const bool in = t < n && c < D;
+      Q[t * LD + c] = in ? conv(s0 + t, kvh * D + c) : 0.f;
+      K[t * LD + c] = in ? conv(s0 + t, nqk + kvh * D + c) : 0.f;
+      G[t * LD + c] = in ? na * softplus_x(ldv(zrow + (size_t)(s0 + t) * a.ldza + c) + dd.dt_bias[(size_t)h * D + c]) : 0.f;
+    }
+    for (int i = tid; i < C * Vq; i += 256) {
+      const int t = i / Vq, c = i - t * Vq;
+      X[i] = t < n && c < V ? conv(s0 + t, 2 * nqk + h * V + c) : 0.f;
+    }
+  }
+  __syncthreads();
+  // unit q and k, and the diagonal of B: eight lanes per token; running sums: a channel per thread
+  {
+    const int t = tid >> 3, l8 = tid & 7;
+    float *q = Q + t * LD, *k = K + t * LD, sq = 0.f, sk = 0.f, qk = 0.f;
+    for (int c = 4 * l8; c < Dp; c += 32) {
+      const float4 x = *reinterpret_cast<const float4*>(q + c), y = *reinterpret_cast<const float4*>(k + c);
+      sq += ((x.x * x.x + x.y * x.y) + x.z * x.z) + x.w * x.w;
+      sk += ((y.x * y.x + y.y * y.y) + y.z * y.z) + y.w * y.w;
+      qk += ((x.x * y.x + x.y * y.y) + x.z * y.z) + x.w * y.w;
+    }
+    const float iq = (1.0f / sqrtf(lanes_sum<4, 1>(sq) + UNIT_EPS)) * (1.0f / sqrtf((float)D));
+    const float ik = 1.0f / sqrtf(lanes_sum<4, 1>(sk) + UNIT_EPS);
+    qk = lanes_sum<4, 1>(qk) * iq * ik;
+    for (int c = 4 * l8; c < Dp; c += 32) {
+      float4* x = reinterpret_cast<float4*>(q + c);
+      float4* y = reinterpret_cast<float4*>(k + c);
+      *x = make_float4(x->x * iq, x->y * iq, x->z * iq, x->w * iq);
+      *y = make_float4(y->x * ik, y->y * ik, y->z * ik, y->w * ik);
+    }
+    if (l8 == 0) B[t * (C + 4) + t] = qk;
+  }
+  for (int c = tid; c < Dp; c += 256) {
+    float v[C];
+#pragma unroll
+    for (int t = 0; t < C; ++t) v[t] = G[t * LD + c];
+#pragma unroll
+    for (int t = 1; t < C; ++t) v[t] += v[t - 1];
+#pragma unroll
+    for (int t = 1; t < C; ++t) G[t * LD + c] = v[t];
+  }
+  // above the diagonal
+  for (int i = tid; i < C * C; i += 256) {
+    const int r = i / C, c = i % C;
+    if (c > r) B[r * (C + 4) + c] = 0.f;
+    if (c >= r) A[r * (C + 4) + c] = 0.f;
+  }
+  __syncthreads();
+  // Below the diagonal inside the two 16 x 16 blocks: a pair (i, j) per thread (120 each), exponents as they are.
+  if (tid < 240) {
+    const int blk = tid >= 120, q = tid - 120 * blk;
+    int i = (int)((1.0f + sqrtf(1.0f + 8.0f * (float)q)) * 0.5f);  // row of the q-th pair: i (i - 1) / 2 <= q
+    while (i * (i - 1) / 2 > q) --i;
+    while (i * (i + 1) / 2 <= q) ++i;
+    const int j = q - i * (i - 1) / 2 + 16 * blk;
+    i += 16 * blk;
+    const float *ki = K + i * LD, *qi = Q + i * LD, *gi = G + i * LD, *kj = K + j * LD, *gj = G + j * LD;
+    float sa = 0.f, sb = 0.f;
+#pragma unroll 2
+    for (int c = 0; c < D; c += 4) {  // columns past D are zero
+      const float4 k1 = *reinterpret_cast<const float4*>(ki + c), q1 = *reinterpret_cast<const float4*>(qi + c);
+      const float4 g1 = *reinterpret_cast<const float4*>(gi + c), k2 = *reinterpret_cast<const float4*>(kj + c);
+      const float4 g2 = *reinterpret_cast<const float4*>(gj + c);
+      const float e0 = k2.x * __expf(g1.x - g2.x), e1 = k2.y * __expf(g1.y - g2.y);
+      const float e2 = k2.z * __expf(g1.z - g2.z), e3 = k2.w * __expf(g1.w - g2.w);
+      sa += k1.x * e0; sa += k1.y * e1; sa += k1.z * e2; sa += k1.w * e3;
+      sb += q1.x * e0; sb += q1.y * e1; sb += q1.z * e2; sb += q1.w * e3;
+    }
+    A[i * (C + 4) + j] = sa * beta[i];
     B[i * (C + 4) + j] = sb;
+  }
+  // The block of tokens 16 .. 31 against 0 .. 15 on MFMA, both sides scaled to the sum R at token 15:
+  // exp(G_i - G_j) = exp(G_i - R) exp(R - G_j), neither exponent positive.  Waves 0, 1: A; 2, 3: B; each half of the
+  // channels.  (A product's k-slot g of step j stands for channel 4 g + j of its 16.)
+  {
+    const int m = lane & 15, g = lane >> 4;
+    const float* left = (wave < 2 ? K : Q) + (16 + m) * LD;
+    const float *gl = G + (16 + m) * LD, *kr = K + m * LD, *gr = G + m * LD, *R = G + 15 * LD;
+    f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int c = (wave & 1) * (Dp / 2) + 4 * g; c < (wave & 1) * (Dp / 2) + Dp / 2; c += 16) {
+      const float4 l = *reinterpret_cast<const float4*>(left + c), g1 = *reinterpret_cast<const float4*>(gl + c);
+      const float4 r = *reinterpret_cast<const float4*>(kr + c), g2 = *reinterpret_cast<const float4*>(gr + c);
+      const float4 ref = *reinterpret_cast<const float4*>(R + c);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(l.x * __expf(g1.x - ref.x), r.x * __expf(ref.x - g2.x), acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(l.y * __expf(g1.y - ref.y), r.y * __expf(ref.y - g2.y), acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(l.z * __expf(g1.z - ref.z), r.z * __expf(ref.z - g2.z), acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(l.w * __expf(g1.w - ref.w), r.w * __expf(ref.w - g2.w), acc, 0, 0, 0);
+    }
+    float* dst = (wave < 2 ? A : B) + (16 + 4 * g) * (C + 4) + m;
+    if (wave & 1) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) dst[r * (C + 4)] = acc[r];
+    }
+    __syncthreads();
+    if (!(wave & 1)) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float v = dst[r * (C + 4)] + acc[r];
+        dst[r * (C + 4)] = wave < 2 ? v * beta[16 + 4 * g + r] : v;
+      }
+    }
   }
   __syncthreads();
   float* w = a.ws + (((size_t)b * H + h) * a.nchunks + ci) * chunk_floats(D, V);
@@ -298,45 +450,58 @@ __global__ __launch_bounds__(256) void chunk_solve_kernel(DeltaArgs<T> a) {
   float* wU = wK + C * Dp;
   float* wB = wU + C * Vq;
   float* wG = wB + C * C;
-  // forward substitution, a column per thread: rows of A are read by all lanes at once
+  // forward substitution, a column per thread: rows of A are read by all lanes at once, the next one ahead of its use
   for (int c = tid; c < Dp + Vq; c += 256) {
     float x[C];
     const bool isw = c < Dp;
     const int vc = c - Dp;
 #pragma unroll
-    for (int t = 0; t < C; ++t) x[t] = beta[t] * (isw ? K[t * LD + c] * expf(G[t * LD + c]) : X[t * Vq + vc]);
+    for (int t = 0; t < C; ++t) x[t] = beta[t] * (isw ? K[t * LD + c] * __expf(G[t * LD + c]) : X[t * Vq + vc]);
     float* dst = isw ? wW + c : wU + vc;
     const int ld = isw ? Dp : Vq;
+    float4 row[2][C / 4];
+    row[1][0] = *reinterpret_cast<const float4*>(A + (C + 4));
     dst[0] = x[0];
 #pragma unroll
     for (int t = 1; t < C; ++t) {
-      const float* ar = A + t * (C + 4);
+      if (t + 1 < C) {
+#pragma unroll
+        for (int j = 0; j < (t + 4) / 4; ++j) row[(t + 1) & 1][j] = *reinterpret_cast<const float4*>(A + (t + 1) * (C + 4) + 4 * j);
+      }
       float s = x[t];
 #pragma unroll
-      for (int j = 0; j < t; ++j) s -= ar[j] * x[j];
+      for (int j = 0; j < t; ++j) {
+        const float4 r = row[t & 1][j / 4];
+        s -= ((j & 3) == 0 ? r.x : ((j & 3) == 1 ? r.y : ((j & 3) == 2 ? r.z : r.w))) * x[j];
+      }
       x[t] = s;
       dst[(size_t)t * ld] = s;
       __builtin_amdgcn_sched_barrier(0);  // row by row: hoisting the reads of all of A would spill
     }
   }
-  for (int i = tid; i < C * Dp; i += 256) {
+  for (int i = 4 * tid; i < C * Dp; i += 1024) {
     const int t = i / Dp, c = i - t * Dp;
-    wQ[i] = Q[t * LD + c] * expf(G[t * LD + c]);
+    const float4 q = *reinterpret_cast<const float4*>(Q + t * LD + c), g = *reinterpret_cast<const float4*>(G + t * LD + c);
+    *reinterpret_cast<float4*>(wQ + i) = make_float4(q.x * __expf(g.x), q.y * __expf(g.y), q.z * __expf(g.z), q.w * __expf(g.w));
   }
-  for (int i = tid; i < C * Dp; i += 256) {
+  for (int i = 4 * tid; i < C * Dp; i += 1024) {
     const int c = i / C, t = i - c * C;
-    wK[i] = K[t * LD + c] * expf(G[(C - 1) * LD + c] - G[t * LD + c]);
+    const float last = G[(C - 1) * LD + c];
+    float v[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) v[u] = K[(t + u) * LD + c] * __expf(last - G[(t + u) * LD + c]);
+    *reinterpret_cast<float4*>(wK + i) = make_float4(v[0], v[1], v[2], v[3]);
   }
   for (int i = tid; i < C * C; i += 256) wB[i] = B[(i / C) * (C + 4) + (i % C)];
-  for (int c = tid; c < Dp; c += 256) wG[c] = expf(G[(C - 1) * LD + c]);
+  for (int c = tid; c < Dp; c += 256) wG[c] = __expf(G[(C - 1) * LD + c]);
 }
 
 // The state over the chunks.  v_mfma_f32_16x16x4_f32: A lane (row = lane & 15, k = lane >> 4), B lane (k = lane >> 4,
 // column = lane & 15), result row 4 (lane >> 4) + r, column lane & 15.  A step of 16 k's takes four products whose k-slot g
 // of product j stands for k = 4 g + j, so a lane fetches the four A elements it needs as one float4.
 template <typename T, int DPT>  // Dp / 16
-__global__ __launch_bounds__(256) void chunk_walk_kernel(DeltaArgs<T> a) {
-  constexpr int Dp = 16 * DPT, MT = (DPT + 3) / 4, LS = 17;
+__global__ __launch_bounds__(256, (DPT > 8 ? 1 : 2)) void chunk_walk_kernel(DeltaArgs<T> a) {
+  constexpr int Dp = 16 * DPT, MT = (DPT + 3) / 4, LS = 20;  // row stride: the four k-slots of a product on different banks
   __shared__ float Sl[Dp * LS];
   __shared__ float Un[C * LS];
   const OharaDelta& dd = a.d;
@@ -364,32 +529,34 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(DeltaArgs<T> a) {
   const float* w = a.ws + ((size_t)b * H + h) * a.nchunks * cf;
   const bool left = wave < 2;           // waves 0, 1: u; waves 2, 3: o
   const int mrow = 16 * (wave & 1);     // this wave's token rows
-  // operands of a chunk, fetched one chunk ahead
-  float4 fa[DPT], fk[MT][2], fg[MT], fb[2];
-  float fu[4];
-  auto fetch = [&](const float* x) {
+  // operands of a chunk: two sets, the next chunk's loads are in flight during this one's products
+  struct Operands {
+    float4 a[DPT], k[MT][2], g[MT], b[2];
+    float u[4];
+  } op[2];
+  auto fetch = [&](const float* x, Operands& f) {
     const float* ap = x + (left ? 0 : C * Dp) + (size_t)(mrow + m) * Dp + 4 * g;
 #pragma unroll
-    for (int i = 0; i < DPT; ++i) fa[i] = *reinterpret_cast<const float4*>(ap + 16 * i);
+    for (int i = 0; i < DPT; ++i) f.a[i] = *reinterpret_cast<const float4*>(ap + 16 * i);
     const float* kp = x + 2 * C * Dp;
     const float* up_ = kp + C * Dp;
     const float* bp = up_ + C * Vq;
     const float* gp = bp + C * C;
+    if (left) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) f.u[r] = up_[(size_t)(mrow + 4 * g + r) * Vq + v0 + m];
+    } else {
+#pragma unroll
+      for (int j = 0; j < 2; ++j) f.b[j] = *reinterpret_cast<const float4*>(bp + (size_t)(mrow + m) * C + 16 * j + 4 * g);
+    }
 #pragma unroll
     for (int i = 0; i < MT; ++i) {
       const int tile = wave + 4 * i;
       if (tile < DPT) {
 #pragma unroll
-        for (int j = 0; j < 2; ++j) fk[i][j] = *reinterpret_cast<const float4*>(kp + (size_t)(16 * tile + m) * C + 16 * j + 4 * g);
-        fg[i] = *reinterpret_cast<const float4*>(gp + 16 * tile + 4 * g);
+        for (int j = 0; j < 2; ++j) f.k[i][j] = *reinterpret_cast<const float4*>(kp + (size_t)(16 * tile + m) * C + 16 * j + 4 * g);
+        f.g[i] = *reinterpret_cast<const float4*>(gp + 16 * tile + 4 * g);
       }
-    }
-    if (left) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) fu[r] = up_[(size_t)(mrow + 4 * g + r) * Vq + v0 + m];
-    } else {
-#pragma unroll
-      for (int j = 0; j < 2; ++j) fb[j] = *reinterpret_cast<const float4*>(bp + (size_t)(mrow + m) * C + 16 * j + 4 * g);
     }
   };
   auto mul4 = [&](float4 av, const float* bcol, f32x4 c) {  // bcol: row 4 g of the step's B rows, column m
@@ -398,44 +565,50 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(DeltaArgs<T> a) {
     c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.z, bcol[2 * LS], c, 0, 0, 0);
     return __builtin_amdgcn_mfma_f32_16x16x4f32(av.w, bcol[3 * LS], c, 0, 0, 0);
   };
-  fetch(w);
-  __syncthreads();
-  for (int ci = 0; ci < nch; ++ci) {
+  auto chunk = [&](int ci, const Operands& f) {
     f32x4 x = (f32x4){0.f, 0.f, 0.f, 0.f}, x2 = x;
 #pragma unroll
     for (int i = 0; i < DPT; i += 2) {
-      x = mul4(fa[i], Sl + (16 * i + 4 * g) * LS + m, x);
-      x2 = mul4(fa[i + 1], Sl + (16 * (i + 1) + 4 * g) * LS + m, x2);
+      x = mul4(f.a[i], Sl + (16 * i + 4 * g) * LS + m, x);
+      x2 = mul4(f.a[i + 1], Sl + (16 * (i + 1) + 4 * g) * LS + m, x2);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) x[r] += x2[r];
     if (left) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) Un[(mrow + 4 * g + r) * LS + m] = fu[r] - x[r];
+      for (int r = 0; r < 4; ++r) Un[(mrow + 4 * g + r) * LS + m] = f.u[r] - x[r];
     }
     __syncthreads();  // u is complete; the state in LDS has been read
+#pragma unroll
+    for (int i = 0; i < MT; ++i) {
+      const int tile = wave + 4 * i;
+      if (tile < DPT) {
+        acc[i][0] *= f.g[i].x; acc[i][1] *= f.g[i].y; acc[i][2] *= f.g[i].z; acc[i][3] *= f.g[i].w;
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i] = mul4(f.k[i][j], Un + (16 * j + 4 * g) * LS + m, acc[i]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) Sl[(16 * tile + 4 * g + r) * LS + m] = acc[i][r];
+      }
+    }
     if (!left) {
 #pragma unroll
-      for (int j = 0; j < 2; ++j) x = mul4(fb[j], Un + (16 * j + 4 * g) * LS + m, x);
+      for (int j = 0; j < 2; ++j) x = mul4(f.b[j], Un + (16 * j + 4 * g) * LS + m, x);
       const int s = (a.chunk0 + ci) * C + mrow + 4 * g;
       float* op = a.o + ((size_t)b * a.seq.seq_len + s) * H * V + (size_t)h * V + v0 + m;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         if (s + r < len && v0 + m < V) op[(size_t)r * H * V] = x[r];
     }
-#pragma unroll
-    for (int i = 0; i < MT; ++i) {
-      const int tile = wave + 4 * i;
-      if (tile < DPT) {
-        acc[i][0] *= fg[i].x; acc[i][1] *= fg[i].y; acc[i][2] *= fg[i].z; acc[i][3] *= fg[i].w;
-#pragma unroll
-        for (int j = 0; j < 2; ++j) acc[i] = mul4(fk[i][j], Un + (16 * j + 4 * g) * LS + m, acc[i]);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) Sl[(16 * tile + 4 * g + r) * LS + m] = acc[i][r];
-      }
-    }
-    if (ci + 1 < nch) fetch(w + (size_t)(ci + 1) * cf);
     __syncthreads();  // the new state is in LDS; u has been read
+  };
+  fetch(w, op[0]);
+  __syncthreads();
+  for (int ci = 0; ci < nch; ci += 2) {
+    if (ci + 1 < nch) fetch(w + (size_t)(ci + 1) * cf, op[1]);
+    chunk(ci, op[0]);
+    if (ci + 1 >= nch) break;
+    if (ci + 2 < nch) fetch(w + (size_t)(ci + 2) * cf, op[0]);
+    chunk(ci + 1, op[1]);
   }
 #pragma unroll
   for (int i = 0; i < MT; ++i) {
@@ -497,10 +670,14 @@ int delta_step(const OharaDelta* d, const T* p, int ldp, float* state, T* ring, 
   a.d = *d; a.p = p; a.ldp = ldp; a.state = state; a.ring = ring; a.out = out; a.ldo = ldo; a.seq = *seq;
   const dim3 grid((unsigned)(seq->batch * d->heads));
   const int c4 = up(d->vdim, 4) / 4;
-  // enough threads that no one holds more than STEP_ROWS rows of the state
-  if ((256 / c4) * STEP_ROWS >= d->dim) hipLaunchKernelGGL((delta_step_kernel<T, 256>), grid, dim3(256), 0, st, a);
-  else if ((512 / c4) * STEP_ROWS >= d->dim) hipLaunchKernelGGL((delta_step_kernel<T, 512>), grid, dim3(512), 0, st, a);
-  else hipLaunchKernelGGL((delta_step_kernel<T, 1024>), grid, dim3(1024), 0, st, a);
+  // 1024 threads from 64 x 64 states on: the launch is a chain of round trips, and with more threads each round fetches
+  // more of the low-rank weights and the state.
+  if (d->dim * d->vdim < 4096 && (256 / c4) * 16 >= d->dim)
+    hipLaunchKernelGGL((delta_step_kernel<T, 256, 16>), grid, dim3(256), 0, st, a);
+  else if ((1024 / c4) * 4 >= d->dim)
+    hipLaunchKernelGGL((delta_step_kernel<T, 1024, 4>), grid, dim3(1024), 0, st, a);
+  else
+    hipLaunchKernelGGL((delta_step_kernel<T, 1024, 16>), grid, dim3(1024), 0, st, a);
   return ohara_launch_status();
 }
 
@@ -519,14 +696,22 @@ int delta_prefill(const OharaDelta* d, const T* p, int ldp, const T* za, int ldz
   int fit = (int)(ws_bytes / per_chunk < all ? ws_bytes / per_chunk : all);
   if (fit < 1) return OHARA_EINVAL;
   const size_t smem = ((size_t)3 * C * (Dp + 4) + (size_t)C * up(d->vdim, 16) + 2 * C * (C + 4) + C) * sizeof(float);
-  if (smem > 64 * 1024)
-    (void)hipFuncSetAttribute((const void*)chunk_solve_kernel<T>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+  const int fast = ((d->dim | d->vdim) & 7) == 0 && d->taps <= 4 ? d->taps : 0;
+  auto solve = [&](auto kernel) {
+    if (smem > 64 * 1024) (void)hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+    hipLaunchKernelGGL(kernel, dim3((unsigned)a.nchunks, (unsigned)d->heads, (unsigned)seq->batch), dim3(256), smem, st, a);
+  };
   const dim3 wgrid((unsigned)((d->vdim + 15) / 16), (unsigned)d->heads, (unsigned)seq->batch);
   for (int c0 = 0; c0 < all; c0 += fit) {
     a.chunk0 = c0;
     a.nchunks = all - c0 < fit ? all - c0 : fit;
-    hipLaunchKernelGGL((chunk_solve_kernel<T>), dim3((unsigned)a.nchunks, (unsigned)d->heads, (unsigned)seq->batch), dim3(256),
-                       smem, st, a);
+    switch (fast) {
+      case 1: solve(chunk_solve_kernel<T, 1>); break;
+      case 2: solve(chunk_solve_kernel<T, 2>); break;
+      case 3: solve(chunk_solve_kernel<T, 3>); break;
+      case 4: solve(chunk_solve_kernel<T, 4>); break;
+      default: solve(chunk_solve_kernel<T, 0>); break;
+    }
     switch (Dp) {
       case 32: hipLaunchKernelGGL((chunk_walk_kernel<T, 2>), wgrid, dim3(256), 0, st, a); break;
       case 64: hipLaunchKernelGGL((chunk_walk_kernel<T, 4>), wgrid, dim3(256), 0, st, a); break;
