@@ -227,28 +227,37 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
     for (int u = 0; u < 8; ++u) gacc[r][grp][e0 + u] = acc[r][u];
   }
   __syncthreads();
+  // weight of every lane group, once per head
+  __shared__ float hm[RB], hd[RB];
+  if (tid < RB * 64) {
+    const int r = tid >> 6, n = tid & 63;
+    float mm = n < NG ? gm[r][n] : -INFINITY;
+    const float M = wave_max(mm);  // -inf: this chunk lies past the query's position
+    const float wg = mm == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mm - M);
+    const float den = wave_sum(n < NG ? wg * gl[r][n] : 0.f);
+    if (n < NG) gm[r][n] = wg;
+    if (n == 0) {
+      hm[r] = M;
+      hd[r] = den;
+    }
+  }
+  __syncthreads();
   for (int i = tid; i < nh * a.V; i += 256) {
     const int r = i / a.V, c = i - r * a.V, h = h0 + r;
-    float M = -INFINITY;
-    for (int n = 0; n < NG; ++n) M = fmaxf(M, gm[r][n]);
-    float num = 0.f, den = 0.f;
-    for (int n = 0; n < NG; ++n) {
-      if (gm[r][n] == -INFINITY) continue;  // a group that saw no position
-      const float wg = __builtin_amdgcn_exp2f(gm[r][n] - M);
-      num += wg * gacc[r][n][c];
-      den += wg * gl[r][n];
-    }
+    float num = 0.f;
+#pragma unroll
+    for (int n = 0; n < NG; ++n) num += gm[r][n] * gacc[r][n][c];
     if (a.ns > 1) {
       // write-through stores: the workgroup that merges may sit on another XCD
       float* o = a.ws + (((size_t)row * a.H + h) * a.ns + blockIdx.y) * (Vp + 2);
       st_coh4(o + c, __float_as_uint(num));
       if (c == 0) {
-        st_coh4(o + Vp, __float_as_uint(M));  // -inf: this chunk lies past the query's position
-        st_coh4(o + Vp + 1, __float_as_uint(den));
+        st_coh4(o + Vp, __float_as_uint(hm[r]));
+        st_coh4(o + Vp + 1, __float_as_uint(hd[r]));
       }
     } else {
       const float gt = a.gate ? sigmoid_x(ldv(a.gate + (size_t)row * a.ldg + h)) : 1.0f;
-      stv(a.out + (size_t)row * a.ldo + h * a.V + c, num / den * gt);
+      stv(a.out + (size_t)row * a.ldo + h * a.V + c, num / hd[r] * gt);
     }
   }
   if (a.ns == 1) return;
@@ -264,37 +273,37 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
   }
   __syncthreads();
   if (!is_last) return;
-  // chunk maxima and sums into LDS (ns <= 64 = at most RB * 64 pairs)
-  float* cm = &gacc[0][0][0];  // RB * NG * W >= 2 * RB * 64 floats
-  float* cl = cm + RB * 64;
-  for (int i = tid; i < nh * a.ns; i += 256) {
-    const int r = i / a.ns, c = i - r * a.ns;
-    const float* o = a.ws + (((size_t)row * a.H + h0 + r) * a.ns + c) * (Vp + 2);
-    cm[r * 64 + c] = __uint_as_float(ld_coh4(o + Vp));
-    cl[r * 64 + c] = __uint_as_float(ld_coh4(o + Vp + 1));
+  // weights of the chunks (ns <= 64: a lane each), a wave per head; then the columns, in chunk order
+  float* cw = &gacc[0][0][0];  // [RB][64]
+  if (tid < RB * 64) {
+    const int r = tid >> 6, n = tid & 63;
+    const bool in = r < nh && n < a.ns;
+    const float* o = a.ws + (((size_t)row * a.H + h0 + (r < nh ? r : 0)) * a.ns + (in ? n : 0)) * (Vp + 2);
+    const float mm = in ? __uint_as_float(ld_coh4(o + Vp)) : -INFINITY, ll = __uint_as_float(ld_coh4(o + Vp + 1));
+    const float M = wave_max(mm);
+    const float wg = mm == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mm - M);
+    const float den = wave_sum(wg == 0.f ? 0.f : wg * ll);
+    cw[tid] = wg;
+    if (n == 0) hd[r] = den;
   }
   __syncthreads();
   for (int i = tid; i < nh * a.V; i += 256) {
     const int r = i / a.V, c = i - r * a.V, h = h0 + r;
     const float* o = a.ws + ((size_t)row * a.H + h) * a.ns * (Vp + 2) + c;
-    float M = -INFINITY;
-    for (int n = 0; n < a.ns; ++n) M = fmaxf(M, cm[r * 64 + n]);
-    float num = 0.f, den = 0.f;
-    for (int n0 = 0; n0 < a.ns; n0 += 16) {  // sixteen chunks' values in flight, every load unconditional
-      float av[16];
+    float num = 0.f;
+    for (int n0 = 0; n0 < a.ns; n0 += 32) {  // 32 chunks' values in flight, every load unconditional
+      float av[32];
 #pragma unroll
-      for (int n = 0; n < 16; ++n) av[n] = __uint_as_float(ld_coh4(o + (size_t)min(n0 + n, a.ns - 1) * (Vp + 2)));
+      for (int n = 0; n < 32; ++n) av[n] = __uint_as_float(ld_coh4(o + (size_t)min(n0 + n, a.ns - 1) * (Vp + 2)));
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int n = 0; n < 16; ++n) {
-        if (n0 + n >= a.ns || cm[r * 64 + n0 + n] == -INFINITY) continue;
-        const float wg = __builtin_amdgcn_exp2f(cm[r * 64 + n0 + n] - M);
-        num += wg * av[n];
-        den += wg * cl[r * 64 + n0 + n];
+      for (int n = 0; n < 32; ++n) {
+        const float wg = n0 + n < a.ns ? cw[r * 64 + n0 + n] : 0.f;
+        num += wg == 0.f ? 0.f : wg * av[n];
       }
     }
     const float gt = a.gate ? sigmoid_x(ldv(a.gate + (size_t)row * a.ldg + h)) : 1.0f;
-    stv(a.out + (size_t)row * a.ldo + h * a.V + c, num / den * gt);
+    stv(a.out + (size_t)row * a.ldo + h * a.V + c, num / hd[r] * gt);
   }
 }
 

@@ -208,8 +208,11 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaArgs<T> a) {
 }
 
 // ---- prompts: workspace ------------------------------------------------------------------------
-// Per (sequence, head, chunk), floats: W [C][Dp] | q exp(G) [C][Dp] | (k exp(G_C - G))^T [Dp][C] | U [C][Vq] | B [C][C] | exp(G_C) [Dp]
-// with Dp = dim rounded up to 32 / 64 / 128 / 256 and Vq = vdim rounded up to 16; padding is zero.
+// Per (sequence, head, chunk): W [C][Dp], q exp(G) [C][Dp], k exp(G_C - G) [Dp][C], U [C][Vq], B [C][C] and exp(G_C) [Dp] as
+// floats, Dp = dim rounded up to 32 / 64 / 128 / 256, Vq = vdim rounded up to 16, padding zero.  The matrices lie in the
+// order the walk's waves read them: 16 x 16 tiles of 64 float4, one per lane.  W, q, k and B: tile (row / 16, column / 16),
+// lane (row % 16, g = column % 16 / 4) holds columns 4 g .. 4 g + 3; U: tile (column / 16, token / 16), lane (column % 16, g)
+// holds tokens 4 g .. 4 g + 3.
 __host__ __device__ __forceinline__ int dim_padded(int d) { return d <= 32 ? 32 : (d <= 64 ? 64 : (d <= 128 ? 128 : 256)); }
 __host__ __device__ __forceinline__ size_t chunk_floats(int D, int V) {
   const int Dp = dim_padded(D), Vq = up(V, 16);
@@ -450,6 +453,26 @@ __global__ __launch_bounds__(256, 2) void chunk_solve_kernel(DeltaArgs<T> a) {
   float* wU = wK + C * Dp;
   float* wB = wU + C * Vq;
   float* wG = wB + C * C;
+  const int ct = Dp / 16;  // column tiles
+  for (int i = tid; i < C * Dp / 4; i += 256) {
+    const int t = 16 * (i / (64 * ct)) + (i & 15), c = 16 * (i / 64 % ct) + 4 * (i >> 4 & 3);
+    const float4 q = *reinterpret_cast<const float4*>(Q + t * LD + c), g = *reinterpret_cast<const float4*>(G + t * LD + c);
+    *reinterpret_cast<float4*>(wQ + 4 * i) = make_float4(q.x * __expf(g.x), q.y * __expf(g.y), q.z * __expf(g.z), q.w * __expf(g.w));
+  }
+  for (int i = tid; i < C * Dp / 4; i += 256) {
+    const int c = 16 * (i >> 7) + (i & 15), t = 16 * (i >> 6 & 1) + 4 * (i >> 4 & 3);
+    const float last = G[(C - 1) * LD + c];
+    float v[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) v[u] = K[(t + u) * LD + c] * __expf(last - G[(t + u) * LD + c]);
+    *reinterpret_cast<float4*>(wK + 4 * i) = make_float4(v[0], v[1], v[2], v[3]);
+  }
+  {
+    const int t = 16 * (tid >> 7) + (tid & 15), c = 16 * (tid >> 6 & 1) + 4 * (tid >> 4 & 3);
+    *reinterpret_cast<float4*>(wB + 4 * tid) = *reinterpret_cast<const float4*>(B + t * (C + 4) + c);
+  }
+  for (int c = tid; c < Dp; c += 256) wG[c] = __expf(G[(C - 1) * LD + c]);
+  __syncthreads();  // q has been read: its place takes W
   // forward substitution, a column per thread: rows of A are read by all lanes at once, the next one ahead of its use
   for (int c = tid; c < Dp + Vq; c += 256) {
     float x[C];
@@ -457,11 +480,8 @@ __global__ __launch_bounds__(256, 2) void chunk_solve_kernel(DeltaArgs<T> a) {
     const int vc = c - Dp;
 #pragma unroll
     for (int t = 0; t < C; ++t) x[t] = beta[t] * (isw ? K[t * LD + c] * __expf(G[t * LD + c]) : X[t * Vq + vc]);
-    float* dst = isw ? wW + c : wU + vc;
-    const int ld = isw ? Dp : Vq;
     float4 row[2][C / 4];
     row[1][0] = *reinterpret_cast<const float4*>(A + (C + 4));
-    dst[0] = x[0];
 #pragma unroll
     for (int t = 1; t < C; ++t) {
       if (t + 1 < C) {
@@ -475,144 +495,179 @@ __global__ __launch_bounds__(256, 2) void chunk_solve_kernel(DeltaArgs<T> a) {
         s -= ((j & 3) == 0 ? r.x : ((j & 3) == 1 ? r.y : ((j & 3) == 2 ? r.z : r.w))) * x[j];
       }
       x[t] = s;
-      dst[(size_t)t * ld] = s;
       __builtin_amdgcn_sched_barrier(0);  // row by row: hoisting the reads of all of A would spill
     }
-  }
-  for (int i = 4 * tid; i < C * Dp; i += 1024) {
-    const int t = i / Dp, c = i - t * Dp;
-    const float4 q = *reinterpret_cast<const float4*>(Q + t * LD + c), g = *reinterpret_cast<const float4*>(G + t * LD + c);
-    *reinterpret_cast<float4*>(wQ + i) = make_float4(q.x * __expf(g.x), q.y * __expf(g.y), q.z * __expf(g.z), q.w * __expf(g.w));
-  }
-  for (int i = 4 * tid; i < C * Dp; i += 1024) {
-    const int c = i / C, t = i - c * C;
-    const float last = G[(C - 1) * LD + c];
-    float v[4];
+    if (isw) {
 #pragma unroll
-    for (int u = 0; u < 4; ++u) v[u] = K[(t + u) * LD + c] * __expf(last - G[(t + u) * LD + c]);
-    *reinterpret_cast<float4*>(wK + i) = make_float4(v[0], v[1], v[2], v[3]);
+      for (int t = 0; t < C; ++t) Q[t * LD + c] = x[t];
+    } else {
+#pragma unroll
+      for (int t = 0; t < C; t += 4)
+        *reinterpret_cast<float4*>(wU + 4 * ((2 * (vc >> 4) + (t >> 4)) * 64 + 16 * (t >> 2 & 3) + (vc & 15))) =
+            make_float4(x[t], x[t + 1], x[t + 2], x[t + 3]);
+    }
   }
-  for (int i = tid; i < C * C; i += 256) wB[i] = B[(i / C) * (C + 4) + (i % C)];
-  for (int c = tid; c < Dp; c += 256) wG[c] = __expf(G[(C - 1) * LD + c]);
+  __syncthreads();
+  for (int i = tid; i < C * Dp / 4; i += 256) {
+    const int t = 16 * (i / (64 * ct)) + (i & 15), c = 16 * (i / 64 % ct) + 4 * (i >> 4 & 3);
+    *reinterpret_cast<float4*>(wW + 4 * i) = *reinterpret_cast<const float4*>(Q + t * LD + c);
+  }
 }
 
 // The state over the chunks.  v_mfma_f32_16x16x4_f32: A lane (row = lane & 15, k = lane >> 4), B lane (k = lane >> 4,
 // column = lane & 15), result row 4 (lane >> 4) + r, column lane & 15.  A step of 16 k's takes four products whose k-slot g
 // of product j stands for k = 4 g + j, so a lane fetches the four A elements it needs as one float4.
+//
+// Eight waves: (u or o) x (two 16-token row tiles) x (two halves of the key channels); the state's 16-channel tiles are
+// spread over all of them.  The halves of u meet where u is read, those of o in LDS one barrier later.
 template <typename T, int DPT>  // Dp / 16
-__global__ __launch_bounds__(256, (DPT > 8 ? 1 : 2)) void chunk_walk_kernel(DeltaArgs<T> a) {
-  constexpr int Dp = 16 * DPT, MT = (DPT + 3) / 4, LS = 20;  // row stride: the four k-slots of a product on different banks
-  __shared__ float Sl[Dp * LS];
-  __shared__ float Un[C * LS];
+__global__ __launch_bounds__(512) void chunk_walk_kernel(DeltaArgs<T> a) {
+  constexpr int Dp = 16 * DPT, MT = (DPT + 7) / 8, HT = DPT / 2, LS = Dp + 4, LU = C + 4;
+  // by value column, so the four rows a lane holds of a result and the four k's it needs of an operand are one float4
+  __shared__ __align__(16) float Sl[16 * LS];
+  __shared__ __align__(16) float Un[2][16 * LU];
+  __shared__ __align__(16) float On[16 * LU];
   const OharaDelta& dd = a.d;
   const int H = dd.heads, D = dd.dim, V = dd.vdim, Vp = up(V, 4), Vq = up(V, 16);
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 15, g = lane >> 4;
-  const int v0 = blockIdx.x * 16, h = blockIdx.y, b = blockIdx.z;
+  const int tid = threadIdx.x, lane = tid & 63, m = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  // Workgroups are handed to the eight XCDs in turn: the column slices of one (sequence, head) get ids eight apart, so the
+  // chunk operands they all read are fetched into one L2.
+  const int nv = Vq / 16, local = blockIdx.x >> 3, pair = (local / nv) * 8 + (blockIdx.x & 7);
+  if (pair >= a.seq.batch * H) return;
+  const int v0 = (local % nv) * 16, h = pair % H, b = pair / H;
   const int len = seq_tokens(a.seq, b);
   const int nch = min(a.nchunks, (len + C - 1) / C - a.chunk0);
   if (nch < 1) return;
   const int pos0 = seq_start(a.seq, b);
   float* S = a.state + ((size_t)seq_slot(a.seq, b) * H + h) * D * Vp;
   const bool fresh = a.chunk0 == 0 && pos0 == 0;
+  auto put4 = [](float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; };
   f32x4 acc[MT];
 #pragma unroll
   for (int i = 0; i < MT; ++i) {
-    const int tile = wave + 4 * i;
+    const int tile = wave + 8 * i;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int d = 16 * tile + 4 * g + r;
       acc[i][r] = (!fresh && tile < DPT && d < D && v0 + m < V) ? S[(size_t)d * Vp + v0 + m] : 0.f;
-      if (tile < DPT) Sl[d * LS + m] = acc[i][r];
     }
+    if (tile < DPT) put4(Sl + m * LS + 16 * tile + 4 * g, acc[i]);
   }
   const size_t cf = chunk_floats(D, V);
   const float* w = a.ws + ((size_t)b * H + h) * a.nchunks * cf;
-  const bool left = wave < 2;           // waves 0, 1: u; waves 2, 3: o
+  const bool left = wave < 4;           // waves 0 - 3: u; 4 - 7: o
+  const int half = (wave >> 1) & 1;     // of the key channels
   const int mrow = 16 * (wave & 1);     // this wave's token rows
-  // operands of a chunk: two sets, the next chunk's loads are in flight during this one's products
+  const int s_first = a.chunk0 * C + mrow + 4 * g;  // token of the lane's first result row, chunk 0
+  float* ob = a.o + (size_t)b * a.seq.seq_len * H * V + (size_t)h * V + v0 + m;
+  // Operands of a chunk: three sets (two where registers end), the next chunks' loads are in flight during this one's
+  // products.  No branch around a
+  // load (what a wave does not need is fetched from a valid address and ignored), so the compiler can count them.
   struct Operands {
-    float4 a[DPT], k[MT][2], g[MT], b[2];
-    float u[4];
-  } op[2];
-  auto fetch = [&](const float* x, Operands& f) {
-    const float* ap = x + (left ? 0 : C * Dp) + (size_t)(mrow + m) * Dp + 4 * g;
+    float4 a[HT], k[MT][2], g[MT], b;
+    f32x4 u;
+  } op[DPT > 8 ? 2 : 3];
+  auto fetch = [&](int ci, Operands& f) {
+    const float* x = w + (size_t)min(ci, nch - 1) * cf;
+    const float4* ap = reinterpret_cast<const float4*>(x + (left ? 0 : C * Dp)) + ((wave & 1) * DPT + half * HT) * 64 + lane;
 #pragma unroll
-    for (int i = 0; i < DPT; ++i) f.a[i] = *reinterpret_cast<const float4*>(ap + 16 * i);
+    for (int i = 0; i < HT; ++i) f.a[i] = ap[64 * i];
     const float* kp = x + 2 * C * Dp;
     const float* up_ = kp + C * Dp;
     const float* bp = up_ + C * Vq;
     const float* gp = bp + C * C;
-    if (left) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) f.u[r] = up_[(size_t)(mrow + 4 * g + r) * Vq + v0 + m];
-    } else {
-#pragma unroll
-      for (int j = 0; j < 2; ++j) f.b[j] = *reinterpret_cast<const float4*>(bp + (size_t)(mrow + m) * C + 16 * j + 4 * g);
-    }
+    f.u = reinterpret_cast<const f32x4*>(up_)[(2 * (v0 >> 4) + (wave & 1)) * 64 + lane];
+    f.b = reinterpret_cast<const float4*>(bp)[(2 * (wave & 1) + half) * 64 + lane];
 #pragma unroll
     for (int i = 0; i < MT; ++i) {
-      const int tile = wave + 4 * i;
-      if (tile < DPT) {
+      const int tile = DPT % 8 == 0 ? wave + 8 * i : min(wave + 8 * i, DPT - 1);
 #pragma unroll
-        for (int j = 0; j < 2; ++j) f.k[i][j] = *reinterpret_cast<const float4*>(kp + (size_t)(16 * tile + m) * C + 16 * j + 4 * g);
-        f.g[i] = *reinterpret_cast<const float4*>(gp + 16 * tile + 4 * g);
-      }
+      for (int j = 0; j < 2; ++j) f.k[i][j] = reinterpret_cast<const float4*>(kp)[(2 * tile + j) * 64 + lane];
+      f.g[i] = *reinterpret_cast<const float4*>(gp + 16 * tile + 4 * g);
     }
   };
-  auto mul4 = [&](float4 av, const float* bcol, f32x4 c) {  // bcol: row 4 g of the step's B rows, column m
-    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.x, bcol[0], c, 0, 0, 0);
-    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.y, bcol[LS], c, 0, 0, 0);
-    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.z, bcol[2 * LS], c, 0, 0, 0);
-    return __builtin_amdgcn_mfma_f32_16x16x4f32(av.w, bcol[3 * LS], c, 0, 0, 0);
+  auto mul4 = [&](float4 av, float4 bv, f32x4 c) {
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.x, bv.x, c, 0, 0, 0);
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.y, bv.y, c, 0, 0, 0);
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(av.z, bv.z, c, 0, 0, 0);
+    return __builtin_amdgcn_mfma_f32_16x16x4f32(av.w, bv.w, c, 0, 0, 0);
   };
-  auto chunk = [&](int ci, const Operands& f) {
-    f32x4 x = (f32x4){0.f, 0.f, 0.f, 0.f}, x2 = x;
-#pragma unroll
-    for (int i = 0; i < DPT; i += 2) {
-      x = mul4(f.a[i], Sl + (16 * i + 4 * g) * LS + m, x);
-      x2 = mul4(f.a[i + 1], Sl + (16 * (i + 1) + 4 * g) * LS + m, x2);
-    }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) x[r] += x2[r];
-    if (left) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) Un[(mrow + 4 * g + r) * LS + m] = f.u[r] - x[r];
-    }
-    __syncthreads();  // u is complete; the state in LDS has been read
-#pragma unroll
-    for (int i = 0; i < MT; ++i) {
-      const int tile = wave + 4 * i;
-      if (tile < DPT) {
-        acc[i][0] *= f.g[i].x; acc[i][1] *= f.g[i].y; acc[i][2] *= f.g[i].z; acc[i][3] *= f.g[i].w;
-#pragma unroll
-        for (int j = 0; j < 2; ++j) acc[i] = mul4(f.k[i][j], Un + (16 * j + 4 * g) * LS + m, acc[i]);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) Sl[(16 * tile + 4 * g + r) * LS + m] = acc[i][r];
-      }
-    }
-    if (!left) {
-#pragma unroll
-      for (int j = 0; j < 2; ++j) x = mul4(f.b[j], Un + (16 * j + 4 * g) * LS + m, x);
-      const int s = (a.chunk0 + ci) * C + mrow + 4 * g;
-      float* op = a.o + ((size_t)b * a.seq.seq_len + s) * H * V + (size_t)h * V + v0 + m;
+  f32x4 o = (f32x4){0.f, 0.f, 0.f, 0.f};
+  // the other half of the last chunk's o is in LDS: add and store (waves of the first half)
+  auto store_o = [&](int ci) {
+    if (!left && half == 0) {
+      const f32x4 p = *reinterpret_cast<const f32x4*>(On + m * LU + mrow + 4 * g);
+      const int s = s_first + ci * C;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if (s + r < len && v0 + m < V) op[(size_t)r * H * V] = x[r];
+        if (s + r < len && v0 + m < V) ob[(size_t)(s + r) * H * V] = o[r] + p[r];
+    }
+  };
+  auto chunk = [&](int ci, const Operands& f) {
+    float4 sv[HT];
+#pragma unroll
+    for (int i = 0; i < HT; ++i) sv[i] = *reinterpret_cast<const float4*>(Sl + m * LS + half * (Dp / 2) + 16 * i + 4 * g);
+    if (ci > 0) store_o(ci - 1);
+    f32x4 x = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < HT; ++i) x = mul4(f.a[i], sv[i], x);
+    if (left) {
+      if (half) put4(Un[1] + m * LU + mrow + 4 * g, (f32x4){-x[0], -x[1], -x[2], -x[3]});
+      else put4(Un[0] + m * LU + mrow + 4 * g, (f32x4){f.u[0] - x[0], f.u[1] - x[1], f.u[2] - x[2], f.u[3] - x[3]});
+    }
+    __syncthreads();  // u is complete; the state and the last o in LDS have been read
+    float4 uv[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const float4 p = *reinterpret_cast<const float4*>(Un[0] + m * LU + 16 * j + 4 * g);
+      const float4 q = *reinterpret_cast<const float4*>(Un[1] + m * LU + 16 * j + 4 * g);
+      uv[j] = make_float4(p.x + q.x, p.y + q.y, p.z + q.z, p.w + q.w);
+    }
+#pragma unroll
+    for (int i = 0; i < MT; ++i) {
+      const int tile = wave + 8 * i;
+      if (DPT % 8 == 0 || tile < DPT) {
+        acc[i][0] *= f.g[i].x; acc[i][1] *= f.g[i].y; acc[i][2] *= f.g[i].z; acc[i][3] *= f.g[i].w;
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i] = mul4(f.k[i][j], uv[j], acc[i]);
+        put4(Sl + m * LS + 16 * tile + 4 * g, acc[i]);
+      }
+    }
+    if (!left) {  // each half takes 16 of the chunk's tokens of B u
+      o = mul4(f.b, half ? uv[1] : uv[0], x);
+      if (half) put4(On + m * LU + mrow + 4 * g, o);
     }
     __syncthreads();  // the new state is in LDS; u has been read
   };
-  fetch(w, op[0]);
-  __syncthreads();
-  for (int ci = 0; ci < nch; ci += 2) {
-    if (ci + 1 < nch) fetch(w + (size_t)(ci + 1) * cf, op[1]);
-    chunk(ci, op[0]);
-    if (ci + 1 >= nch) break;
-    if (ci + 2 < nch) fetch(w + (size_t)(ci + 2) * cf, op[0]);
-    chunk(ci + 1, op[1]);
+  fetch(0, op[0]);
+  if constexpr (DPT > 8) {
+    __syncthreads();
+    for (int ci = 0; ci < nch; ci += 2) {
+      fetch(ci + 1, op[1]);
+      chunk(ci, op[0]);
+      if (ci + 1 >= nch) break;
+      fetch(ci + 2, op[0]);
+      chunk(ci + 1, op[1]);
+    }
+  } else {
+    fetch(1, op[1]);
+    __syncthreads();
+    for (int ci = 0; ci < nch; ci += 3) {
+      fetch(ci + 2, op[2]);
+      chunk(ci, op[0]);
+      if (ci + 1 >= nch) break;
+      fetch(ci + 3, op[0]);
+      chunk(ci + 1, op[1]);
+      if (ci + 2 >= nch) break;
+      fetch(ci + 4, op[1]);
+      chunk(ci + 2, op[2]);
+    }
   }
+  store_o(nch - 1);
 #pragma unroll
   for (int i = 0; i < MT; ++i) {
-    const int tile = wave + 4 * i;
+    const int tile = wave + 8 * i;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int d = 16 * tile + 4 * g + r;
@@ -701,7 +756,7 @@ int delta_prefill(const OharaDelta* d, const T* p, int ldp, const T* za, int ldz
     if (smem > 64 * 1024) (void)hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
     hipLaunchKernelGGL(kernel, dim3((unsigned)a.nchunks, (unsigned)d->heads, (unsigned)seq->batch), dim3(256), smem, st, a);
   };
-  const dim3 wgrid((unsigned)((d->vdim + 15) / 16), (unsigned)d->heads, (unsigned)seq->batch);
+  const dim3 wgrid((unsigned)((d->heads * seq->batch + 7) / 8 * 8 * ((d->vdim + 15) / 16)));
   for (int c0 = 0; c0 < all; c0 += fit) {
     a.chunk0 = c0;
     a.nchunks = all - c0 < fit ? all - c0 : fit;
@@ -713,10 +768,10 @@ int delta_prefill(const OharaDelta* d, const T* p, int ldp, const T* za, int ldz
       default: solve(chunk_solve_kernel<T, 0>); break;
     }
     switch (Dp) {
-      case 32: hipLaunchKernelGGL((chunk_walk_kernel<T, 2>), wgrid, dim3(256), 0, st, a); break;
-      case 64: hipLaunchKernelGGL((chunk_walk_kernel<T, 4>), wgrid, dim3(256), 0, st, a); break;
-      case 128: hipLaunchKernelGGL((chunk_walk_kernel<T, 8>), wgrid, dim3(256), 0, st, a); break;
-      default: hipLaunchKernelGGL((chunk_walk_kernel<T, 16>), wgrid, dim3(256), 0, st, a); break;
+      case 32: hipLaunchKernelGGL((chunk_walk_kernel<T, 2>), wgrid, dim3(512), 0, st, a); break;
+      case 64: hipLaunchKernelGGL((chunk_walk_kernel<T, 4>), wgrid, dim3(512), 0, st, a); break;
+      case 128: hipLaunchKernelGGL((chunk_walk_kernel<T, 8>), wgrid, dim3(512), 0, st, a); break;
+      default: hipLaunchKernelGGL((chunk_walk_kernel<T, 16>), wgrid, dim3(512), 0, st, a); break;
     }
   }
   const int rows = seq->batch * seq->seq_len;

@@ -51,10 +51,17 @@ __device__ __forceinline__ int seq_start(const OharaSeq& q, int b) {
 __device__ __forceinline__ int seq_tokens(const OharaSeq& q, int b) { return q.lens ? min(q.lens[b], q.seq_len) : q.seq_len; }
 __device__ __forceinline__ int seq_slot(const OharaSeq& q, int b) { return q.slots ? q.slots[b] : b; }
 
-// sigmoid, silu and softplus in full fp32
-__device__ __forceinline__ float sigmoid_x(float v) { return 1.0f / (1.0f + expf(-v)); }
-__device__ __forceinline__ float silu_x(float v) { return v / (1.0f + expf(-v)); }
-__device__ __forceinline__ float softplus_x(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
+// sigmoid, silu and softplus in fp32 on the hardware exponential, logarithm and reciprocal (each within a few units of the
+// last place; the library functions and the IEEE division are several times the instructions)
+__device__ __forceinline__ float sigmoid_x(float v) { return __frcp_rn(1.0f + __expf(-v)); }
+__device__ __forceinline__ float silu_x(float v) { return v * __frcp_rn(1.0f + __expf(-v)); }
+// max(v, 0) + log(1 + e) with e = exp(-|v|).  1 + e rounds; dividing by what it rounded to, log(u) * e / (u - 1) with
+// u = fl(1 + e), keeps the relative precision for small e.
+__device__ __forceinline__ float softplus_x(float v) {
+  const float e = __expf(-fabsf(v)), u = 1.0f + e, d = u - 1.0f;
+  const float l = d == 0.f ? e : __logf(u) * e * __frcp_rn(d);
+  return fmaxf(v, 0.f) + l;
+}
 
 inline bool seq_ok(const OharaSeq* q) {
   return q && q->batch >= 1 && q->seq_len >= 1 && (int64_t)q->batch * q->seq_len <= INT32_MAX &&

@@ -144,6 +144,132 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualArgs<T> a) {
   }
 }
 
+// The same for rows of at most 1024 * NP columns (all sizes multiples of 4): a thread owns NP pieces of four columns and
+// keeps them in registers, and everything that does not depend on the norm - residual, weights, the convolution's past
+// inputs (MT: taps at most) - is requested before the sums.  One round trip instead of four.
+template <typename T, int NP, int MT>
+__global__ __launch_bounds__(256) void residual_norm_regs_kernel(ResidualArgs<T> a) {
+  extern __shared__ __align__(16) float smem[];  // groups > 1: a partial sum per piece, then 1 / rms per group
+  __shared__ float red[2][4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, row = blockIdx.x, d = a.d;
+  const int gs4 = d / a.groups / 4;  // pieces per group
+  float* xr = a.x + (size_t)row * d;
+  const bool add = !a.ids && a.y;
+  float x[NP][4], y[NP][4], w[NP][4], past[NP][MT][4], cw[NP][MT][4];
+  int64_t id = 0;
+  if (a.ids) {
+    id = a.ids[row];
+    if (id < 0 || id >= a.vocab) id = 0;  // the host validates ids; never read out of bounds
+  }
+  int pos = 0;
+  float* ring = nullptr;
+  if (MT > 1) {
+    pos = seq_start(a.seq, row);
+    ring = a.ring + (size_t)seq_slot(a.seq, row) * a.taps * d;
+  }
+#pragma unroll
+  for (int p = 0; p < NP; ++p) {
+    const int i = 4 * tid + 1024 * p;
+    const bool in = i < d;
+    const float zero[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int u = 0; u < 4; ++u) x[p][u] = y[p][u] = w[p][u] = zero[u];
+    if (!in) continue;
+    if (a.ids) ld4(a.table + (size_t)id * d + i, x[p]);
+    else ld4(xr + i, x[p]);
+    if (add) {
+      ld4(a.y + (size_t)row * a.ldy + i, y[p]);
+      ld4(a.norm_w + i, w[p]);
+    }
+    if (MT > 1) {
+#pragma unroll
+      for (int lag = 0; lag < MT; ++lag) {
+        if (lag < a.taps) ld4(a.conv_w + (size_t)(a.taps - 1 - lag) * d + i, cw[p][lag]);
+        if (lag > 0 && lag < a.taps && pos >= lag) ld4(ring + (size_t)((pos - lag) % a.taps) * d + i, past[p][lag]);
+      }
+    }
+  }
+  auto inverse = [&](float (&v)[NP][4], float* r4, float (&inv)[NP]) {
+    float s[NP], tot = 0.f;
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      s[p] = ((v[p][0] * v[p][0] + v[p][1] * v[p][1]) + v[p][2] * v[p][2]) + v[p][3] * v[p][3];
+      tot += s[p];
+    }
+    if (a.groups == 1) {
+      tot = wave_sum(tot);
+      if (lane == 0) r4[wave] = tot;
+      __syncthreads();
+      const float r = 1.0f / sqrtf((((r4[0] + r4[1]) + r4[2]) + r4[3]) / (float)d + a.eps);
+#pragma unroll
+      for (int p = 0; p < NP; ++p) inv[p] = r;
+      return;
+    }
+    float* ginv = smem + 256 * NP;
+    __syncthreads();  // an earlier use of the sums is over
+#pragma unroll
+    for (int p = 0; p < NP; ++p) smem[tid + 256 * p] = s[p];
+    __syncthreads();
+    for (int g = wave; g < a.groups; g += 4) {
+      float t = 0.f;
+      for (int i = lane; i < gs4; i += 64) t += smem[g * gs4 + i];
+      t = wave_sum(t);
+      if (lane == 0) ginv[g] = 1.0f / sqrtf(t / (float)(4 * gs4) + a.eps);
+    }
+    __syncthreads();
+#pragma unroll
+    for (int p = 0; p < NP; ++p) inv[p] = ginv[min((tid + 256 * p) / gs4, a.groups - 1)];
+  };
+  if (add) {
+    float inv[NP];
+    inverse(y, red[0], inv);
+#pragma unroll
+    for (int p = 0; p < NP; ++p)
+#pragma unroll
+      for (int u = 0; u < 4; ++u) x[p][u] += y[p][u] * inv[p] * w[p][u];
+  }
+  if (add || a.ids) {
+#pragma unroll
+    for (int p = 0; p < NP; ++p)
+      if (4 * tid + 1024 * p < d) st4(xr + 4 * tid + 1024 * p, x[p]);
+  }
+  if (a.mode == OHARA_OUT_NONE) return;
+  T* o = a.out + (size_t)row * a.ldo;
+  for (int i = d + tid; i < a.ldo; i += 256) stv(o + i, 0.f);
+  float inv[NP];
+  if (a.mode == OHARA_OUT_NORM) inverse(x, red[1], inv);
+  const bool live = MT > 1 && seq_tokens(a.seq, row) > 0 && pos >= 0;
+#pragma unroll
+  for (int p = 0; p < NP; ++p) {
+    const int i = 4 * tid + 1024 * p;
+    if (i >= d) continue;
+    float r[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) r[u] = x[p][u];
+    if (a.mode == OHARA_OUT_NORM) {
+      float w2[4];
+      ld4(a.norm2_w + i, w2);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) r[u] = x[p][u] * inv[p] * w2[u];
+    }
+    if (MT > 1) {
+      float c[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) c[u] = cw[p][0][u] * x[p][u];
+#pragma unroll
+      for (int lag = 1; lag < MT; ++lag)
+        if (lag < a.taps && pos >= lag) {
+#pragma unroll
+          for (int u = 0; u < 4; ++u) c[u] += cw[p][lag][u] * past[p][lag][u];
+        }
+      if (live) st4(ring + (size_t)(pos % a.taps) * d + i, x[p]);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) r[u] += c[u];
+    }
+    st4(o + i, r);
+  }
+}
+
 // out = x + conv(x): a workgroup per (row, 1024 columns), four columns per thread
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void input_conv_kernel(const float* x, int d, const float* w, int taps, const float* ring,
@@ -225,6 +351,16 @@ int launch_residual(ResidualArgs<T> a, const OharaSeq* seq, hipStream_t st) {
   if (smem > 64 * 1024) return OHARA_ESIZE;
   const dim3 grid((unsigned)(seq->batch * seq->seq_len));
   const bool vec = (a.d & 3) == 0 && ((a.d / a.groups) & 3) == 0 && (a.ldy & 3) == 0 && (a.ldo & 3) == 0;
+  const bool conv = a.mode == OHARA_OUT_CONV;
+  if (vec && a.d <= 4096 && (!conv || a.taps <= 4)) {
+    auto regs = [&](auto kernel, int np) {
+      hipLaunchKernelGGL(kernel, grid, dim3(256), a.groups > 1 ? (256 * np + a.groups) * sizeof(float) : 0, st, a);
+    };
+    if (a.d <= 1024) conv ? regs(residual_norm_regs_kernel<T, 1, 4>, 1) : regs(residual_norm_regs_kernel<T, 1, 1>, 1);
+    else if (a.d <= 2048) conv ? regs(residual_norm_regs_kernel<T, 2, 4>, 2) : regs(residual_norm_regs_kernel<T, 2, 1>, 2);
+    else conv ? regs(residual_norm_regs_kernel<T, 4, 4>, 4) : regs(residual_norm_regs_kernel<T, 4, 1>, 4);
+    return ohara_launch_status();
+  }
   if (vec) hipLaunchKernelGGL((residual_norm_kernel<T, true>), grid, dim3(256), smem, st, a);
   else hipLaunchKernelGGL((residual_norm_kernel<T, false>), grid, dim3(256), smem, st, a);
   return ohara_launch_status();

@@ -115,7 +115,7 @@ class BiasedAttention:
     q, k, v, gate, out: (weight, bias or None) pairs of the projections off the same input."""
 
     WORKGROUPS = 1024   # decode: a context is cut into chunks until about this many workgroups run
-    MIN_CHUNK = 64      # positions of a chunk at least (of the cache's capacity)
+    MIN_CHUNK = 128     # positions of a chunk at least (of the cache's capacity)
 
     def __init__(self, q, k, v, gate, out, q_norm, k_norm, *, heads: int, kv_heads: int, dim: int, vdim: int, scale: float,
                  eps: float, slopes: torch.Tensor, dtype=BF16, device="cuda"):
@@ -140,6 +140,7 @@ class BiasedAttention:
 
     def state(self, rows: int, max_seq_length: int) -> dict:
         zeros = lambda n: torch.zeros(rows, max_seq_length, self.kv_heads, ops.round8(n), dtype=self.dtype, device=self.device)  # noqa: E731
+        self._split(rows, max_seq_length)  # a step captured before any eager one finds its workspace initialised
         return {"key": zeros(self.dim), "value": zeros(self.vdim)}
 
     def n_split(self, batch: int, max_seq_length: int) -> int:
@@ -147,17 +148,22 @@ class BiasedAttention:
         sets = self.kv_heads * -(-rep // (4 if rep >= 4 else (2 if rep >= 2 else 1)))
         return max(1, min(64, self.WORKGROUPS // (batch * sets), max_seq_length // self.MIN_CHUNK))
 
+    def _split(self, batch: int, max_seq_length: int):
+        """(chunks, workspace) of a decode step; steps of the same batch size share the workspace, so they must run on one
+        stream or otherwise in turn."""
+        ns = self.n_split(batch, max_seq_length)
+        if ns == 1:
+            return 1, None
+        ws = self._ws.get((batch, ns))
+        if ws is None:
+            ws = self._ws[(batch, ns)] = ops.attn_bias_workspace(batch, self.heads, self.vdim, ns, self.device)
+        return ns, ws
+
     def __call__(self, h, state, seq: ops.Seq):
         p = self.proj(h)
         q = ops.qkv_norm_append(p, self.heads, self.kv_heads, self.dim, self.vdim, self.q_norm, self.k_norm, self.eps,
                                 state.key, state.value, seq)
-        ns, ws = 1, None
-        if seq.seq_len == 1:
-            ns = self.n_split(seq.batch, state.key.shape[1])
-            if ns > 1:
-                ws = self._ws.get((seq.batch, ns))
-                if ws is None:
-                    ws = self._ws[(seq.batch, ns)] = ops.attn_bias_workspace(seq.batch, self.heads, self.vdim, ns, self.device)
+        ns, ws = self._split(seq.batch, state.key.shape[1]) if seq.seq_len == 1 else (1, None)
         gate = p[:, self.gate_at:self.gate_at + self.heads]
         att = ops.attn_bias(q, state.key, state.value, self.heads, self.kv_heads, self.dim, self.vdim, self.scale, self.slopes,
                             gate, seq, ns, ws)
@@ -175,7 +181,7 @@ class ChannelDelta:
     per head.  q, k: (kv_heads * dim, width); v: (heads * vdim, width); convs: (channels, taps) each."""
 
     WORKSPACE = 1 << 30  # bytes of per-chunk intermediates at most; longer prompts are walked in segments
-    _workspaces: dict = {}  # device -> the workspace every layer on that device shares
+    _workspaces: dict = {}  # device -> the workspace every layer on that device shares (prompts run on one stream)
 
     def __init__(self, q, k, v, q_conv, k_conv, v_conv, beta, a_log, a1, a2, dt_bias, g1, g2, norm_w, out, *, heads: int,
                  kv_heads: int, dim: int, vdim: int, eps: float, dtype=BF16, device="cuda"):
