@@ -48,7 +48,7 @@ def close(got, want, dtype, scale=None, tol=None):
 
 
 @pytest.mark.parametrize("dtype", [F32, BF])
-@pytest.mark.parametrize("d, groups", [(60, 3), (40, 1), (64, 8), (35, 5), (2048, 2)])
+@pytest.mark.parametrize("d, groups", [(60, 3), (40, 1), (64, 8), (35, 5), (2048, 2), (3000, 3), (4096, 1), (5000, 5)])
 def test_residual_norm(cuda, dtype, d, groups):
     from ohara_amd import ops
 
