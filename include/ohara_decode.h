@@ -633,6 +633,10 @@ typedef struct OharaSeq {
 #define OHARA_OUT_COPY 1 /* x */
 #define OHARA_OUT_CONV 2 /* x + causal depthwise convolution of x over time (seq_len 1; see conv_w / ring) */
 #define OHARA_OUT_NORM 3 /* group RMS norm of x times norm2_w */
+/* May be added to out_mode (groups 1 only): the norm of y / of OHARA_OUT_NORM is a layer norm without bias,
+ * i.e. the row's mean is taken off before the root mean square. */
+#define OHARA_CENTER_Y 16
+#define OHARA_CENTER_OUT 32
 
 /* Residual update of a block with norms on the sublayer outputs, one launch:
  *   ids != NULL:  x = table[id]              (table: activation type, vocab rows of d)
@@ -672,6 +676,14 @@ int ohara_gemm_f32(const float* x, int ldx, const float* w, const float* w_up, c
 int ohara_gemm_softcap_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, float cap, int rows,
                             uint16_t* out, int ldo, void* stream);
 
+/* out[row, i] = gelu_tanh((x W^T)[row, i]) * table[ids[row] * ldt + i], gelu_tanh(z) = z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))),
+ * i < n: a projection gated onto an embedding of the row's token (table: rows of ldt entries, the layer's n from the pointer on).
+ * The sum stays fp32 up to the product.  bf16: packed weight, n and ldt multiples of 4, any rows; f32: W (n, k) row-major. */
+int ohara_gemm_gelu_lookup_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, const uint16_t* table, int ldt,
+                                const int64_t* ids, int vocab, int rows, uint16_t* out, int ldo, void* stream);
+int ohara_gemm_gelu_lookup_f32(const float* x, int ldx, const float* w, int n, int k, const float* table, int ldt,
+                               const int64_t* ids, int vocab, int rows, float* out, int ldo, void* stream);
+
 /* Attention front end off one projection p with row layout [q (h*dh); k (h_kv*dh); v (h_kv*dv); ...]:
  * q and k are each divided by the root mean square of ALL their elements of the row and multiplied by
  * qn / kn; every value head is divided by its own root mean square.  q -> q_out (rows, h, dhp), keys and
@@ -683,6 +695,14 @@ int ohara_qkv_norm_append_bf16(const uint16_t* p, int ldp, int h, int h_kv, int 
 int ohara_qkv_norm_append_f32(const float* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn, const float* kn,
                               float eps, float* q_out, float* kcache, float* vcache, int t_max, const OharaSeq* seq,
                               void* stream);
+/* The same layout without norms: the first rot dimensions of every q and k head are rotated in neighbouring pairs,
+ * (u, v) -> (u cos - v sin, v cos + u sin) with the angles' tables cos, sin (t_max, rot / 2) fp32 at the token's position. */
+int ohara_qkv_rotate_append_bf16(const uint16_t* p, int ldp, int h, int h_kv, int dh, int dv, const float* cos,
+                                 const float* sin, int rot, uint16_t* q_out, uint16_t* kcache, uint16_t* vcache, int t_max,
+                                 const OharaSeq* seq, void* stream);
+int ohara_qkv_rotate_append_f32(const float* p, int ldp, int h, int h_kv, int dh, int dv, const float* cos, const float* sin,
+                                int rot, float* q_out, float* kcache, float* vcache, int t_max, const OharaSeq* seq,
+                                void* stream);
 /* Causal attention over the cache with a linear distance bias and a per-head output gate:
  *   o[row, hd, :] = sigmoid(gate[row, hd]) * sum_j softmax_j(scale q . k_j - slopes[hd] (i - j)) v_j,  j <= i = position.
  * Scores, softmax weights and sums are fp32 (the _bf16 prefill product carries every fp32 weight as three
@@ -699,6 +719,49 @@ int ohara_attn_bias_f32(const float* q, const float* kcache, const float* vcache
                         int t_max, float scale, const float* slopes, const float* gate, int ldg, int n_split,
                         void* workspace, float* out, int ldo, const OharaSeq* seq, void* stream);
 
+/* The same with other score functions and windows.  Score of query position i and key position j <= i:
+ *   s = scale q . k_j;  cap > 0: s = cap tanh(s / cap);  slopes: s -= slopes[head] (i - j);
+ * chunk > 0: only keys of the query's own chunk, floor(i / chunk) = floor(j / chunk), are visible.
+ * ld_k, ld_v > 0: elements between neighbouring positions of the keys / values (0: h_kv * dhp, h_kv * dvp).
+ * gate_elements: the gate has one entry per output element (rows of h*dv) instead of one per head. */
+typedef struct OharaScores {
+  float scale, cap;
+  int chunk, gate_elements, ld_k, ld_v;
+  const float* slopes;
+} OharaScores;
+int ohara_attn_scored_bf16(const uint16_t* q, const uint16_t* kcache, const uint16_t* vcache, int h, int h_kv, int dh,
+                           int dv, int t_max, const OharaScores* sc, const uint16_t* gate, int ldg, int n_split,
+                           void* workspace, uint16_t* out, int ldo, const OharaSeq* seq, void* stream);
+int ohara_attn_scored_f32(const float* q, const float* kcache, const float* vcache, int h, int h_kv, int dh, int dv,
+                          int t_max, const OharaScores* sc, const float* gate, int ldg, int n_split, void* workspace,
+                          float* out, int ldo, const OharaSeq* seq, void* stream);
+
+/* Latent attention: all heads read one cached latent c (rank rp = rank rounded up to 8 per position) that is key and value at
+ * once; a head's key and value projections are applied to its query and to its weighted sum instead.
+ *   latent_front   p row [cq (q_rank) at 0; c (rank) at off_c]: each over its root mean square times qn / cn;
+ *                  cq -> q_out (rows, q_rank rounded up to 8), c -> cache (cache rows, t_max, rp) and, if c_out, c_out (rows, rp)
+ *   head_linear    out[row, head, :] = W[head] x[row, head, :], W (h, n, k) row-major, n and k multiples of 8; x rows of ldx with
+ *                  heads k apart; out rows of ldo with heads n_out <= n apart (entries n_out .. n-1 are dropped, columns past
+ *                  h * n_out are set to zero); gate (rows of ldg, h * n_out entries): times sigmoid(gate)
+ *   attn_latent    q (rows, h, rp) -> out (rows, h, rp): sum_j softmax_j(scale q . c_j) c_j over j <= position, rank <= 512.
+ *                  n_split > 1: the context is cut into that many chunks that meet in `workspace`
+ *                  (ohara_attn_latent_workspace_bytes); a second launch merges them in chunk order. */
+int ohara_latent_front_bf16(const uint16_t* p, int ldp, int q_rank, int off_c, int rank, const float* qn, const float* cn,
+                            float eps, uint16_t* q_out, uint16_t* cache, int t_max, uint16_t* c_out, const OharaSeq* seq,
+                            void* stream);
+int ohara_latent_front_f32(const float* p, int ldp, int q_rank, int off_c, int rank, const float* qn, const float* cn,
+                           float eps, float* q_out, float* cache, int t_max, float* c_out, const OharaSeq* seq,
+                           void* stream);
+int ohara_head_linear_bf16(const uint16_t* x, int ldx, const uint16_t* w, int h, int n, int k, int n_out, int rows,
+                           const uint16_t* gate, int ldg, uint16_t* out, int ldo, void* stream);
+int ohara_head_linear_f32(const float* x, int ldx, const float* w, int h, int n, int k, int n_out, int rows, const float* gate,
+                          int ldg, float* out, int ldo, void* stream);
+int64_t ohara_attn_latent_workspace_bytes(int rows, int h, int rank, int n_split);
+int ohara_attn_latent_bf16(const uint16_t* q, const uint16_t* cache, int h, int rank, int t_max, float scale, int n_split,
+                           void* workspace, uint16_t* out, const OharaSeq* seq, void* stream);
+int ohara_attn_latent_f32(const float* q, const float* cache, int h, int rank, int t_max, float scale, int n_split,
+                          void* workspace, float* out, const OharaSeq* seq, void* stream);
+
 /* Gated delta rule with one decay per head and key channel.  Per value head: S (dim x vdim) fp32,
  *   S <- diag(exp(lg)) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q,
  *   q, k, v: short causal convolution per channel (taps), silu; q, k over sqrt(sum of squares + 1e-6), q also times
@@ -709,11 +772,15 @@ int ohara_attn_bias_f32(const float* q, const float* kcache, const float* vcache
  * a2 (heads*dim, rank_a), g2 (heads*vdim, rank_g) row-major in the activation type; conv_w (taps, channels) fp32 with the
  * current token's row last; state (cache rows, heads, dim, vdim rounded up to a multiple of 4) fp32; ring (cache rows,
  * taps, channels) in the activation type.  A sequence whose first token sits at position 0 starts from zero
- * whatever its state and ring hold.  dim, vdim <= 256. */
+ * whatever its state and ring hold.  dim, vdim <= 256.
+ * a2 == NULL: one decay per head, lg = neg_a[head] * softplus(a + dt_bias[head]) with the heads columns a from off_a (any offset;
+ * rank_a is not read).  g2 == NULL: the gate's heads*vdim columns come from off_g as they are (rank_g is not read).
+ * flags: OHARA_DELTA_SILU_GATE: the gate is silu instead of sigmoid. */
+#define OHARA_DELTA_SILU_GATE 1
 typedef struct OharaDelta {
   int heads, kv_heads, dim, vdim, taps, rank_a, rank_g, off_a, off_g, off_b;
   float eps;
-  int reserved;
+  int flags;
   const float* conv_w;
   const void* a2;
   const void* g2;
@@ -727,7 +794,7 @@ int ohara_delta_step_bf16(const OharaDelta* d, const uint16_t* p, int ldp, float
 int ohara_delta_step_f32(const OharaDelta* d, const float* p, int ldp, float* state, float* ring, float* out, int ldo,
                          const OharaSeq* seq, void* stream);
 /* Any number of tokens per sequence, in chunks of 32 tokens: za (rows, heads*dim) = W_a2 a1 and zg (rows, heads*vdim)
- * = W_g2 g1 come from the caller.  First the chunks are solved on their own in parallel, then the state walks
+ * = W_g2 g1 come from the caller (NULL where a2 / g2 is).  First the chunks are solved on their own in parallel, then the state walks
  * over them on fp32 matrix products; state is updated, the ring is only read (follow with
  * ohara_conv_ring_store over the first 2*kv_heads*dim + heads*vdim columns of p).  workspace:
  * ohara_delta_workspace_bytes for the number of tokens per sequence worked on at a time (the call cuts

@@ -11,8 +11,8 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "lib", "libohara_decode.so")
-# fewer sources, the same entry points where present (ohara_amd.build.ensure); loaded if the full library is not built
-PARTIAL_LIB_PATH = os.path.join(_HERE, "lib", "libohara_serving.so")
+# fewer sources, the same entry points where present: what ohara_amd.build.ensure built, loaded if the full library is not built
+partial_path = None
 
 OK, EINVAL, ELAUNCH, ESIZE = 0, -1, -2, -3
 _ERR = {EINVAL: "invalid argument", ELAUNCH: "HIP launch failed", ESIZE: "size not supported"}
@@ -68,12 +68,18 @@ class OharaSeq(C.Structure):
 class OharaDelta(C.Structure):
     _fields_ = [
         ("heads", _i), ("kv_heads", _i), ("dim", _i), ("vdim", _i), ("taps", _i), ("rank_a", _i), ("rank_g", _i),
-        ("off_a", _i), ("off_g", _i), ("off_b", _i), ("eps", _f), ("reserved", _i),
+        ("off_a", _i), ("off_g", _i), ("off_b", _i), ("eps", _f), ("flags", _i),
         ("conv_w", _p), ("a2", _p), ("g2", _p), ("neg_a", _p), ("dt_bias", _p), ("norm_w", _p),
     ]
 
 
+class OharaScores(C.Structure):
+    _fields_ = [("scale", _f), ("cap", _f), ("chunk", _i), ("gate_elements", _i), ("ld_k", _i), ("ld_v", _i), ("slopes", _p)]
+
+
 OUT_NONE, OUT_COPY, OUT_CONV, OUT_NORM = 0, 1, 2, 3
+CENTER_Y, CENTER_OUT = 16, 32
+DELTA_SILU_GATE = 1
 OHARA_LOGITS_NONE, OHARA_LOGITS_LAST, OHARA_LOGITS_ALL = 0, 1, 2
 
 _PROTOS = {
@@ -149,6 +155,12 @@ _PROTOS = {
         "conv_ring_store": (_i, [_p, _i, _i, _i, _p, C.POINTER(OharaSeq), _p]),
         "qkv_norm_append": (_i, [_p, _i, _i, _i, _i, _i, _p, _p, _f, _p, _p, _p, _i, C.POINTER(OharaSeq), _p]),
         "attn_bias": (_i, [_p, _p, _p, _i, _i, _i, _i, _i, _f, _p, _p, _i, _i, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "attn_scored": (_i, [_p, _p, _p, _i, _i, _i, _i, _i, C.POINTER(OharaScores), _p, _i, _i, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "qkv_rotate_append": (_i, [_p, _i, _i, _i, _i, _i, _p, _p, _i, _p, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "gemm_gelu_lookup": (_i, [_p, _i, _p, _i, _i, _p, _i, _p, _i, _i, _p, _i, _p]),
+        "latent_front": (_i, [_p, _i, _i, _i, _i, _p, _p, _f, _p, _p, _i, _p, C.POINTER(OharaSeq), _p]),
+        "head_linear": (_i, [_p, _i, _p, _i, _i, _i, _i, _i, _p, _i, _p, _i, _p]),
+        "attn_latent": (_i, [_p, _p, _i, _i, _i, _f, _i, _p, _p, C.POINTER(OharaSeq), _p]),
         "delta_step": (_i, [C.POINTER(OharaDelta), _p, _i, _p, _p, _p, _i, C.POINTER(OharaSeq), _p]),
         "delta_prefill": (_i, [C.POINTER(OharaDelta), _p, _i, _p, _i, _p, _i, _p, _p, _p, _i64, _p, _p, _i,
                                C.POINTER(OharaSeq), _p]),
@@ -156,6 +168,7 @@ _PROTOS = {
     "ohara_gemm_f32": (_i, [_p, _i, _p, _p, _p, _f, _i, _i, _i, _p, _i, _p]),
     "ohara_gemm_softcap_bf16": (_i, [_p, _i, _p, _i, _i, _f, _i, _p, _i, _p]),
     "ohara_attn_bias_workspace_bytes": (_i64, [_i, _i, _i, _i]),
+    "ohara_attn_latent_workspace_bytes": (_i64, [_i, _i, _i, _i]),
     "ohara_delta_workspace_bytes": (_i64, [_i, _i, _i, _i, _i]),
     "ohara_event_create": (_i, [C.POINTER(_p)]),
     "ohara_event_destroy": (_i, [_p]),
@@ -170,7 +183,7 @@ def lib():
     """The loaded library; raises if it was never built."""
     global _lib
     if _lib is None:
-        path = LIB_PATH if os.path.exists(LIB_PATH) else PARTIAL_LIB_PATH
+        path = LIB_PATH if os.path.exists(LIB_PATH) or partial_path is None else partial_path
         if not os.path.exists(path):
             raise RuntimeError(
                 f"{LIB_PATH} is missing: build the HIP kernels first (python -m ohara_amd.build). "
@@ -178,7 +191,7 @@ def lib():
             )
         handle = C.CDLL(path)
         for name, (res, args) in _PROTOS.items():
-            if path == PARTIAL_LIB_PATH and not hasattr(handle, name):
+            if path != LIB_PATH and not hasattr(handle, name):
                 continue  # an entry point of another kind of model: calling it raises
             fn = getattr(handle, name)
             fn.restype = res

@@ -18,10 +18,14 @@ INCLUDE = os.path.join(os.path.dirname(HERE), "include")
 LIB_DIR = os.path.join(HERE, "lib")
 OBJ_DIR = os.path.join(LIB_DIR, "obj")
 LIB_PATH = os.path.join(LIB_DIR, "libohara_decode.so")
-# A library of fewer sources for programs that serve one kind of model from a fresh checkout (``ensure``): the same
-# entry points, those of other models absent.
-PARTIAL_LIB_PATH = os.path.join(LIB_DIR, "libohara_serving.so")
-SERVING = ("attention_bias", "delta_rule", "gemm_f32", "gemm_skinny", "gemm_tile", "misc", "residual_norm", "sampler")
+# Libraries of fewer sources for programs that serve one design from a fresh checkout (``ensure``): the same entry
+# points, those of other models absent.
+_HYBRID = ("attention_bias", "delta_rule", "gemm_f32", "gemm_skinny", "gemm_tile", "misc", "residual_norm", "sampler")
+SERVING = {"Povazen": _HYBRID, "Vavelorn": (*_HYBRID, "latent")}
+
+
+def partial_path(design: str) -> str:
+    return os.path.join(LIB_DIR, f"libohara_{design.lower()}.so")
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = [
@@ -54,13 +58,14 @@ def _run(cmd: list[str]) -> str:
     return err
 
 
-def build_library(verbose: bool = False, incremental: bool = False, jobs: int = 8, only=None) -> str:
-    """One object per source (compiled in parallel), then one link.  ``only``: the names of the sources to build into
-    the partial library instead of all of them into the full one."""
+def build_library(verbose: bool = False, incremental: bool = False, jobs: int = 8, design: str | None = None) -> str:
+    """One object per source (compiled in parallel), then one link.  ``design``: only what that design needs, into its
+    partial library."""
+    only = None if design is None else SERVING[design]
     os.makedirs(OBJ_DIR, exist_ok=True)
     hdr = _headers_mtime()
     todo, objs = [], []
-    target = LIB_PATH if only is None else PARTIAL_LIB_PATH
+    target = LIB_PATH if design is None else partial_path(design)
     for src in sources():
         if only is not None and os.path.basename(src)[:-4] not in only:
             continue
@@ -82,15 +87,22 @@ def build_library(verbose: bool = False, incremental: bool = False, jobs: int = 
     return target
 
 
-def ensure(only) -> str:
-    """The full library if it is built, else the partial one with the sources ``only``, built now if it is missing or older than its sources."""
+def ensure(design: str | None = None) -> str:
+    """The full library if it is built, else the partial one of ``design`` (no such design: the full one), built now if it is
+    missing or older than its sources; ``_lib.lib()`` loads it from here on."""
+    from . import _lib
+
     if os.path.exists(LIB_PATH):
         return LIB_PATH
-    srcs = [s for s in sources() if os.path.basename(s)[:-4] in only]
+    if design not in SERVING:
+        return build_library(incremental=True)
+    path = partial_path(design)
+    srcs = [s for s in sources() if os.path.basename(s)[:-4] in SERVING[design]]
     newest = max(_headers_mtime(), *(os.path.getmtime(s) for s in srcs))
-    if not os.path.exists(PARTIAL_LIB_PATH) or os.path.getmtime(PARTIAL_LIB_PATH) < newest:
-        build_library(incremental=True, only=only)
-    return PARTIAL_LIB_PATH
+    if not os.path.exists(path) or os.path.getmtime(path) < newest:
+        build_library(incremental=True, design=design)
+    _lib.partial_path = path
+    return path
 
 
 if __name__ == "__main__":

@@ -128,7 +128,14 @@ def loop_moe_config(config: Config) -> Config:
 # config class (``from_dict``) and of the model class (config, state dict, device, dtype).
 ARCHITECTURES = {
     "Povazen": ("povazen", "PovazenConfig", "Povazen"),
+    "Vavelorn": ("vavelorn", "VavelornConfig", "Vavelorn"),
 }
+
+
+def architecture_of(path) -> str | None:
+    """The "architecture" that a folder's config.json names (None: no such file or entry)."""
+    cfg = Path(path) / "config.json"
+    return json.loads(cfg.read_text(encoding="utf-8")).get("architecture") if cfg.exists() else None
 
 
 def _architecture(name: str):

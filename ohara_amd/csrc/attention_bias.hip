@@ -1,7 +1,9 @@
-// Attention over the KV cache with a linear distance bias, norms over whole projections and a gate per head.
+// Attention over the KV cache with a linear distance bias or a soft cap on the scores, over the whole context or inside chunks,
+// and a gate per head or per element.
 //
 //   qkv_norm_append   q and k over the root mean square of the whole projection row, values over each head's,
 //                     keys and values into the cache: a workgroup per token
+//   qkv_rotate_append the same without norms, q and k rotated in neighbouring pairs
 //   attn_bias_kernel  one query token per workgroup (decode; any head width up to 256; bf16 or fp32)
 //   attn_bias_prefill many query tokens on bf16 MFMA
 //
@@ -110,6 +112,66 @@ __global__ __launch_bounds__(256) void qkv_norm_append_kernel(FrontArgs<T> a) {
   }
 }
 
+template <typename T>
+struct RotateArgs {
+  const T* p;
+  const float* cos;
+  const float* sin;
+  T* q;
+  T* kc;
+  T* vc;
+  int ldp, H, G, D, V, Tmax, rot;
+  OharaSeq seq;
+};
+
+// A thread takes P consecutive elements of one head (P = 4 where all sizes are multiples of 4, so that no rotated pair
+// is split, else 1).
+template <typename T, int P>
+__global__ __launch_bounds__(256) void qkv_rotate_append_kernel(RotateArgs<T> a) {
+  const int row = blockIdx.x, b = row / a.seq.seq_len, s = row - b * a.seq.seq_len;
+  const int pos = seq_start(a.seq, b) + s;
+  if (s >= seq_tokens(a.seq, b) || pos < 0 || pos >= a.Tmax) return;
+  const int Dp = (a.D + 7) & ~7, Vp = (a.V + 7) & ~7, half = a.rot / 2;
+  const T* p = a.p + (size_t)row * a.ldp;
+  const float *cs = a.cos + (size_t)pos * half, *sn = a.sin + (size_t)pos * half;
+  T* qo = a.q + (size_t)row * a.H * Dp;
+  const size_t crow = (size_t)seq_slot(a.seq, b) * a.Tmax + pos;
+  T* ko = a.kc + crow * a.G * Dp;
+  T* vo = a.vc + crow * a.G * Vp;
+  const int nqk = (a.H + a.G) * Dp, all = nqk + a.G * Vp;
+  for (int i = (blockIdx.y * 256 + threadIdx.x) * P; i < all; i += gridDim.y * 256 * P) {
+    const bool isv = i >= nqk;
+    const int j = isv ? i - nqk : i, w = isv ? Vp : Dp, h = j / w, c = j - h * w, n = isv ? a.V : a.D;
+    const T* src = p + (isv ? (a.H + a.G) * a.D + h * a.V : h * a.D);
+    T* dst = isv ? vo + h * Vp : (h < a.H ? qo + h * Dp : ko + (h - a.H) * Dp);
+    float v[4] = {0.f, 0.f, 0.f, 0.f};
+    if (P == 4) {
+      if (c < n) ld4(src + c, v);
+    } else if (c < n) {
+      v[0] = ldv(src + c);
+    }
+    if (!isv && c < a.rot) {
+      if (P == 1) {
+        const float x = ldv(src + (c ^ 1)), co = cs[c >> 1], si = sn[c >> 1];
+        v[0] = (c & 1) ? v[0] * co + x * si : v[0] * co - x * si;
+      } else {
+#pragma unroll
+        for (int u = 0; u < 4; u += 2)
+          if (c + u < a.rot) {
+            const float co = cs[(c + u) >> 1], si = sn[(c + u) >> 1], e = v[u], o = v[u + 1];
+            v[u] = e * co - o * si;
+            v[u + 1] = o * co + e * si;
+          }
+      }
+    }
+    if (P == 4) {
+      st4(dst + c, v);
+    } else {
+      stv(dst + c, v[0]);
+    }
+  }
+}
+
 // ---- one query token per workgroup -----------------------------------------------------------
 template <typename T>
 struct AttnBiasArgs {
@@ -120,6 +182,10 @@ struct AttnBiasArgs {
   const float* slopes;
   T* out;
   int H, G, D, V, Tmax, ldg, ldo;
+  int kd, vd;      // elements between neighbouring positions of the keys / values
+  int chunk;       // > 0: only keys of the query's own chunk are visible
+  int gate_elem;   // the gate has an entry per output element
+  float cap;       // CAP kernels: cap * tanh(score / cap)
   int rb, nhb;     // query heads served together (at most RB) and such sets per KV head
   int ns;
   float scale;
@@ -128,10 +194,17 @@ struct AttnBiasArgs {
   OharaSeq seq;
 };
 
+// tanh with an absolute error of about an ulp of 1: what a capped score of the bf16 kernels needs
+__device__ __forceinline__ float tanh_x(float v) { return 1.0f - 2.0f * __frcp_rn(1.0f + __expf(2.0f * v)); }
+template <typename T>
+__device__ __forceinline__ float gate_of(const AttnBiasArgs<T>& a, size_t row, int h, int c) {
+  return a.gate ? sigmoid_x(ldv(a.gate + row * a.ldg + (a.gate_elem ? h * a.V + c : h))) : 1.0f;
+}
+
 // LP lanes own one cached position (lane l elements 8l .. 8l+7 of key and value), so a workgroup walks 256 / LP
 // positions per round with an online softmax per lane group and query head; the groups are merged through LDS.
 // Scores are in log2 units.
-template <typename T, int LP, int RB>
+template <typename T, int LP, int RB, bool CAP>
 __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
   constexpr int NG = 256 / LP, W = 8 * LP;
   __shared__ float gm[RB][NG], gl[RB][NG];
@@ -158,7 +231,7 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
 #pragma unroll
   for (int r = 0; r < RB; ++r) {
     const int h = h0 + min(r, nh - 1);
-    slope[r] = a.slopes[h] * OHARA_LOG2E;
+    slope[r] = a.slopes ? a.slopes[h] * OHARA_LOG2E : 0.f;
     Raw8<T> v;
     v.load(a.q + ((size_t)row * a.H + h) * Dp + (ownk ? e0 : 0));
     v.get(qr[r]);
@@ -174,13 +247,13 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
     for (int u = 0; u < 8; ++u) acc[r][u] = 0.f;
   }
   // lanes past a row's end read its first elements: their products are zeroed (keys) or never stored (values)
-  const size_t kd = (size_t)a.G * Dp, vd = (size_t)a.G * Vp, base = (size_t)seq_slot(a.seq, b) * a.Tmax;
+  const size_t kd = a.kd, vd = a.vd, base = (size_t)seq_slot(a.seq, b) * a.Tmax;
   const T* kb = a.kc + base * kd + (size_t)g * Dp + (ownk ? e0 : 0);
   const T* vb = a.vc + base * vd + (size_t)g * Vp + (ownv ? e0 : 0);
-  int t_lo = 0, t_hi = pq;
+  int t_lo = a.chunk > 0 ? pq / a.chunk * a.chunk : 0, t_hi = pq;
   if (a.ns > 1) {
-    const int per = ((pq + a.ns) / a.ns + NG - 1) / NG * NG;  // ceil((pq + 1) / ns) in whole rounds
-    t_lo = blockIdx.y * per;
+    const int per = ((pq - t_lo + a.ns) / a.ns + NG - 1) / NG * NG;  // the visible positions over ns, in whole rounds
+    t_lo += blockIdx.y * per;
     t_hi = min(pq, t_lo + per - 1);
   }
   constexpr int R = 2;  // positions a lane group has in flight
@@ -207,7 +280,13 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
 #pragma unroll
         for (int u = 0; u < 8; ++u) dot = __builtin_fmaf(k[u], qr[r][u], dot);
         dot = lanes_sum<LP / 2, 1>(dot);
-        const float sc = dot * sl2 - slope[r] * dist;
+        float sc;
+        if constexpr (CAP) {
+          const float z = dot * a.scale / a.cap;
+          sc = a.cap * OHARA_LOG2E * (sizeof(T) == 4 ? tanhf(z) : tanh_x(z)) - slope[r] * dist;
+        } else {
+          sc = dot * sl2 - slope[r] * dist;
+        }
         const float mn = fmaxf(m[r], sc);
         const float corr = __builtin_amdgcn_exp2f(m[r] - mn), p = __builtin_amdgcn_exp2f(sc - mn);
         lsum[r] = lsum[r] * corr + p;
@@ -256,7 +335,7 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
         st_coh4(o + Vp + 1, __float_as_uint(hd[r]));
       }
     } else {
-      const float gt = a.gate ? sigmoid_x(ldv(a.gate + (size_t)row * a.ldg + h)) : 1.0f;
+      const float gt = gate_of(a, row, h, c);
       stv(a.out + (size_t)row * a.ldo + h * a.V + c, num / hd[r] * gt);
     }
   }
@@ -302,7 +381,7 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
         num += wg == 0.f ? 0.f : wg * av[n];
       }
     }
-    const float gt = a.gate ? sigmoid_x(ldv(a.gate + (size_t)row * a.ldg + h)) : 1.0f;
+    const float gt = gate_of(a, row, h, c);
     stv(a.out + (size_t)row * a.ldo + h * a.V + c, num / hd[r] * gt);
   }
 }
@@ -314,7 +393,7 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
 // the B operand of the second product (k-slot 8 g + i of window w <-> position 32 w + 4 g + i for i < 4,
 // 32 w + 16 + 4 g + i - 4 otherwise).  The running maximum is kept as an integer in log2 units, so most tiles leave it
 // alone and the accumulators need no rescaling.
-template <int DP, int VP, int QW>
+template <int DP, int VP, int QW, bool CAP>
 __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias_prefill_kernel(AttnBiasArgs<bf16_t> a, int nqb) {
   constexpr int KT = 64, NK = DP / 32, ND = VP / 16;
   constexpr int LDK = DP + 8, LDV = KT + 4;
@@ -335,22 +414,24 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
   if (q0 >= len || pos0 < 0 || pos0 + len > a.Tmax) return;
   const int Dq = (a.D + 7) & ~7, Vq = (a.V + 7) & ~7;
   const int kvh = h / (a.H / a.G);
-  const size_t kd = (size_t)a.G * Dq, vd = (size_t)a.G * Vq, base = (size_t)seq_slot(a.seq, b) * a.Tmax;
+  const size_t kd = a.kd, vd = a.vd, base = (size_t)seq_slot(a.seq, b) * a.Tmax;
   const bf16_t* kb = a.kc + base * kd + (size_t)kvh * Dq;
   const bf16_t* vb = a.vc + base * vd + (size_t)kvh * Vq;
   const int Lall = pos0 + len;
   const int kv_end = min(pos0 + q0 + 64 * QW, Lall);
   const int wq0 = q0 + wave * 16 * QW;
   const int wave_last = min(pos0 + wq0 + 16 * QW - 1, Lall - 1);
-  const float sl2 = a.scale * OHARA_LOG2E, slope = a.slopes[h] * OHARA_LOG2E;
+  const float sl2 = a.scale * OHARA_LOG2E, slope = a.slopes ? a.slopes[h] * OHARA_LOG2E : 0.f;
+  const float icap = CAP ? a.scale / a.cap : 0.f, cap2 = CAP ? a.cap * OHARA_LOG2E : 0.f;
 
   uint4 qf[QW][NK];
-  int qpos[QW];
+  int qpos[QW], qlow[QW];  // a query's own position and the first one it sees
   size_t qrow[QW];
 #pragma unroll
   for (int u = 0; u < QW; ++u) {
     const int qi = min(wq0 + 16 * u + m, len - 1);  // lanes past the end repeat the last query and are not stored
     qpos[u] = pos0 + qi;
+    qlow[u] = a.chunk > 0 ? qpos[u] / a.chunk * a.chunk : 0;
     qrow[u] = (size_t)b * a.seq.seq_len + qi;
 #pragma unroll
     for (int j = 0; j < NK; ++j)
@@ -360,7 +441,7 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
   float mrun[QW], lrun[QW];
 #pragma unroll
   for (int u = 0; u < QW; ++u) {
-    mrun[u] = -INFINITY;
+    mrun[u] = -1e30f;  // finite: a tile may lie wholly outside a query's window
     lrun[u] = 0.f;
 #pragma unroll
     for (int t = 0; t < ND; ++t) o[u][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -419,13 +500,20 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
     }
   };
 
-  load_tile(0);
-  for (int t0 = 0; t0 < kv_end; t0 += KT) {
+  // with chunks: from the tile of the first position the workgroup's / the wave's first query sees
+  int t_first = 0, wave_low = 0, wave_low_last = 0;
+  if (a.chunk > 0) {
+    t_first = (pos0 + q0) / a.chunk * a.chunk / KT * KT;
+    wave_low = (pos0 + min(wq0, len - 1)) / a.chunk * a.chunk;
+    wave_low_last = wave_last / a.chunk * a.chunk;
+  }
+  load_tile(t_first);
+  for (int t0 = t_first; t0 < kv_end; t0 += KT) {
     __syncthreads();  // everyone is done with the previous tile
     store_tile();
     __syncthreads();
     if (t0 + KT < kv_end) load_tile(t0 + KT);  // in flight during the products
-    if (t0 > wave_last) continue;               // wholly masked for this wave (barriers stay uniform)
+    if (t0 > wave_last || t0 + KT <= wave_low) continue;  // wholly masked for this wave (barriers stay uniform)
     f32x4 s[4][QW];
 #pragma unroll
     for (int kk = 0; kk < 4; ++kk) {
@@ -442,7 +530,8 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
           s[kk][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kf[j]), __builtin_bit_cast(bf16x8, qf[u][j]),
                                                              s[kk][u], 0, 0, 0);
     }
-    const bool edge = t0 + KT - 1 > pos0 + wq0;  // (wave-uniform) the tile reaches past the wave's first query
+    // (wave-uniform) the tile reaches past the wave's first query or before what its last one sees
+    const bool edge = t0 + KT - 1 > pos0 + wq0 || t0 < wave_low_last;
 #pragma unroll
     for (int u = 0; u < QW; ++u) {
       float tmax = -INFINITY;
@@ -451,13 +540,15 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
       for (int kk = 0; kk < 4; ++kk)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          float v = __builtin_fmaf(s[kk][u][i], sl2, __builtin_fmaf(slope, (float)(16 * kk + i), b0));
-          if (edge && t0 + 16 * kk + 4 * g + i > qpos[u]) v = -INFINITY;
+          const float bias = __builtin_fmaf(slope, (float)(16 * kk + i), b0);
+          float v = CAP ? __builtin_fmaf(cap2, tanh_x(s[kk][u][i] * icap), bias) : __builtin_fmaf(s[kk][u][i], sl2, bias);
+          const int t = t0 + 16 * kk + 4 * g + i;
+          if (edge && (t > qpos[u] || t < qlow[u])) v = -INFINITY;
           s[kk][u][i] = v;
           tmax = fmaxf(tmax, v);
         }
       tmax = lane_xor_max<32>(lane_xor_max<16>(tmax));
-      const float mn = fmaxf(mrun[u], ceilf(tmax));  // finite: position 0 is visible to every query
+      const float mn = fmaxf(mrun[u], ceilf(tmax));
       const float corr = __builtin_amdgcn_exp2f(mrun[u] - mn);
       mrun[u] = mn;
       float ts = 0.f;
@@ -522,19 +613,21 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
   for (int u = 0; u < QW; ++u) {
     const float l = lane_xor_sum<32>(lane_xor_sum<16>(lrun[u]));
     if (wq0 + 16 * u + m >= len) continue;
-    const float inv = (a.gate ? sigmoid_x(ldv(a.gate + qrow[u] * a.ldg + h)) : 1.0f) / l;
+    const float inv = (a.gate_elem ? 1.0f : gate_of(a, qrow[u], h, 0)) / l;
     bf16_t* orow = a.out + qrow[u] * a.ldo;
     const bool wide = ((a.V | a.ldo) & 3) == 0;
 #pragma unroll
     for (int t = 0; t < ND; ++t) {
       const int c = 16 * t + 4 * g;
+      float v[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = o[u][t][i] * inv * (a.gate_elem && c + i < a.V ? gate_of(a, qrow[u], h, c + i) : 1.0f);
       if (wide) {
-        const float v[4] = {o[u][t][0] * inv, o[u][t][1] * inv, o[u][t][2] * inv, o[u][t][3] * inv};
         if (c < a.V) st4(orow + (size_t)h * a.V + c, v);
       } else {
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          if (c + i < a.V) orow[(size_t)h * a.V + c + i] = f2bf(o[u][t][i] * inv);
+          if (c + i < a.V) orow[(size_t)h * a.V + c + i] = f2bf(v[i]);
       }
     }
     if (h == 0 && g == 0)
@@ -542,8 +635,8 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
   }
 }
 
-template <int DP, int VP>
-int launch_prefill_dv(const AttnBiasArgs<bf16_t>& a, hipStream_t st) {
+template <int DP, int VP, bool CAP>
+int launch_prefill_cap(const AttnBiasArgs<bf16_t>& a, hipStream_t st) {
   // 32 queries per wave where there are enough workgroups for it: half the LDS reads per product
   constexpr int QW = DP + VP <= 256 ? 2 : 1;
   static int cus = 0;
@@ -554,12 +647,17 @@ int launch_prefill_dv(const AttnBiasArgs<bf16_t>& a, hipStream_t st) {
   }
   const int n2 = (a.seq.seq_len + 64 * QW - 1) / (64 * QW), n1 = (a.seq.seq_len + 63) / 64;
   if (QW > 1 && (int64_t)n2 * a.H * a.seq.batch >= 2 * (int64_t)cus)
-    hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, VP, QW>), dim3((unsigned)n2, (unsigned)a.H, (unsigned)a.seq.batch), dim3(256),
+    hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, VP, QW, CAP>), dim3((unsigned)n2, (unsigned)a.H, (unsigned)a.seq.batch), dim3(256),
                        0, st, a, n2);
   else
-    hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, VP, 1>), dim3((unsigned)n1, (unsigned)a.H, (unsigned)a.seq.batch), dim3(256),
+    hipLaunchKernelGGL((attn_bias_prefill_kernel<DP, VP, 1, CAP>), dim3((unsigned)n1, (unsigned)a.H, (unsigned)a.seq.batch), dim3(256),
                        0, st, a, n1);
   return ohara_launch_status();
+}
+
+template <int DP, int VP>
+int launch_prefill_dv(const AttnBiasArgs<bf16_t>& a, hipStream_t st) {
+  return a.cap > 0.f ? launch_prefill_cap<DP, VP, true>(a, st) : launch_prefill_cap<DP, VP, false>(a, st);
 }
 
 template <int DP>
@@ -588,7 +686,23 @@ int launch_front(const FrontArgs<T>& a, hipStream_t st) {
   return ohara_launch_status();
 }
 
-template <typename T, int LP>
+template <typename T>
+int launch_rotate(const RotateArgs<T>& a, hipStream_t st) {
+  if (!a.p || !a.q || !a.kc || !a.vc || !seq_ok(&a.seq)) return OHARA_EINVAL;
+  if (a.H < 1 || a.G < 1 || a.H % a.G || a.D < 1 || a.V < 1 || a.Tmax < 1) return OHARA_EINVAL;
+  if (a.rot < 0 || (a.rot & 1) || a.rot > a.D || (a.rot && (!a.cos || !a.sin))) return OHARA_EINVAL;
+  if (a.ldp < a.H * a.D + a.G * (a.D + a.V)) return OHARA_EINVAL;
+  if (!a.seq.pos_dev && a.seq.pos + a.seq.seq_len > a.Tmax) return OHARA_EINVAL;
+  const int all = (a.H + a.G) * ((a.D + 7) & ~7) + a.G * ((a.V + 7) & ~7);
+  const int P = ((a.D | a.V | a.ldp) & 3) == 0 ? 4 : 1;
+  const int ny = (all + 256 * P - 1) / (256 * P);
+  const dim3 grid((unsigned)(a.seq.batch * a.seq.seq_len), (unsigned)(ny < 8 ? ny : 8));
+  if (P == 4) hipLaunchKernelGGL((qkv_rotate_append_kernel<T, 4>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((qkv_rotate_append_kernel<T, 1>), grid, dim3(256), 0, st, a);
+  return ohara_launch_status();
+}
+
+template <typename T, int LP, bool CAP>
 int launch_bias_rb(AttnBiasArgs<T> a, hipStream_t st) {
   const int rep = a.H / a.G;
   a.rb = rep >= 4 ? 4 : (rep >= 2 ? 2 : 1);
@@ -596,18 +710,31 @@ int launch_bias_rb(AttnBiasArgs<T> a, hipStream_t st) {
   const int64_t gx = (int64_t)a.seq.batch * a.seq.seq_len * a.G * a.nhb;
   if (gx > INT32_MAX) return OHARA_ESIZE;
   const dim3 grid((unsigned)gx, (unsigned)a.ns);
-  if (a.rb == 4) hipLaunchKernelGGL((attn_bias_kernel<T, LP, 4>), grid, dim3(256), 0, st, a);
-  else if (a.rb == 2) hipLaunchKernelGGL((attn_bias_kernel<T, LP, 2>), grid, dim3(256), 0, st, a);
-  else hipLaunchKernelGGL((attn_bias_kernel<T, LP, 1>), grid, dim3(256), 0, st, a);
+  if (a.rb == 4) hipLaunchKernelGGL((attn_bias_kernel<T, LP, 4, CAP>), grid, dim3(256), 0, st, a);
+  else if (a.rb == 2) hipLaunchKernelGGL((attn_bias_kernel<T, LP, 2, CAP>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((attn_bias_kernel<T, LP, 1, CAP>), grid, dim3(256), 0, st, a);
   return ohara_launch_status();
+}
+
+template <typename T, bool CAP>
+int launch_bias_lp(const AttnBiasArgs<T>& a, hipStream_t st) {
+  const int w = a.D > a.V ? a.D : a.V;
+  if (w <= 64) return launch_bias_rb<T, 8, CAP>(a, st);
+  if (w <= 128) return launch_bias_rb<T, 16, CAP>(a, st);
+  return launch_bias_rb<T, 32, CAP>(a, st);
 }
 
 template <typename T>
 int launch_bias(AttnBiasArgs<T> a, void* workspace, hipStream_t st) {
-  if (!a.q || !a.kc || !a.vc || !a.slopes || !a.out || !seq_ok(&a.seq)) return OHARA_EINVAL;
+  if (!a.q || !a.kc || !a.vc || !a.out || !seq_ok(&a.seq)) return OHARA_EINVAL;
   if (a.H < 1 || a.G < 1 || a.H % a.G || a.D < 1 || a.V < 1 || a.Tmax < 1) return OHARA_EINVAL;
   if (a.D > 256 || a.V > 256) return OHARA_ESIZE;
-  if (a.ldo < a.H * a.V || (a.gate && a.ldg < 1)) return OHARA_EINVAL;
+  if (a.ldo < a.H * a.V || (a.gate && a.ldg < (a.gate_elem ? a.H * a.V : 1))) return OHARA_EINVAL;
+  if (a.chunk < 0 || !(a.cap >= 0.f)) return OHARA_EINVAL;
+  const int kd = a.G * ((a.D + 7) & ~7), vd = a.G * ((a.V + 7) & ~7);
+  if (!a.kd) a.kd = kd;
+  if (!a.vd) a.vd = vd;
+  if (a.kd < kd || a.vd < vd || ((a.kd | a.vd) & 7)) return OHARA_EINVAL;  // 16-byte loads
   if (!a.seq.pos_dev && a.seq.pos + a.seq.seq_len > a.Tmax) return OHARA_EINVAL;
   if (a.ns < 1 || a.ns > 64 || (a.ns > 1 && (!workspace || a.seq.seq_len != 1))) return OHARA_EINVAL;
   const size_t cbytes = (((size_t)a.seq.batch * a.H * sizeof(int)) + 255) & ~(size_t)255;
@@ -616,10 +743,20 @@ int launch_bias(AttnBiasArgs<T> a, void* workspace, hipStream_t st) {
   if constexpr (sizeof(T) == 2) {
     if (a.seq.seq_len >= 16 && a.H <= 65535 && a.seq.batch <= 65535) return launch_prefill(a, st);
   }
-  const int w = a.D > a.V ? a.D : a.V;
-  if (w <= 64) return launch_bias_rb<T, 8>(a, st);
-  if (w <= 128) return launch_bias_rb<T, 16>(a, st);
-  return launch_bias_rb<T, 32>(a, st);
+  return a.cap > 0.f ? launch_bias_lp<T, true>(a, st) : launch_bias_lp<T, false>(a, st);
+}
+
+template <typename T>
+int attn_scored(const T* q, const T* kcache, const T* vcache, int h, int h_kv, int dh, int dv, int t_max,
+                const OharaScores* sc, const T* gate, int ldg, int n_split, void* workspace, T* out, int ldo,
+                const OharaSeq* seq, void* stream) {
+  if (!seq || !sc) return OHARA_EINVAL;
+  AttnBiasArgs<T> a{};
+  a.q = q; a.kc = kcache; a.vc = vcache; a.gate = gate; a.slopes = sc->slopes; a.out = out;
+  a.H = h; a.G = h_kv; a.D = dh; a.V = dv; a.Tmax = t_max; a.ldg = ldg; a.ldo = ldo; a.ns = n_split; a.scale = sc->scale;
+  a.cap = sc->cap; a.chunk = sc->chunk; a.gate_elem = sc->gate_elements != 0; a.kd = sc->ld_k; a.vd = sc->ld_v;
+  a.seq = *seq;
+  return launch_bias<T>(a, workspace, (hipStream_t)stream);
 }
 
 }  // namespace
@@ -650,22 +787,42 @@ int64_t ohara_attn_bias_workspace_bytes(int rows, int h, int dv, int n_split) {
 int ohara_attn_bias_bf16(const uint16_t* q, const uint16_t* kcache, const uint16_t* vcache, int h, int h_kv, int dh,
                          int dv, int t_max, float scale, const float* slopes, const uint16_t* gate, int ldg, int n_split,
                          void* workspace, uint16_t* out, int ldo, const OharaSeq* seq, void* stream) {
-  if (!seq) return OHARA_EINVAL;
-  AttnBiasArgs<bf16_t> a{};
-  a.q = q; a.kc = kcache; a.vc = vcache; a.gate = gate; a.slopes = slopes; a.out = out;
-  a.H = h; a.G = h_kv; a.D = dh; a.V = dv; a.Tmax = t_max; a.ldg = ldg; a.ldo = ldo; a.ns = n_split; a.scale = scale;
-  a.seq = *seq;
-  return launch_bias<bf16_t>(a, workspace, (hipStream_t)stream);
+  if (!slopes) return OHARA_EINVAL;
+  const OharaScores sc{scale, 0.f, 0, 0, 0, 0, slopes};
+  return attn_scored<bf16_t>(q, kcache, vcache, h, h_kv, dh, dv, t_max, &sc, gate, ldg, n_split, workspace, out, ldo, seq, stream);
 }
 int ohara_attn_bias_f32(const float* q, const float* kcache, const float* vcache, int h, int h_kv, int dh, int dv,
                         int t_max, float scale, const float* slopes, const float* gate, int ldg, int n_split,
                         void* workspace, float* out, int ldo, const OharaSeq* seq, void* stream) {
+  if (!slopes) return OHARA_EINVAL;
+  const OharaScores sc{scale, 0.f, 0, 0, 0, 0, slopes};
+  return attn_scored<float>(q, kcache, vcache, h, h_kv, dh, dv, t_max, &sc, gate, ldg, n_split, workspace, out, ldo, seq, stream);
+}
+
+int ohara_attn_scored_bf16(const uint16_t* q, const uint16_t* kcache, const uint16_t* vcache, int h, int h_kv, int dh,
+                           int dv, int t_max, const OharaScores* sc, const uint16_t* gate, int ldg, int n_split,
+                           void* workspace, uint16_t* out, int ldo, const OharaSeq* seq, void* stream) {
+  return attn_scored<bf16_t>(q, kcache, vcache, h, h_kv, dh, dv, t_max, sc, gate, ldg, n_split, workspace, out, ldo, seq, stream);
+}
+int ohara_attn_scored_f32(const float* q, const float* kcache, const float* vcache, int h, int h_kv, int dh, int dv,
+                          int t_max, const OharaScores* sc, const float* gate, int ldg, int n_split, void* workspace,
+                          float* out, int ldo, const OharaSeq* seq, void* stream) {
+  return attn_scored<float>(q, kcache, vcache, h, h_kv, dh, dv, t_max, sc, gate, ldg, n_split, workspace, out, ldo, seq, stream);
+}
+
+int ohara_qkv_rotate_append_bf16(const uint16_t* p, int ldp, int h, int h_kv, int dh, int dv, const float* cos,
+                                 const float* sin, int rot, uint16_t* q_out, uint16_t* kcache, uint16_t* vcache, int t_max,
+                                 const OharaSeq* seq, void* stream) {
   if (!seq) return OHARA_EINVAL;
-  AttnBiasArgs<float> a{};
-  a.q = q; a.kc = kcache; a.vc = vcache; a.gate = gate; a.slopes = slopes; a.out = out;
-  a.H = h; a.G = h_kv; a.D = dh; a.V = dv; a.Tmax = t_max; a.ldg = ldg; a.ldo = ldo; a.ns = n_split; a.scale = scale;
-  a.seq = *seq;
-  return launch_bias<float>(a, workspace, (hipStream_t)stream);
+  return launch_rotate<bf16_t>(RotateArgs<bf16_t>{p, cos, sin, q_out, kcache, vcache, ldp, h, h_kv, dh, dv, t_max, rot, *seq},
+                               (hipStream_t)stream);
+}
+int ohara_qkv_rotate_append_f32(const float* p, int ldp, int h, int h_kv, int dh, int dv, const float* cos, const float* sin,
+                                int rot, float* q_out, float* kcache, float* vcache, int t_max, const OharaSeq* seq,
+                                void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  return launch_rotate<float>(RotateArgs<float>{p, cos, sin, q_out, kcache, vcache, ldp, h, h_kv, dh, dv, t_max, rot, *seq},
+                              (hipStream_t)stream);
 }
 
 }  // extern "C"

@@ -308,6 +308,11 @@ __device__ __forceinline__ void wait_own_stores() {
 // epilogue made a fifth of that kernel's time.
 __device__ __forceinline__ float silu_f(float x) { return x * __frcp_rn(1.0f + __expf(-x)); }
 
+// z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))) in fp32
+__device__ __forceinline__ float gelu_tanh(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+
 // Host-side launch check: every entry point returns OHARA_ELAUNCH when the
 // launch itself was rejected.
 static inline int ohara_launch_status() {

@@ -1,5 +1,5 @@
-// Gated delta rule with one decay per head and key channel, with its short convolutions, unit norms, step sizes and
-// gated output norm.  Per value head, S (dim x vdim, fp32) from zero:
+// Gated delta rule with one decay per head and key channel or one per head, with its short convolutions, unit norms, step
+// sizes and gated output norm.  Per value head, S (dim x vdim, fp32) from zero:
 //   S <- diag(exp(lg)) S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q.
 //
 // delta_step_kernel: one token per sequence, everything in one launch, a workgroup per (sequence, value head).  The
@@ -37,6 +37,10 @@ struct DeltaArgs {
   int chunk0, nchunks;  // chunks of this segment
   OharaSeq seq;
 };
+
+__device__ __forceinline__ float out_gate(const OharaDelta& d, float z) {
+  return d.flags & OHARA_DELTA_SILU_GATE ? silu_x(z) : sigmoid_x(z);
+}
 
 __host__ __device__ __forceinline__ int up(int v, int m) { return (v + m - 1) / m * m; }
 
@@ -89,11 +93,18 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaArgs<T> a) {
     else vs[i - 2 * D] = y;
   }
   // decays and output gates: eight lanes per row of a2 / g2, two rows and 128 columns in flight
-  {
+  const float na = dd.neg_a[h];
+  if (!dd.a2) {
+    const float g = expf(na * softplus_x(ldv(p + dd.off_a + h) + dd.dt_bias[h]));
+    for (int i = tid; i < D; i += NT) gs[i] = g;
+  }
+  if (!dd.g2)
+    for (int i = tid; i < V; i += NT) gate[i] = out_gate(dd, ldv(p + dd.off_g + h * V + i));
+  if (dd.a2 || dd.g2) {
     const int l8 = tid & 7;
-    const float na = dd.neg_a[h];
     constexpr int RP = NT / 8;  // rows per pass
-    for (int r0 = 0; r0 < D + V; r0 += 2 * RP) {
+    const int r_end = dd.g2 ? D + V : D;
+    for (int r0 = dd.a2 ? 0 : D; r0 < r_end; r0 += 2 * RP) {
       float s[2] = {0.f, 0.f};
       const int nmax = max(dd.rank_a, dd.rank_g);
       for (int i0 = 0; i0 < nmax; i0 += 128) {
@@ -108,7 +119,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaArgs<T> a) {
 #pragma unroll
           for (int e = 0; e < 2; ++e) {
             const int i = i0 + 64 * e + 8 * l8;
-            if (r < D + V && i < n) {
+            if (r < r_end && i < n) {
               wv[u][e].load(wrow + i);
               xv[u][e].load(xr + i);
             } else {
@@ -132,9 +143,9 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(DeltaArgs<T> a) {
       for (int u = 0; u < 2; ++u) {
         const int r = r0 + u * RP + (tid >> 3);
         const float z = lanes_sum<4, 1>(s[u]);
-        if (r < D + V && l8 == 0) {
+        if (r < r_end && l8 == 0) {
           if (r < D) gs[r] = expf(na * softplus_x(z + dd.dt_bias[(size_t)h * D + r]));
-          else gate[r - D] = sigmoid_x(z);
+          else gate[r - D] = out_gate(dd, z);
         }
       }
     }
@@ -284,6 +295,7 @@ __global__ __launch_bounds__(256, 2) void chunk_solve_kernel(DeltaArgs<T> a) {
   const T* prow = a.p + (size_t)b * a.seq.seq_len * a.ldp;  // row of the sequence's first token in this call
   const T* zrow = a.za + (size_t)b * a.seq.seq_len * a.ldza + (size_t)h * D;
   const float na = dd.neg_a[h];
+  const bool per_head = !dd.a2;  // one decay for all channels
   if (tid < C) beta[tid] = tid < n ? sigmoid_x(ldv(prow + (size_t)(s0 + tid) * a.ldp + dd.off_b + h)) : 0.f;
   if constexpr (TAPS > 0) {
     const int d8 = D / 8, v8 = V / 8;
@@ -302,7 +314,7 @@ __global__ __launch_bounds__(256, 2) void chunk_solve_kernel(DeltaArgs<T> a) {
       }
     }
     // decays: 8 channels of two tokens per thread and round
-    for (int it = tid; it < d8 * (C / 2); it += 256) {
+    for (int it = tid; !per_head && it < d8 * (C / 2); it += 256) {
       const int t = it / d8, c = 8 * (it % d8);
       Raw8<T> z[2];
 #pragma unroll
@@ -346,12 +358,17 @@ __global__ __launch_bounds__(256, 2) void chunk_solve_kernel(DeltaArgs<T> a) {
       const bool in = t < n && c < D;
       Q[t * LD + c] = in ? conv(s0 + t, kvh * D + c) : 0.f;
       K[t * LD + c] = in ? conv(s0 + t, nqk + kvh * D + c) : 0.f;
-      G[t * LD + c] = in ? na * softplus_x(ldv(zrow + (size_t)(s0 + t) * a.ldza + c) + dd.dt_bias[(size_t)h * D + c]) : 0.f;
+      G[t * LD + c] = in && !per_head ? na * softplus_x(ldv(zrow + (size_t)(s0 + t) * a.ldza + c) + dd.dt_bias[(size_t)h * D + c]) : 0.f;
     }
     for (int i = tid; i < C * Vq; i += 256) {
       const int t = i / Vq, c = i - t * Vq;
       X[i] = t < n && c < V ? conv(s0 + t, 2 * nqk + h * V + c) : 0.f;
     }
+  }
+  if (per_head) {
+    if (tid < C) A[tid] = tid < n ? na * softplus_x(ldv(prow + (size_t)(s0 + tid) * a.ldp + dd.off_a + h) + dd.dt_bias[h]) : 0.f;
+    __syncthreads();
+    for (int i = tid; i < C * D; i += 256) G[i / D * LD + i % D] = A[i / D];
   }
   __syncthreads();
   // unit q and k, and the diagonal of B: eight lanes per token; running sums: a channel per thread
@@ -676,7 +693,7 @@ __global__ __launch_bounds__(512) void chunk_walk_kernel(DeltaArgs<T> a) {
   }
 }
 
-// out = o / rms(o) * norm_w * sigmoid(zg): a wave per (row, head)
+// out = o / rms(o) * norm_w * gate: a wave per (row, head)
 template <typename T>
 __global__ __launch_bounds__(256) void delta_out_kernel(DeltaArgs<T> a) {
   const OharaDelta& dd = a.d;
@@ -684,6 +701,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaArgs<T> a) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int row = blockIdx.x, b = row / a.seq.seq_len, s = row - b * a.seq.seq_len;
   T* orow = a.out + (size_t)row * a.ldo;
+  const T* zg = dd.g2 ? a.zg + (size_t)row * a.ldzg : a.p + (size_t)row * a.ldp + dd.off_g;
   for (int i = H * V + threadIdx.x; i < a.ldo; i += 256) stv(orow + i, 0.f);
   if (s >= seq_tokens(a.seq, b)) return;
   for (int h = blockIdx.y * 4 + wave; h < H; h += 4 * gridDim.y) {
@@ -693,25 +711,27 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaArgs<T> a) {
     for (int u = 0; u < 4; ++u) {
       const int c = lane + 64 * u;
       v[u] = c < V ? o[c] : 0.f;
-      z[u] = c < V ? ldv(a.zg + (size_t)row * a.ldzg + (size_t)h * V + c) : 0.f;
+      z[u] = c < V ? ldv(zg + (size_t)h * V + c) : 0.f;
       ss += v[u] * v[u];
     }
     const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)V + dd.eps);
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
       const int c = lane + 64 * u;
-      if (c < V) stv(orow + h * V + c, v[u] * inv * dd.norm_w[c] * sigmoid_x(z[u]));
+      if (c < V) stv(orow + h * V + c, v[u] * inv * dd.norm_w[c] * out_gate(dd, z[u]));
     }
   }
 }
 
 bool delta_ok(const OharaDelta* d, int ldp) {
-  if (!d || !d->conv_w || !d->a2 || !d->g2 || !d->neg_a || !d->dt_bias || !d->norm_w) return false;
+  if (!d || !d->conv_w || !d->neg_a || !d->dt_bias || !d->norm_w) return false;
   if (d->heads < 1 || d->kv_heads < 1 || d->heads % d->kv_heads || d->dim < 1 || d->vdim < 1 || d->taps < 1) return false;
   const int channels = 2 * d->kv_heads * d->dim + d->heads * d->vdim;
-  if (d->rank_a < 8 || d->rank_g < 8 || ((d->rank_a | d->rank_g | d->off_a | d->off_g | ldp) & 7)) return false;
-  return ldp >= channels && d->off_a >= channels && d->off_a + d->rank_a <= ldp && d->off_g >= channels &&
-         d->off_g + d->rank_g <= ldp && d->off_b >= channels && d->off_b + d->heads <= ldp;
+  if (d->a2 && (d->rank_a < 8 || ((d->rank_a | d->off_a) & 7))) return false;
+  if (d->g2 && (d->rank_g < 8 || ((d->rank_g | d->off_g) & 7))) return false;
+  const int na = d->a2 ? d->rank_a : d->heads, ng = d->g2 ? d->rank_g : d->heads * d->vdim;
+  return (ldp & 7) == 0 && ldp >= channels && d->off_a >= channels && d->off_a + na <= ldp && d->off_g >= channels &&
+         d->off_g + ng <= ldp && d->off_b >= channels && d->off_b + d->heads <= ldp;
 }
 
 template <typename T>
@@ -739,8 +759,8 @@ int delta_step(const OharaDelta* d, const T* p, int ldp, float* state, T* ring, 
 template <typename T>
 int delta_prefill(const OharaDelta* d, const T* p, int ldp, const T* za, int ldza, const T* zg, int ldzg, float* state,
                   const T* ring, void* ws, int64_t ws_bytes, float* o, T* out, int ldo, const OharaSeq* seq, hipStream_t st) {
-  if (!delta_ok(d, ldp) || !p || !za || !zg || !state || !ring || !ws || !o || !out || !seq_ok(seq)) return OHARA_EINVAL;
-  if (ldo < d->heads * d->vdim || ldza < d->heads * d->dim || ldzg < d->heads * d->vdim) return OHARA_EINVAL;
+  if (!delta_ok(d, ldp) || !p || (d->a2 && !za) || (d->g2 && !zg) || !state || !ring || !ws || !o || !out || !seq_ok(seq)) return OHARA_EINVAL;
+  if (ldo < d->heads * d->vdim || (d->a2 && ldza < d->heads * d->dim) || (d->g2 && ldzg < d->heads * d->vdim)) return OHARA_EINVAL;
   if (d->dim > 256 || d->vdim > 256 || d->heads > 65535 || seq->batch > 65535) return OHARA_ESIZE;
   DeltaArgs<T> a{};
   a.d = *d; a.p = p; a.ldp = ldp; a.za = za; a.ldza = ldza; a.zg = zg; a.ldzg = ldzg; a.state = state;

@@ -5,10 +5,11 @@
 //   rotary + KV append ohara/embeddings_pos/rotary.py:55-93, ohara/modules/kv_cache.py:104-105
 //   bias / new_gelu / parallel-block sum of Phi   ohara/models/phi.py:37-52, :147-151
 //   soft cap of the fp32 sum (vocabulary projections with capped logits)
+//   gelu of the fp32 sum times an embedding of the row's token
 #pragma once
 #include "common.h"
 
-enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3, EPI_BIAS = 4, EPI_BIAS_GELU = 5, EPI_BIAS_ADD2 = 6, EPI_PHI_IN = 7, EPI_SOFTCAP = 8 };
+enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3, EPI_BIAS = 4, EPI_BIAS_GELU = 5, EPI_BIAS_ADD2 = 6, EPI_PHI_IN = 7, EPI_SOFTCAP = 8, EPI_GELU_LOOKUP = 9 };
 
 struct GemmArgs {
   const uint4* wp;
@@ -45,6 +46,10 @@ struct GemmArgs {
   bf16_t* out2;
   int ldo2;
   float cap;  // EPI_SOFTCAP: cap * tanh(acc / cap)
+  // EPI_GELU_LOOKUP: bf16(gelu_tanh(acc) * table[ids[row] * ldt + n]); ids belong to the rows of `out`
+  const bf16_t* table;
+  const int64_t* ids;
+  int ldt, vocab;
 };
 
 // gemm_tile.hip: the tiled kernel for calls with many rows (a.B rows, no fused norm).
@@ -103,6 +108,18 @@ __device__ __forceinline__ void gemm_epilogue(const GemmArgs& a, int b, int stri
       for (int i = 0; i < 4; ++i)
         if (r0 + i < a.N) o[i] = f2bf(v[i]);
     }
+    return;
+  }
+  if (EPI == EPI_GELU_LOOKUP) {  // N, ldo and ldt are multiples of 4
+    if (r0 >= a.N) return;
+    int64_t id = a.ids[b];
+    if (id < 0 || id >= a.vocab) id = 0;  // the host validates ids; never read out of bounds
+    const uint2 ev = *reinterpret_cast<const uint2*>(a.table + (size_t)id * a.ldt + r0);
+    const float e[4] = {lo_bf(ev.x), hi_bf(ev.x), lo_bf(ev.y), hi_bf(ev.y)};
+    float v[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = gelu_tanh(acc[i]) * e[i];
+    *reinterpret_cast<uint2*>(a.out + (size_t)b * a.ldo + r0) = make_uint2(pack_bf(v[0], v[1]), pack_bf(v[2], v[3]));
     return;
   }
   const float y0 = rbf(acc[0]), y1 = rbf(acc[1]), y2 = rbf(acc[2]), y3 = rbf(acc[3]);

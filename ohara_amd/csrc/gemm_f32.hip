@@ -1,4 +1,4 @@
-// fp32 matrix product for models served in 32-bit: y = x W^T with bias, SwiGLU or soft-cap epilogues, on
+// fp32 matrix product for models served in 32-bit: y = x W^T with bias, SwiGLU, soft-cap or gelu-lookup epilogues, on
 // v_mfma_f32_16x16x4_f32 (true fp32 products and sums).  A workgroup owns 64 rows x 64 weight rows, a wave a
 // 32 x 32 quarter; 16 columns of both operands per step go through LDS, the next step's loads are in flight
 // during the products.
@@ -14,6 +14,9 @@ struct GemmF32Args {
   float* out;
   int ldx, ldo, n, k, rows;
   float cap;
+  const float* table;  // gelu_tanh(y) * table[ids[row] * ldt + column]
+  const int64_t* ids;
+  int ldt, vocab;
 };
 
 constexpr int GT = 64, GK = 16, GL = GK + 4;
@@ -86,6 +89,11 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32Args a) {
         float v = acc[0][i][j][r];
         if (SWIGLU) v = silu_x(v) * acc[NB - 1][i][j][r];
         if (a.bias) v += a.bias[c];
+        if (a.table) {
+          int64_t id = a.ids[row];
+          if (id < 0 || id >= a.vocab) id = 0;  // the host validates ids; never read out of bounds
+          v = gelu_tanh(v) * a.table[(size_t)id * a.ldt + c];
+        }
         if (a.cap > 0.f) v = a.cap * tanhf(v / a.cap);
         a.out[(size_t)row * a.ldo + c] = v;
       }
@@ -101,9 +109,20 @@ extern "C" int ohara_gemm_f32(const float* x, int ldx, const float* w, const flo
   if (w_up && (bias || cap > 0.f)) return OHARA_EINVAL;
   const int64_t ny = ((int64_t)rows + GT - 1) / GT;
   if (ny > 65535) return OHARA_ESIZE;
-  const GemmF32Args a{x, w, w_up, bias, out, ldx, ldo, n, k, rows, cap};
+  const GemmF32Args a{x, w, w_up, bias, out, ldx, ldo, n, k, rows, cap, nullptr, nullptr, 0, 0};
   const dim3 grid((unsigned)((n + GT - 1) / GT), (unsigned)ny);
   if (w_up) hipLaunchKernelGGL((gemm_f32_kernel<true>), grid, dim3(256), 0, (hipStream_t)stream, a);
   else hipLaunchKernelGGL((gemm_f32_kernel<false>), grid, dim3(256), 0, (hipStream_t)stream, a);
+  return ohara_launch_status();
+}
+
+extern "C" int ohara_gemm_gelu_lookup_f32(const float* x, int ldx, const float* w, int n, int k, const float* table, int ldt,
+                                          const int64_t* ids, int vocab, int rows, float* out, int ldo, void* stream) {
+  if (!x || !w || !table || !ids || !out || n < 1 || k < 1 || rows < 1 || vocab < 1) return OHARA_EINVAL;
+  if ((k & 3) || (ldx & 3) || ldx < k || ldo < n || ldt < n) return OHARA_EINVAL;  // 16-byte loads
+  const int64_t ny = ((int64_t)rows + GT - 1) / GT;
+  if (ny > 65535) return OHARA_ESIZE;
+  const GemmF32Args a{x, w, nullptr, nullptr, out, ldx, ldo, n, k, rows, 0.f, table, ids, ldt, vocab};
+  hipLaunchKernelGGL((gemm_f32_kernel<false>), dim3((unsigned)((n + GT - 1) / GT), (unsigned)ny), dim3(256), 0, (hipStream_t)stream, a);
   return ohara_launch_status();
 }

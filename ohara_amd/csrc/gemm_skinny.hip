@@ -96,7 +96,7 @@ __global__ __launch_bounds__(NW * 64) void skinny_kernel(GemmArgs a) {
   // the weights of the whole share in one go - the rows arrive first (loads return in order), the norm's sums run
   // while the weights are still on their way, and the rows are not fetched a second time.
   constexpr int SP = 8;
-  const bool pre_ok = ((a.N | a.ldo | a.ldr | a.ldr2) & 3) == 0 && EPI != EPI_STORE && EPI != EPI_SWIGLU && EPI != EPI_SOFTCAP;
+  const bool pre_ok = ((a.N | a.ldo | a.ldr | a.ldr2) & 3) == 0 && EPI != EPI_STORE && EPI != EPI_SWIGLU && EPI != EPI_SOFTCAP && EPI != EPI_GELU_LOOKUP;
   EpiPre ep[BT];
   if (wave == 0 && pre_ok) {
 #pragma unroll
@@ -471,6 +471,7 @@ int launch_epi(const GemmArgs& a, int epi, int strips, hipStream_t st) {
     case EPI_SWIGLU: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_SWIGLU>), grid, block, 0, st, a); break;
     case EPI_ROPE: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_ROPE>), grid, block, 0, st, a); break;
     case EPI_SOFTCAP: hipLaunchKernelGGL((skinny_kernel<BT, false, EPI_SOFTCAP>), grid, block, 0, st, a); break;  // never with a norm
+    case EPI_GELU_LOOKUP: hipLaunchKernelGGL((skinny_kernel<BT, false, EPI_GELU_LOOKUP>), grid, block, 0, st, a); break;
     case EPI_BIAS: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS>), grid, block, 0, st, a); break;
     case EPI_BIAS_GELU: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS_GELU>), grid, block, 0, st, a); break;
     case EPI_BIAS_ADD2: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS_ADD2>), grid, block, 0, st, a); break;
@@ -518,6 +519,7 @@ int launch_skinny(const GemmArgs& a0, int epi, int packed_rows, hipStream_t st) 
     } else {
       a.out = a0.out + (size_t)r * a0.ldo;
       if (a0.resid) a.resid = a0.resid + (size_t)r * a0.ldr;
+      if (a0.ids) a.ids = a0.ids + r;
       if (a0.resid2) a.resid2 = a0.resid2 + (size_t)r * a0.ldr2;
     }
     const int rc = launch_chunk(a, epi, strips, st);
@@ -635,6 +637,18 @@ int ohara_gemm_softcap_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int 
   a.x = x; a.ldx = ldx; a.B = rows; a.N = n; a.K = k; a.out = out; a.ldo = ldo; a.cap = cap;
   if (rows > 64) return ohara_launch_gemm_tile(a, EPI_SOFTCAP, (n + 15) / 16 * 16, (hipStream_t)stream);
   return launch_skinny(a, EPI_SOFTCAP, (n + 15) / 16 * 16, (hipStream_t)stream);
+}
+
+int ohara_gemm_gelu_lookup_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, const uint16_t* table, int ldt,
+                                const int64_t* ids, int vocab, int rows, uint16_t* out, int ldo, void* stream) {
+  if (!x || !wp || !table || !ids || !out || n < 1 || k < 1 || rows < 1 || vocab < 1) return OHARA_EINVAL;
+  if ((k & 7) || (ldx & 7) || ldx < k || ldo < n || ldt < n || ((n | ldo | ldt) & 3)) return OHARA_EINVAL;
+  GemmArgs a{};
+  a.wp = reinterpret_cast<const uint4*>(wp);
+  a.x = x; a.ldx = ldx; a.B = rows; a.N = n; a.K = k; a.out = out; a.ldo = ldo;
+  a.table = table; a.ldt = ldt; a.ids = ids; a.vocab = vocab;
+  if (rows > 64) return ohara_launch_gemm_tile(a, EPI_GELU_LOOKUP, (n + 15) / 16 * 16, (hipStream_t)stream);
+  return launch_skinny(a, EPI_GELU_LOOKUP, (n + 15) / 16 * 16, (hipStream_t)stream);
 }
 
 int ohara_gemm_skinny_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, const uint16_t* norm_w,

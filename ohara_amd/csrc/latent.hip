@@ -1,0 +1,553 @@
+// Latent attention: every head's keys and values are projections of one cached latent per position, so decode steps
+// apply the projections to the query and to the weighted sum instead and read only the latents.
+//
+//   latent_front         RMS norms of the query latent and of the cached one, append: a workgroup per token
+//   head_linear          one small matrix per head (both projections), optional gate per output element
+//   attn_latent_kernel   bf16 MFMA: 16 heads are the 16 query columns of a tile of 64 positions
+//   latent_plain_kernel  the same one position per wave at a time (fp32)
+//   latent_merge_kernel  the chunks of a split context, in chunk order
+//
+// Scores, softmax weights and sums are fp32; the second MFMA product keeps the fp32 weights by splitting each into three
+// bf16 terms (8 + 8 + 8 significant bits).
+#include "hybrid.h"
+
+namespace {
+
+template <typename T>
+struct LatentFrontArgs {
+  const T* p;
+  const float* qn;
+  const float* cn;
+  T* q;
+  T* cache;
+  T* c_out;
+  int ldp, q_rank, off_c, rank, Tmax;
+  float eps;
+  OharaSeq seq;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_front_kernel(LatentFrontArgs<T> a) {
+  __shared__ float red[2][4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int row = blockIdx.x, b = row / a.seq.seq_len, s = row - b * a.seq.seq_len;
+  const int pos = seq_start(a.seq, b) + s;
+  if (s >= seq_tokens(a.seq, b) || pos < 0 || pos >= a.Tmax) return;
+  const int Qp = (a.q_rank + 7) & ~7, Rp = (a.rank + 7) & ~7;
+  const T *pq = a.p + (size_t)row * a.ldp, *pc = pq + a.off_c;
+  const bool vec = ((a.q_rank | a.off_c | a.rank | a.ldp) & 3) == 0;
+  float sq = 0.f, sc = 0.f;
+  auto sum = [&](const T* src, int n) {
+    float t = 0.f;
+    if (vec) {
+      for (int i = 4 * tid; i < n; i += 1024) {
+        float v[4];
+        ld4(src + i, v);
+        t += ((v[0] * v[0] + v[1] * v[1]) + v[2] * v[2]) + v[3] * v[3];
+      }
+    } else {
+      for (int i = tid; i < n; i += 256) {
+        const float v = ldv(src + i);
+        t += v * v;
+      }
+    }
+    return t;
+  };
+  sq = wave_sum(sum(pq, a.q_rank));
+  sc = wave_sum(sum(pc, a.rank));
+  if (lane == 0) {
+    red[0][wave] = sq;
+    red[1][wave] = sc;
+  }
+  __syncthreads();
+  const float iq = 1.0f / sqrtf((((red[0][0] + red[0][1]) + red[0][2]) + red[0][3]) / (float)a.q_rank + a.eps);
+  const float ic = 1.0f / sqrtf((((red[1][0] + red[1][1]) + red[1][2]) + red[1][3]) / (float)a.rank + a.eps);
+  auto put = [&](const T* src, int n, int np, const float* w, float inv, T* d0, T* d1) {
+    if (vec) {
+      for (int i = 4 * tid; i < np; i += 1024) {
+        float v[4] = {0.f, 0.f, 0.f, 0.f}, g[4];
+        if (i < n) {
+          ld4(src + i, v);
+          ld4(w + i, g);
+#pragma unroll
+          for (int u = 0; u < 4; ++u) v[u] = v[u] * inv * g[u];
+        }
+        st4(d0 + i, v);
+        if (d1) st4(d1 + i, v);
+      }
+    } else {
+      for (int i = tid; i < np; i += 256) {
+        const float v = i < n ? ldv(src + i) * inv * w[i] : 0.f;
+        stv(d0 + i, v);
+        if (d1) stv(d1 + i, v);
+      }
+    }
+  };
+  put(pq, a.q_rank, Qp, a.qn, iq, a.q + (size_t)row * Qp, (T*)nullptr);
+  put(pc, a.rank, Rp, a.cn, ic, a.cache + ((size_t)seq_slot(a.seq, b) * a.Tmax + pos) * Rp,
+      a.c_out ? a.c_out + (size_t)row * Rp : nullptr);
+}
+
+// ---- one matrix per head -----------------------------------------------------------------------
+template <typename T>
+struct HeadLinearArgs {
+  const T* x;
+  const T* w;
+  const T* gate;
+  T* out;
+  int ldx, h, n, k, n_out, rows, ldg, ldo;
+};
+
+template <typename T>
+__device__ __forceinline__ void head_linear_pad(const HeadLinearArgs<T>& a, int row0, int nrows) {
+  const int used = a.h * a.n_out, pad = a.ldo - used;
+  for (int i = threadIdx.x; i < pad * nrows; i += blockDim.x)
+    stv(a.out + (size_t)(row0 + i / pad) * a.ldo + used + i % pad, 0.f);
+}
+
+// A wave: 16 output entries x 16 rows of one head; the weights are the A operand straight from memory.
+__global__ __launch_bounds__(256) void head_linear_kernel(HeadLinearArgs<bf16_t> a) {
+  constexpr int CH = 8;  // k-steps whose loads are issued together
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 15, g = lane >> 4;
+  const int h = blockIdx.y, row0 = blockIdx.z * 16, strip = (blockIdx.x * 4 + wave) * 16;
+  if (h == 0 && blockIdx.x == 0) head_linear_pad(a, row0, min(16, a.rows - row0));
+  if (strip >= a.n_out) return;
+  const int o = min(strip + m, a.n - 1), row = min(row0 + m, a.rows - 1);
+  const bf16_t* w = a.w + ((size_t)h * a.n + o) * a.k;
+  const bf16_t* x = a.x + (size_t)row * a.ldx + (size_t)h * a.k;
+  const uint4 zero = make_uint4(0, 0, 0, 0);
+  f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int j0 = 0; j0 < a.k; j0 += 32 * CH) {
+    uint4 wv[CH], xv[CH];
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+      const int k0 = j0 + 32 * c + 8 * g;
+      const bool in = k0 < a.k;  // k is a multiple of 8
+      wv[c] = in ? ldg16(w + k0) : zero;
+      xv[c] = in ? ldg16(x + k0) : zero;
+    }
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int c = 0; c < CH; ++c)
+      if (j0 + 32 * c < a.k)
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wv[c]), __builtin_bit_cast(bf16x8, xv[c]), acc, 0, 0, 0);
+  }
+  if (row0 + m >= a.rows) return;
+  const int c0 = strip + 4 * g;
+  float v[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    v[i] = a.gate && c0 + i < a.n_out ? acc[i] * sigmoid_x(ldv(a.gate + (size_t)row * a.ldg + h * a.n_out + c0 + i)) : acc[i];
+  bf16_t* dst = a.out + (size_t)row * a.ldo + (size_t)h * a.n_out + c0;
+  if (((a.n_out | a.ldo) & 3) == 0) {
+    if (c0 < a.n_out) st4(dst, v);
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (c0 + i < a.n_out) dst[i] = f2bf(v[i]);
+  }
+}
+
+// fp32: a workgroup per (row, head), a wave per output entry
+__global__ __launch_bounds__(256) void head_linear_f32_kernel(HeadLinearArgs<float> a) {
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, row = blockIdx.x, h = blockIdx.y;
+  if (h == 0) head_linear_pad(a, row, 1);
+  const float* x = a.x + (size_t)row * a.ldx + (size_t)h * a.k;
+  for (int o = wave; o < a.n_out; o += 4) {
+    const float* w = a.w + ((size_t)h * a.n + o) * a.k;
+    float s = 0.f;
+    for (int i = lane; i < a.k; i += 64) s = __builtin_fmaf(w[i], x[i], s);
+    s = wave_sum(s);
+    if (lane == 0) {
+      if (a.gate) s *= sigmoid_x(a.gate[(size_t)row * a.ldg + h * a.n_out + o]);
+      a.out[(size_t)row * a.ldo + (size_t)h * a.n_out + o] = s;
+    }
+  }
+}
+
+// ---- attention over the latents ------------------------------------------------------------------
+template <typename T>
+struct LatentArgs {
+  const T* q;      // (rows, H, Rp)
+  const T* cache;  // (cache rows, Tmax, Rp)
+  T* out;          // (rows, H, Rp)
+  float* ws;       // ns > 1: per (row, head, chunk) Rp + 4 floats {weighted sum, max, sum}
+  int H, Rp, Tmax, ns, nhb;
+  float scale;
+  OharaSeq seq;
+};
+
+constexpr int KT = 64;  // positions per tile
+
+// visible positions of a row that chunk `part` works on; false: the row is padding
+template <typename T>
+__device__ __forceinline__ bool latent_range(const LatentArgs<T>& a, int row, int part, int& slot, int& lo, int& hi) {
+  const int b = row / a.seq.seq_len, s = row - b * a.seq.seq_len, pq = seq_start(a.seq, b) + s;
+  if (s >= seq_tokens(a.seq, b) || pq < 0 || pq >= a.Tmax) return false;
+  slot = seq_slot(a.seq, b);
+  const int per = a.ns > 1 ? ((pq + a.ns) / a.ns + KT - 1) / KT * KT : pq + 1;  // ceil((pq + 1) / ns) in whole tiles
+  lo = part * per;
+  hi = min(pq, lo + per - 1);
+  return true;
+}
+
+// Four waves share a tile of 64 latents in LDS, once as it is (keys) and once transposed (values).  Scores: a wave's 16 positions
+// x 16 heads over the whole rank.  Weighted sum: a wave's quarter of the rank x 16 heads over all 64 positions.  The running
+// maximum is an integer in log2 units, so most tiles leave it alone.
+template <int RT>  // 32-element steps of the rank
+__global__ __launch_bounds__(256) void attn_latent_kernel(LatentArgs<bf16_t> a) {
+  constexpr int R = 32 * RT, LDK = R + 8, LDV = KT + 8, LDP = KT + 4, CV = R / 8, NG = RT / 4, NT = RT / 2;
+  extern __shared__ __align__(16) unsigned char latent_smem[];
+  bf16_t* Ks = reinterpret_cast<bf16_t*>(latent_smem);        // [KT][LDK]
+  bf16_t* Vt = Ks + KT * LDK;                                  // [R][LDV]
+  float* Ps = reinterpret_cast<float*>(Vt + R * LDV);          // [16][LDP]
+  float* wm = Ps + 16 * LDP;                                   // [4][16]
+  // A column's positions are rotated by eight per group of eight columns: the threads that write one position group write
+  // columns eight apart, which would land on two banks.
+  auto vt_off = [](int col, int p) { return (p + 8 * (col >> 3)) & (KT - 1); };
+  const int tid = threadIdx.x, lane = tid & 63, m = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int row = blockIdx.x / a.nhb, h0 = (blockIdx.x - row * a.nhb) * 16, part = blockIdx.y;
+  int slot, t_lo, t_hi;
+  if (!latent_range(a, row, part, slot, t_lo, t_hi)) return;
+  const bf16_t* cb = a.cache + (size_t)slot * a.Tmax * a.Rp;
+  const int h = h0 + m;
+  const uint4 zero = make_uint4(0, 0, 0, 0);
+  uint4 qf[RT], cr[RT];
+#pragma unroll
+  for (int j = 0; j < RT; ++j)
+    qf[j] = (h < a.H && 32 * j + 8 * g < a.Rp) ? ldg16(a.q + ((size_t)row * a.H + h) * a.Rp + 32 * j + 8 * g) : zero;
+  const int vrow = tid / CV, vcol = 8 * (tid % CV);
+  auto load_tile = [&](int t0) {
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {  // four consecutive positions per thread and group: the transposed write is wide
+      const int p = 4 * (vrow + (i / 4) * (256 / CV)) + i % 4;
+      cr[i] = (t0 + p <= t_hi && vcol < a.Rp) ? ldg16(cb + (size_t)(t0 + p) * a.Rp + vcol) : zero;
+    }
+  };
+  auto store_tile = [&]() {
+#pragma unroll
+    for (int grp = 0; grp < NG; ++grp) {
+      const int p0 = 4 * (vrow + grp * (256 / CV));
+      uint32_t w[4][4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const uint4 v = cr[4 * grp + r];
+        *reinterpret_cast<uint4*>(Ks + (p0 + r) * LDK + vcol) = v;
+        w[r][0] = v.x; w[r][1] = v.y; w[r][2] = v.z; w[r][3] = v.w;
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int at = vt_off(vcol, p0);  // the same for the eight columns of the piece
+        *reinterpret_cast<uint2*>(Vt + (vcol + 2 * e) * LDV + at) =
+            make_uint2((w[0][e] & 0xffffu) | (w[1][e] << 16), (w[2][e] & 0xffffu) | (w[3][e] << 16));
+        *reinterpret_cast<uint2*>(Vt + (vcol + 2 * e + 1) * LDV + at) =
+            make_uint2((w[0][e] >> 16) | (w[1][e] & 0xffff0000u), (w[2][e] >> 16) | (w[3][e] & 0xffff0000u));
+      }
+    }
+  };
+  f32x4 o[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) o[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float mrun = -1e30f, lrun = 0.f;
+  const float sl2 = a.scale * OHARA_LOG2E;
+  if (t_lo <= t_hi) load_tile(t_lo);
+  for (int t0 = t_lo; t0 <= t_hi; t0 += KT) {
+    __syncthreads();  // everyone is done with the previous tile
+    store_tile();
+    __syncthreads();
+    if (t0 + KT <= t_hi) load_tile(t0 + KT);  // in flight during the products
+    f32x4 s = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < RT; ++j) {
+      const uint4 kf = *reinterpret_cast<const uint4*>(Ks + (16 * wave + m) * LDK + 32 * j + 8 * g);
+      s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kf), __builtin_bit_cast(bf16x8, qf[j]), s, 0, 0, 0);
+    }
+    float mx = -1e30f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      s[i] = t0 + 16 * wave + 4 * g + i <= t_hi ? s[i] * sl2 : -INFINITY;
+      mx = fmaxf(mx, s[i]);
+    }
+    mx = lane_xor_max<32>(lane_xor_max<16>(mx));
+    if (g == 0) wm[16 * wave + m] = mx;
+    __syncthreads();
+    const float tmax = fmaxf(fmaxf(wm[m], wm[16 + m]), fmaxf(wm[32 + m], wm[48 + m]));
+    const float mn = fmaxf(mrun, ceilf(tmax));
+    const float corr = __builtin_amdgcn_exp2f(mrun - mn);
+    mrun = mn;
+    f32x4 p;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) p[i] = __builtin_amdgcn_exp2f(s[i] - mn);
+    lrun = lrun * corr + (((p[0] + p[1]) + p[2]) + p[3]);  // this lane's share
+    *reinterpret_cast<f32x4*>(Ps + m * LDP + 16 * wave + 4 * g) = p;
+    if (__any(corr != 1.0f)) {
+#pragma unroll
+      for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[t][i] *= corr;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int w = 0; w < 2; ++w) {
+      const float4 pa = *reinterpret_cast<const float4*>(Ps + m * LDP + 32 * w + 8 * g);
+      const float4 pb = *reinterpret_cast<const float4*>(Ps + m * LDP + 32 * w + 8 * g + 4);
+      const float pv[8] = {pa.x, pa.y, pa.z, pa.w, pb.x, pb.y, pb.z, pb.w};
+      uint32_t hi[4], mid[4], lo[4];  // p = hi + mid + lo exactly
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float p0 = pv[2 * e], p1 = pv[2 * e + 1];
+        hi[e] = pack_bf(p0, p1);
+        const float r0 = p0 - lo_bf(hi[e]), r1 = p1 - hi_bf(hi[e]);
+        mid[e] = pack_bf(r0, r1);
+        lo[e] = pack_bf(r0 - lo_bf(mid[e]), r1 - hi_bf(mid[e]));
+      }
+      const uint4 pt[3] = {make_uint4(hi[0], hi[1], hi[2], hi[3]), make_uint4(mid[0], mid[1], mid[2], mid[3]),
+                           make_uint4(lo[0], lo[1], lo[2], lo[3])};
+      uint4 vf[NT];
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        const int col = 16 * (wave * NT + t) + m;
+        vf[t] = *reinterpret_cast<const uint4*>(Vt + col * LDV + vt_off(col, 32 * w + 8 * g));
+      }
+#pragma unroll
+      for (int k = 0; k < 3; ++k)
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+          o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, vf[t]), __builtin_bit_cast(bf16x8, pt[k]), o[t], 0, 0, 0);
+    }
+  }
+  // sums of the four waves; the maximum is the same in all of them
+  const float lw = lane_xor_sum<32>(lane_xor_sum<16>(lrun));
+  __syncthreads();
+  if (g == 0) wm[16 * wave + m] = lw;
+  __syncthreads();
+  if (h >= a.H) return;
+  const float l = (wm[m] + wm[16 + m]) + (wm[32 + m] + wm[48 + m]);
+  if (a.ns > 1) {
+    float* w = a.ws + (((size_t)row * a.H + h) * a.ns + part) * (a.Rp + 4);
+    if (t_lo <= t_hi) {
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        const int c = 16 * (wave * NT + t) + 4 * g;
+        if (c < a.Rp) *reinterpret_cast<f32x4*>(w + c) = o[t];
+      }
+    }
+    if (wave == 0 && g == 0) {
+      w[a.Rp] = mrun;
+      w[a.Rp + 1] = l;
+    }
+    return;
+  }
+  const float inv = 1.0f / l;
+  bf16_t* dst = a.out + ((size_t)row * a.H + h) * a.Rp;
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int c = 16 * (wave * NT + t) + 4 * g;
+    const float v[4] = {o[t][0] * inv, o[t][1] * inv, o[t][2] * inv, o[t][3] * inv};
+    if (c < a.Rp) st4(dst + c, v);
+  }
+}
+
+// A workgroup per (row, head, chunk): a wave takes every fourth position, a lane eight elements of it (rank <= 512).
+template <typename T>
+__global__ __launch_bounds__(256) void latent_plain_kernel(LatentArgs<T> a) {
+  __shared__ __align__(16) float acc_s[4][512];
+  __shared__ float wm[4], wl[4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int row = blockIdx.x / a.H, h = blockIdx.x - row * a.H, part = blockIdx.y;
+  int slot, t_lo, t_hi;
+  if (!latent_range(a, row, part, slot, t_lo, t_hi)) return;
+  const int e0 = 8 * lane;
+  const bool own = e0 < a.Rp;
+  float q[8], acc[8], mr = -1e30f, lr = 0.f;
+  {
+    Raw8<T> v;
+    v.load(a.q + ((size_t)row * a.H + h) * a.Rp + (own ? e0 : 0));
+    v.get(q);
+  }
+#pragma unroll
+  for (int u = 0; u < 8; ++u) {
+    q[u] = own ? q[u] * a.scale * OHARA_LOG2E : 0.f;
+    acc[u] = 0.f;
+  }
+  const T* cb = a.cache + (size_t)slot * a.Tmax * a.Rp + (own ? e0 : 0);
+  for (int t = t_lo + wave; t <= t_hi; t += 4) {
+    Raw8<T> v;
+    v.load(cb + (size_t)t * a.Rp);
+    float c[8], dot = 0.f;
+    v.get(c);
+#pragma unroll
+    for (int u = 0; u < 8; ++u) dot = __builtin_fmaf(c[u], q[u], dot);
+    dot = wave_sum(dot);
+    const float mn = fmaxf(mr, dot), corr = __builtin_amdgcn_exp2f(mr - mn), p = __builtin_amdgcn_exp2f(dot - mn);
+    lr = lr * corr + p;
+#pragma unroll
+    for (int u = 0; u < 8; ++u) acc[u] = acc[u] * corr + p * c[u];
+    mr = mn;
+  }
+#pragma unroll
+  for (int u = 0; u < 8; ++u) acc_s[wave][e0 + u] = acc[u];
+  if (lane == 0) {
+    wm[wave] = mr;
+    wl[wave] = lr;
+  }
+  __syncthreads();
+  const float M = fmaxf(fmaxf(wm[0], wm[1]), fmaxf(wm[2], wm[3]));
+  float f[4], l = 0.f;
+#pragma unroll
+  for (int w = 0; w < 4; ++w) {
+    f[w] = __builtin_amdgcn_exp2f(wm[w] - M);
+    l += f[w] * wl[w];
+  }
+  float* ws = a.ns > 1 ? a.ws + (((size_t)row * a.H + h) * a.ns + part) * (a.Rp + 4) : nullptr;
+  for (int c = tid; c < a.Rp; c += 256) {
+    const float v = ((f[0] * acc_s[0][c] + f[1] * acc_s[1][c]) + f[2] * acc_s[2][c]) + f[3] * acc_s[3][c];
+    if (ws) ws[c] = v;
+    else stv(a.out + ((size_t)row * a.H + h) * a.Rp + c, v / l);
+  }
+  if (ws && tid == 0) {
+    ws[a.Rp] = M;
+    ws[a.Rp + 1] = l;
+  }
+}
+
+// A workgroup per (row, head), four columns per thread.
+template <typename T>
+__global__ __launch_bounds__(128) void latent_merge_kernel(LatentArgs<T> a) {
+  __shared__ float wt[64];
+  __shared__ float total;
+  const int row = blockIdx.x / a.H, tid = threadIdx.x;
+  int slot, lo, hi;
+  if (!latent_range(a, row, 0, slot, lo, hi)) return;
+  const int per = hi - lo + 1, b = row / a.seq.seq_len, pq = seq_start(a.seq, b) + row - b * a.seq.seq_len;
+  const int used = min(a.ns, (pq + per) / per);  // chunks that hold a visible position
+  const float* ws = a.ws + (size_t)blockIdx.x * a.ns * (a.Rp + 4);
+  if (tid < 64) {
+    const bool in = tid < used;
+    const float mm = in ? ws[(size_t)tid * (a.Rp + 4) + a.Rp] : -1e30f, ll = in ? ws[(size_t)tid * (a.Rp + 4) + a.Rp + 1] : 0.f;
+    const float M = wave_max(mm), w = in ? __builtin_amdgcn_exp2f(mm - M) : 0.f, L = wave_sum(w * ll);
+    wt[tid] = w;
+    if (tid == 0) total = 1.0f / L;
+  }
+  __syncthreads();
+  const int c = 4 * tid;
+  if (c >= a.Rp) return;
+  f32x4 s = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int n0 = 0; n0 < used; n0 += 8) {
+    f32x4 v[8];
+#pragma unroll
+    for (int n = 0; n < 8; ++n) v[n] = *reinterpret_cast<const f32x4*>(ws + (size_t)min(n0 + n, used - 1) * (a.Rp + 4) + c);
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int n = 0; n < 8; ++n) {
+      const float w = n0 + n < used ? wt[n0 + n] : 0.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) s[i] += w * v[n][i];
+    }
+  }
+  const float t = total, r[4] = {s[0] * t, s[1] * t, s[2] * t, s[3] * t};
+  st4(a.out + (size_t)blockIdx.x * a.Rp + c, r);
+}
+
+template <typename T>
+int launch_front(const LatentFrontArgs<T>& a, hipStream_t st) {
+  if (!a.p || !a.qn || !a.cn || !a.q || !a.cache || !seq_ok(&a.seq)) return OHARA_EINVAL;
+  if (a.q_rank < 1 || a.rank < 1 || a.Tmax < 1 || a.off_c < a.q_rank || a.ldp < a.off_c + a.rank) return OHARA_EINVAL;
+  if (!a.seq.pos_dev && a.seq.pos + a.seq.seq_len > a.Tmax) return OHARA_EINVAL;
+  hipLaunchKernelGGL((latent_front_kernel<T>), dim3((unsigned)(a.seq.batch * a.seq.seq_len)), dim3(256), 0, st, a);
+  return ohara_launch_status();
+}
+
+template <typename T>
+bool head_linear_ok(const HeadLinearArgs<T>& a) {
+  if (!a.x || !a.w || !a.out || a.h < 1 || a.n < 1 || a.k < 1 || a.rows < 1 || a.n_out < 1 || a.n_out > a.n) return false;
+  if (((a.n | a.k | a.ldx) & 7) || a.ldx < a.h * a.k || a.ldo < a.h * a.n_out) return false;
+  return !a.gate || a.ldg >= a.h * a.n_out;
+}
+
+template <int RT>
+int launch_latent(const LatentArgs<bf16_t>& a, dim3 grid, hipStream_t st) {
+  constexpr int R = 32 * RT;
+  const size_t smem = (size_t)(KT * (R + 8) + R * (KT + 8)) * sizeof(bf16_t) + (16 * (KT + 4) + 64) * sizeof(float);
+  if (smem > 64 * 1024)
+    (void)hipFuncSetAttribute((const void*)attn_latent_kernel<RT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+  hipLaunchKernelGGL((attn_latent_kernel<RT>), grid, dim3(256), smem, st, a);
+  return ohara_launch_status();
+}
+
+template <typename T>
+int attn_latent(const T* q, const T* cache, int h, int rank, int t_max, float scale, int n_split, void* workspace, T* out,
+                const OharaSeq* seq, hipStream_t st) {
+  if (!q || !cache || !out || !seq_ok(seq) || h < 1 || rank < 1 || t_max < 1) return OHARA_EINVAL;
+  if (rank > 512) return OHARA_ESIZE;
+  if (n_split < 1 || n_split > 64 || (n_split > 1 && !workspace)) return OHARA_EINVAL;
+  if (!seq->pos_dev && seq->pos + seq->seq_len > t_max) return OHARA_EINVAL;
+  LatentArgs<T> a{q, cache, out, reinterpret_cast<float*>(workspace), h, (rank + 7) & ~7, t_max, n_split, (h + 15) / 16, scale, *seq};
+  const int64_t rows = (int64_t)seq->batch * seq->seq_len;
+  if (rows * h > INT32_MAX) return OHARA_ESIZE;
+  int rc;
+  if constexpr (sizeof(T) == 2) {
+    const dim3 grid((unsigned)(rows * a.nhb), (unsigned)n_split);
+    rc = a.Rp <= 128 ? launch_latent<4>(a, grid, st) : (a.Rp <= 256 ? launch_latent<8>(a, grid, st) : launch_latent<16>(a, grid, st));
+  } else {
+    hipLaunchKernelGGL((latent_plain_kernel<T>), dim3((unsigned)(rows * h), (unsigned)n_split), dim3(256), 0, st, a);
+    rc = ohara_launch_status();
+  }
+  if (rc || n_split == 1) return rc;
+  hipLaunchKernelGGL((latent_merge_kernel<T>), dim3((unsigned)(rows * h)), dim3(128), 0, st, a);
+  return ohara_launch_status();
+}
+
+}  // namespace
+
+extern "C" {
+
+int ohara_latent_front_bf16(const uint16_t* p, int ldp, int q_rank, int off_c, int rank, const float* qn, const float* cn,
+                            float eps, uint16_t* q_out, uint16_t* cache, int t_max, uint16_t* c_out, const OharaSeq* seq,
+                            void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  return launch_front<bf16_t>(LatentFrontArgs<bf16_t>{p, qn, cn, q_out, cache, c_out, ldp, q_rank, off_c, rank, t_max, eps, *seq},
+                              (hipStream_t)stream);
+}
+int ohara_latent_front_f32(const float* p, int ldp, int q_rank, int off_c, int rank, const float* qn, const float* cn,
+                           float eps, float* q_out, float* cache, int t_max, float* c_out, const OharaSeq* seq,
+                           void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  return launch_front<float>(LatentFrontArgs<float>{p, qn, cn, q_out, cache, c_out, ldp, q_rank, off_c, rank, t_max, eps, *seq},
+                             (hipStream_t)stream);
+}
+
+int ohara_head_linear_bf16(const uint16_t* x, int ldx, const uint16_t* w, int h, int n, int k, int n_out, int rows,
+                           const uint16_t* gate, int ldg, uint16_t* out, int ldo, void* stream) {
+  const HeadLinearArgs<bf16_t> a{x, w, gate, out, ldx, h, n, k, n_out, rows, ldg, ldo};
+  if (!head_linear_ok(a)) return OHARA_EINVAL;
+  const int nz = (rows + 15) / 16;
+  if (h > 65535 || nz > 65535) return OHARA_ESIZE;
+  hipLaunchKernelGGL(head_linear_kernel, dim3((unsigned)((n_out + 63) / 64), (unsigned)h, (unsigned)nz), dim3(256), 0,
+                     (hipStream_t)stream, a);
+  return ohara_launch_status();
+}
+int ohara_head_linear_f32(const float* x, int ldx, const float* w, int h, int n, int k, int n_out, int rows, const float* gate,
+                          int ldg, float* out, int ldo, void* stream) {
+  const HeadLinearArgs<float> a{x, w, gate, out, ldx, h, n, k, n_out, rows, ldg, ldo};
+  if (!head_linear_ok(a)) return OHARA_EINVAL;
+  if (h > 65535) return OHARA_ESIZE;
+  hipLaunchKernelGGL(head_linear_f32_kernel, dim3((unsigned)rows, (unsigned)h), dim3(256), 0, (hipStream_t)stream, a);
+  return ohara_launch_status();
+}
+
+int64_t ohara_attn_latent_workspace_bytes(int rows, int h, int rank, int n_split) {
+  if (rows < 1 || h < 1 || rank < 1 || n_split < 1) return OHARA_EINVAL;
+  return (int64_t)rows * h * n_split * (((rank + 7) & ~7) + 4) * (int64_t)sizeof(float);
+}
+int ohara_attn_latent_bf16(const uint16_t* q, const uint16_t* cache, int h, int rank, int t_max, float scale, int n_split,
+                           void* workspace, uint16_t* out, const OharaSeq* seq, void* stream) {
+  return attn_latent<bf16_t>(q, cache, h, rank, t_max, scale, n_split, workspace, out, seq, (hipStream_t)stream);
+}
+int ohara_attn_latent_f32(const float* q, const float* cache, int h, int rank, int t_max, float scale, int n_split,
+                          void* workspace, float* out, const OharaSeq* seq, void* stream) {
+  return attn_latent<float>(q, cache, h, rank, t_max, scale, n_split, workspace, out, seq, (hipStream_t)stream);
+}
+
+}  // extern "C"

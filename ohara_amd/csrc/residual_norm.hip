@@ -1,5 +1,5 @@
-// Residual stream of blocks whose norm sits on the sublayer output, and the causal depthwise convolution in
-// front of a mixer.  The residual is fp32 throughout.
+// Residual stream of blocks whose norm (RMS or layer norm) sits on the sublayer output, and the causal depthwise
+// convolution in front of a mixer.  The residual is fp32 throughout.
 //
 // Decode (one token per sequence): embedding or residual update, group norm, input convolution and its ring
 // update are ONE launch, a workgroup per row.  Prompts: the residual update is a workgroup per row, the
@@ -20,9 +20,23 @@ struct ResidualArgs {
   const float* conv_w;
   float* ring;
   int d, vocab, ldy, groups, ldo, mode, taps;
+  int center_y, center_out;  // norm of y / of the output: layer norm (the mean is taken off first) instead of RMS
   float eps;
   OharaSeq seq;
 };
+
+// Takes the row's mean off a row in LDS (layer norms: one group).  Ends with a barrier.
+__device__ __forceinline__ void center_row(float* row, int d, float* red) {
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  float s = 0.f;
+  for (int i = tid; i < d; i += 256) s += row[i];
+  s = wave_sum(s);
+  if (lane == 0) red[wave] = s;
+  __syncthreads();
+  const float mean = (((red[0] + red[1]) + red[2]) + red[3]) / (float)d;
+  for (int i = tid; i < d; i += 256) row[i] -= mean;
+  __syncthreads();
+}
 
 // inv[g] = 1 / sqrt(mean square of group g + eps) for a row in LDS.  Ends with a barrier.
 __device__ __forceinline__ void group_inverse(const float* row, int d, int groups, float eps, float* inv, float* red) {
@@ -89,6 +103,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualArgs<T> a) {
       for (int i = tid; i < d; i += 256) ys[i] = ldv(yr + i);
     }
     __syncthreads();
+    if (a.center_y) center_row(ys, d, red);
     group_inverse(ys, d, a.groups, a.eps, inv, red);
     if (VEC) {
       for (int i = tid * 4; i < d; i += 1024) {
@@ -117,6 +132,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualArgs<T> a) {
   T* o = a.out + (size_t)row * a.ldo;
   for (int i = d + tid; i < a.ldo; i += 256) stv(o + i, 0.f);
   if (a.mode == OHARA_OUT_NORM) {
+    if (a.center_out) center_row(ys, d, red);
     group_inverse(ys, d, a.groups, a.eps, inv, red);
     for (int i = tid; i < d; i += 256) stv(o + i, ys[i] * inv[i / gs] * a.norm2_w[i]);
   } else if (a.mode == OHARA_OUT_COPY) {
@@ -150,7 +166,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualArgs<T> a) {
 template <typename T, int NP, int MT>
 __global__ __launch_bounds__(256) void residual_norm_regs_kernel(ResidualArgs<T> a) {
   extern __shared__ __align__(16) float smem[];  // groups > 1: a partial sum per piece, then 1 / rms per group
-  __shared__ float red[2][4];
+  __shared__ float red[4][4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, row = blockIdx.x, d = a.d;
   const int gs4 = d / a.groups / 4;  // pieces per group
   float* xr = a.x + (size_t)row * d;
@@ -189,6 +205,19 @@ __global__ __launch_bounds__(256) void residual_norm_regs_kernel(ResidualArgs<T>
       }
     }
   }
+  auto center = [&](float (&v)[NP][4], float* r4) {  // layer norms: v minus the row's mean
+    float tot = 0.f;
+#pragma unroll
+    for (int p = 0; p < NP; ++p) tot += ((v[p][0] + v[p][1]) + v[p][2]) + v[p][3];  // zeros past the row's end
+    tot = wave_sum(tot);
+    if (lane == 0) r4[wave] = tot;
+    __syncthreads();
+    const float mean = (((r4[0] + r4[1]) + r4[2]) + r4[3]) / (float)d;
+#pragma unroll
+    for (int p = 0; p < NP; ++p)
+#pragma unroll
+      for (int u = 0; u < 4; ++u) v[p][u] = 4 * tid + 1024 * p < d ? v[p][u] - mean : 0.f;
+  };
   auto inverse = [&](float (&v)[NP][4], float* r4, float (&inv)[NP]) {
     float s[NP], tot = 0.f;
 #pragma unroll
@@ -222,6 +251,7 @@ __global__ __launch_bounds__(256) void residual_norm_regs_kernel(ResidualArgs<T>
   };
   if (add) {
     float inv[NP];
+    if (a.center_y) center(y, red[2]);
     inverse(y, red[0], inv);
 #pragma unroll
     for (int p = 0; p < NP; ++p)
@@ -237,7 +267,10 @@ __global__ __launch_bounds__(256) void residual_norm_regs_kernel(ResidualArgs<T>
   T* o = a.out + (size_t)row * a.ldo;
   for (int i = d + tid; i < a.ldo; i += 256) stv(o + i, 0.f);
   float inv[NP];
-  if (a.mode == OHARA_OUT_NORM) inverse(x, red[1], inv);
+  if (a.mode == OHARA_OUT_NORM) {  // x has been stored: it may be changed
+    if (a.center_out) center(x, red[3]);
+    inverse(x, red[1], inv);
+  }
   const bool live = MT > 1 && seq_tokens(a.seq, row) > 0 && pos >= 0;
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
@@ -339,6 +372,10 @@ __global__ __launch_bounds__(256) void ring_store_kernel(const T* src, int ld, i
 
 template <typename T>
 int launch_residual(ResidualArgs<T> a, const OharaSeq* seq, hipStream_t st) {
+  a.center_y = (a.mode & OHARA_CENTER_Y) != 0;
+  a.center_out = (a.mode & OHARA_CENTER_OUT) != 0;
+  a.mode &= ~(OHARA_CENTER_Y | OHARA_CENTER_OUT);
+  if ((a.center_y || a.center_out) && a.groups != 1) return OHARA_EINVAL;
   if (!a.x || a.d < 1 || a.groups < 1 || a.d % a.groups || !seq_ok(seq)) return OHARA_EINVAL;
   if (a.ids && (!a.table || a.vocab < 1)) return OHARA_EINVAL;
   if (!a.ids && a.y && (!a.norm_w || a.ldy < a.d)) return OHARA_EINVAL;
@@ -398,14 +435,14 @@ int ohara_residual_norm_bf16(float* x, int d, const int64_t* ids, const uint16_t
                              const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
                              void* stream) {
   return launch_residual<bf16_t>(ResidualArgs<bf16_t>{x, ids, table, y, norm_w, out, norm2_w, conv_w, ring, d, vocab, ldy,
-                                                      groups, ldo, out_mode, taps, eps, {}}, seq, (hipStream_t)stream);
+                                                      groups, ldo, out_mode, taps, 0, 0, eps, {}}, seq, (hipStream_t)stream);
 }
 int ohara_residual_norm_f32(float* x, int d, const int64_t* ids, const float* table, int vocab, const float* y, int ldy,
                             const float* norm_w, int groups, float eps, int out_mode, float* out, int ldo,
                             const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
                             void* stream) {
   return launch_residual<float>(ResidualArgs<float>{x, ids, table, y, norm_w, out, norm2_w, conv_w, ring, d, vocab, ldy, groups,
-                                                    ldo, out_mode, taps, eps, {}}, seq, (hipStream_t)stream);
+                                                    ldo, out_mode, taps, 0, 0, eps, {}}, seq, (hipStream_t)stream);
 }
 
 int ohara_input_conv_bf16(const float* x, int d, const float* conv_w, int taps, const float* ring, uint16_t* out, int ldo,

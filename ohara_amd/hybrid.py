@@ -13,7 +13,7 @@ import torch
 import torch.nn.functional as F
 
 from . import ops
-from ._lib import OharaDelta
+from ._lib import DELTA_SILU_GATE, OharaDelta
 
 BF16, F32 = torch.bfloat16, torch.float32
 
@@ -38,16 +38,16 @@ class Linear:
         self.bias = None if bias is None else _pad(bias.detach().to(device=device, dtype=dtype), self.n).contiguous()
         self.w = w if dtype == F32 else ops.pack_linear(w)
 
-    def __call__(self, x: torch.Tensor) -> torch.Tensor:
+    def __call__(self, x: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
         if self.dtype == F32:
-            return ops.gemm_f32(x, self.w, self.bias, cap=self.cap)
+            return ops.gemm_f32(x, self.w, self.bias, cap=self.cap, out=out)
         if self.cap:
-            return ops.gemm_softcap(x, self.w, self.cap)
+            return ops.gemm_softcap(x, self.w, self.cap, out=out)
         if self.bias is not None:
-            return ops.linear_bias(x, self.w, self.bias)
+            return ops.linear_bias(x, self.w, self.bias, out=out)
         if x.stride(0) != x.shape[1]:
-            return ops.gemm(x, self.w)  # a column slice of a wider buffer
-        return ops.gemm_skinny(x, self.w)
+            return ops.gemm(x, self.w, out=out)  # a column slice of a wider buffer
+        return ops.gemm_skinny(x, self.w, out=out)
 
     def tensors(self):
         yield self.w if self.dtype == F32 else self.w.data
@@ -87,6 +87,27 @@ class GroupNorm:
         self.w = w.detach().to(device=device, dtype=F32).contiguous()
         self.groups, self.eps = groups, float(eps)
 
+    def of(self, y) -> dict:
+        """What ``ops.residual_norm`` needs to add the norm of y."""
+        return dict(y=y, norm_w=self.w, groups=self.groups, eps=self.eps)
+
+    def out(self) -> dict:
+        """What ``ops.residual_norm`` needs to return the norm of the residual."""
+        return dict(mode="norm", norm2_w=self.w, groups=self.groups, eps=self.eps)
+
+
+class LayerNorm(GroupNorm):
+    """(x - mean) / sqrt(variance + eps) times w, no bias (applied inside ``ops.residual_norm``)."""
+
+    def __init__(self, w, eps: float, device="cuda"):
+        super().__init__(w, 1, eps, device)
+
+    def of(self, y) -> dict:
+        return dict(super().of(y), center_y=True)
+
+    def out(self) -> dict:
+        return dict(super().out(), center_out=True)
+
 
 class InputConv:
     """h + causal depthwise convolution of h over time; w (width, taps), the last column is the current token's."""
@@ -108,35 +129,26 @@ def distance_slopes(heads: int) -> torch.Tensor:
     return torch.tensor([2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)], dtype=F32)
 
 
-class BiasedAttention:
-    """Causal attention without rotation: q and k normed over the whole projection, values over each head without a
-    weight, a linear distance bias on the scores, one sigmoid gate per head on the outputs.
-
-    q, k, v, gate, out: (weight, bias or None) pairs of the projections off the same input."""
+class CachedAttention:
+    """Keys and values per position, and the split of a decode step's context, for the attention classes below."""
 
     WORKGROUPS = 1024   # decode: a context is cut into chunks until about this many workgroups run
-    MIN_CHUNK = 128     # positions of a chunk at least (of the cache's capacity)
+    MIN_CHUNK = 128     # positions of a chunk at least (of what a query can see of the cache's capacity)
 
-    def __init__(self, q, k, v, gate, out, q_norm, k_norm, *, heads: int, kv_heads: int, dim: int, vdim: int, scale: float,
-                 eps: float, slopes: torch.Tensor, dtype=BF16, device="cuda"):
+    def _sizes(self, heads: int, kv_heads: int, dim: int, vdim: int, projections, dtype, device) -> None:
         if heads < 1 or kv_heads < 1 or heads % kv_heads:
             raise ValueError("kv_heads must divide heads")
-        for name, (w, b), n in (("q", q, heads * dim), ("k", k, kv_heads * dim), ("v", v, kv_heads * vdim), ("gate", gate, heads)):
-            if w.shape[0] != n or (b is not None and b.numel() != n):
+        for name, w, n in projections:
+            if w.shape[0] != n:
                 raise ValueError(f"attention {name} projection has {w.shape[0]} rows, {n} expected")
         if max(dim, vdim) > 256:
             raise ValueError("attention head sizes up to 256 are supported")
         self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
-        self.scale, self.eps, self.dtype, self.device = float(scale), float(eps), dtype, device
-        pairs = (q, k, v, gate)
-        biases = [b if b is not None else torch.zeros(w.shape[0], dtype=w.dtype, device=w.device) for w, b in pairs]
-        has_bias = any(b is not None for _, b in pairs)
-        self.proj = Linear(torch.cat([w for w, _ in pairs]), torch.cat(biases) if has_bias else None, dtype=dtype, device=device)
-        self.out = Linear(out, dtype=dtype, device=device)
-        dev = lambda t: t.detach().to(device=device, dtype=F32).contiguous()  # noqa: E731
-        self.q_norm, self.k_norm, self.slopes = dev(q_norm), dev(k_norm), dev(slopes)
-        self.gate_at = heads * dim + kv_heads * (dim + vdim)
+        self.dtype, self.device = dtype, device
         self._ws: dict = {}
+
+    def _visible(self, max_seq_length: int) -> int:
+        return max_seq_length
 
     def state(self, rows: int, max_seq_length: int) -> dict:
         zeros = lambda n: torch.zeros(rows, max_seq_length, self.kv_heads, ops.round8(n), dtype=self.dtype, device=self.device)  # noqa: E731
@@ -146,7 +158,7 @@ class BiasedAttention:
     def n_split(self, batch: int, max_seq_length: int) -> int:
         rep = self.heads // self.kv_heads
         sets = self.kv_heads * -(-rep // (4 if rep >= 4 else (2 if rep >= 2 else 1)))
-        return max(1, min(64, self.WORKGROUPS // (batch * sets), max_seq_length // self.MIN_CHUNK))
+        return max(1, min(64, self.WORKGROUPS // (batch * sets), self._visible(max_seq_length) // self.MIN_CHUNK))
 
     def _split(self, batch: int, max_seq_length: int):
         """(chunks, workspace) of a decode step; steps of the same batch size share the workspace, so they must run on one
@@ -158,6 +170,27 @@ class BiasedAttention:
         if ws is None:
             ws = self._ws[(batch, ns)] = ops.attn_bias_workspace(batch, self.heads, self.vdim, ns, self.device)
         return ns, ws
+
+
+class BiasedAttention(CachedAttention):
+    """Causal attention without rotation: q and k normed over the whole projection, values over each head without a
+    weight, a linear distance bias on the scores, one sigmoid gate per head on the outputs.
+
+    q, k, v, gate, out: (weight, bias or None) pairs of the projections off the same input."""
+
+    def __init__(self, q, k, v, gate, out, q_norm, k_norm, *, heads: int, kv_heads: int, dim: int, vdim: int, scale: float,
+                 eps: float, slopes: torch.Tensor, dtype=BF16, device="cuda"):
+        parts = (("q", q, heads * dim), ("k", k, kv_heads * dim), ("v", v, kv_heads * vdim), ("gate", gate, heads))
+        self._sizes(heads, kv_heads, dim, vdim, [(name, t, n) for name, pair, n in parts for t in pair if t is not None], dtype, device)
+        self.scale, self.eps = float(scale), float(eps)
+        pairs = (q, k, v, gate)
+        biases = [b if b is not None else torch.zeros(w.shape[0], dtype=w.dtype, device=w.device) for w, b in pairs]
+        has_bias = any(b is not None for _, b in pairs)
+        self.proj = Linear(torch.cat([w for w, _ in pairs]), torch.cat(biases) if has_bias else None, dtype=dtype, device=device)
+        self.out = Linear(out, dtype=dtype, device=device)
+        dev = lambda t: t.detach().to(device=device, dtype=F32).contiguous()  # noqa: E731
+        self.q_norm, self.k_norm, self.slopes = dev(q_norm), dev(k_norm), dev(slopes)
+        self.gate_at = heads * dim + kv_heads * (dim + vdim)
 
     def __call__(self, h, state, seq: ops.Seq):
         p = self.proj(h)
@@ -175,20 +208,185 @@ class BiasedAttention:
         yield from (self.q_norm, self.k_norm)
 
 
-class ChannelDelta:
-    """Gated delta rule with one decay per head and key channel (see csrc/delta_rule.hip for the equations): short
-    convolutions with silu on q, k and v, unit q and k, low-rank decay and output-gate projections, gated norm
-    per head.  q, k: (kv_heads * dim, width); v: (heads * vdim, width); convs: (channels, taps) each."""
+_ROTARY: dict = {}
+
+
+def rotary_tables(base: float, dims: int, positions: int, device):
+    """(cos, sin) of position * base^(-2i / dims), i < dims / 2, as (positions, dims / 2) fp32; one pair for all layers that share
+    the constants."""
+    device = torch.device(device)
+    key = (float(base), dims, positions, device.type, device.index)
+    if key not in _ROTARY:
+        f = float(base) ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / max(dims, 1))
+        a = torch.arange(positions, dtype=torch.float64).unsqueeze(1) * f
+        _ROTARY[key] = (a.cos().to(device, F32).contiguous(), a.sin().to(device, F32).contiguous())
+    return _ROTARY[key]
+
+
+class RotaryAttention(CachedAttention):
+    """Causal attention with the first ``rot_dims`` dimensions of q and k rotated in neighbouring pairs, soft-capped scores (``cap``,
+    0: none) and, with ``chunk`` > 0, keys of the query's own chunk of that many positions only."""
+
+    def __init__(self, q, k, v, out, *, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, rot_base: float, rot_dims: int,
+                 cap: float = 0.0, chunk: int = 0, dtype=BF16, device="cuda"):
+        self._sizes(heads, kv_heads, dim, vdim, (("q", q, heads * dim), ("k", k, kv_heads * dim), ("v", v, kv_heads * vdim)), dtype, device)
+        if rot_dims < 0 or rot_dims % 2 or rot_dims > dim:
+            raise ValueError("rotated dimensions must be an even number up to the head size")
+        if cap < 0 or chunk < 0:
+            raise ValueError("soft cap and chunk size cannot be negative")
+        self.scale, self.cap, self.chunk, self.rot_base, self.rot_dims = float(scale), float(cap), chunk, float(rot_base), rot_dims
+        self.proj = Linear(torch.cat([q, k, v]), dtype=dtype, device=device)
+        self.out = Linear(out, dtype=dtype, device=device)
+
+    def _visible(self, max_seq_length: int) -> int:
+        return min(max_seq_length, self.chunk) if self.chunk else max_seq_length
+
+    def state(self, rows: int, max_seq_length: int) -> dict:
+        rotary_tables(self.rot_base, self.rot_dims, max_seq_length, self.device)
+        return super().state(rows, max_seq_length)
+
+    def __call__(self, h, state, seq: ops.Seq):
+        p, t_max = self.proj(h), state.key.shape[1]
+        cos, sin = rotary_tables(self.rot_base, self.rot_dims, t_max, self.device)
+        q = ops.qkv_rotate_append(p, self.heads, self.kv_heads, self.dim, self.vdim, cos, sin, self.rot_dims, state.key, state.value, seq)
+        ns, ws = self._split(seq.batch, t_max) if seq.seq_len == 1 else (1, None)
+        att = ops.attn_scored(q, state.key, state.value, self.heads, self.kv_heads, self.dim, self.vdim, t_max, self.scale, seq,
+                              cap=self.cap, chunk=self.chunk, n_split=ns, workspace=ws)
+        return self.out(att)
+
+    def tensors(self):
+        yield from self.proj.tensors()
+        yield from self.out.tensors()
+
+
+class LatentAttention:
+    """Causal attention without positions whose queries come from one normed latent and whose keys and values are per-head
+    projections of another, the only thing cached; every output element times a sigmoid gate.
+
+    q_down (q_rank, width), q_up (heads * dim, q_rank); kv_down (rank, width), k_up (heads * dim, rank), v_up (heads * vdim, rank);
+    gate (heads * vdim, width).  Calls of ``EXPAND`` tokens and more form keys and values of all their positions once; shorter
+    ones apply k_up to the query and v_up to the weighted sum of the latents."""
+
+    EXPAND = 16
+    WORKGROUPS = 256    # a context is cut into chunks until about this many workgroups run
+    TILE = 64           # positions of a chunk at least
+
+    def __init__(self, q_down, q_norm, q_up, kv_down, kv_norm, k_up, v_up, gate, out, *, heads: int, dim: int, vdim: int, scale: float,
+                 eps: float, dtype=BF16, device="cuda"):
+        rq, r = q_down.shape[0], kv_down.shape[0]
+        for name, w, n in (("q_up", q_up, heads * dim), ("k_up", k_up, heads * dim), ("v_up", v_up, heads * vdim), ("gate", gate, heads * vdim)):
+            if w.shape[0] != n:
+                raise ValueError(f"latent attention {name} projection has {w.shape[0]} rows, {n} expected")
+        if max(dim, vdim) > 256 or r > 512:
+            raise ValueError("latent attention head sizes up to 256 and cached latents up to 512 are supported")
+        self.heads, self.dim, self.vdim, self.q_rank, self.rank = heads, dim, vdim, rq, r
+        self.scale, self.eps, self.dtype, self.device = float(scale), float(eps), dtype, device
+        kw = dict(dtype=dtype, device=device)
+        r8 = ops.round8
+        self.off_c = r8(rq)
+        self.off_g = self.off_c + r8(r)
+        self.proj = Linear(torch.cat([_pad(q_down, self.off_c), _pad(kv_down, r8(r)), gate]), **kw)
+        self.out = Linear(out, **kw)
+
+        def per_head(w, n):  # (heads * n, k) -> (heads, n, k), rows and columns padded to multiples of 8
+            w = w.detach().view(heads, n, w.shape[1])
+            return F.pad(w, (0, r8(w.shape[2]) - w.shape[2], 0, r8(n) - n))
+
+        k_heads, v_heads = per_head(k_up, dim), per_head(v_up, vdim)
+        self.q_up = Linear(per_head(q_up, dim).flatten(0, 1), **kw)
+        self.kv_up = Linear(torch.cat([k_heads.flatten(0, 1), v_heads.flatten(0, 1)]), **kw)
+        self.k_absorb = k_heads.transpose(1, 2).to(device=device, dtype=dtype).contiguous()
+        self.v_absorb = v_heads.to(device=device, dtype=dtype).contiguous()
+        dev = lambda t: t.detach().to(device=device, dtype=F32).contiguous()  # noqa: E731
+        self.q_norm, self.kv_norm = dev(q_norm), dev(kv_norm)
+        self._ws: dict = {}
+
+    def state(self, rows: int, max_seq_length: int) -> dict:
+        self._split(rows, max_seq_length)
+        return {"latent": torch.zeros(rows, max_seq_length, ops.round8(self.rank), dtype=self.dtype, device=self.device)}
+
+    def _split(self, rows: int, max_seq_length: int):
+        """(chunks, workspace) of a call over ``rows`` query tokens; calls of as many rows share the workspace."""
+        ns = max(1, min(64, self.WORKGROUPS // (rows * -(-self.heads // 16)), max_seq_length // self.TILE))
+        if ns == 1:
+            return 1, None
+        ws = self._ws.get((rows, ns))
+        if ws is None:
+            ws = self._ws[(rows, ns)] = ops.attn_latent_workspace(rows, self.heads, self.rank, ns, self.device)
+        return ns, ws
+
+    def _expanded(self, c, state, seq: ops.Seq):
+        """Keys and values of all positions of every sequence (batch, longest, [heads * dim; heads * vdim]).  ``c``: the call's own
+        latents where that is all of them."""
+        if c is not None:
+            return self.kv_up(c), seq.seq_len
+        starts, counts, rows = seq.host
+        ends = [s + n for s, n in zip(starts, counts)]
+        kv = torch.empty(seq.batch, max(ends), self.kv_up.n, dtype=self.dtype, device=self.device)
+        for b, (row, end) in enumerate(zip(rows, ends)):
+            self.kv_up(state.latent[row, :end], out=kv[b, :end])
+        return kv.view(-1, self.kv_up.n), max(ends)
+
+    def __call__(self, h, state, seq: ops.Seq):
+        p = self.proj(h)
+        H, n = self.heads, self.heads * self.vdim
+        gate = p[:, self.off_g:self.off_g + n]
+        expand = seq.seq_len >= self.EXPAND and seq.host is not None
+        whole = expand and not any(seq.host[0])
+        cq, c = ops.latent_front(p, self.q_rank, self.off_c, self.rank, self.q_norm, self.kv_norm, self.eps, state.latent, seq, whole)
+        q = self.q_up(cq)
+        if expand:
+            kv, length = self._expanded(c, state, seq)
+            at = ops.Seq(seq.batch, seq.seq_len, int(seq.c.pos), seq.pos_dev, bool(seq.c.pos_stride), seq.lens)
+            att = ops.attn_scored(q, kv, kv[:, H * ops.round8(self.dim):], H, H, self.dim, self.vdim, length, self.scale, at, gate=gate,
+                                  gate_elements=True, ld_k=kv.stride(0), ld_v=kv.stride(0))
+            return self.out(att)
+        ns, ws = self._split(seq.rows, state.latent.shape[1])
+        mixed = ops.attn_latent(ops.head_linear(q, self.k_absorb, ops.round8(self.rank)), state.latent, H, self.rank, self.scale, seq, ns, ws)
+        return self.out(ops.head_linear(mixed, self.v_absorb, self.vdim, gate))
+
+    def tensors(self):
+        for lin in (self.proj, self.q_up, self.kv_up, self.out):
+            yield from lin.tensors()
+        yield from (self.q_norm, self.kv_norm)
+
+
+class TokenSide:
+    """What a layer adds to the residual for its token: proj(gelu_tanh(gate x) * e) with e the row's ``dim`` entries of an embedding
+    table from ``column`` on, over its own root mean square times norm_w (``norm``)."""
+
+    def __init__(self, gate, proj, norm_w, table, column: int, *, eps: float, dtype=BF16, device="cuda"):
+        self.gate, self.proj = Linear(gate, dtype=dtype, device=device), Linear(proj, dtype=dtype, device=device)
+        self.norm = GroupNorm(norm_w, 1, eps, device)
+        self.table, self.column = table, column
+
+    @staticmethod
+    def lay_out(table, layers: int, *, dtype=BF16, device="cuda") -> torch.Tensor:
+        """(vocab, layers * dim) -> (vocab, layers * dim rounded up to 8), each layer's entries followed by zeros."""
+        vocab, n = table.shape
+        t = table.detach().view(vocab, layers, n // layers)
+        return F.pad(t, (0, ops.round8(t.shape[2]) - t.shape[2])).flatten(1).to(device=device, dtype=dtype).contiguous()
+
+    def __call__(self, x, ids):
+        return self.proj(ops.gemm_gelu_lookup(x, self.gate.w, self.table, self.column, ids))
+
+    def tensors(self):
+        yield from self.gate.tensors()
+        yield from self.proj.tensors()
+        yield self.norm.w
+
+
+class DeltaRule:
+    """Gated delta rule (see csrc/delta_rule.hip for the equations): short convolutions with silu on q, k and v, unit q and k,
+    gated norm per head.  The subclasses give decays and output gates."""
 
     WORKSPACE = 1 << 30  # bytes of per-chunk intermediates at most; longer prompts are walked in segments
     _workspaces: dict = {}  # device -> the workspace every layer on that device shares (prompts run on one stream)
 
-    def __init__(self, q, k, v, q_conv, k_conv, v_conv, beta, a_log, a1, a2, dt_bias, g1, g2, norm_w, out, *, heads: int,
-                 kv_heads: int, dim: int, vdim: int, eps: float, dtype=BF16, device="cuda"):
+    def _sizes(self, heads: int, kv_heads: int, dim: int, vdim: int, q, k, v, more, convs, a_log, dt_bias, norm_w, eps: float, dtype, device):
         if heads < 1 or kv_heads < 1 or heads % kv_heads:
             raise ValueError("kv_heads must divide heads")
-        for name, w, n in (("q", q, kv_heads * dim), ("k", k, kv_heads * dim), ("v", v, heads * vdim), ("beta", beta, heads),
-                           ("a2", a2, heads * dim), ("g2", g2, heads * vdim)):
+        for name, w, n in (("q", q, kv_heads * dim), ("k", k, kv_heads * dim), ("v", v, heads * vdim), *more):
             if w.shape[0] != n:
                 raise ValueError(f"delta rule {name} projection has {w.shape[0]} rows, {n} expected")
         if max(dim, vdim) > 256:
@@ -196,26 +394,18 @@ class ChannelDelta:
         self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
         self.dtype, self.device = dtype, torch.device(device)
         self.channels = 2 * kv_heads * dim + heads * vdim
-        self.taps = q_conv.shape[1]
-        ra, rg = ops.round8(a1.shape[0]), ops.round8(g1.shape[0])
+        self.taps = convs[0].shape[1]
         self.off_a = ops.round8(self.channels)
-        self.off_g, self.off_b = self.off_a + ra, self.off_a + ra + rg
-        qkv = _pad(torch.cat([q, k, v]), self.off_a)
-        self.proj = Linear(torch.cat([qkv, _pad(a1, ra), _pad(g1, rg), beta]), dtype=dtype, device=device)
-        a2, g2 = _pad(a2, a2.shape[0], ra), _pad(g2, g2.shape[0], rg)
-        self.a2_proj, self.g2_proj = (Linear(w, dtype=dtype, device=device) for w in (a2, g2))
-        self.out = Linear(out, dtype=dtype, device=device)
-        dev = lambda t, dt=F32: t.detach().to(device=device, dtype=dt).contiguous()  # noqa: E731
-        self.a2, self.g2 = dev(a2, dtype), dev(g2, dtype)
-        self.conv_w = dev(torch.cat([q_conv, k_conv, v_conv]).t())
-        self.neg_a = -torch.exp(dev(a_log))
-        self.dt_bias, self.norm_w = dev(dt_bias), dev(norm_w)
+        self.conv_w = self._dev(torch.cat(convs).t())
+        self.neg_a = -torch.exp(self._dev(a_log))
+        self.dt_bias, self.norm_w = self._dev(dt_bias), self._dev(norm_w)
         d = OharaDelta()
-        d.heads, d.kv_heads, d.dim, d.vdim, d.taps = heads, kv_heads, dim, vdim, self.taps
-        d.rank_a, d.rank_g, d.off_a, d.off_g, d.off_b, d.eps = ra, rg, self.off_a, self.off_g, self.off_b, float(eps)
-        d.conv_w, d.a2, d.g2 = self.conv_w.data_ptr(), self.a2.data_ptr(), self.g2.data_ptr()
-        d.neg_a, d.dt_bias, d.norm_w = self.neg_a.data_ptr(), self.dt_bias.data_ptr(), self.norm_w.data_ptr()
+        d.heads, d.kv_heads, d.dim, d.vdim, d.taps, d.eps = heads, kv_heads, dim, vdim, self.taps, float(eps)
+        d.conv_w, d.neg_a, d.dt_bias, d.norm_w = (t.data_ptr() for t in (self.conv_w, self.neg_a, self.dt_bias, self.norm_w))
         self._c = d
+
+    def _dev(self, t, dtype=F32):
+        return t.detach().to(device=self.device, dtype=dtype).contiguous()
 
     def state(self, rows: int, max_seq_length: int) -> dict:
         return {"delta": torch.zeros(rows, self.heads, self.dim, (self.vdim + 3) // 4 * 4, dtype=F32, device=self.device),
@@ -224,21 +414,68 @@ class ChannelDelta:
     def _workspace(self, batch: int, tokens: int) -> torch.Tensor:
         need = ops.delta_workspace_bytes(self.heads, self.dim, self.vdim, batch, tokens)
         need = max(min(need, self.WORKSPACE), ops.delta_workspace_bytes(self.heads, self.dim, self.vdim, batch, 1))
-        ws = ChannelDelta._workspaces.get(self.device)
+        ws = DeltaRule._workspaces.get(self.device)
         if ws is None or ws.numel() < need:
-            ws = ChannelDelta._workspaces[self.device] = torch.empty(need, dtype=torch.uint8, device=self.device)
+            ws = DeltaRule._workspaces[self.device] = torch.empty(need, dtype=torch.uint8, device=self.device)
         return ws
+
+    def _low_rank(self, p):
+        """(decay logits, output gates) of a prompt that are not columns of p."""
+        return None, None
 
     def __call__(self, h, state, seq: ops.Seq):
         p = self.proj(h)
         if seq.seq_len == 1:
             return self.out(ops.delta_step(self._c, p, state.delta, state.ring, seq))
-        za = self.a2_proj(p[:, self.off_a:self.off_g])
-        zg = self.g2_proj(p[:, self.off_g:self.off_b])
+        za, zg = self._low_rank(p)
         o = ops.delta_prefill(self._c, p, za, zg, state.delta, state.ring, self._workspace(seq.batch, seq.seq_len), seq)
         return self.out(o)
 
     def tensors(self):
-        for lin in (self.proj, self.a2_proj, self.g2_proj, self.out):
-            yield from lin.tensors()
+        yield from self.proj.tensors()
+        yield from self.out.tensors()
         yield from (self.conv_w, self.neg_a, self.dt_bias, self.norm_w)
+
+
+class ChannelDelta(DeltaRule):
+    """One decay per head and key channel, low-rank decay and output-gate projections, sigmoid gate.  q, k: (kv_heads * dim, width);
+    v: (heads * vdim, width); convs: (channels, taps) each."""
+
+    def __init__(self, q, k, v, q_conv, k_conv, v_conv, beta, a_log, a1, a2, dt_bias, g1, g2, norm_w, out, *, heads: int,
+                 kv_heads: int, dim: int, vdim: int, eps: float, dtype=BF16, device="cuda"):
+        self._sizes(heads, kv_heads, dim, vdim, q, k, v, (("beta", beta, heads), ("a2", a2, heads * dim), ("g2", g2, heads * vdim)),
+                    (q_conv, k_conv, v_conv), a_log, dt_bias, norm_w, eps, dtype, device)
+        ra, rg = ops.round8(a1.shape[0]), ops.round8(g1.shape[0])
+        self.off_g, self.off_b = self.off_a + ra, self.off_a + ra + rg
+        qkv = _pad(torch.cat([q, k, v]), self.off_a)
+        self.proj = Linear(torch.cat([qkv, _pad(a1, ra), _pad(g1, rg), beta]), dtype=dtype, device=device)
+        a2, g2 = _pad(a2, a2.shape[0], ra), _pad(g2, g2.shape[0], rg)
+        self.a2_proj, self.g2_proj = (Linear(w, dtype=dtype, device=device) for w in (a2, g2))
+        self.out = Linear(out, dtype=dtype, device=device)
+        self.a2, self.g2 = self._dev(a2, dtype), self._dev(g2, dtype)
+        d = self._c
+        d.rank_a, d.rank_g, d.off_a, d.off_g, d.off_b = ra, rg, self.off_a, self.off_g, self.off_b
+        d.a2, d.g2 = self.a2.data_ptr(), self.g2.data_ptr()
+
+    def _low_rank(self, p):
+        return self.a2_proj(p[:, self.off_a:self.off_g]), self.g2_proj(p[:, self.off_g:self.off_b])
+
+    def tensors(self):
+        yield from super().tensors()
+        for lin in (self.a2_proj, self.g2_proj):
+            yield from lin.tensors()
+
+
+class HeadDelta(DeltaRule):
+    """One decay per head, output gate by a projection of its own through silu.  q, k: (kv_heads * dim, width); v, gate:
+    (heads * vdim, width); beta, decay: (heads, width); convs: (channels, taps) each."""
+
+    def __init__(self, q, k, v, q_conv, k_conv, v_conv, beta, a_log, decay, dt_bias, gate, norm_w, out, *, heads: int, kv_heads: int,
+                 dim: int, vdim: int, eps: float, dtype=BF16, device="cuda"):
+        self._sizes(heads, kv_heads, dim, vdim, q, k, v, (("beta", beta, heads), ("decay", decay, heads), ("gate", gate, heads * vdim)),
+                    (q_conv, k_conv, v_conv), a_log, dt_bias, norm_w, eps, dtype, device)
+        self.proj = Linear(torch.cat([_pad(torch.cat([q, k, v]), self.off_a), gate, decay, beta]), dtype=dtype, device=device)
+        self.out = Linear(out, dtype=dtype, device=device)
+        d, n = self._c, heads * vdim
+        d.off_g, d.off_a, d.off_b = self.off_a, self.off_a + n, self.off_a + n + heads
+        d.flags = DELTA_SILU_GATE

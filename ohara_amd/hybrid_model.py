@@ -1,0 +1,170 @@
+"""What the hybrid decoders share: the call surface of the other models around a list of layer blocks.
+
+A design's class builds ``self.layers`` (one dict per layer with a "mixer" of ``ohara_amd.hybrid``) and gives ``_run``, the
+launches of one call; positions, cache rows, checks, sessions and greedy generation are here.  ``position`` may be one
+per sequence, prompts of one call may have different lengths (``seq_lens``) and sit in chosen cache rows
+(``slots``).
+"""
+
+from __future__ import annotations
+
+import torch
+
+from . import ops
+from ._lib import lib
+from .hybrid import BF16, F32
+from .llama import _check_ids_on_host
+from .session import GraphDecodeSession
+from .state_cache import LayerState
+
+
+class HybridDecoder:
+    supports_last_only = True   # forward(..., last_only=True) computes the last row of logits only
+    supports_seq_lens = True    # forward(..., seq_lens=, slots=): prompts of different lengths, chosen cache rows
+
+    def __init__(self, config, device, dtype):
+        if dtype not in (BF16, F32):
+            raise ValueError(f"{type(self).__name__} is served in bfloat16 or float32")
+        lib()  # fail loudly now if the HIP library is missing
+        self.config, self.device, self.dtype = config, torch.device(device), dtype
+        self.layers = []
+        self.trace = None  # a list: forward() appends the residual stream after every layer to it
+
+    @staticmethod
+    def _tensor(state: dict, name: str, *shape) -> torch.Tensor:
+        t = state[name]
+        if tuple(t.shape) != shape:
+            raise ValueError(f"{name} has shape {tuple(t.shape)}, the config says {shape}")
+        return t
+
+    def _layer_state(self, block: dict, rows: int, max_seq_length: int) -> dict:
+        """The tensors a layer keeps per sequence."""
+        return block["mixer"].state(rows, max_seq_length)
+
+    def eval(self):
+        return self
+
+    def to(self, *args, **kwargs):
+        """A request for the device / dtype the model was built with is a no-op, anything else raises."""
+        for a in (*args, kwargs.get("device"), kwargs.get("dtype")):
+            if isinstance(a, torch.dtype):
+                if a != self.dtype:
+                    raise ValueError(f"ohara_amd: the model was built in {self.dtype}; build it in {a} instead of casting it")
+            elif a is not None:
+                want = torch.device(a)
+                if want.type != self.device.type or (want.index is not None and want.index != (self.device.index or 0)):
+                    raise ValueError(f"ohara_amd: the model lives on {self.device}; build it on {want} instead of moving it")
+        return self
+
+    def build_kv_cache(self, batch_size: int = 1, int8: bool = False) -> list[LayerState]:
+        """One ``LayerState`` per layer: what its mixer keeps per sequence (keys and values, latents, a recurrent state and its
+        convolution's past inputs) and what the design adds (``_layer_state``)."""
+        if batch_size < 1:
+            raise ValueError("batch_size must be at least 1")
+        if int8:
+            raise ValueError(f"{type(self).__name__} keeps its caches in the model's dtype (no int8 mode)")
+        t = self.config.max_sequence_length
+        return [LayerState(t, self._layer_state(b, batch_size, t), i) for i, b in enumerate(self.layers)]
+
+    @torch.no_grad()
+    def forward(self, x: torch.Tensor, kv_cache: list | None = None, position_ids=None, *, last_only: bool = False,
+                seq_pos: torch.Tensor | None = None, seq_lens=None, slots=None) -> torch.Tensor:
+        """Logits (B, S, vocab), or (B, 1, vocab) of every sequence's last token with ``last_only``.  ``position_ids``: one
+        position, or a list with one per sequence (``seq_pos``: the same as an int32 device tensor the caller keeps up to
+        date).  ``seq_lens``: tokens of each sequence in this call, the rest of its row is padding.  ``slots``: the cache row
+        of each sequence (rows not named are left alone)."""
+        c = self.config
+        if x.ndim != 2:
+            raise ValueError("input token IDs must have shape (batch, sequence)")
+        B, S = x.shape
+        if isinstance(position_ids, torch.Tensor):
+            position_ids = [int(p) for p in position_ids.tolist()] if position_ids.numel() > 1 else int(position_ids.item())
+        if S < 1:
+            raise ValueError("input sequence cannot be empty")
+        if kv_cache is None:
+            if position_ids is not None or slots is not None:
+                raise ValueError("position_ids is only valid when using a KV cache")
+            if S > c.max_sequence_length:
+                raise ValueError("input exceeds max_sequence_length")
+            kv_cache, position_ids = self.build_kv_cache(B), 0
+        if len(kv_cache) != c.num_hidden_layers:
+            raise ValueError("KV cache must contain one entry per model layer")
+        lens = [S] * B if seq_lens is None else [int(n) for n in seq_lens]
+        if len(lens) != B or min(lens) < 1 or max(lens) > S:
+            raise ValueError("seq_lens must hold one count in [1, sequence] per sequence")
+        ragged = isinstance(position_ids, (list, tuple))
+        starts = [int(p) for p in position_ids] if ragged else [position_ids] * B
+        if len(starts) != B:
+            raise ValueError("one position per sequence is required")
+        if any(p is None or p < 0 for p in starts):
+            raise ValueError("a non-negative position_ids is required with KV cache")
+        if max(p + n for p, n in zip(starts, lens)) > c.max_sequence_length:
+            raise ValueError("input exceeds max_sequence_length")
+        if slots is not None:
+            slots = [int(s) for s in slots]
+            if len(slots) != B:
+                raise ValueError("one slot per sequence is required")
+            ends = [cc._reserve_rows(slots, lens, starts) for cc in kv_cache]
+        elif ragged or len(set(lens)) > 1:
+            ends = [cc._reserve_ragged(B, lens, starts) for cc in kv_cache]
+        else:
+            ends = [cc._reserve(B, lens[0], starts[0]) for cc in kv_cache]
+        _check_ids_on_host(x, c.vocab_size)
+
+        def dev32(values):
+            return torch.tensor(values, dtype=torch.int32).to(self.device)
+
+        per_sequence = seq_pos is not None or len(set(starts)) > 1
+        if per_sequence and seq_pos is None:
+            seq_pos = dev32(starts)
+        seq = ops.Seq(B, S, starts[0], seq_pos, per_sequence, None if lens == [S] * B else dev32(lens),
+                      None if slots is None else dev32(slots), (starts, lens, slots or list(range(B))))
+        logits = self._run(x.reshape(-1).to(device=self.device, dtype=torch.int64), kv_cache, seq, last_only)
+        for cc, end in zip(kv_cache, ends):
+            if slots is not None:
+                cc._commit_rows(slots, end)
+            elif isinstance(end, list):
+                cc._commit_ragged(B, end)
+            else:
+                cc._commit(B, end)
+        return logits.view(B, 1 if last_only else S, c.vocab_size)
+
+    __call__ = forward
+
+    def _run(self, ids: torch.Tensor, kv_cache: list, seq: ops.Seq, last_only: bool) -> torch.Tensor:
+        """The launches of one call; no host-side state, so a one-token call can be captured in a graph."""
+        raise NotImplementedError
+
+    @staticmethod
+    def _last_rows(h: torch.Tensor, seq: ops.Seq) -> torch.Tensor:
+        """The rows of every sequence's last token."""
+        last = torch.arange(seq.batch, device=h.device) * seq.seq_len - 1
+        return h[last + (seq.seq_len if seq.lens is None else seq.lens)]
+
+    # -- device-resident loop ------------------------------------------------------------------
+
+    def supports_persistent(self, batch: int) -> bool:
+        """There is no single-launch decode kernel for this model: sessions replay the captured chain."""
+        return False
+
+    def session(self, batch: int, max_new_tokens: int, valid_vocab: int = 0, kv_cache: list | None = None,
+                persistent: bool | None = None, sampling=None, u=None) -> GraphDecodeSession:
+        if persistent:
+            raise ValueError("the persistent decode kernel does not cover this shape")
+        return GraphDecodeSession(self, batch, max_new_tokens, valid_vocab, kv_cache, sampling, u)
+
+    def decode_step(self, ids: torch.Tensor, kv_cache: list, pos_dev: torch.Tensor) -> torch.Tensor:
+        """Logits (B, vocab) of one more token per sequence at the shared position ``pos_dev[0]`` (int32, on the device);
+        touches no host-side bookkeeping."""
+        return self._run(ids, kv_cache, ops.Seq(ids.numel(), 1, 0, pos_dev), False)
+
+    @torch.no_grad()
+    def generate_greedy(self, prompt_ids: torch.Tensor, steps: int, *, use_graph: bool = True, valid_vocab: int = 0,
+                        kv_cache: list | None = None) -> torch.Tensor:
+        """Prefill the prompts, then ``steps`` greedy tokens with no host round trip per token -> (B, steps) ids."""
+        if steps < 1:
+            return torch.zeros(prompt_ids.shape[0], 0, dtype=torch.int64, device=self.device)
+        sess = self.session(prompt_ids.shape[0], steps, valid_vocab, kv_cache)
+        sess.prefill(prompt_ids)
+        sess.run(steps - 1, use_graph=use_graph)
+        return sess.tokens()

@@ -608,17 +608,23 @@ class Seq:
     position for all sequences, or one per sequence with ``per_sequence``; ``lens`` / ``slots`` (int32, one entry per
     sequence): tokens of each sequence in the call, cache row of each sequence."""
 
-    __slots__ = ("c", "batch", "seq_len", "lens", "_keep")
+    __slots__ = ("c", "batch", "seq_len", "lens", "host", "_keep")
 
-    def __init__(self, batch: int, seq_len: int, pos: int = 0, pos_dev=None, per_sequence: bool = False, lens=None, slots=None):
+    def __init__(self, batch: int, seq_len: int, pos: int = 0, pos_dev=None, per_sequence: bool = False, lens=None, slots=None,
+                 host=None):
+        """``host``: (starts, counts, rows of the cache) of the sequences as lists, where the caller knows them."""
         for name, t in (("pos_dev", pos_dev), ("lens", lens), ("slots", slots)):
             if t is not None:
                 _need(t, torch.int32, name)
                 if t.numel() < (1 if name == "pos_dev" and not per_sequence else batch):
                     raise ValueError(f"{name}: one entry per sequence is required")
-        self.batch, self.seq_len, self.lens = batch, seq_len, lens
+        self.batch, self.seq_len, self.lens, self.host = batch, seq_len, lens, host
         self._keep = (pos_dev, lens, slots)
         self.c = _lib.OharaSeq(batch, seq_len, int(pos), int(per_sequence), _ptr(pos_dev), _ptr(lens), _ptr(slots))
+
+    @property
+    def pos_dev(self):
+        return self._keep[0]
 
     @property
     def rows(self) -> int:
@@ -630,13 +636,15 @@ class Seq:
 
 
 def residual_norm(x, seq: Seq, dtype, *, ids=None, table=None, y=None, norm_w=None, groups=1, eps=0.0, mode="none",
-                  norm2_w=None, conv_w=None, ring=None):
+                  norm2_w=None, conv_w=None, ring=None, center_y=False, center_out=False):
     """x (rows, d) fp32 <- table[ids], or x + norm_w * group_rms(y), in place; returns what ``mode`` asks for as
     (rows, d rounded up to 8) in ``dtype``: "copy" of x, "conv" (x + causal depthwise convolution over time, one token per
-    sequence, ring updated), "norm" (group RMS norm of x times norm2_w), or None."""
+    sequence, ring updated), "norm" (group RMS norm of x times norm2_w), or None.  ``center_y`` / ``center_out``: the norm
+    of y / of the output is a layer norm without bias."""
     _need(x, F32, "x")
     rows, d = x.shape
     m = {"none": _lib.OUT_NONE, "copy": _lib.OUT_COPY, "conv": _lib.OUT_CONV, "norm": _lib.OUT_NORM}[mode]
+    m |= (_lib.CENTER_Y if center_y else 0) | (_lib.CENTER_OUT if center_out else 0)
     if rows != seq.rows:
         raise ValueError("x has one row per token of the call")
     for t, name in ((y, "y"), (table, "table")):
@@ -696,6 +704,35 @@ def gemm_softcap(x, w: PackedLinear, cap: float, out=None):
     return out
 
 
+def gemm_gelu_lookup(x, w, table, column: int, ids, out=None):
+    """gelu_tanh(x W^T) * table[ids, column: column + n]; w: a packed weight (bf16) or (n, k) fp32, table (vocab, columns), ids
+    (rows,) int64 on the device."""
+    f32 = x.dtype == F32
+    n, k = w.shape if f32 else (w.n, w.k)
+    if not x.is_cuda or x.stride(1) != 1 or x.shape[1] != k or table.dtype != x.dtype or not table.is_contiguous():
+        raise ValueError("x and table must be device matrices of one dtype, x with W's columns")
+    if column < 0 or column + n > table.shape[1] or ids.dtype != torch.int64 or ids.numel() != x.shape[0]:
+        raise ValueError("the table has no such columns, or ids are not one int64 per row")
+    if out is None:
+        out = torch.empty(x.shape[0], n, dtype=x.dtype, device=x.device)
+    check(_typed("gemm_gelu_lookup", x.dtype)(
+        _ptr(x), x.stride(0), _ptr(w if f32 else w.data), n, k, _ptr(table) + column * table.element_size(), table.stride(0),
+        _ptr(ids), table.shape[0], x.shape[0], _ptr(out), out.stride(0), _stream()), "gemm_gelu_lookup")
+    return out
+
+
+def qkv_rotate_append(p, h, h_kv, dh, dv, cos, sin, rot, kcache, vcache, seq: Seq):
+    """p rows [q; k; v; ...] -> q (rows, h * round8(dh)); keys and values into the caches; the first ``rot`` dimensions of q and
+    k heads rotated in neighbouring pairs by the tables cos, sin (positions, rot / 2) fp32."""
+    if rot and (cos.shape != (cos.shape[0], rot // 2) or cos.shape[0] < kcache.shape[1] or cos.shape != sin.shape):
+        raise ValueError("rotary tables must cover the cache's positions with rot / 2 angles each")
+    q = torch.empty(p.shape[0], h * round8(dh), dtype=p.dtype, device=p.device)
+    check(_typed("qkv_rotate_append", p.dtype)(
+        _ptr(p), p.stride(0), h, h_kv, dh, dv, _ptr(cos), _ptr(sin), rot, _ptr(q), _ptr(kcache), _ptr(vcache), kcache.shape[1],
+        seq.ref, _stream()), "qkv_rotate_append")
+    return q
+
+
 def qkv_norm_append(p, h, h_kv, dh, dv, qn, kn, eps, kcache, vcache, seq: Seq):
     """p rows [q; k; v; ...] -> normalised q (rows, h * round8(dh)); keys and values into the caches."""
     q = torch.empty(p.shape[0], h * round8(dh), dtype=p.dtype, device=p.device)
@@ -722,6 +759,58 @@ def attn_bias(q, kcache, vcache, h, h_kv, dh, dv, scale, slopes, gate, seq: Seq,
     return out
 
 
+def attn_scored(q, keys, values, h, h_kv, dh, dv, t_max, scale, seq: Seq, *, cap=0.0, chunk=0, slopes=None, gate=None,
+                gate_elements=False, ld_k=0, ld_v=0, n_split=1, workspace=None):
+    """Causal attention over positions of ``keys`` / ``values`` (cache rows of t_max positions, ``ld_k`` / ``ld_v`` elements apart if
+    not densely packed) -> (rows, round8(h * dv)).  Scores: scale q . k, soft-capped by ``cap``, minus slopes[head] * distance;
+    ``chunk``: inside chunks of that many positions.  gate: a (rows, h) or, ``gate_elements``, (rows, h * dv) column slice,
+    through the sigmoid."""
+    out = torch.empty(q.shape[0], round8(h * dv), dtype=q.dtype, device=q.device)
+    sc = _lib.OharaScores(scale, cap, chunk, int(gate_elements), ld_k, ld_v, _ptr(slopes))
+    check(_typed("attn_scored", q.dtype)(
+        _ptr(q), _ptr(keys), _ptr(values), h, h_kv, dh, dv, t_max, C.byref(sc), _ptr(gate), 0 if gate is None else gate.stride(0),
+        n_split, _ptr(workspace), _ptr(out), out.stride(0), seq.ref, _stream()), "attn_scored")
+    return out
+
+
+def latent_front(p, q_rank, off_c, rank, qn, cn, eps, cache, seq: Seq, compact: bool = False):
+    """p rows [query latent; cached latent at off_c] -> RMS-normed query latent (rows, round8(q_rank)) and, with ``compact``, the
+    normed cached latent (rows, round8(rank)), which goes into the cache (cache rows, positions, round8(rank)) either way."""
+    q = torch.empty(p.shape[0], round8(q_rank), dtype=p.dtype, device=p.device)
+    c = torch.empty(p.shape[0], round8(rank), dtype=p.dtype, device=p.device) if compact else None
+    check(_typed("latent_front", p.dtype)(
+        _ptr(p), p.stride(0), q_rank, off_c, rank, _ptr(qn), _ptr(cn), eps, _ptr(q), _ptr(cache), cache.shape[1], _ptr(c), seq.ref,
+        _stream()), "latent_front")
+    return q, c
+
+
+def head_linear(x, w, n_out: int, gate=None):
+    """x (rows, >= h * k), w (h, n, k) -> (rows, round8(h * n_out)): one matrix per head, the first n_out entries of each, times
+    sigmoid(gate) with gate a (rows, h * n_out) column slice."""
+    h, n, k = w.shape
+    out = torch.empty(x.shape[0], round8(h * n_out), dtype=x.dtype, device=x.device)
+    check(_typed("head_linear", x.dtype)(
+        _ptr(x), x.stride(0), _ptr(w), h, n, k, n_out, x.shape[0], _ptr(gate), 0 if gate is None else gate.stride(0), _ptr(out),
+        out.stride(0), _stream()), "head_linear")
+    return out
+
+
+def attn_latent_workspace(rows, h, rank, n_split, device) -> torch.Tensor:
+    n = lib().ohara_attn_latent_workspace_bytes(rows, h, rank, n_split)
+    if n < 0:
+        raise ValueError("bad latent attention workspace shape")
+    return torch.empty(n, dtype=torch.uint8, device=device)
+
+
+def attn_latent(q, cache, h, rank, scale, seq: Seq, n_split=1, workspace=None):
+    """q (rows, h * round8(rank)) against the cached latents (cache rows, positions, round8(rank)), which are keys and values at
+    once -> weighted sums (rows, h * round8(rank))."""
+    out = torch.empty_like(q)
+    check(_typed("attn_latent", q.dtype)(_ptr(q), _ptr(cache), h, rank, cache.shape[1], scale, n_split, _ptr(workspace), _ptr(out),
+                                         seq.ref, _stream()), "attn_latent")
+    return out
+
+
 def delta_step(d: "_lib.OharaDelta", p, state, ring, seq: Seq):
     """One token per sequence of the gated delta rule -> (rows, round8(heads * vdim)); state and ring updated."""
     out = torch.empty(p.shape[0], round8(d.heads * d.vdim), dtype=p.dtype, device=p.device)
@@ -738,12 +827,12 @@ def delta_workspace_bytes(heads, dim, vdim, batch, tokens) -> int:
 
 
 def delta_prefill(d: "_lib.OharaDelta", p, za, zg, state, ring, workspace, seq: Seq):
-    """Any number of tokens per sequence of the gated delta rule; the ring is updated after the call's convolutions."""
+    """Any number of tokens per sequence of the gated delta rule (za, zg: the low-rank products, None where d has no such matrix); the ring is updated after the call's convolutions."""
     rows = p.shape[0]
     out = torch.empty(rows, round8(d.heads * d.vdim), dtype=p.dtype, device=p.device)
     o_tmp = torch.empty(rows, d.heads * d.vdim, dtype=F32, device=p.device)
     check(_typed("delta_prefill", p.dtype)(
-        C.byref(d), _ptr(p), p.stride(0), _ptr(za), za.stride(0), _ptr(zg), zg.stride(0), _ptr(state), _ptr(ring),
+        C.byref(d), _ptr(p), p.stride(0), _ptr(za), 0 if za is None else za.stride(0), _ptr(zg), 0 if zg is None else zg.stride(0), _ptr(state), _ptr(ring),
         _ptr(workspace), workspace.numel(), _ptr(o_tmp), _ptr(out), out.stride(0), seq.ref, _stream()), "delta_prefill")
     conv_ring_store(p, 2 * d.kv_heads * d.dim + d.heads * d.vdim, ring, seq)
     return out

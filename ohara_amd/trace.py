@@ -54,12 +54,12 @@ def main(argv=None) -> int:
 
     from . import build
 
-    build.ensure(build.SERVING)
+    from .checkpoint import architecture_of, build_model, load_checkpoint
+
+    build.ensure(architecture_of(args.model))
 
     import numpy as np
     import torch
-
-    from .checkpoint import build_model, load_checkpoint
 
     config, state = load_checkpoint(args.model, max_sequence_length=max(2, args.max_tokens))
     model = build_model(config, state, dtype=getattr(torch, args.dtype))

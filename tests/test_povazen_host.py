@@ -10,7 +10,7 @@ import torch
 
 from _povazen import CONFIGS
 from ohara_amd import _lib, build
-from ohara_amd.checkpoint import _architecture, load_checkpoint
+from ohara_amd.checkpoint import ARCHITECTURES, _architecture, load_checkpoint
 from ohara_amd.povazen import Povazen, PovazenConfig
 from ohara_amd.state_cache import LayerState
 
@@ -93,7 +93,7 @@ def test_entry_points_check_their_arguments():
 
 def test_partial_library_sources_exist():
     names = {os.path.basename(s)[:-4] for s in build.sources()}
-    assert set(build.SERVING) <= names
+    assert set().union(*build.SERVING.values()) <= names and set(build.SERVING) == set(ARCHITECTURES)
 
 
 class _Model:
