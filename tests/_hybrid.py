@@ -1,0 +1,78 @@
+"""Helpers of the hybrid decoders' tests: random inputs, comparisons with float64, caches full of an earlier owner's leftovers."""
+
+import torch
+
+BF, F32 = torch.bfloat16, torch.float32
+
+
+def tokens(cfg, n, seed=0):
+    return torch.randint(0, cfg["vocab"], (n,), generator=torch.Generator().manual_seed(seed)).tolist()
+
+
+def doubled(weights):
+    return {k: v.double() for k, v in weights.items()}
+
+
+def row_errors(got, want):
+    """Root mean square of the logits' difference, row by row, over that of the logits."""
+    want = want.double()
+    d = got.double().cpu() - want
+    return d.pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
+
+
+def error(got, want):
+    return row_errors(got, want).max().item()
+
+
+def agrees(got, want, dtype):
+    """Logits row by row against float64, as a share of their root mean square.  32-bit: 2e-5.  bfloat16: the CPU statement
+    with its activations rounded to bf16 lies 0.5 - 1 % away on average on these random models and 6 % at single
+    ill-conditioned positions (a norm over small values)."""
+    rows = row_errors(got, want)
+    if dtype == F32:
+        return rows.max() < 2e-5
+    return rows.max() < 0.12 and rows.median() < (0.025 if len(rows) >= 8 else 0.12)
+
+
+def rnd(*shape, seed=0, s=1.0):
+    return torch.randn(*shape, generator=torch.Generator().manual_seed(seed)) * s
+
+
+def dev(t, dtype=None):
+    return t.to("cuda", dtype if dtype is not None else t.dtype).contiguous()
+
+
+def close(got, want, dtype, scale=None, tol=None):
+    """bf16: one rounding of the result (2^-9 of it) plus fp32 noise; fp32: noise."""
+    got, want = got.double().cpu(), want.double()
+    scale = want.abs().max().item() if scale is None else scale
+    bound = (2.0 ** -8 * want.abs() if dtype == BF else 0.0) + (tol or 1e-5) * scale
+    bad = (got - want).abs() > bound
+    assert not bad.any(), ((got - want).abs().max().item(), int(bad.sum()), scale)
+
+
+def poisoned(model, rows):
+    cache = model.build_kv_cache(rows)
+    for c in cache:
+        for t in c.tensors.values():
+            t.fill_(float("nan"))
+    return cache
+
+
+class Tok:
+    eos_token_id = bos_token_id = None
+
+    def __init__(self, vocab):
+        self.vocab = vocab
+
+    def __len__(self):
+        return self.vocab
+
+    def get_vocab(self):
+        return {}
+
+    def encode(self, text, add_special_tokens=False):
+        return [int(t) for t in text.split()]
+
+    def decode(self, ids, skip_special_tokens=True):
+        return "".join(f"{i} " for i in ids)

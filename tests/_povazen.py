@@ -1,8 +1,7 @@
 """Small Povazen configs with random weights for the tests (every size differs between layers; none is a multiple of
 everything), and helpers to run the product and the oracle on them."""
 
-import torch
-
+from _hybrid import doubled, error, row_errors, tokens  # noqa: F401
 from oracle import povazen_ref as R
 
 
@@ -36,29 +35,10 @@ CONFIGS = {
 }
 
 
-def tokens(cfg, n, seed=0):
-    return torch.randint(0, cfg["vocab"], (n,), generator=torch.Generator().manual_seed(seed)).tolist()
-
-
 def build(cfg, weights, dtype, max_len=512):
     from ohara_amd.povazen import Povazen, PovazenConfig
 
     return Povazen(PovazenConfig.from_dict(cfg, max_len), weights, dtype=dtype)
-
-
-def doubled(weights):
-    return {k: v.double() for k, v in weights.items()}
-
-
-def row_errors(got, want):
-    """Root mean square of the logits' difference, row by row, over that of the logits."""
-    want = want.double()
-    d = got.double().cpu() - want
-    return d.pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
-
-
-def error(got, want):
-    return row_errors(got, want).max().item()
 
 
 def reference(cfg, weights, toks):
