@@ -176,6 +176,8 @@ def random_weights(cfg: dict, seed: int = 0) -> dict:
             K = m["kv_heads"]
             for nm, k in (("q", K * D), ("k", K * D), ("v", H * V)):
                 w[p + nm], w[p + nm + ".conv"] = lin(k, d), n(k, m["conv"], s=0.6)
+            for nm in ("k", "k.conv"):  # keys near the queries: a read-out of nearly nothing is all rounding after its norm
+                w[p + nm] = 0.8 * w[p + nm.replace("k", "q", 1)] + 0.6 * w[p + nm]
             w[p + "b"], w[p + "a"], w[p + "g"], w[p + "norm"] = lin(H, d), lin(H, d), lin(H * V, d), norm(V)
             w[p + "A_log"] = torch.linspace(-3.0, 1.0, H) if H > 1 else torch.zeros(1)
             w[p + "dt_bias"] = n(H) - 1.5

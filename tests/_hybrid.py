@@ -24,14 +24,12 @@ def error(got, want):
     return row_errors(got, want).max().item()
 
 
-def agrees(got, want, dtype):
-    """Logits row by row against float64, as a share of their root mean square.  32-bit: 2e-5.  bfloat16: the CPU statement
-    with its activations rounded to bf16 lies 0.5 - 1 % away on average on these random models and 6 % at single
-    ill-conditioned positions (a norm over small values)."""
-    rows = row_errors(got, want)
-    if dtype == F32:
-        return rows.max() < 2e-5
-    return rows.max() < 0.12 and rows.median() < (0.025 if len(rows) >= 8 else 0.12)
+def agrees(got, want, dtype, f32=(2e-5, 2e-5), bf16=(0.12, 0.025)):
+    """Logits row by row against float64, as a share of their root mean square: (largest, median) row.  The defaults are for
+    norms on the sublayer outputs only, where the CPU statement with its activations rounded to bf16 lies 0.5 - 1 % away on
+    average on random models and 6 % at single ill-conditioned positions (a norm over small values)."""
+    rows, (largest, median) = row_errors(got, want), f32 if dtype == F32 else bf16
+    return rows.max() < largest and (len(rows) < 8 or rows.median() < median)
 
 
 def rnd(*shape, seed=0, s=1.0):

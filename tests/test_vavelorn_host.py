@@ -1,0 +1,96 @@
+"""Vavelorn's host side without a GPU: configuration and registry, layout of the side embedding, rotary tables, argument checks of
+the entry points."""
+
+import ctypes
+import json
+
+import pytest
+import torch
+
+from _vavelorn import CONFIGS
+from ohara_amd import _lib
+from ohara_amd.checkpoint import _architecture, architecture_of, load_checkpoint
+from ohara_amd.hybrid import TokenSide, rotary_tables
+from ohara_amd.vavelorn import Vavelorn, VavelornConfig
+
+
+def test_config_from_json_and_registry(tmp_path):
+    from safetensors.torch import save_file
+
+    save_file({"embed": torch.zeros(2, 2, dtype=torch.bfloat16)}, str(tmp_path / "model.safetensors"))
+    assert architecture_of(tmp_path) is None
+    (tmp_path / "config.json").write_text(json.dumps(CONFIGS["odd"]))
+    assert architecture_of(tmp_path) == "Vavelorn"
+    cfg, state = load_checkpoint(tmp_path, max_sequence_length=77)
+    assert isinstance(cfg, VavelornConfig) and list(state) == ["embed"]
+    assert (cfg.vocab_size, cfg.hidden_size, cfg.side_dim, cfg.norm_eps, cfg.max_sequence_length) == (97, 60, 5, 2e-3, 77)
+    assert cfg.num_hidden_layers == 6 and cfg.num_attention_heads == 6
+    d, a, l = cfg.layers[:3]
+    assert (d.type, d.heads, d.kv_heads, d.dim, d.vdim, d.conv, d.ff) == ("delta", 4, 2, 24, 20, 2, 44)
+    assert (a.type, a.heads, a.kv_heads, a.dim, a.vdim, a.scale, a.rot_base, a.rot_dims, a.softcap, a.chunk, a.ff) == (
+        "attention", 6, 2, 20, 12, 0.3, 300.0, 12, 8.0, 45, 0)
+    assert (l.type, l.heads, l.dim, l.vdim, l.kv_rank, l.q_rank, l.scale, l.ff) == ("latent_attention", 3, 12, 28, 40, 20, 0.4, 100)
+    assert load_checkpoint(tmp_path)[0].max_sequence_length == VavelornConfig.max_sequence_length
+    assert _architecture("Vavelorn") == (VavelornConfig, Vavelorn)
+
+
+@pytest.mark.parametrize("change, message", [
+    (dict(type="window"), "unknown mixer"),
+    (dict(mlp={"kind": "experts", "ff": 8}), "unknown feed-forward"),
+])
+def test_config_rejects_what_it_does_not_know(change, message):
+    layer = {**CONFIGS["odd"]["layers"][0], **change}
+    with pytest.raises(ValueError, match=message):
+        VavelornConfig.from_dict({**CONFIGS["odd"], "layers": [layer]})
+
+
+def test_side_table_layout():
+    t = torch.arange(2 * 15, dtype=torch.float32).view(2, 15)
+    got = TokenSide.lay_out(t, 3, dtype=torch.float32, device="cpu")
+    assert got.shape == (2, 24)
+    for i in range(3):
+        assert torch.equal(got[:, 8 * i:8 * i + 5], t[:, 5 * i:5 * i + 5]) and not got[:, 8 * i + 5:8 * i + 8].any()
+
+
+def test_rotary_tables_are_exact_far_out():
+    cos, sin = rotary_tables(2e5, 10, 5000, "cpu")
+    assert cos.shape == (5000, 5) and cos.dtype == torch.float32 and rotary_tables(2e5, 10, 5000, "cpu")[0] is cos
+    a = 4999 * 2e5 ** (-torch.arange(0, 10, 2, dtype=torch.float64) / 10)
+    assert (cos[4999] - a.cos()).abs().max() < 1e-7 and (sin[4999] - a.sin()).abs().max() < 1e-7
+    assert rotary_tables(2.0, 0, 7, "cpu")[0].shape == (7, 0)
+
+
+def test_entry_points_check_their_arguments():
+    L, r = _lib.lib(), ctypes.byref
+    seq, late = _lib.OharaSeq(1, 1, 0, 0, None, None, None), _lib.OharaSeq(1, 1, 16, 0, None, None, None)
+    buf = ctypes.create_string_buffer(4096)
+    p = ctypes.addressof(buf)
+    E = _lib.EINVAL
+    scores = lambda **kw: r(_lib.OharaScores(*[kw.get(k, 0) for k in ("scale", "cap", "chunk", "gate_elements", "ld_k", "ld_v")], None))  # noqa: E731
+    attn = lambda sc, seq=seq, ns=1, ldo=16, gate=0, ldg=0: L.ohara_attn_scored_bf16(  # noqa: E731
+        p, p, p, 2, 1, 8, 8, 16, sc, gate, ldg, ns, 0, p, ldo, r(seq), 0)
+    assert attn(scores(chunk=-1)) == E and attn(scores(cap=-1.0)) == E and attn(scores(cap=float("nan"))) == E
+    assert attn(scores(ld_k=4)) == E and attn(scores(ld_v=12)) == E and attn(scores(), ldo=8) == E
+    assert attn(scores(gate_elements=1), gate=p, ldg=2) == E  # a gate per element has h * dv columns
+    assert attn(scores(), ns=2) == E and attn(scores(), seq=late) == E
+    # layer norms have one group
+    assert L.ohara_residual_norm_bf16(p, 8, 0, 0, 0, p, 8, p, 2, 1e-5, 16, 0, 0, 0, 0, 0, 0, r(seq), 0) == E
+    assert L.ohara_gemm_gelu_lookup_bf16(p, 8, p, 8, 8, p, 4, p, 3, 1, p, 8, 0) == E  # table rows shorter than n
+    assert L.ohara_gemm_gelu_lookup_f32(p, 8, p, 4, 6, p, 4, p, 3, 1, p, 4, 0) == E   # k % 4
+    # rotated dimensions: even, inside the head, with tables
+    rotate = lambda rot, tab=p, seq=seq: L.ohara_qkv_rotate_append_f32(p, 32, 2, 1, 8, 8, tab, tab, rot, p, p, p, 16, r(seq), 0)  # noqa: E731
+    assert rotate(3) == E and rotate(10) == E and rotate(4, 0) == E and rotate(4, p, late) == E
+    assert L.ohara_latent_front_bf16(p, 24, 16, 8, 8, p, p, 1e-5, p, p, 16, 0, r(seq), 0) == E  # the latents overlap
+    assert L.ohara_latent_front_f32(p, 24, 16, 16, 8, p, p, 1e-5, p, p, 16, 0, r(late), 0) == E
+    assert L.ohara_head_linear_bf16(p, 16, p, 2, 12, 8, 12, 1, 0, 0, p, 24, 0) == E   # n % 8
+    assert L.ohara_head_linear_f32(p, 16, p, 2, 8, 8, 9, 1, 0, 0, p, 24, 0) == E      # more entries than rows
+    assert L.ohara_attn_latent_bf16(p, p, 2, 520, 16, 1.0, 1, 0, p, r(seq), 0) == _lib.ESIZE
+    assert L.ohara_attn_latent_f32(p, p, 2, 8, 16, 1.0, 2, 0, p, r(seq), 0) == E      # no workspace
+    assert L.ohara_attn_latent_workspace_bytes(3, 2, 20, 4) == 4 * 3 * 2 * 4 * 28
+    # a delta rule without low-rank matrices takes its decays and gates from the projection's columns
+    d = _lib.OharaDelta()
+    d.heads = d.kv_heads = d.taps = 1
+    d.dim = d.vdim = 8
+    d.conv_w = d.neg_a = d.dt_bias = d.norm_w = p
+    d.off_g, d.off_a, d.off_b = 24, 32, 40  # b past the row's end
+    assert L.ohara_delta_step_f32(r(d), p, 40, p, p, p, 8, r(seq), 0) == E
