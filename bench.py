@@ -702,17 +702,36 @@ def bitnet_phase_timeline(dev, batch=1, steps=16):
     return out
 
 
+HYBRID_SIZES = {"d1024": (1024, 8, 8, 4, 128, 2816), "d2048": (2048, 8, 16, 4, 128, 5632)}  # width, layers, heads, KV heads, head size, ff
+
+
+def hybrid_llama(name, dev):
+    """A Llama of a size's width, depth, heads and feed-forward with random weights."""
+    from ohara_amd.llama import Config, Llama
+
+    d, layers, H, G, dh, ff = HYBRID_SIZES[name]
+    cfg = Config(vocab_size=32000, hidden_size=d, intermediate_size=ff, num_attention_heads=H, num_key_value_heads=G,
+                 num_hidden_layers=layers, dropout=0.0, max_sequence_length=4608)
+    g = torch.Generator(device=dev).manual_seed(0)
+    n = lambda *shape: (torch.randn(*shape, generator=g, device=dev) * 0.02).to(torch.bfloat16)  # noqa: E731
+    one = torch.ones(d, dtype=torch.bfloat16, device=dev)
+    st = {"token_emb.weight": n(32000, d), "vocab_proj.weight": n(32000, d), "norm.weight": one}
+    for i in range(layers):
+        p = f"layers.{i}."
+        st.update({p + "attn.query.weight": n(d, d), p + "attn.key.weight": n(G * dh, d), p + "attn.value.weight": n(G * dh, d),
+                   p + "attn.proj.weight": n(d, d), p + "ff.up.weight": n(ff, d), p + "ff.gate.weight": n(ff, d),
+                   p + "ff.down.weight": n(d, ff), p + "norm1.weight": one, p + "norm2.weight": one})
+    return Llama(cfg, st, device=dev)
+
+
 def povazen_size(name):
-    """(config dict of the hybrid model, Config keywords of a Llama of the same width, depth, heads and feed-forward)."""
-    d, n, H, G, dh, ff = {"d1024": (1024, 8, 8, 4, 128, 2816), "d2048": (2048, 8, 16, 4, 128, 5632)}[name]
+    """The config dict of the hybrid model."""
+    d, n, H, G, dh, ff = HYBRID_SIZES[name]
     mlp = {"kind": "dense", "ff": ff}
     delta = {"type": "channel_delta", "mixer": {"heads": H, "kv_heads": H, "dim": dh, "vdim": dh, "conv": 4}, "mlp": mlp}
     att = {"type": "attention", "mixer": {"heads": H, "kv_heads": G, "dim": dh, "vdim": dh, "scale": dh ** -0.5}, "mlp": mlp}
-    cfg = {"width": d, "vocab": 32000, "canon": {"taps": 4}, "norm": {"eps": 1e-6, "groups": 1}, "logit_softcap": 30.0,
-           "layers": ([delta] * 3 + [att]) * (n // 4)}
-    llama = dict(vocab_size=32000, hidden_size=d, intermediate_size=ff, num_attention_heads=H, num_key_value_heads=G,
-                 num_hidden_layers=n, dropout=0.0)
-    return cfg, llama
+    return {"width": d, "vocab": 32000, "canon": {"taps": 4}, "norm": {"eps": 1e-6, "groups": 1}, "logit_softcap": 30.0,
+            "layers": ([delta] * 3 + [att]) * (n // 4)}
 
 
 def povazen_state(cfg, dev, rank=128, seed=5):
@@ -872,39 +891,207 @@ def bench_povazen_kernels(cfg, dev):
     return rows
 
 
+def bench_models(name, models, dev):
+    """Prefill and decode figures of (label, constructor) pairs, one model in memory at a time."""
+    out = {}
+    for label, make in models:
+        model = make()
+        out[label] = {"parameters": sum(t.numel() for t in model.parameters()),
+                      "prefill": {f"{B}x{S}": _time_model_prefill(model, B, S, dev) for B, S in ((1, 512), (1, 4096), (8, 1024))},
+                      "decode": {f"batch {B}, context {L}": _time_model_decode(model, B, L)
+                                 for B, L in ((1, 1024), (1, 4096), (8, 4096), (32, 2048))}}
+        del model
+        torch.cuda.empty_cache()
+    return out
+
+
 def bench_povazen(dev, sizes=("d1024", "d2048"), kernels=True):
     """Prefill and decode of the hybrid model (three delta-rule layers to one attention layer, SwiGLU everywhere, random
     weights) beside Llama at the same width, depth, heads and feed-forward."""
-    from ohara_amd.llama import Config, Llama
     from ohara_amd.povazen import Povazen, PovazenConfig
 
     out = {}
     for name in sizes:
-        cfg, kw = povazen_size(name)
-        res = {"layers": len(cfg["layers"]), "width": cfg["width"]}
-        lcfg = Config(**kw, max_sequence_length=4608)
-        g = torch.Generator(device=dev).manual_seed(0)
-        d, f, kvw = lcfg.hidden_size, lcfg.intermediate_size, lcfg.num_key_value_heads * (lcfg.hidden_size // lcfg.num_attention_heads)
-        n = lambda *shape: (torch.randn(*shape, generator=g, device=dev) * 0.02).to(torch.bfloat16)  # noqa: E731
-        one = torch.ones(d, dtype=torch.bfloat16, device=dev)
-        st = {"token_emb.weight": n(32000, d), "vocab_proj.weight": n(32000, d), "norm.weight": one}
-        for i in range(lcfg.num_hidden_layers):
-            p = f"layers.{i}."
-            st.update({p + "attn.query.weight": n(d, d), p + "attn.key.weight": n(kvw, d), p + "attn.value.weight": n(kvw, d),
-                       p + "attn.proj.weight": n(d, d), p + "ff.up.weight": n(f, d), p + "ff.gate.weight": n(f, d),
-                       p + "ff.down.weight": n(d, f), p + "norm1.weight": one, p + "norm2.weight": one})
-        for label, make in (("povazen", lambda: Povazen(PovazenConfig.from_dict(cfg, 4608), povazen_state(cfg, dev), device=dev)),
-                            ("llama", lambda: Llama(lcfg, st, device=dev))):
-            model = make()
-            res[label] = {"parameters": sum(t.numel() for t in model.parameters()),
-                          "prefill": {f"{B}x{S}": _time_model_prefill(model, B, S, dev) for B, S in ((1, 512), (1, 4096), (8, 1024))},
-                          "decode": {f"batch {B}, context {L}": _time_model_decode(model, B, L)
-                                     for B, L in ((1, 1024), (1, 4096), (8, 4096), (32, 2048))}}
-            del model
-            torch.cuda.empty_cache()
+        cfg = povazen_size(name)
+        out[name] = {"layers": len(cfg["layers"]), "width": cfg["width"], **bench_models(name, (
+            ("povazen", lambda: Povazen(PovazenConfig.from_dict(cfg, 4608), povazen_state(cfg, dev), device=dev)),
+            ("llama", lambda: hybrid_llama(name, dev))), dev)}
         if kernels:
-            res["kernels"] = bench_povazen_kernels(cfg, dev)
-        out[name] = res
+            out[name]["kernels"] = bench_povazen_kernels(cfg, dev)
+    return out
+
+
+def vavelorn_size(name):
+    """The config dict: two delta-rule layers to one of latent and one of chunked rotary attention."""
+    d, n, H, G, dh, ff = HYBRID_SIZES[name]
+    layer = lambda kind, **m: {"type": kind, "mixer": {"heads": H, "dim": dh, "vdim": dh, **m}, "mlp": {"kind": "dense", "ff": ff}}  # noqa: E731
+    delta = layer("delta", kv_heads=H, conv=4)
+    latent = layer("latent_attention", kv_rank=512, q_rank=d // 2, scale=dh ** -0.5)
+    att = layer("attention", kv_heads=G, scale=dh ** -0.5, rot={"base": 1e4, "dims": dh // 2}, softcap=30.0, mask={"size": 4096})
+    return {"width": d, "vocab": 32000, "token_side": {"dim": 64}, "norm": {"eps": 1e-5}, "layers": [delta, latent, delta, att] * (n // 4)}
+
+
+def vavelorn_state(cfg, dev, seed=5):
+    """Random weights: matrices N(0, 1/columns), unit norms, decays of some tens of tokens."""
+    g = torch.Generator(device=dev).manual_seed(seed)
+    n = lambda *shape, s=1.0: (torch.randn(*shape, generator=g, device=dev) * s).to(torch.bfloat16)  # noqa: E731
+    lin = lambda o, i: n(o, i, s=i ** -0.5)  # noqa: E731
+    one = lambda k: torch.ones(k, device=dev, dtype=torch.bfloat16)  # noqa: E731
+    d, side = cfg["width"], cfg["token_side"]["dim"]
+    st = {"embed": n(cfg["vocab"], d), "side.embed": n(cfg["vocab"], side * len(cfg["layers"])), "head": lin(cfg["vocab"], d),
+          "final.norm": one(d)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, ff = f"l{i}.", layer["mixer"], layer["mlp"]["ff"]
+        H, K, D, V = m["heads"], m.get("kv_heads"), m["dim"], m["vdim"]
+        st.update({p + f"norm{k}": one(d) for k in ("1", "1b", "2", "2b")})
+        st.update({p + "mlp.gate": lin(ff, d), p + "mlp.up": lin(ff, d), p + "mlp.down": lin(d, ff), p + "side.gate": lin(side, d),
+                   p + "side.proj": lin(d, side), p + "side.norm": one(d)})
+        p += "mix."
+        st[p + "o"] = lin(d, H * V)
+        if layer["type"] == "latent_attention":
+            r, rq = m["kv_rank"], m["q_rank"]
+            st.update({p + "dq": lin(rq, d), p + "dq.norm": one(rq), p + "uq": lin(H * D, rq), p + "dkv": lin(r, d), p + "dkv.norm": one(r),
+                       p + "uk": lin(H * D, r), p + "uv": lin(H * V, r), p + "g": lin(H * V, d)})
+            continue
+        vrows = K * V if layer["type"] == "attention" else H * V
+        st.update({p + "q": lin(H * D if layer["type"] == "attention" else K * D, d), p + "k": lin(K * D, d), p + "v": lin(vrows, d)})
+        if layer["type"] == "delta":
+            st.update({p + "b": lin(H, d), p + "a": lin(H, d), p + "g": lin(H * V, d), p + "norm": one(V), p + "dt_bias": n(H) - 3.0,
+                       p + "A_log": torch.zeros(H, device=dev, dtype=torch.bfloat16)})
+            for c, k in (("q", K * D), ("k", K * D), ("v", H * V)):
+                st[p + c + ".conv"] = n(k, m["conv"], s=0.5)
+    return st
+
+
+def _sole_layers(build, config_of, state, cfg, kinds, dev):
+    """The mixers of the first layer of each kind, from a model of just those layers."""
+    at = [next(i for i, layer in enumerate(cfg["layers"]) if layer["type"] == kind) for kind in kinds]
+    names = {f"l{i}.": f"l{k}." for k, i in enumerate(at)}
+    if "side.embed" in state:
+        side = cfg["token_side"]["dim"]
+        state = {**state, "side.embed": state["side.embed"][:, :side * len(at)]}
+    keep = {names.get(k.split(".")[0] + ".", "") + (k.split(".", 1)[1] if k.split(".")[0] + "." in names else k): v for k, v in state.items()
+            if k.split(".")[0] + "." in names or not k.startswith("l")}
+    return build(config_of({**cfg, "layers": [cfg["layers"][i] for i in at]}, 4096), keep, device=dev)
+
+
+def bench_vavelorn_kernels(name, dev):
+    """The design's own kernels at one layer's sizes, each beside the like kernel of Llama or Povazen."""
+    from ohara_amd import ops
+    from ohara_amd.hybrid import distance_slopes
+    from ohara_amd.povazen import Povazen, PovazenConfig
+    from ohara_amd.vavelorn import Vavelorn, VavelornConfig
+
+    bf, cfg, pcfg = torch.bfloat16, vavelorn_size(name), povazen_size(name)
+    model = _sole_layers(Vavelorn, VavelornConfig.from_dict, vavelorn_state(cfg, dev), cfg, ("delta", "latent_attention", "attention"), dev)
+    pov = _sole_layers(Povazen, PovazenConfig.from_dict, povazen_state(pcfg, dev), pcfg, ("channel_delta", "attention"), dev)
+    delta, lat, att = (b["mixer"] for b in model.layers)
+    pdelta, patt = (b["mixer"] for b in pov.layers)
+    H, G, D, V, d, R = att.heads, att.kv_heads, att.dim, att.vdim, cfg["width"], lat.rank
+    slopes = distance_slopes(H).to(dev)
+    rnd = lambda *shape, dt=bf: torch.randn(*shape, device=dev).to(dt)  # noqa: E731
+    rows = []
+
+    def timed(fn, n=8):  # n calls per graph: what a single-launch graph costs to start would swamp the small kernels
+        return graph_time(lambda: [fn() for _ in range(n)], iters=20) / n
+
+    for B, L in ((1, 4096), (8, 4096), (32, 2048)):
+        seq = ops.Seq(B, 1, L - 1)
+        q, k, v = rnd(B, H * D), rnd(B, L, G, D), rnd(B, L, G, V)
+        ns, ws = att._split(B, L)
+        t_att = timed(lambda: ops.attn_scored(q, k, v, H, G, D, V, L, 0.1, seq, cap=30.0, chunk=4096, n_split=ns, workspace=ws))
+        n2 = max(1, min(1024 // (B * G), L // 128, 64))
+        ws2 = ops.attn_workspace(B, H, G, D, n2, dev)
+        t_llama = timed(lambda: ops.attn_decode(q, k, v, H, G, D, L, n2, ws2))
+        by = 2.0 * G * (D + V) * B * L
+        c, ql = rnd(B, L, R), rnd(B, H * R)
+        nl, wl = lat._split(B, L)
+        t_lat = timed(lambda: ops.attn_latent(ql, c, H, R, 0.1, seq, nl, wl))
+        rows.append({"kernel": "decode attention", "batch": B, "context": L, "attn_bias_kernel (cap, chunk)": _hbm(t_att, by),
+                     "llama attn_decode_kernel": _hbm(t_llama, by), "attn_latent_kernel + merge": _hbm(t_lat, 2.0 * R * B * L)})
+    for B, S in ((1, 4096), (8, 1024)):
+        seq = ops.Seq(B, S, 0)
+        q, k, v = rnd(B * S, H * D), rnd(B, S, G, D), rnd(B, S, G, V)
+        fl = 2.0 * B * H * (D + V) * S * (S + 1) / 2
+        gate, ge, kv = rnd(B * S, H), rnd(B * S, H * V), rnd(B * S, H * (D + V))
+        rows.append({
+            "kernel": "prompt attention", "batch": B, "tokens": S,
+            "attn_bias_prefill_kernel (cap, chunk)": _flops(timed(lambda: ops.attn_scored(
+                q, k, v, H, G, D, V, S, 0.1, seq, cap=30.0, chunk=4096)), fl, MFMA_BF16_PEAK_TFLOPS),
+            "latent: attn_bias_prefill_kernel (expanded, gated)": _flops(timed(lambda: ops.attn_scored(
+                q, kv, kv[:, H * D:], H, H, D, V, S, 0.1, seq, gate=ge, gate_elements=True, ld_k=H * (D + V), ld_v=H * (D + V))), fl,
+                MFMA_BF16_PEAK_TFLOPS),
+            "povazen attn_bias_prefill_kernel": _flops(timed(lambda: ops.attn_bias(q, k, v, H, G, D, V, 0.1, slopes, gate, seq)), fl,
+                                                       MFMA_BF16_PEAK_TFLOPS),
+            "llama attn_prefill_kernel": _flops(timed(lambda: ops.attn_prefill(q, k, v, H, G, D, 0, S)), fl, MFMA_BF16_PEAK_TFLOPS)})
+    side, norm = model.layers[0]["side"], model.layers[0]["norm1b"]
+    plain = ops.pack_linear(rnd(side.gate.n, d))
+    for B in (1, 8, 32):
+        seq, ids = ops.Seq(B, 1, 100), torch.randint(0, 32000, (B,), device=dev)
+        row = {"kernel": "one token", "batch": B}
+        for label, mix, more in (("delta_step_kernel", delta, 2.0 * B * H * V), ("povazen delta_step_kernel", pdelta, 2.0 * (pdelta.a2.numel() + pdelta.g2.numel()))):
+            st, p = mix.state(B, 4096), rnd(B, mix.proj.n)
+            row[label] = _hbm(timed(lambda: ops.delta_step(mix._c, p, st["delta"], st["ring"], seq)), 8.0 * B * H * D * V + more)
+        x, xl, gate = rnd(B, H * D), rnd(B, H * R), rnd(B, H * V)
+        by = 2.0 * H * R * D
+        row["head_linear_kernel (keys)"] = _hbm(timed(lambda: ops.head_linear(x, lat.k_absorb, R)), by)
+        row["head_linear_kernel (values, gate)"] = _hbm(timed(lambda: ops.head_linear(xl, lat.v_absorb, V, gate)), by)
+        w = ops.pack_linear(rnd(R * 2, H * D // 2))
+        xs = rnd(B, H * D // 2)
+        row["llama gemm_skinny, as many weights"] = _hbm(timed(lambda: ops.gemm_skinny(xs, w)), by)
+        hx = rnd(B, d)
+        row["gemm_gelu_lookup"] = _hbm(timed(lambda: ops.gemm_gelu_lookup(hx, side.gate.w, side.table, 0, ids)), 2.0 * side.gate.n * d)
+        row["llama gemm_skinny, same weights"] = _hbm(timed(lambda: ops.gemm_skinny(hx, plain)), 2.0 * side.gate.n * d)
+        xf, y = rnd(B, d, dt=torch.float32), rnd(B, d)
+        row["residual_norm_kernel (two layer norms)"] = _hbm(timed(lambda: ops.residual_norm(
+            xf, seq, bf, **{**norm.of(y), **norm.out()})), B * d * 12.0)
+        row["povazen residual_norm_kernel (two norms)"] = _hbm(timed(lambda: ops.residual_norm(
+            xf, seq, bf, y=y, norm_w=norm.w, groups=1, eps=1e-5, mode="norm", norm2_w=norm.w)), B * d * 12.0)
+        rows.append(row)
+    for B, S in ((1, 4096), (8, 1024)):
+        seq, n, ids = ops.Seq(B, S, 0), B * S, torch.randint(0, 32000, (B * S,), device=dev)
+        row = {"kernel": "prompt, other kernels", "batch": B, "tokens": S}
+        for label, mix in (("delta_prefill (3 kernels)", delta), ("povazen delta_prefill (3 kernels)", pdelta)):
+            st, p = mix.state(B, 4096), rnd(n, mix.proj.n)
+            za, zg = (None, None) if mix is delta else (rnd(n, H * D) - 3.0, rnd(n, H * V))
+            ws = mix._workspace(B, S)
+            row[label] = _flops(timed(lambda: ops.delta_prefill(mix._c, p, za, zg, st["delta"], st["ring"], ws, seq)),
+                                7.0 * n * H * D * V, FP32_MFMA_PEAK_TFLOPS)
+        kc, vc, big = rnd(B, S, G, D), rnd(B, S, G, V), rnd(n, max(att.proj.n, patt.proj.n, lat.proj.n))
+        cos, sin = (torch.ones(S, D // 4, device=dev) for _ in range(2))
+        by = 4.0 * n * (H * D + G * (D + V))
+        row["qkv_rotate_append_kernel"] = _hbm(timed(lambda: ops.qkv_rotate_append(big, H, G, D, V, cos, sin, D // 2, kc, vc, seq)), by)
+        row["povazen qkv_norm_append_kernel"] = _hbm(timed(lambda: ops.qkv_norm_append(
+            big, H, G, D, V, patt.q_norm, patt.k_norm, 1e-6, kc, vc, seq)), by)
+        cl = rnd(B, S, R)
+        row["latent_front_kernel"] = _hbm(timed(lambda: ops.latent_front(
+            big, lat.q_rank, lat.off_c, R, lat.q_norm, lat.kv_norm, 1e-5, cl, seq, True)), 2.0 * n * (2 * lat.q_rank + 3 * R))
+        hx = rnd(n, d)
+        fl = 2.0 * n * side.gate.n * d
+        row["gemm_gelu_lookup"] = _flops(timed(lambda: ops.gemm_gelu_lookup(hx, side.gate.w, side.table, 0, ids)), fl, MFMA_BF16_PEAK_TFLOPS)
+        row["llama gemm, same weights"] = _flops(timed(lambda: ops.gemm_skinny(hx, plain)), fl, MFMA_BF16_PEAK_TFLOPS)
+        xf, y = rnd(n, d, dt=torch.float32), rnd(n, d)
+        row["residual_norm_kernel (two layer norms)"] = _hbm(timed(lambda: ops.residual_norm(
+            xf, seq, bf, **{**norm.of(y), **norm.out()})), n * d * 12.0)
+        row["povazen residual_norm_kernel (two norms)"] = _hbm(timed(lambda: ops.residual_norm(
+            xf, seq, bf, y=y, norm_w=norm.w, groups=1, eps=1e-5, mode="norm", norm2_w=norm.w)), n * d * 12.0)
+        rows.append(row)
+    return rows
+
+
+def bench_vavelorn(dev, sizes=("d1024", "d2048")):
+    """Prefill and decode of Vavelorn with random weights beside Povazen and Llama at the same width, depth, heads and feed-forward."""
+    from ohara_amd.povazen import Povazen, PovazenConfig
+    from ohara_amd.vavelorn import Vavelorn, VavelornConfig
+
+    out = {}
+    for name in sizes:
+        cfg, pcfg = vavelorn_size(name), povazen_size(name)
+        out[name] = {"layers": len(cfg["layers"]), "width": cfg["width"], **bench_models(name, (
+            ("vavelorn", lambda: Vavelorn(VavelornConfig.from_dict(cfg, 4608), vavelorn_state(cfg, dev), device=dev)),
+            ("povazen", lambda: Povazen(PovazenConfig.from_dict(pcfg, 4608), povazen_state(pcfg, dev), device=dev)),
+            ("llama", lambda: hybrid_llama(name, dev))), dev)}
+        out[name]["kernels"] = bench_vavelorn_kernels(name, dev)
     return out
 
 
@@ -939,6 +1126,8 @@ def main():
                     help="run the GQA decode-attention figures (bf16 and int8 cache) alone and exit")
     ap.add_argument("--povazen-only", type=str, nargs="?", const="d1024,d2048", default="", metavar="SIZES",
                     help="run the Povazen prefill, decode and kernel figures beside Llama at equal sizes alone and exit")
+    ap.add_argument("--vavelorn-only", type=str, nargs="?", const="d1024,d2048", default="", metavar="SIZES",
+                    help="run the Vavelorn prefill, decode and kernel figures beside Povazen and Llama at equal sizes alone and exit")
     ap.add_argument("--phi-decode-only", type=int, default=0, metavar="B",
                     help="run 12 eager Phi-2 decode steps of B sequences at context 1024 and exit (profiling workload)")
     args = ap.parse_args()
@@ -962,6 +1151,9 @@ def main():
         del src, dst
     if args.povazen_only:
         print(json.dumps(bench_povazen(dev, tuple(args.povazen_only.split(","))), indent=1))
+        return
+    if args.vavelorn_only:
+        print(json.dumps(bench_vavelorn(dev, tuple(args.vavelorn_only.split(","))), indent=1))
         return
     if args.phi_decode_only:
         print(json.dumps(phi_decode_only(dev, args.phi_decode_only)))
