@@ -1024,7 +1024,7 @@ def bench_vavelorn_kernels(name, dev):
             "povazen attn_bias_prefill_kernel": _flops(timed(lambda: ops.attn_bias(q, k, v, H, G, D, V, 0.1, slopes, gate, seq)), fl,
                                                        MFMA_BF16_PEAK_TFLOPS),
             "llama attn_prefill_kernel": _flops(timed(lambda: ops.attn_prefill(q, k, v, H, G, D, 0, S)), fl, MFMA_BF16_PEAK_TFLOPS)})
-    side, norm = model.layers[0]["side"], model.layers[0]["norm1b"]
+    side, norm, after = model.layers[0]["side"], model.layers[0]["norm2b"], model.layers[1]["norm1"]
     plain = ops.pack_linear(rnd(side.gate.n, d))
     for B in (1, 8, 32):
         seq, ids = ops.Seq(B, 1, 100), torch.randint(0, 32000, (B,), device=dev)
@@ -1047,6 +1047,13 @@ def bench_vavelorn_kernels(name, dev):
             xf, seq, bf, **{**norm.of(y), **norm.out()})), B * d * 12.0)
         row["povazen residual_norm_kernel (two norms)"] = _hbm(timed(lambda: ops.residual_norm(
             xf, seq, bf, y=y, norm_w=norm.w, groups=1, eps=1e-5, mode="norm", norm2_w=norm.w)), B * d * 12.0)
+        row["token_side_kernel (update, side embedding, norm)"] = _hbm(timed(lambda: ops.token_side(
+            xf, y, norm.w, side.gate.w, side.proj.w, side.table, side.column, ids, side.norm.w, norm.eps, after.w, center_y=True,
+            center_out=True)),
+                                                                      B * d * 12.0 + 4.0 * side.gate.n * d)
+        row["the same unfused (4 launches)"] = _hbm(timed(lambda: (
+            ops.residual_norm(xf, seq, bf, **{**side.norm.of(side(ops.residual_norm(xf, seq, bf, **{**norm.of(y), "mode": "copy"}), ids)),
+                                              **after.out()}))), B * d * 12.0 + 4.0 * side.gate.n * d)
         rows.append(row)
     for B, S in ((1, 4096), (8, 1024)):
         seq, n, ids = ops.Seq(B, S, 0), B * S, torch.randint(0, 32000, (B * S,), device=dev)
@@ -1075,6 +1082,13 @@ def bench_vavelorn_kernels(name, dev):
             xf, seq, bf, **{**norm.of(y), **norm.out()})), n * d * 12.0)
         row["povazen residual_norm_kernel (two norms)"] = _hbm(timed(lambda: ops.residual_norm(
             xf, seq, bf, y=y, norm_w=norm.w, groups=1, eps=1e-5, mode="norm", norm2_w=norm.w)), n * d * 12.0)
+        row["token_side_kernel (update, side embedding, norm)"] = _hbm(timed(lambda: ops.token_side(
+            xf, y, norm.w, side.gate.w, side.proj.w, side.table, side.column, ids, side.norm.w, norm.eps, after.w, center_y=True,
+            center_out=True)),
+                                                                      n * d * 12.0 + 4.0 * side.gate.n * d)
+        row["the same unfused (4 launches)"] = _hbm(timed(lambda: (
+            ops.residual_norm(xf, seq, bf, **{**side.norm.of(side(ops.residual_norm(xf, seq, bf, **{**norm.of(y), "mode": "copy"}), ids)),
+                                              **after.out()}))), n * d * 12.0 + 4.0 * side.gate.n * d)
         rows.append(row)
     return rows
 

@@ -684,6 +684,16 @@ int ohara_gemm_gelu_lookup_bf16(const uint16_t* x, int ldx, const uint16_t* wp, 
 int ohara_gemm_gelu_lookup_f32(const float* x, int ldx, const float* w, int n, int k, const float* table, int ldt,
                                const int64_t* ids, int vocab, int rows, float* out, int ldo, void* stream);
 
+/* A layer's side embedding with the residual updates on either side, one launch (every norm over the whole row with eps):
+ *   x += norm_w * norm(y);  z = gelu_tanh(Wg x) * table[ids[row] * ldt + i];  x += side_w * rms(Wp z);  out = out_w * norm(x)
+ * x: (rows, d) fp32, updated in place; y: rows of ldy; gate, proj: packed Wg (n, d rounded up to 8) and Wp (d rounded up to 8, n);
+ * center_y / center_out: that norm is a layer norm without bias.  d, ldy and ldo multiples of 4, n <= 256.  x, z and Wp z are
+ * rounded to bf16 for the products.  rows_per_group: rows of a workgroup (a power of two up to 16), rows_per_group * d <= 16384. */
+int ohara_token_side_bf16(float* x, int d, const uint16_t* y, int ldy, const float* norm_w, int center_y, const uint16_t* gate,
+                          const uint16_t* proj, int n, const uint16_t* table, int ldt, const int64_t* ids, int vocab,
+                          const float* side_w, float eps, const float* out_w, int center_out, int rows, int rows_per_group,
+                          uint16_t* out, int ldo, void* stream);
+
 /* Attention front end off one projection p with row layout [q (h*dh); k (h_kv*dh); v (h_kv*dv); ...]:
  * q and k are each divided by the root mean square of ALL their elements of the row and multiplied by
  * qn / kn; every value head is divided by its own root mean square.  q -> q_out (rows, h, dhp), keys and

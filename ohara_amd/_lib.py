@@ -167,6 +167,7 @@ _PROTOS = {
     }.items()},
     "ohara_gemm_f32": (_i, [_p, _i, _p, _p, _p, _f, _i, _i, _i, _p, _i, _p]),
     "ohara_gemm_softcap_bf16": (_i, [_p, _i, _p, _i, _i, _f, _i, _p, _i, _p]),
+    "ohara_token_side_bf16": (_i, [_p, _i, _p, _i, _p, _i, _p, _p, _i, _p, _i, _p, _i, _p, _f, _p, _i, _i, _i, _p, _i, _p]),
     "ohara_attn_bias_workspace_bytes": (_i64, [_i, _i, _i, _i]),
     "ohara_attn_latent_workspace_bytes": (_i64, [_i, _i, _i, _i]),
     "ohara_delta_workspace_bytes": (_i64, [_i, _i, _i, _i, _i]),

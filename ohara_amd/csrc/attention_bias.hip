@@ -195,7 +195,11 @@ struct AttnBiasArgs {
 };
 
 // tanh with an absolute error of about an ulp of 1: what a capped score of the bf16 kernels needs
-__device__ __forceinline__ float tanh_x(float v) { return 1.0f - 2.0f * __frcp_rn(1.0f + __expf(2.0f * v)); }
+// (hardware exponential and reciprocal: the correctly rounded reciprocal is several times the instructions)
+__device__ __forceinline__ float tanh_x(float v) {
+  return __builtin_fmaf(-2.0f, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.0f * OHARA_LOG2E * v)), 1.0f);
+}
+
 template <typename T>
 __device__ __forceinline__ float gate_of(const AttnBiasArgs<T>& a, size_t row, int h, int c) {
   return a.gate ? sigmoid_x(ldv(a.gate + row * a.ldg + (a.gate_elem ? h * a.V + c : h))) : 1.0f;

@@ -355,6 +355,8 @@ class TokenSide:
     """What a layer adds to the residual for its token: proj(gelu_tanh(gate x) * e) with e the row's ``dim`` entries of an embedding
     table from ``column`` on, over its own root mean square times norm_w (``norm``)."""
 
+    ONE_CU = 1 << 16  # elements of either matrix up to which a single workgroup reads them as fast as several launches do
+
     def __init__(self, gate, proj, norm_w, table, column: int, *, eps: float, dtype=BF16, device="cuda"):
         self.gate, self.proj = Linear(gate, dtype=dtype, device=device), Linear(proj, dtype=dtype, device=device)
         self.norm = GroupNorm(norm_w, 1, eps, device)
@@ -369,6 +371,19 @@ class TokenSide:
 
     def __call__(self, x, ids):
         return self.proj(ops.gemm_gelu_lookup(x, self.gate.w, self.table, self.column, ids))
+
+    def update(self, x, seq: ops.Seq, ids, y, norm, after):
+        """The residual x plus norm(y), plus what the side embedding makes of that; returns ``after`` of it (``norm``, ``after``:
+        norms over the whole row with this one's eps).  One launch where the sizes allow it; a few rows of a wide model take
+        four, whose weights more than one CU reads."""
+        rows, d = x.shape
+        same = norm.groups == after.groups == 1 and norm.eps == after.eps == self.norm.eps
+        fits = d % 4 == 0 and d <= ops.TOKEN_SIDE_ELEMENTS and self.gate.n <= 256
+        if self.gate.dtype == BF16 and same and fits and (rows > 64 or self.gate.n * d <= self.ONE_CU):
+            return ops.token_side(x, y, norm.w, self.gate.w, self.proj.w, self.table, self.column, ids, self.norm.w, norm.eps, after.w,
+                                  center_y=isinstance(norm, LayerNorm), center_out=isinstance(after, LayerNorm))
+        h = ops.residual_norm(x, seq, self.gate.dtype, **{**norm.of(y), "mode": "copy"})
+        return ops.residual_norm(x, seq, self.gate.dtype, **{**self.norm.of(self(h, ids)), **after.out()})
 
     def tensors(self):
         yield from self.gate.tensors()

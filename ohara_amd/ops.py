@@ -721,6 +721,32 @@ def gemm_gelu_lookup(x, w, table, column: int, ids, out=None):
     return out
 
 
+TOKEN_SIDE_ELEMENTS = 16384  # of the residual that a workgroup of token_side holds
+
+
+def token_side(x, y, norm_w, gate: PackedLinear, proj: PackedLinear, table, column: int, ids, side_w, eps: float, out_w, *,
+               center_y=False, center_out=False, rows_per_group: int | None = None):
+    """x (rows, d) fp32 += norm_w * norm(y); x += side_w * rms(proj(gelu_tanh(gate x) * table[ids, column: column + n])); returns
+    out_w * norm(x) as (rows, round8(d)) bf16.  One launch; d a multiple of 4."""
+    _need(x, F32, "x")
+    _need(y, BF16, "y")
+    rows, d = x.shape
+    if gate.k != round8(d) or proj.n != round8(d) or proj.k != gate.n or y.shape[0] != rows or ids.numel() != rows or ids.dtype != torch.int64:
+        raise ValueError("token_side: operands do not fit the residual")
+    if table.dtype != BF16 or not table.is_contiguous() or column < 0 or column + gate.n > table.shape[1]:
+        raise ValueError("the table has no such columns")
+    if rows_per_group is None:  # four, and more where that fills the 256 CUs more than once
+        rows_per_group = 1
+        while rows_per_group < 16 and 2 * rows_per_group * d <= TOKEN_SIDE_ELEMENTS and (rows_per_group < 4 or rows > 256 * rows_per_group):
+            rows_per_group *= 2
+    out = torch.empty(rows, round8(d), dtype=BF16, device=x.device)
+    check(lib().ohara_token_side_bf16(
+        _ptr(x), d, _ptr(y), y.stride(0), _ptr(norm_w), int(center_y), _ptr(gate.data), _ptr(proj.data), gate.n,
+        _ptr(table) + column * table.element_size(), table.stride(0), _ptr(ids), table.shape[0], _ptr(side_w), eps, _ptr(out_w),
+        int(center_out), rows, rows_per_group, _ptr(out), out.stride(0), _stream()), "token_side")
+    return out
+
+
 def qkv_rotate_append(p, h, h_kv, dh, dv, cos, sin, rot, kcache, vcache, seq: Seq):
     """p rows [q; k; v; ...] -> q (rows, h * round8(dh)); keys and values into the caches; the first ``rot`` dimensions of q and
     k heads rotated in neighbouring pairs by the tables cos, sin (positions, rot / 2) fp32."""

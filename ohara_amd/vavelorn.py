@@ -7,7 +7,7 @@ its config lists them, with layer norms before and after every sublayer and an e
 The call surface is the other models' (``ohara_amd.hybrid_model``).  ``dtype`` float32 serves the model in 32-bit throughout.
 
 Residual update and the norm of the next sublayer are one launch.  Decode steps run 3 launches per recurrent mixer, 4 per rotary
-attention and 7 or 8 per latent attention, 3 per feed-forward and 4 per side embedding, all capturable.
+attention and 7 or 8 per latent attention, 3 per feed-forward and 1 (wide models: 4) per side embedding, all capturable.
 """
 
 from __future__ import annotations
@@ -158,11 +158,10 @@ class Vavelorn(HybridDecoder):
         nexts = [block["norm1"] for block in self.layers[1:]] + [self.final_norm]
         h = update(dict(ids=ids, table=self.embed), self.layers[0]["norm1"].out())
         for block, state, after in zip(self.layers, kv_cache, nexts):
-            source = block["norm1b"].of(block["mixer"](h, state, seq))
+            y, norm = block["mixer"](h, state, seq), block["norm1b"]
             if block["mlp"] is not None:
-                source = block["norm2b"].of(block["mlp"](update(source, block["norm2"].out())))
-            side = block["side"]
-            h = update(side.norm.of(side(update(source, dict(mode="copy")), ids)), after.out())
+                y, norm = block["mlp"](update(norm.of(y), block["norm2"].out())), block["norm2b"]
+            h = block["side"].update(x, seq, ids, y, norm, after)
             if self.trace is not None:
                 self.trace.append(x.clone())
         if last_only and seq.seq_len > 1:

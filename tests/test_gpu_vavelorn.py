@@ -439,6 +439,50 @@ def test_token_side(cuda, dtype, dim):
             assert diff < (1e-5 if dtype == F32 else 2e-2), (rows, i, diff)
 
 
+@pytest.mark.parametrize("d, dim", [(36, 5), (60, 16), (4, 1), (1000, 40), (1024, 64), (2048, 100), (5000, 256), (35, 7)])
+def test_token_side_and_updates_in_one_launch(cuda, d, dim):
+    """Against float64 with the launch's roundings (residual, gated embedding and projection to bf16), and against the
+    separate launches of the 32-bit build."""
+    from ohara_amd import ops
+    from ohara_amd.hybrid import GroupNorm, LayerNorm, TokenSide
+
+    vocab, layers, eps = 13, 2, 1e-4
+    table, gate, proj = rnd(vocab, layers * dim).to(BF), rnd(dim, d, seed=1, s=2 / d ** 0.5).to(BF), rnd(d, dim, seed=2).to(BF)
+    w1, w2, w3 = (rnd(d, seed=s) for s in (3, 4, 5))
+    rounded = lambda t: t.to(BF).double()  # noqa: E731
+    for rows in (1, 7, 70):
+        x, y = rnd(rows, d, seed=rows), (rnd(rows, ops.round8(d), seed=rows + 1) + 0.5).to(BF)
+        y[:, d:] = 0
+        ids = torch.randint(0, vocab, (rows,), generator=torch.Generator().manual_seed(rows))
+        yd, e = y[:, :d].double(), table[ids, dim:].double()
+        for center in (True, False):
+            kind = (lambda w: LayerNorm(w, eps)) if center else (lambda w: GroupNorm(w, 1, eps))
+            norm = (lambda t, w: R.layer_norm(t, w.double(), eps)) if center else (lambda t, w: R.rms(t, eps) * w.double())  # noqa: E731
+            mid = x.double() + norm(yd, w1)
+            z = rounded(R.gelu_tanh(rounded(mid) @ gate.double().t()) * e)
+            want = mid + R.rms(rounded(z @ proj.double().t()), eps) * w2.double()
+            for groups in (None, 1, 2, 4, 8, 16):
+                if groups and (groups * d > ops.TOKEN_SIDE_ELEMENTS or d % 4):
+                    continue
+                side = TokenSide(gate, proj, w2, TokenSide.lay_out(table, layers), ops.round8(dim), eps=eps)
+                xd = dev(x)
+                if groups is None:
+                    out = side.update(xd, ops.Seq(rows, 1), ids.cuda(), dev(y), kind(w1), kind(w3))
+                else:
+                    out = ops.token_side(xd, dev(y), dev(w1), side.gate.w, side.proj.w, side.table, side.column, ids.cuda(), dev(w2), eps,
+                                         dev(w3), center_y=center, center_out=center, rows_per_group=groups)
+                # a rounding that falls the other way moves z, and with it everything after, by a bf16 step of one entry
+                assert ((xd.double().cpu() - want).abs() <= 0.02 + 2.0 ** -6 * (want - mid).abs()).all(), (rows, groups)
+                close(out[:, :d], norm(xd.double().cpu(), w3), BF)
+                assert not out[:, d:].any()
+            side = TokenSide(gate, proj, w2, TokenSide.lay_out(table, layers, dtype=F32), ops.round8(dim), eps=eps, dtype=F32)
+            xd = dev(x)
+            out = side.update(xd, ops.Seq(rows, 1), ids.cuda(), dev(y, F32), kind(w1), kind(w3))
+            want = mid + R.rms((R.gelu_tanh(mid @ gate.double().t()) * e) @ proj.double().t(), eps) * w2.double()
+            close(xd, want, F32, tol=3e-5)
+            close(out[:, :d], norm(want, w3), F32, tol=1e-4)
+
+
 # ---- the model ------------------------------------------------------------------------------------
 
 

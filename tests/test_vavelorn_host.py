@@ -77,6 +77,10 @@ def test_entry_points_check_their_arguments():
     assert L.ohara_residual_norm_bf16(p, 8, 0, 0, 0, p, 8, p, 2, 1e-5, 16, 0, 0, 0, 0, 0, 0, r(seq), 0) == E
     assert L.ohara_gemm_gelu_lookup_bf16(p, 8, p, 8, 8, p, 4, p, 3, 1, p, 8, 0) == E  # table rows shorter than n
     assert L.ohara_gemm_gelu_lookup_f32(p, 8, p, 4, 6, p, 4, p, 3, 1, p, 4, 0) == E   # k % 4
+    side = lambda d=8, ldy=8, n=8, R=1, ldo=8: L.ohara_token_side_bf16(  # noqa: E731
+        p, d, p, ldy, p, 1, p, p, n, p, 512, p, 3, p, 1e-5, p, 1, 1, R, p, ldo, 0)
+    assert side(d=6) == E and side(ldy=4) == E and side(R=3) == E and side(n=264) == _lib.ESIZE
+    assert side(d=4096, ldy=4096, ldo=4096, R=16) == _lib.ESIZE  # more of the residual than a workgroup holds
     # rotated dimensions: even, inside the head, with tables
     rotate = lambda rot, tab=p, seq=seq: L.ohara_qkv_rotate_append_f32(p, 32, 2, 1, 8, 8, tab, tab, rot, p, p, p, 16, r(seq), 0)  # noqa: E731
     assert rotate(3) == E and rotate(10) == E and rotate(4, 0) == E and rotate(4, p, late) == E
