@@ -1029,7 +1029,8 @@ def bench_vavelorn_kernels(name, dev):
     for B in (1, 8, 32):
         seq, ids = ops.Seq(B, 1, 100), torch.randint(0, 32000, (B,), device=dev)
         row = {"kernel": "one token", "batch": B}
-        for label, mix, more in (("delta_step_kernel", delta, 2.0 * B * H * V), ("povazen delta_step_kernel", pdelta, 2.0 * (pdelta.a2.numel() + pdelta.g2.numel()))):
+        for label, mix, more in (("delta_step_kernel", delta, 2.0 * B * H * V),
+                                 ("povazen delta_step_kernel", pdelta, 2.0 * (pdelta.a2.numel() + pdelta.g2.numel()))):
             st, p = mix.state(B, 4096), rnd(B, mix.proj.n)
             row[label] = _hbm(timed(lambda: ops.delta_step(mix._c, p, st["delta"], st["ring"], seq)), 8.0 * B * H * D * V + more)
         x, xl, gate = rnd(B, H * D), rnd(B, H * R), rnd(B, H * V)

@@ -853,12 +853,13 @@ def delta_workspace_bytes(heads, dim, vdim, batch, tokens) -> int:
 
 
 def delta_prefill(d: "_lib.OharaDelta", p, za, zg, state, ring, workspace, seq: Seq):
-    """Any number of tokens per sequence of the gated delta rule (za, zg: the low-rank products, None where d has no such matrix); the ring is updated after the call's convolutions."""
+    """Any number of tokens per sequence of the gated delta rule (za, zg: the low-rank products, None where d has no such
+    matrix); the ring is updated after the call's convolutions."""
     rows = p.shape[0]
     out = torch.empty(rows, round8(d.heads * d.vdim), dtype=p.dtype, device=p.device)
     o_tmp = torch.empty(rows, d.heads * d.vdim, dtype=F32, device=p.device)
     check(_typed("delta_prefill", p.dtype)(
-        C.byref(d), _ptr(p), p.stride(0), _ptr(za), 0 if za is None else za.stride(0), _ptr(zg), 0 if zg is None else zg.stride(0), _ptr(state), _ptr(ring),
-        _ptr(workspace), workspace.numel(), _ptr(o_tmp), _ptr(out), out.stride(0), seq.ref, _stream()), "delta_prefill")
+        C.byref(d), _ptr(p), p.stride(0), _ptr(za), 0 if za is None else za.stride(0), _ptr(zg), 0 if zg is None else zg.stride(0),
+        _ptr(state), _ptr(ring), _ptr(workspace), workspace.numel(), _ptr(o_tmp), _ptr(out), out.stride(0), seq.ref, _stream()), "delta_prefill")
     conv_ring_store(p, 2 * d.kv_heads * d.dim + d.heads * d.vdim, ring, seq)
     return out
