@@ -638,21 +638,35 @@ typedef struct OharaSeq {
 #define OHARA_CENTER_Y 16
 #define OHARA_CENTER_OUT 32
 
+/* Output of routed experts before it is summed: row n of the layer's output is
+ *   sum_j w[n*top + j] * (idx[n*top + j] < experts ? y[pos_of[n*top + j]] : h[n]) + shared[n]   (shared: NULL for none),
+ * in fp32 and in the order of j; rows of y, h, shared in the activation type, leading dimensions multiples of 4. */
+typedef struct OharaMixture {
+  int top, experts, ldy, ldh, lds, reserved;
+  const float* w;
+  const int32_t* idx;
+  const int32_t* pos_of;
+  const void* y;
+  const void* h;
+  const void* shared;
+} OharaMixture;
+
 /* Residual update of a block with norms on the sublayer outputs, one launch:
- *   ids != NULL:  x = table[id]              (table: activation type, vocab rows of d)
- *   y != NULL:    x += norm_w * group_rms(y) (groups equal runs of the row, each over sqrt(mean square + eps))
+ *   ids != NULL:  x = table_scale * table[id] (table: activation type, vocab rows of d)
+ *   y != NULL:    x += norm_w * group_rms(y)  (groups equal runs of the row, each over sqrt(mean square + eps))
+ *   mix != NULL:  the same with the rows of an OharaMixture as y
  * x: (rows, d) fp32, updated in place.  out (leading dimension ldo >= d, columns past d are set to zero)
  * per out_mode.  OHARA_OUT_CONV: conv_w (taps, d) fp32 with the current token's row last, ring
  * (cache rows, taps, d) fp32 holds the inputs of the last tokens at index position mod taps and is
  * updated; inputs before position 0 count as zero, so a ring needs no clearing when its row is reused.
  * OHARA_OUT_NORM takes norm2_w. */
-int ohara_residual_norm_bf16(float* x, int d, const int64_t* ids, const uint16_t* table, int vocab, const uint16_t* y,
+int ohara_residual_norm_bf16(float* x, int d, const int64_t* ids, const uint16_t* table, int vocab, float table_scale, const uint16_t* y,
                              int ldy, const float* norm_w, int groups, float eps, int out_mode, uint16_t* out, int ldo,
-                             const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
+                             const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaMixture* mix, const OharaSeq* seq,
                              void* stream);
-int ohara_residual_norm_f32(float* x, int d, const int64_t* ids, const float* table, int vocab, const float* y, int ldy,
+int ohara_residual_norm_f32(float* x, int d, const int64_t* ids, const float* table, int vocab, float table_scale, const float* y, int ldy,
                             const float* norm_w, int groups, float eps, int out_mode, float* out, int ldo,
-                            const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
+                            const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaMixture* mix, const OharaSeq* seq,
                             void* stream);
 /* out = x + causal depthwise convolution of x over time for any seq_len (the ring is only read: follow with
  * ohara_conv_ring_store_f32), columns d .. ldo-1 of out are set to zero. */
@@ -675,6 +689,18 @@ int ohara_gemm_f32(const float* x, int ldx, const float* w, const float* w_up, c
  * (vocabulary projections with soft-capped logits). */
 int ohara_gemm_softcap_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, float cap, int rows,
                             uint16_t* out, int ldo, void* stream);
+
+/* Constants of a clamped gated unit. */
+typedef struct OharaGlu {
+  float limit, alpha, offset;
+  int reserved;
+} OharaGlu;
+/* Clamped gated unit: out = g sigmoid(alpha g) (u + offset), g = min(x Wg^T, limit), u = min(max(x Wu^T, -limit), limit), in fp32 up
+ * to the store.  bf16: packed weight in the order of ohara_swiglu_perm, any rows; f32: two matrices (n, k) row-major. */
+int ohara_gemm_glu_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, float limit, float alpha, float offset,
+                        int rows, uint16_t* out, int ldo, void* stream);
+int ohara_gemm_glu_f32(const float* x, int ldx, const float* w_gate, const float* w_up, int n, int k, float limit, float alpha,
+                       float offset, int rows, float* out, int ldo, void* stream);
 
 /* out[row, i] = gelu_tanh((x W^T)[row, i]) * table[ids[row] * ldt + i], gelu_tanh(z) = z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))),
  * i < n: a projection gated onto an embedding of the row's token (table: rows of ldt entries, the layer's n from the pointer on).
@@ -713,12 +739,21 @@ int ohara_qkv_rotate_append_bf16(const uint16_t* p, int ldp, int h, int h_kv, in
 int ohara_qkv_rotate_append_f32(const float* p, int ldp, int h, int h_kv, int dh, int dv, const float* cos, const float* sin,
                                 int rot, float* q_out, float* kcache, float* vcache, int t_max, const OharaSeq* seq,
                                 void* stream);
+/* The same with every q and k head first divided by its own root mean square and multiplied by qn / kn (dh entries, shared by
+ * the heads).  dh, dv <= 256. */
+int ohara_qkv_headnorm_rotate_append_bf16(const uint16_t* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn,
+                                          const float* kn, float eps, const float* cos, const float* sin, int rot,
+                                          uint16_t* q_out, uint16_t* kcache, uint16_t* vcache, int t_max, const OharaSeq* seq,
+                                          void* stream);
+int ohara_qkv_headnorm_rotate_append_f32(const float* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn,
+                                         const float* kn, float eps, const float* cos, const float* sin, int rot, float* q_out,
+                                         float* kcache, float* vcache, int t_max, const OharaSeq* seq, void* stream);
 /* Causal attention over the cache with a linear distance bias and a per-head output gate:
  *   o[row, hd, :] = sigmoid(gate[row, hd]) * sum_j softmax_j(scale q . k_j - slopes[hd] (i - j)) v_j,  j <= i = position.
  * Scores, softmax weights and sums are fp32 (the _bf16 prefill product carries every fp32 weight as three
  * bfloat16 terms).  q / caches as written by ohara_qkv_norm_append; gate (leading dimension ldg, in the
  * activation type; NULL: none); out rows of h*dv with leading dimension ldo, columns past h*dv are set to
- * zero.  dh, dv <= 256.  n_split > 1 (seq_len 1): the context of a (sequence, KV head) is cut into that many chunks
+ * zero up to the next multiple of 8 (ldo may go further).  dh, dv <= 256.  n_split > 1 (seq_len 1): the context of a (sequence, KV head) is cut into that many chunks
  * that meet in `workspace` (ohara_attn_bias_workspace_bytes, zero-filled once; calls sharing it must not
  * overlap). */
 int64_t ohara_attn_bias_workspace_bytes(int rows, int h, int dv, int n_split);
@@ -733,11 +768,17 @@ int ohara_attn_bias_f32(const float* q, const float* kcache, const float* vcache
  *   s = scale q . k_j;  cap > 0: s = cap tanh(s / cap);  slopes: s -= slopes[head] (i - j);
  * chunk > 0: only keys of the query's own chunk, floor(i / chunk) = floor(j / chunk), are visible.
  * ld_k, ld_v > 0: elements between neighbouring positions of the keys / values (0: h_kv * dhp, h_kv * dvp).
- * gate_elements: the gate has one entry per output element (rows of h*dv) instead of one per head. */
+ * gate_elements: the gate has one entry per output element (rows of h*dv) instead of one per head.
+ * window > 0: only the window keys up to and including the query's own are visible (with chunk: those of them in the chunk).
+ * sinks: per head a score that joins the softmax without a value, p_j = exp(s_j) / (exp(sinks[head]) + sum exp(s)).
+ * out_scale: factor of the output, applied before it is rounded. */
 typedef struct OharaScores {
   float scale, cap;
   int chunk, gate_elements, ld_k, ld_v;
   const float* slopes;
+  const float* sinks;
+  int window;
+  float out_scale;
 } OharaScores;
 int ohara_attn_scored_bf16(const uint16_t* q, const uint16_t* kcache, const uint16_t* vcache, int h, int h_kv, int dh,
                            int dv, int t_max, const OharaScores* sc, const uint16_t* gate, int ldg, int n_split,
@@ -817,6 +858,64 @@ int ohara_delta_prefill_bf16(const OharaDelta* d, const uint16_t* p, int ldp, co
 int ohara_delta_prefill_f32(const OharaDelta* d, const float* p, int ldp, const float* za, int ldza, const float* zg,
                             int ldzg, float* state, const float* ring, void* workspace, int64_t workspace_bytes,
                             float* o_tmp, float* out, int ldo, const OharaSeq* seq, void* stream);
+
+/* Retention: linear attention with one fixed decay per head and no normaliser.  Per head, S (dim x vdim) fp32 from zero:
+ *   S <- decay S + k_scale k v^T;   o = S^T q;   out = out_scale * o / sqrt(mean of o^2 over vdim_used + eps) * silu(g).
+ * A projection row p holds q, k (heads*dim each), v, g (heads*vdim each) from columns off_q, off_k, off_v, off_g; dim, vdim and the
+ * offsets are multiples of 8, vdim, dim <= 256; of each head's vdim columns the first vdim_used count (the others must be zero).
+ * powers (heads, OHARA_RETENTION_CHUNK + 1) fp32: decay to the power of 0, 1, ...  state (cache rows, heads, dim, vdim) fp32; a
+ * sequence whose first token sits at position 0 starts from zero whatever its state holds.  out: heads*vdim columns. */
+#define OHARA_RETENTION_CHUNK 128
+typedef struct OharaRetention {
+  int heads, dim, vdim, vdim_used, off_q, off_k, off_v, off_g;
+  float eps, k_scale, out_scale;
+  int reserved;
+  const float* powers;
+} OharaRetention;
+/* One token per sequence (seq_len 1), one launch. */
+int ohara_retention_step_bf16(const OharaRetention* r, const uint16_t* p, int ldp, float* state, uint16_t* out, int ldo,
+                              const OharaSeq* seq, void* stream);
+int ohara_retention_step_f32(const OharaRetention* r, const float* p, int ldp, float* state, float* out, int ldo,
+                             const OharaSeq* seq, void* stream);
+/* Any number of tokens per sequence in chunks: what every chunk adds to the state (all chunks in parallel), the states before
+ * the chunks, the outputs (in parallel again).  workspace: ohara_retention_workspace_bytes for the number of tokens per sequence
+ * worked on at a time (the call cuts longer sequences into segments that fit). */
+int64_t ohara_retention_workspace_bytes(int heads, int dim, int vdim, int batch, int tokens);
+int ohara_retention_prefill_bf16(const OharaRetention* r, const uint16_t* p, int ldp, float* state, void* workspace,
+                                 int64_t workspace_bytes, uint16_t* out, int ldo, const OharaSeq* seq, void* stream);
+int ohara_retention_prefill_f32(const OharaRetention* r, const float* p, int ldp, float* state, void* workspace,
+                                int64_t workspace_bytes, float* out, int ldo, const OharaSeq* seq, void* stream);
+
+/* ---- routed experts with clamped gated units, fp32 router, groups, identity outputs ---------------------------------
+ * router: z = W x in fp32 (w (n_out, k) row-major in the activation type), s = softmax(z) over all n_out outputs; the choice looks
+ * at s + correction (fp32, NULL: s) inside the `keep` of `groups` equal groups of neighbouring outputs whose largest entry is
+ * largest; the `top` best are chosen (ties: lowest index) -> idx (rows, top), weights s / (sum of the chosen s + 1e-20) -> wgt
+ * (rows, top) fp32.  Sorted by expert: offs (n_out + 1), pair_of (rows*top) sorted position -> row*top + j, pos_of its inverse.
+ * hist: workspace of ceil(rows*top / 1024) * n_out ints; counter: one zeroed int (left zero).  n_out <= 1024, top <= 64,
+ * groups <= 64. */
+int ohara_moe_router_bf16(const uint16_t* x, int ldx, const uint16_t* w, int ldw, const float* correction, int rows, int k, int n_out,
+                          int top, int groups, int keep, int32_t* idx, float* wgt, int32_t* offs, int32_t* pair_of,
+                          int32_t* pos_of, int32_t* hist, int32_t* counter, void* stream);
+int ohara_moe_router_f32(const float* x, int ldx, const float* w, int ldw, const float* correction, int rows, int k, int n_out,
+                         int top, int groups, int keep, int32_t* idx, float* wgt, int32_t* offs, int32_t* pair_of,
+                         int32_t* pos_of, int32_t* hist, int32_t* counter, void* stream);
+/* Products of the first n_experts experts over their sorted pairs.  glu: act[position] = clamped unit (ohara_gemm_glu_*) of row
+ * pair_of[position] / top of x; down: y[position] = W_down act[position], not weighted.  bf16: packed weights expert_stride_bytes
+ * apart; few pairs stream the weights (the shared expert, if given, rides along with its n_tokens rows), many run in tiles
+ * of 128 (no shared expert).  f32: row-major (n_experts, n, k) matrices. */
+int ohara_moe_glu_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int64_t expert_stride_bytes, int n_experts, int hidden, int d,
+                       int top, int n_pairs, const int32_t* offs, const int32_t* pair_of, const OharaGlu* glu, uint16_t* act,
+                       int ld_act, const uint16_t* wp_shared, int hidden_shared, int n_tokens, const OharaGlu* glu_shared,
+                       uint16_t* act_shared, int ld_act_shared, void* stream);
+int ohara_moe_down_bf16(const uint16_t* act, int ld_act, const uint16_t* wp, int64_t expert_stride_bytes, int n_experts, int d,
+                        int hidden, int n_pairs, const int32_t* offs, uint16_t* y, int ldy, const uint16_t* wp_shared,
+                        int hidden_shared, int n_tokens, const uint16_t* act_shared, int ld_act_shared, uint16_t* y_shared,
+                        int ldy_shared, void* stream);
+int ohara_moe_glu_f32(const float* x, int ldx, const float* w_gate, const float* w_up, int n_experts, int hidden, int d, int top,
+                      int n_pairs, const int32_t* offs, const int32_t* pair_of, const OharaGlu* glu, float* act, int ld_act,
+                      void* stream);
+int ohara_moe_down_f32(const float* act, int ld_act, const float* w, int n_experts, int d, int hidden, int n_pairs,
+                       const int32_t* offs, float* y, int ldy, void* stream);
 
 /* ---- timing helpers (measurement only; no counterpart in the reference) -----------
  * Thin wrappers over hipEventCreate / hipEventDestroy / hipEventElapsedTime so that a

@@ -74,12 +74,28 @@ class OharaDelta(C.Structure):
 
 
 class OharaScores(C.Structure):
-    _fields_ = [("scale", _f), ("cap", _f), ("chunk", _i), ("gate_elements", _i), ("ld_k", _i), ("ld_v", _i), ("slopes", _p)]
+    _fields_ = [("scale", _f), ("cap", _f), ("chunk", _i), ("gate_elements", _i), ("ld_k", _i), ("ld_v", _i), ("slopes", _p),
+                ("sinks", _p), ("window", _i), ("out_scale", _f)]
+
+
+class OharaMixture(C.Structure):
+    _fields_ = [("top", _i), ("experts", _i), ("ldy", _i), ("ldh", _i), ("lds", _i), ("reserved", _i), ("w", _p), ("idx", _p),
+                ("pos_of", _p), ("y", _p), ("h", _p), ("shared", _p)]
+
+
+class OharaGlu(C.Structure):
+    _fields_ = [("limit", _f), ("alpha", _f), ("offset", _f), ("reserved", _i)]
+
+
+class OharaRetention(C.Structure):
+    _fields_ = [("heads", _i), ("dim", _i), ("vdim", _i), ("vdim_used", _i), ("off_q", _i), ("off_k", _i), ("off_v", _i), ("off_g", _i),
+                ("eps", _f), ("k_scale", _f), ("out_scale", _f), ("reserved", _i), ("powers", _p)]
 
 
 OUT_NONE, OUT_COPY, OUT_CONV, OUT_NORM = 0, 1, 2, 3
 CENTER_Y, CENTER_OUT = 16, 32
 DELTA_SILU_GATE = 1
+RETENTION_CHUNK = 128
 OHARA_LOGITS_NONE, OHARA_LOGITS_LAST, OHARA_LOGITS_ALL = 0, 1, 2
 
 _PROTOS = {
@@ -150,13 +166,18 @@ _PROTOS = {
     "ohara_bitnet_decode_persistent": (_i, [C.POINTER(OharaBitModel), C.POINTER(OharaDecodeState), _p, _i, _i, _i,
                                             C.c_uint, _p]),
     **{f"ohara_{name}_{dt}": proto for dt in ("bf16", "f32") for name, proto in {
-        "residual_norm": (_i, [_p, _i, _p, _p, _i, _p, _i, _p, _i, _f, _i, _p, _i, _p, _p, _i, _p, C.POINTER(OharaSeq), _p]),
+        "residual_norm": (_i, [_p, _i, _p, _p, _i, _f, _p, _i, _p, _i, _f, _i, _p, _i, _p, _p, _i, _p, C.POINTER(OharaMixture),
+                               C.POINTER(OharaSeq), _p]),
         "input_conv": (_i, [_p, _i, _p, _i, _p, _p, _i, C.POINTER(OharaSeq), _p]),
         "conv_ring_store": (_i, [_p, _i, _i, _i, _p, C.POINTER(OharaSeq), _p]),
         "qkv_norm_append": (_i, [_p, _i, _i, _i, _i, _i, _p, _p, _f, _p, _p, _p, _i, C.POINTER(OharaSeq), _p]),
         "attn_bias": (_i, [_p, _p, _p, _i, _i, _i, _i, _i, _f, _p, _p, _i, _i, _p, _p, _i, C.POINTER(OharaSeq), _p]),
         "attn_scored": (_i, [_p, _p, _p, _i, _i, _i, _i, _i, C.POINTER(OharaScores), _p, _i, _i, _p, _p, _i, C.POINTER(OharaSeq), _p]),
         "qkv_rotate_append": (_i, [_p, _i, _i, _i, _i, _i, _p, _p, _i, _p, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "qkv_headnorm_rotate_append": (_i, [_p, _i, _i, _i, _i, _i, _p, _p, _f, _p, _p, _i, _p, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "retention_step": (_i, [C.POINTER(OharaRetention), _p, _i, _p, _p, _i, C.POINTER(OharaSeq), _p]),
+        "retention_prefill": (_i, [C.POINTER(OharaRetention), _p, _i, _p, _p, _i64, _p, _i, C.POINTER(OharaSeq), _p]),
+        "moe_router": (_i, [_p, _i, _p, _i, _p, _i, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _p, _p, _p]),
         "gemm_gelu_lookup": (_i, [_p, _i, _p, _i, _i, _p, _i, _p, _i, _i, _p, _i, _p]),
         "latent_front": (_i, [_p, _i, _i, _i, _i, _p, _p, _f, _p, _p, _i, _p, C.POINTER(OharaSeq), _p]),
         "head_linear": (_i, [_p, _i, _p, _i, _i, _i, _i, _i, _p, _i, _p, _i, _p]),
@@ -165,6 +186,14 @@ _PROTOS = {
         "delta_prefill": (_i, [C.POINTER(OharaDelta), _p, _i, _p, _i, _p, _i, _p, _p, _p, _i64, _p, _p, _i,
                                C.POINTER(OharaSeq), _p]),
     }.items()},
+    "ohara_gemm_glu_bf16": (_i, [_p, _i, _p, _i, _i, _f, _f, _f, _i, _p, _i, _p]),
+    "ohara_gemm_glu_f32": (_i, [_p, _i, _p, _p, _i, _i, _f, _f, _f, _i, _p, _i, _p]),
+    "ohara_moe_glu_bf16": (_i, [_p, _i, _p, _i64, _i, _i, _i, _i, _i, _p, _p, C.POINTER(OharaGlu), _p, _i, _p, _i, _i,
+                                C.POINTER(OharaGlu), _p, _i, _p]),
+    "ohara_moe_down_bf16": (_i, [_p, _i, _p, _i64, _i, _i, _i, _i, _p, _p, _i, _p, _i, _i, _p, _i, _p, _i, _p]),
+    "ohara_moe_glu_f32": (_i, [_p, _i, _p, _p, _i, _i, _i, _i, _i, _p, _p, C.POINTER(OharaGlu), _p, _i, _p]),
+    "ohara_moe_down_f32": (_i, [_p, _i, _p, _i, _i, _i, _i, _p, _p, _i, _p]),
+    "ohara_retention_workspace_bytes": (_i64, [_i, _i, _i, _i, _i]),
     "ohara_gemm_f32": (_i, [_p, _i, _p, _p, _p, _f, _i, _i, _i, _p, _i, _p]),
     "ohara_gemm_softcap_bf16": (_i, [_p, _i, _p, _i, _i, _f, _i, _p, _i, _p]),
     "ohara_token_side_bf16": (_i, [_p, _i, _p, _i, _p, _i, _p, _p, _i, _p, _i, _p, _i, _p, _f, _p, _i, _i, _i, _p, _i, _p]),

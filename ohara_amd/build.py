@@ -20,8 +20,9 @@ OBJ_DIR = os.path.join(LIB_DIR, "obj")
 LIB_PATH = os.path.join(LIB_DIR, "libohara_decode.so")
 # Libraries of fewer sources for programs that serve one design from a fresh checkout (``ensure``): the same entry
 # points, those of other models absent.
-_HYBRID = ("attention_bias", "delta_rule", "gemm_f32", "gemm_skinny", "gemm_tile", "misc", "residual_norm", "sampler")
-SERVING = {"Povazen": _HYBRID, "Vavelorn": (*_HYBRID, "latent", "token_side")}
+_HYBRID = ("attention_bias", "gemm_f32", "gemm_skinny", "gemm_tile", "misc", "residual_norm", "sampler")
+SERVING = {"Fibirax": (*_HYBRID, "moe", "retention"), "Povazen": (*_HYBRID, "delta_rule"),
+           "Vavelorn": (*_HYBRID, "delta_rule", "latent", "token_side")}
 
 
 def partial_path(design: str) -> str:

@@ -127,6 +127,7 @@ def loop_moe_config(config: Config) -> Config:
 # Designs other than the reference's Llama, by the "architecture" of their config.json: module and names of the
 # config class (``from_dict``) and of the model class (config, state dict, device, dtype).
 ARCHITECTURES = {
+    "Fibirax": ("fibirax", "FibiraxConfig", "Fibirax"),
     "Povazen": ("povazen", "PovazenConfig", "Povazen"),
     "Vavelorn": ("vavelorn", "VavelornConfig", "Vavelorn"),
 }

@@ -1,9 +1,10 @@
-// Attention over the KV cache with a linear distance bias or a soft cap on the scores, over the whole context or inside chunks,
-// and a gate per head or per element.
+// Attention over the KV cache with a linear distance bias or a soft cap on the scores, over the whole context, inside chunks or
+// in a sliding window, with a sink in the softmax and a gate per head or per element.
 //
 //   qkv_norm_append   q and k over the root mean square of the whole projection row, values over each head's,
 //                     keys and values into the cache: a workgroup per token
 //   qkv_rotate_append the same without norms, q and k rotated in neighbouring pairs
+//   qkv_headnorm_rotate_append  q and k of every head over that head's root mean square, then rotated: a lane group per head
 //   attn_bias_kernel  one query token per workgroup (decode; any head width up to 256; bf16 or fp32)
 //   attn_bias_prefill many query tokens on bf16 MFMA
 //
@@ -172,6 +173,69 @@ __global__ __launch_bounds__(256) void qkv_rotate_append_kernel(RotateArgs<T> a)
   }
 }
 
+template <typename T>
+struct HeadNormArgs {
+  RotateArgs<T> r;
+  const float* qn;
+  const float* kn;
+  float eps;
+};
+
+// LP lanes own one head of a token, four consecutive elements each (heads of up to 4 LP elements), so the norm is a sum over
+// lanes and no rotated pair is split.  Value heads pass through.
+template <typename T, int LP>
+__global__ __launch_bounds__(256) void qkv_headnorm_rotate_append_kernel(HeadNormArgs<T> n) {
+  constexpr int NU = 256 / LP;
+  const RotateArgs<T>& a = n.r;
+  const int row = blockIdx.x, b = row / a.seq.seq_len, s = row - b * a.seq.seq_len;
+  const int pos = seq_start(a.seq, b) + s;
+  if (s >= seq_tokens(a.seq, b) || pos < 0 || pos >= a.Tmax) return;
+  const int Dp = (a.D + 7) & ~7, Vp = (a.V + 7) & ~7, half = a.rot / 2;
+  const T* p = a.p + (size_t)row * a.ldp;
+  const float *cs = a.cos + (size_t)pos * half, *sn = a.sin + (size_t)pos * half;
+  const size_t crow = (size_t)seq_slot(a.seq, b) * a.Tmax + pos;
+  const bool vec = ((a.D | a.V | a.ldp) & 3) == 0;
+  const int c = 4 * (threadIdx.x % LP), heads = a.H + 2 * a.G;
+  for (int u0 = blockIdx.y * NU; u0 < heads; u0 += gridDim.y * NU) {  // the same rounds for all lanes
+    const int u = u0 + threadIdx.x / LP;
+    const bool live = u < heads, isq = u < a.H, isv = u >= a.H + a.G;
+    const int w = isv ? a.V : a.D;
+    const T* src = p + (isv ? (a.H + a.G) * a.D + (u - a.H - a.G) * a.V : u * a.D) + c;
+    float v[4] = {0.f, 0.f, 0.f, 0.f}, g[4] = {1.f, 1.f, 1.f, 1.f};
+    if (live && c < w) {
+      const float* gw = (isq ? n.qn : n.kn) + c;
+      if (vec) {
+        ld4(src, v);
+        if (!isv) ld4(gw, g);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (c + i < w) {
+            v[i] = ldv(src + i);
+            if (!isv) g[i] = gw[i];
+          }
+      }
+    }
+    const float ss = lanes_sum<LP / 2, 1>(((v[0] * v[0] + v[1] * v[1]) + v[2] * v[2]) + v[3] * v[3]);
+    if (!live || c >= (isv ? Vp : Dp)) continue;
+    if (!isv) {
+      const float r = 1.0f / sqrtf(ss / (float)a.D + n.eps);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = v[i] * r * g[i];
+#pragma unroll
+      for (int i = 0; i < 4; i += 2)
+        if (c + i < a.rot) {
+          const float co = cs[(c + i) >> 1], si = sn[(c + i) >> 1], e = v[i], o = v[i + 1];
+          v[i] = e * co - o * si;
+          v[i + 1] = o * co + e * si;
+        }
+    }
+    T* dst = isq ? a.q + ((size_t)row * a.H + u) * Dp
+                 : (isv ? a.vc + (crow * a.G + u - a.H - a.G) * Vp : a.kc + (crow * a.G + u - a.H) * Dp);
+    st4(dst + c, v);
+  }
+}
+
 // ---- one query token per workgroup -----------------------------------------------------------
 template <typename T>
 struct AttnBiasArgs {
@@ -184,6 +248,9 @@ struct AttnBiasArgs {
   int H, G, D, V, Tmax, ldg, ldo;
   int kd, vd;      // elements between neighbouring positions of the keys / values
   int chunk;       // > 0: only keys of the query's own chunk are visible
+  int window;      // > 0: only that many keys up to the query's own are visible
+  const float* sinks;  // per head: a score that takes part in the softmax without a value (null: none)
+  float out_scale; // of the output
   int gate_elem;   // the gate has an entry per output element
   float cap;       // CAP kernels: cap * tanh(score / cap)
   int rb, nhb;     // query heads served together (at most RB) and such sets per KV head
@@ -200,10 +267,21 @@ __device__ __forceinline__ float tanh_x(float v) {
   return __builtin_fmaf(-2.0f, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.0f * OHARA_LOG2E * v)), 1.0f);
 }
 
+// what an output element is multiplied by
 template <typename T>
 __device__ __forceinline__ float gate_of(const AttnBiasArgs<T>& a, size_t row, int h, int c) {
-  return a.gate ? sigmoid_x(ldv(a.gate + row * a.ldg + (a.gate_elem ? h * a.V + c : h))) : 1.0f;
+  return a.gate ? a.out_scale * sigmoid_x(ldv(a.gate + row * a.ldg + (a.gate_elem ? h * a.V + c : h))) : a.out_scale;
 }
+
+// the first position a query sees; grows with pos
+template <typename T>
+__device__ __forceinline__ int first_seen(const AttnBiasArgs<T>& a, int pos) {
+  const int w = a.window > 0 ? max(0, pos - a.window + 1) : 0;
+  return a.chunk > 0 ? max(w, pos / a.chunk * a.chunk) : w;
+}
+// columns past H * V that an output row is padded with zeros to
+template <typename T>
+__device__ __forceinline__ int out_padded(const AttnBiasArgs<T>& a) { return min(a.ldo, (a.H * a.V + 7) & ~7); }
 
 // LP lanes own one cached position (lane l elements 8l .. 8l+7 of key and value), so a workgroup walks 256 / LP
 // positions per round with an online softmax per lane group and query head; the groups are merged through LDS.
@@ -223,7 +301,7 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
   const int b = row / a.seq.seq_len, s = row - b * a.seq.seq_len;
   const int pq = seq_start(a.seq, b) + s;
   if (hb == 0 && g == 0 && blockIdx.y == 0)
-    for (int i = a.H * a.V + tid; i < a.ldo; i += 256) stv(a.out + (size_t)row * a.ldo + i, 0.f);
+    for (int i = a.H * a.V + tid; i < out_padded(a); i += 256) stv(a.out + (size_t)row * a.ldo + i, 0.f);
   if (s >= seq_tokens(a.seq, b) || pq < 0 || pq >= a.Tmax) return;  // the same for every chunk of the row
   const int rep = a.H / a.G;
   const int h0 = g * rep + hb * a.rb, nh = min(a.rb, rep - hb * a.rb);
@@ -245,8 +323,9 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
   float m[RB], lsum[RB], acc[RB][8];
 #pragma unroll
   for (int r = 0; r < RB; ++r) {
-    m[r] = -INFINITY;
-    lsum[r] = 0.f;
+    const bool sink = a.sinks && grp == 0 && blockIdx.y == 0;  // one lane group of one chunk starts from the sink
+    m[r] = sink ? a.sinks[h0 + min(r, nh - 1)] * OHARA_LOG2E : -INFINITY;
+    lsum[r] = sink ? 1.f : 0.f;
 #pragma unroll
     for (int u = 0; u < 8; ++u) acc[r][u] = 0.f;
   }
@@ -254,7 +333,7 @@ __global__ __launch_bounds__(256) void attn_bias_kernel(AttnBiasArgs<T> a) {
   const size_t kd = a.kd, vd = a.vd, base = (size_t)seq_slot(a.seq, b) * a.Tmax;
   const T* kb = a.kc + base * kd + (size_t)g * Dp + (ownk ? e0 : 0);
   const T* vb = a.vc + base * vd + (size_t)g * Vp + (ownv ? e0 : 0);
-  int t_lo = a.chunk > 0 ? pq / a.chunk * a.chunk : 0, t_hi = pq;
+  int t_lo = first_seen(a, pq), t_hi = pq;
   if (a.ns > 1) {
     const int per = ((pq - t_lo + a.ns) / a.ns + NG - 1) / NG * NG;  // the visible positions over ns, in whole rounds
     t_lo += blockIdx.y * per;
@@ -435,7 +514,7 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
   for (int u = 0; u < QW; ++u) {
     const int qi = min(wq0 + 16 * u + m, len - 1);  // lanes past the end repeat the last query and are not stored
     qpos[u] = pos0 + qi;
-    qlow[u] = a.chunk > 0 ? qpos[u] / a.chunk * a.chunk : 0;
+    qlow[u] = first_seen(a, qpos[u]);
     qrow[u] = (size_t)b * a.seq.seq_len + qi;
 #pragma unroll
     for (int j = 0; j < NK; ++j)
@@ -447,6 +526,11 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
   for (int u = 0; u < QW; ++u) {
     mrun[u] = -1e30f;  // finite: a tile may lie wholly outside a query's window
     lrun[u] = 0.f;
+    if (a.sinks) {  // one of the four lane groups starts from the sink
+      const float sk = a.sinks[h] * OHARA_LOG2E;
+      mrun[u] = ceilf(sk);
+      lrun[u] = g == 0 ? __builtin_amdgcn_exp2f(sk - mrun[u]) : 0.f;
+    }
 #pragma unroll
     for (int t = 0; t < ND; ++t) o[u][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
   }
@@ -504,13 +588,9 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
     }
   };
 
-  // with chunks: from the tile of the first position the workgroup's / the wave's first query sees
-  int t_first = 0, wave_low = 0, wave_low_last = 0;
-  if (a.chunk > 0) {
-    t_first = (pos0 + q0) / a.chunk * a.chunk / KT * KT;
-    wave_low = (pos0 + min(wq0, len - 1)) / a.chunk * a.chunk;
-    wave_low_last = wave_last / a.chunk * a.chunk;
-  }
+  // from the tile of the first position the workgroup's first query sees; the first positions of the wave's first and last query
+  const int t_first = first_seen(a, pos0 + q0) / KT * KT;
+  const int wave_low = first_seen(a, pos0 + min(wq0, len - 1)), wave_low_last = first_seen(a, wave_last);
   load_tile(t_first);
   for (int t0 = t_first; t0 < kv_end; t0 += KT) {
     __syncthreads();  // everyone is done with the previous tile
@@ -635,7 +715,7 @@ __global__ __launch_bounds__(256, (DP > 128 || VP > 128 ? 1 : 2)) void attn_bias
       }
     }
     if (h == 0 && g == 0)
-      for (int i = a.H * a.V; i < a.ldo; ++i) orow[i] = 0;
+      for (int i = a.H * a.V; i < out_padded(a); ++i) orow[i] = 0;
   }
 }
 
@@ -691,18 +771,38 @@ int launch_front(const FrontArgs<T>& a, hipStream_t st) {
 }
 
 template <typename T>
+bool rotate_ok(const RotateArgs<T>& a) {
+  if (!a.p || !a.q || !a.kc || !a.vc || !seq_ok(&a.seq)) return false;
+  if (a.H < 1 || a.G < 1 || a.H % a.G || a.D < 1 || a.V < 1 || a.Tmax < 1) return false;
+  if (a.rot < 0 || (a.rot & 1) || a.rot > a.D || (a.rot && (!a.cos || !a.sin))) return false;
+  if (a.ldp < a.H * a.D + a.G * (a.D + a.V)) return false;
+  if (!a.seq.pos_dev && a.seq.pos + a.seq.seq_len > a.Tmax) return false;
+  return true;
+}
+
+template <typename T>
 int launch_rotate(const RotateArgs<T>& a, hipStream_t st) {
-  if (!a.p || !a.q || !a.kc || !a.vc || !seq_ok(&a.seq)) return OHARA_EINVAL;
-  if (a.H < 1 || a.G < 1 || a.H % a.G || a.D < 1 || a.V < 1 || a.Tmax < 1) return OHARA_EINVAL;
-  if (a.rot < 0 || (a.rot & 1) || a.rot > a.D || (a.rot && (!a.cos || !a.sin))) return OHARA_EINVAL;
-  if (a.ldp < a.H * a.D + a.G * (a.D + a.V)) return OHARA_EINVAL;
-  if (!a.seq.pos_dev && a.seq.pos + a.seq.seq_len > a.Tmax) return OHARA_EINVAL;
+  if (!rotate_ok(a)) return OHARA_EINVAL;
   const int all = (a.H + a.G) * ((a.D + 7) & ~7) + a.G * ((a.V + 7) & ~7);
   const int P = ((a.D | a.V | a.ldp) & 3) == 0 ? 4 : 1;
   const int ny = (all + 256 * P - 1) / (256 * P);
   const dim3 grid((unsigned)(a.seq.batch * a.seq.seq_len), (unsigned)(ny < 8 ? ny : 8));
   if (P == 4) hipLaunchKernelGGL((qkv_rotate_append_kernel<T, 4>), grid, dim3(256), 0, st, a);
   else hipLaunchKernelGGL((qkv_rotate_append_kernel<T, 1>), grid, dim3(256), 0, st, a);
+  return ohara_launch_status();
+}
+
+template <typename T>
+int launch_headnorm_rotate(const HeadNormArgs<T>& n, hipStream_t st) {
+  const RotateArgs<T>& a = n.r;
+  if (!rotate_ok(a) || !n.qn || !n.kn) return OHARA_EINVAL;
+  if (a.D > 256 || a.V > 256) return OHARA_ESIZE;
+  const int w = a.D > a.V ? a.D : a.V, heads = a.H + 2 * a.G;
+  const int lp = w <= 64 ? 16 : (w <= 128 ? 32 : 64), ny = (heads + 256 / lp - 1) / (256 / lp);
+  const dim3 grid((unsigned)(a.seq.batch * a.seq.seq_len), (unsigned)(ny < 16 ? ny : 16));
+  if (lp == 16) hipLaunchKernelGGL((qkv_headnorm_rotate_append_kernel<T, 16>), grid, dim3(256), 0, st, n);
+  else if (lp == 32) hipLaunchKernelGGL((qkv_headnorm_rotate_append_kernel<T, 32>), grid, dim3(256), 0, st, n);
+  else hipLaunchKernelGGL((qkv_headnorm_rotate_append_kernel<T, 64>), grid, dim3(256), 0, st, n);
   return ohara_launch_status();
 }
 
@@ -734,7 +834,7 @@ int launch_bias(AttnBiasArgs<T> a, void* workspace, hipStream_t st) {
   if (a.H < 1 || a.G < 1 || a.H % a.G || a.D < 1 || a.V < 1 || a.Tmax < 1) return OHARA_EINVAL;
   if (a.D > 256 || a.V > 256) return OHARA_ESIZE;
   if (a.ldo < a.H * a.V || (a.gate && a.ldg < (a.gate_elem ? a.H * a.V : 1))) return OHARA_EINVAL;
-  if (a.chunk < 0 || !(a.cap >= 0.f)) return OHARA_EINVAL;
+  if (a.chunk < 0 || a.window < 0 || !(a.cap >= 0.f)) return OHARA_EINVAL;
   const int kd = a.G * ((a.D + 7) & ~7), vd = a.G * ((a.V + 7) & ~7);
   if (!a.kd) a.kd = kd;
   if (!a.vd) a.vd = vd;
@@ -758,7 +858,7 @@ int attn_scored(const T* q, const T* kcache, const T* vcache, int h, int h_kv, i
   AttnBiasArgs<T> a{};
   a.q = q; a.kc = kcache; a.vc = vcache; a.gate = gate; a.slopes = sc->slopes; a.out = out;
   a.H = h; a.G = h_kv; a.D = dh; a.V = dv; a.Tmax = t_max; a.ldg = ldg; a.ldo = ldo; a.ns = n_split; a.scale = sc->scale;
-  a.cap = sc->cap; a.chunk = sc->chunk; a.gate_elem = sc->gate_elements != 0; a.kd = sc->ld_k; a.vd = sc->ld_v;
+  a.cap = sc->cap; a.chunk = sc->chunk; a.window = sc->window; a.sinks = sc->sinks; a.out_scale = sc->out_scale; a.gate_elem = sc->gate_elements != 0; a.kd = sc->ld_k; a.vd = sc->ld_v;
   a.seq = *seq;
   return launch_bias<T>(a, workspace, (hipStream_t)stream);
 }
@@ -792,14 +892,14 @@ int ohara_attn_bias_bf16(const uint16_t* q, const uint16_t* kcache, const uint16
                          int dv, int t_max, float scale, const float* slopes, const uint16_t* gate, int ldg, int n_split,
                          void* workspace, uint16_t* out, int ldo, const OharaSeq* seq, void* stream) {
   if (!slopes) return OHARA_EINVAL;
-  const OharaScores sc{scale, 0.f, 0, 0, 0, 0, slopes};
+  const OharaScores sc{scale, 0.f, 0, 0, 0, 0, slopes, nullptr, 0, 1.f};
   return attn_scored<bf16_t>(q, kcache, vcache, h, h_kv, dh, dv, t_max, &sc, gate, ldg, n_split, workspace, out, ldo, seq, stream);
 }
 int ohara_attn_bias_f32(const float* q, const float* kcache, const float* vcache, int h, int h_kv, int dh, int dv,
                         int t_max, float scale, const float* slopes, const float* gate, int ldg, int n_split,
                         void* workspace, float* out, int ldo, const OharaSeq* seq, void* stream) {
   if (!slopes) return OHARA_EINVAL;
-  const OharaScores sc{scale, 0.f, 0, 0, 0, 0, slopes};
+  const OharaScores sc{scale, 0.f, 0, 0, 0, 0, slopes, nullptr, 0, 1.f};
   return attn_scored<float>(q, kcache, vcache, h, h_kv, dh, dv, t_max, &sc, gate, ldg, n_split, workspace, out, ldo, seq, stream);
 }
 
@@ -827,6 +927,22 @@ int ohara_qkv_rotate_append_f32(const float* p, int ldp, int h, int h_kv, int dh
   if (!seq) return OHARA_EINVAL;
   return launch_rotate<float>(RotateArgs<float>{p, cos, sin, q_out, kcache, vcache, ldp, h, h_kv, dh, dv, t_max, rot, *seq},
                               (hipStream_t)stream);
+}
+
+int ohara_qkv_headnorm_rotate_append_bf16(const uint16_t* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn, const float* kn,
+                                          float eps, const float* cos, const float* sin, int rot, uint16_t* q_out, uint16_t* kcache,
+                                          uint16_t* vcache, int t_max, const OharaSeq* seq, void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  const RotateArgs<bf16_t> r{p, cos, sin, q_out, kcache, vcache, ldp, h, h_kv, dh, dv, t_max, rot, *seq};
+  return launch_headnorm_rotate<bf16_t>(HeadNormArgs<bf16_t>{r, qn, kn, eps}, (hipStream_t)stream);
+}
+
+int ohara_qkv_headnorm_rotate_append_f32(const float* p, int ldp, int h, int h_kv, int dh, int dv, const float* qn, const float* kn,
+                                          float eps, const float* cos, const float* sin, int rot, float* q_out, float* kcache,
+                                          float* vcache, int t_max, const OharaSeq* seq, void* stream) {
+  if (!seq) return OHARA_EINVAL;
+  const RotateArgs<float> r{p, cos, sin, q_out, kcache, vcache, ldp, h, h_kv, dh, dv, t_max, rot, *seq};
+  return launch_headnorm_rotate<float>(HeadNormArgs<float>{r, qn, kn, eps}, (hipStream_t)stream);
 }
 
 }  // extern "C"

@@ -308,6 +308,13 @@ __device__ __forceinline__ void wait_own_stores() {
 // epilogue made a fifth of that kernel's time.
 __device__ __forceinline__ float silu_f(float x) { return x * __frcp_rn(1.0f + __expf(-x)); }
 
+// g sigmoid(alpha g) (u + offset) with g capped by limit from above and u from both sides
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float offset) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * __frcp_rn(1.0f + __expf(-alpha * g)) * (u + offset);
+}
+
 // z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))) in fp32
 __device__ __forceinline__ float gelu_tanh(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));

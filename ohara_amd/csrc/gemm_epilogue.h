@@ -6,10 +6,11 @@
 //   bias / new_gelu / parallel-block sum of Phi   ohara/models/phi.py:37-52, :147-151
 //   soft cap of the fp32 sum (vocabulary projections with capped logits)
 //   gelu of the fp32 sum times an embedding of the row's token
+//   clamped gated unit of the fp32 sums
 #pragma once
 #include "common.h"
 
-enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3, EPI_BIAS = 4, EPI_BIAS_GELU = 5, EPI_BIAS_ADD2 = 6, EPI_PHI_IN = 7, EPI_SOFTCAP = 8, EPI_GELU_LOOKUP = 9 };
+enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3, EPI_BIAS = 4, EPI_BIAS_GELU = 5, EPI_BIAS_ADD2 = 6, EPI_PHI_IN = 7, EPI_SOFTCAP = 8, EPI_GELU_LOOKUP = 9, EPI_GLU = 10 };
 
 struct GemmArgs {
   const uint4* wp;
@@ -50,6 +51,7 @@ struct GemmArgs {
   const bf16_t* table;
   const int64_t* ids;
   int ldt, vocab;
+  OharaGlu glu;  // EPI_GLU: packed rows as EPI_SWIGLU
 };
 
 // gemm_tile.hip: the tiled kernel for calls with many rows (a.B rows, no fused norm).
@@ -120,6 +122,14 @@ __device__ __forceinline__ void gemm_epilogue(const GemmArgs& a, int b, int stri
 #pragma unroll
     for (int i = 0; i < 4; ++i) v[i] = gelu_tanh(acc[i]) * e[i];
     *reinterpret_cast<uint2*>(a.out + (size_t)b * a.ldo + r0) = make_uint2(pack_bf(v[0], v[1]), pack_bf(v[2], v[3]));
+    return;
+  }
+  if (EPI == EPI_GLU) {  // rows as in EPI_SWIGLU; N and ldo are multiples of 2
+    const int f = strip * 8 + 2 * g;
+    if (f < a.N)
+      *reinterpret_cast<uint32_t*>(a.out + (size_t)b * a.ldo + f) =
+          pack_bf(clamped_glu(acc[0], acc[2], a.glu.limit, a.glu.alpha, a.glu.offset),
+                  clamped_glu(acc[1], acc[3], a.glu.limit, a.glu.alpha, a.glu.offset));
     return;
   }
   const float y0 = rbf(acc[0]), y1 = rbf(acc[1]), y2 = rbf(acc[2]), y3 = rbf(acc[3]);

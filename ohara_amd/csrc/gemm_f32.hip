@@ -1,4 +1,5 @@
-// fp32 matrix product for models served in 32-bit: y = x W^T with bias, SwiGLU, soft-cap or gelu-lookup epilogues, on
+// fp32 matrix product for models served in 32-bit: y = x W^T with bias, SwiGLU, clamped gated unit, soft-cap or gelu-lookup
+// epilogues, for one matrix or for the sorted rows of several experts (a grid plane per expert), on
 // v_mfma_f32_16x16x4_f32 (true fp32 products and sums).  A workgroup owns 64 rows x 64 weight rows, a wave a
 // 32 x 32 quarter; 16 columns of both operands per step go through LDS, the next step's loads are in flight
 // during the products.
@@ -17,17 +18,33 @@ struct GemmF32Args {
   const float* table;  // gelu_tanh(y) * table[ids[row] * ldt + column]
   const int64_t* ids;
   int ldt, vocab;
+  OharaGlu glu;         // GLU
+  const int32_t* offs;  // experts: rows offs[e] .. offs[e + 1] - 1 of the output, matrices `stride` floats apart
+  const int32_t* pair_of;  // row of x: pair_of[row] / top (null: the row itself)
+  int top;
+  size_t stride;
 };
 
 constexpr int GT = 64, GK = 16, GL = GK + 4;
 
-template <bool SWIGLU>
+enum { ACT_NONE = 0, ACT_SWIGLU = 1, ACT_GLU = 2 };
+
+template <int ACT>
 __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32Args a) {
-  constexpr int NB = SWIGLU ? 2 : 1;
+  constexpr int NB = ACT == ACT_NONE ? 1 : 2;
   __shared__ __align__(16) float xs[GT * GL];
   __shared__ __align__(16) float ws[NB][GT * GL];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 15, g = lane >> 4;
-  const int r0 = blockIdx.y * GT, c0 = blockIdx.x * GT;
+  int r0 = blockIdx.y * GT;
+  const int c0 = blockIdx.x * GT;
+  if (a.offs) {
+    const int e = blockIdx.z;
+    r0 += a.offs[e];
+    a.rows = a.offs[e + 1];
+    if (r0 >= a.rows) return;
+    a.w += e * a.stride;
+    if (NB == 2) a.w2 += e * a.stride;
+  }
   const int wr = (wave & 1) * 32, wc = (wave >> 1) * 32;
   const int lr = tid >> 2, lc = (tid & 3) * 4;  // loader: one float4 per thread and operand
   f32x4 acc[NB][2][2];
@@ -39,10 +56,11 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32Args a) {
       for (int j = 0; j < 2; ++j) acc[u][i][j] = (f32x4){0.f, 0.f, 0.f, 0.f};
   const uint4 zero = make_uint4(0, 0, 0, 0);
   uint4 xv, wv[NB];
+  const int xrow = r0 + lr < a.rows ? (a.pair_of ? a.pair_of[r0 + lr] / a.top : r0 + lr) : -1;
   auto load = [&](int k0) {
     const int k = k0 + lc;
     const bool ink = k < a.k;  // k is a multiple of 4
-    xv = (ink && r0 + lr < a.rows) ? ldg16(a.x + (size_t)(r0 + lr) * a.ldx + k) : zero;
+    xv = (ink && xrow >= 0) ? ldg16(a.x + (size_t)xrow * a.ldx + k) : zero;
 #pragma unroll
     for (int u = 0; u < NB; ++u)
       wv[u] = (ink && c0 + lr < a.n) ? ldg16((u ? a.w2 : a.w) + (size_t)(c0 + lr) * a.k + k) : zero;
@@ -87,7 +105,8 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32Args a) {
         const int row = r0 + wr + 16 * i + 4 * g + r;
         if (row >= a.rows) continue;
         float v = acc[0][i][j][r];
-        if (SWIGLU) v = silu_x(v) * acc[NB - 1][i][j][r];
+        if (ACT == ACT_SWIGLU) v = silu_x(v) * acc[NB - 1][i][j][r];
+        if (ACT == ACT_GLU) v = clamped_glu(v, acc[NB - 1][i][j][r], a.glu.limit, a.glu.alpha, a.glu.offset);
         if (a.bias) v += a.bias[c];
         if (a.table) {
           int64_t id = a.ids[row];
@@ -109,10 +128,10 @@ extern "C" int ohara_gemm_f32(const float* x, int ldx, const float* w, const flo
   if (w_up && (bias || cap > 0.f)) return OHARA_EINVAL;
   const int64_t ny = ((int64_t)rows + GT - 1) / GT;
   if (ny > 65535) return OHARA_ESIZE;
-  const GemmF32Args a{x, w, w_up, bias, out, ldx, ldo, n, k, rows, cap, nullptr, nullptr, 0, 0};
+  const GemmF32Args a{x, w, w_up, bias, out, ldx, ldo, n, k, rows, cap, nullptr, nullptr, 0, 0, {}, nullptr, nullptr, 1, 0};
   const dim3 grid((unsigned)((n + GT - 1) / GT), (unsigned)ny);
-  if (w_up) hipLaunchKernelGGL((gemm_f32_kernel<true>), grid, dim3(256), 0, (hipStream_t)stream, a);
-  else hipLaunchKernelGGL((gemm_f32_kernel<false>), grid, dim3(256), 0, (hipStream_t)stream, a);
+  if (w_up) hipLaunchKernelGGL((gemm_f32_kernel<ACT_SWIGLU>), grid, dim3(256), 0, (hipStream_t)stream, a);
+  else hipLaunchKernelGGL((gemm_f32_kernel<ACT_NONE>), grid, dim3(256), 0, (hipStream_t)stream, a);
   return ohara_launch_status();
 }
 
@@ -122,7 +141,50 @@ extern "C" int ohara_gemm_gelu_lookup_f32(const float* x, int ldx, const float* 
   if ((k & 3) || (ldx & 3) || ldx < k || ldo < n || ldt < n) return OHARA_EINVAL;  // 16-byte loads
   const int64_t ny = ((int64_t)rows + GT - 1) / GT;
   if (ny > 65535) return OHARA_ESIZE;
-  const GemmF32Args a{x, w, nullptr, nullptr, out, ldx, ldo, n, k, rows, 0.f, table, ids, ldt, vocab};
-  hipLaunchKernelGGL((gemm_f32_kernel<false>), dim3((unsigned)((n + GT - 1) / GT), (unsigned)ny), dim3(256), 0, (hipStream_t)stream, a);
+  const GemmF32Args a{x, w, nullptr, nullptr, out, ldx, ldo, n, k, rows, 0.f, table, ids, ldt, vocab, {}, nullptr, nullptr, 1, 0};
+  hipLaunchKernelGGL((gemm_f32_kernel<ACT_NONE>), dim3((unsigned)((n + GT - 1) / GT), (unsigned)ny), dim3(256), 0, (hipStream_t)stream, a);
+  return ohara_launch_status();
+}
+
+extern "C" int ohara_gemm_glu_f32(const float* x, int ldx, const float* w_gate, const float* w_up, int n, int k, float limit, float alpha,
+                                  float offset, int rows, float* out, int ldo, void* stream) {
+  if (!x || !w_gate || !w_up || !out || n < 1 || k < 1 || rows < 1) return OHARA_EINVAL;
+  if ((k & 3) || (ldx & 3) || ldx < k || ldo < n) return OHARA_EINVAL;  // 16-byte loads
+  const int64_t ny = ((int64_t)rows + GT - 1) / GT;
+  if (ny > 65535) return OHARA_ESIZE;
+  GemmF32Args a{};
+  a.x = x; a.w = w_gate; a.w2 = w_up; a.out = out; a.ldx = ldx; a.ldo = ldo; a.n = n; a.k = k; a.rows = rows;
+  a.glu = OharaGlu{limit, alpha, offset, 0};
+  hipLaunchKernelGGL((gemm_f32_kernel<ACT_GLU>), dim3((unsigned)((n + GT - 1) / GT), (unsigned)ny), dim3(256), 0, (hipStream_t)stream, a);
+  return ohara_launch_status();
+}
+
+extern "C" int ohara_moe_glu_f32(const float* x, int ldx, const float* w_gate, const float* w_up, int n_experts, int hidden, int d,
+                                 int top, int n_pairs, const int32_t* offs, const int32_t* pair_of, const OharaGlu* glu, float* act,
+                                 int ld_act, void* stream) {
+  if (!x || !w_gate || !w_up || !offs || !pair_of || !glu || !act || n_experts < 1 || hidden < 1 || d < 1 || top < 1 || n_pairs < 1)
+    return OHARA_EINVAL;
+  if ((d & 3) || (ldx & 3) || ldx < d || ld_act < hidden) return OHARA_EINVAL;
+  const int64_t ny = ((int64_t)n_pairs + GT - 1) / GT;
+  if (ny > 65535 || n_experts > 65535) return OHARA_ESIZE;
+  GemmF32Args a{};
+  a.x = x; a.w = w_gate; a.w2 = w_up; a.out = act; a.ldx = ldx; a.ldo = ld_act; a.n = hidden; a.k = d;
+  a.glu = *glu; a.offs = offs; a.pair_of = pair_of; a.top = top; a.stride = (size_t)hidden * d;
+  hipLaunchKernelGGL((gemm_f32_kernel<ACT_GLU>), dim3((unsigned)((hidden + GT - 1) / GT), (unsigned)ny, (unsigned)n_experts), dim3(256), 0,
+                     (hipStream_t)stream, a);
+  return ohara_launch_status();
+}
+
+extern "C" int ohara_moe_down_f32(const float* act, int ld_act, const float* w, int n_experts, int d, int hidden, int n_pairs,
+                                  const int32_t* offs, float* y, int ldy, void* stream) {
+  if (!act || !w || !offs || !y || n_experts < 1 || hidden < 1 || d < 1 || n_pairs < 1) return OHARA_EINVAL;
+  if ((hidden & 3) || (ld_act & 3) || ld_act < hidden || ldy < d) return OHARA_EINVAL;
+  const int64_t ny = ((int64_t)n_pairs + GT - 1) / GT;
+  if (ny > 65535 || n_experts > 65535) return OHARA_ESIZE;
+  GemmF32Args a{};
+  a.x = act; a.w = w; a.out = y; a.ldx = ld_act; a.ldo = ldy; a.n = d; a.k = hidden; a.offs = offs; a.top = 1;
+  a.stride = (size_t)hidden * d;
+  hipLaunchKernelGGL((gemm_f32_kernel<ACT_NONE>), dim3((unsigned)((d + GT - 1) / GT), (unsigned)ny, (unsigned)n_experts), dim3(256), 0,
+                     (hipStream_t)stream, a);
   return ohara_launch_status();
 }

@@ -96,7 +96,7 @@ __global__ __launch_bounds__(NW * 64) void skinny_kernel(GemmArgs a) {
   // the weights of the whole share in one go - the rows arrive first (loads return in order), the norm's sums run
   // while the weights are still on their way, and the rows are not fetched a second time.
   constexpr int SP = 8;
-  const bool pre_ok = ((a.N | a.ldo | a.ldr | a.ldr2) & 3) == 0 && EPI != EPI_STORE && EPI != EPI_SWIGLU && EPI != EPI_SOFTCAP && EPI != EPI_GELU_LOOKUP;
+  const bool pre_ok = ((a.N | a.ldo | a.ldr | a.ldr2) & 3) == 0 && EPI != EPI_STORE && EPI != EPI_SWIGLU && EPI != EPI_SOFTCAP && EPI != EPI_GELU_LOOKUP && EPI != EPI_GLU;
   EpiPre ep[BT];
   if (wave == 0 && pre_ok) {
 #pragma unroll
@@ -472,6 +472,7 @@ int launch_epi(const GemmArgs& a, int epi, int strips, hipStream_t st) {
     case EPI_ROPE: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_ROPE>), grid, block, 0, st, a); break;
     case EPI_SOFTCAP: hipLaunchKernelGGL((skinny_kernel<BT, false, EPI_SOFTCAP>), grid, block, 0, st, a); break;  // never with a norm
     case EPI_GELU_LOOKUP: hipLaunchKernelGGL((skinny_kernel<BT, false, EPI_GELU_LOOKUP>), grid, block, 0, st, a); break;
+    case EPI_GLU: hipLaunchKernelGGL((skinny_kernel<BT, false, EPI_GLU>), grid, block, 0, st, a); break;
     case EPI_BIAS: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS>), grid, block, 0, st, a); break;
     case EPI_BIAS_GELU: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS_GELU>), grid, block, 0, st, a); break;
     case EPI_BIAS_ADD2: hipLaunchKernelGGL((skinny_kernel<BT, NORM, EPI_BIAS_ADD2>), grid, block, 0, st, a); break;
@@ -637,6 +638,18 @@ int ohara_gemm_softcap_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int 
   a.x = x; a.ldx = ldx; a.B = rows; a.N = n; a.K = k; a.out = out; a.ldo = ldo; a.cap = cap;
   if (rows > 64) return ohara_launch_gemm_tile(a, EPI_SOFTCAP, (n + 15) / 16 * 16, (hipStream_t)stream);
   return launch_skinny(a, EPI_SOFTCAP, (n + 15) / 16 * 16, (hipStream_t)stream);
+}
+
+int ohara_gemm_glu_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, float limit, float alpha, float offset,
+                        int rows, uint16_t* out, int ldo, void* stream) {
+  if (!x || !wp || !out || n < 1 || k < 1 || rows < 1) return OHARA_EINVAL;
+  if ((k & 7) || (ldx & 7) || ldx < k || ldo < n || ((n | ldo) & 1)) return OHARA_EINVAL;
+  GemmArgs a{};
+  a.wp = reinterpret_cast<const uint4*>(wp);
+  a.x = x; a.ldx = ldx; a.B = rows; a.N = n; a.K = k; a.out = out; a.ldo = ldo; a.glu = OharaGlu{limit, alpha, offset, 0};
+  const int packed_rows = 2 * ((n + 7) / 8 * 8);
+  if (rows > 64) return ohara_launch_gemm_tile(a, EPI_GLU, packed_rows, (hipStream_t)stream);
+  return launch_skinny(a, EPI_GLU, packed_rows, (hipStream_t)stream);
 }
 
 int ohara_gemm_gelu_lookup_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int n, int k, const uint16_t* table, int ldt,

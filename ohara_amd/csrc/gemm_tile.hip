@@ -223,6 +223,7 @@ int ohara_launch_gemm_tile(const GemmArgs& a, int epi, int packed_rows, hipStrea
     case EPI_PHI_IN: hipLaunchKernelGGL((gemm_tile_kernel<EPI_PHI_IN>), grid, block, 0, st, a, MT, NT, nstrips); break;
     case EPI_SOFTCAP: hipLaunchKernelGGL((gemm_tile_kernel<EPI_SOFTCAP>), grid, block, 0, st, a, MT, NT, nstrips); break;
     case EPI_GELU_LOOKUP: hipLaunchKernelGGL((gemm_tile_kernel<EPI_GELU_LOOKUP>), grid, block, 0, st, a, MT, NT, nstrips); break;
+    case EPI_GLU: hipLaunchKernelGGL((gemm_tile_kernel<EPI_GLU>), grid, block, 0, st, a, MT, NT, nstrips); break;
     default: return OHARA_EINVAL;
   }
   return ohara_launch_status();

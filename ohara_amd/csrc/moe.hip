@@ -14,7 +14,11 @@
 //   combine  out[token] = sum over its experts in ascending expert id, each add rounded to bf16
 //            (index_add_ in the activation dtype, :184), + shared expert (:206-207,219-220),
 //            + residual (ohara/models/llama.py:200)
-#include "common.h"
+//
+// The second half is a layer of another kind without a counterpart in the reference: fp32 router over experts and identity
+// outputs with groups, clamped gated units, fp32 weights.  It shares the sort and the expert kernel; its sum over the
+// chosen experts is part of the residual update (OharaMixture, residual_norm.hip).
+#include "mfma_frag.h"
 
 namespace {
 
@@ -393,7 +397,7 @@ __global__ __launch_bounds__(256) void moe_route_fused_kernel(RouteFusedArgs a) 
 }
 
 // ---- expert projections --------------------------------------------------------------------------
-enum { X_SWIGLU = 0, X_DOWN = 1 };
+enum { X_SWIGLU = 0, X_DOWN = 1, X_GLU = 2, X_RAW = 3 };  // X_GLU: clamped unit; X_RAW: X_DOWN without weights
 
 struct ExpertArgs {
   const uint4* wp;        // [E][strips][KS][64] packed rows of every expert
@@ -417,6 +421,7 @@ struct ExpertArgs {
   int N_out_sh, K_sh;
   bf16_t* out_sh;
   int ldo_sh;
+  OharaGlu glu, glu_sh;   // X_GLU
 };
 
 // CH: k-steps a wave has in flight at once (the host takes 4 when a wave's share of K is that short).
@@ -424,12 +429,13 @@ struct ExpertArgs {
 // afterwards where it lies beyond the wave's share - so the batch is one run of loads without branches.
 template <int EPI, int CH>
 __global__ __launch_bounds__(256) void moe_expert_kernel(ExpertArgs a) {
+  constexpr bool GATED = EPI == X_SWIGLU || EPI == X_GLU;
   const int strip = blockIdx.x, e = blockIdx.y;
   const bool sh = e >= a.E;  // (workgroup-uniform) a row of the shared expert: 16 tokens each
   const int p0 = sh ? (e - a.E) * 16 : a.offs[e], p1 = sh ? min(a.N_sh, p0 + 16) : a.offs[e + 1];
   if (p0 >= p1) return;
   const int N_out = sh ? a.N_out_sh : a.N_out, K = sh ? a.K_sh : a.K;
-  if (strip * 16 >= (EPI == X_SWIGLU ? 2 * ((N_out + 7) / 8 * 8) : N_out)) return;  // (the grid is as wide as the widest)
+  if (strip * 16 >= (GATED ? 2 * ((N_out + 7) / 8 * 8) : N_out)) return;  // (the grid is as wide as the widest)
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int m = lane & 15, g = lane >> 4;
   const int KS = (K + 31) >> 5;
@@ -443,9 +449,9 @@ __global__ __launch_bounds__(256) void moe_expert_kernel(ExpertArgs a) {
     const int pos = pt + m;
     const bool has = pos < p1;
     const int posc = min(pos, p1 - 1);  // a token of this expert: lanes past the end compute a column nobody stores
-    const int pair = sh ? 0 : a.pair_of[posc];
+    const int pair = sh || EPI == X_RAW ? 0 : a.pair_of[posc];
     const bf16_t* xrow = sh ? a.x_sh + (size_t)posc * a.ldx_sh
-                            : a.x + (size_t)((EPI == X_SWIGLU) ? pair / a.k : posc) * a.ldx;
+                            : a.x + (size_t)(GATED ? pair / a.k : posc) * a.ldx;
     float wt = 1.0f;  // (the shared expert's output is not scaled: a bf16 value times one is itself)
     if (EPI == X_DOWN && !sh) wt = bf2f(a.w[pair]);  // asked for here, used in the epilogue
     f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -475,7 +481,13 @@ __global__ __launch_bounds__(256) void moe_expert_kernel(ExpertArgs a) {
     if (wave == 0) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) acc[i] = ((acc[i] + red[0][lane][i]) + red[1][lane][i]) + red[2][lane][i];
-      if (has) {
+      if (has && EPI == X_GLU) {
+        const OharaGlu u = sh ? a.glu_sh : a.glu;
+        const int f = strip * 8 + 2 * g;
+        bf16_t* o = outp + (size_t)pos * ldo + f;
+        if (f < N_out) o[0] = f2bf(clamped_glu(acc[0], acc[2], u.limit, u.alpha, u.offset));
+        if (f + 1 < N_out) o[1] = f2bf(clamped_glu(acc[1], acc[3], u.limit, u.alpha, u.offset));
+      } else if (has) {
         const float y0 = rbf(acc[0]), y1 = rbf(acc[1]), y2 = rbf(acc[2]), y3 = rbf(acc[3]);
         if (EPI == X_SWIGLU) {
           const int f = strip * 8 + 2 * g;
@@ -494,6 +506,413 @@ __global__ __launch_bounds__(256) void moe_expert_kernel(ExpertArgs a) {
     }
     __syncthreads();
   }
+}
+
+// ---- fp32 router, groups, identity outputs -------------------------------------------------------
+template <typename T>
+struct RouterArgs {
+  const T* x;
+  const T* w;
+  const float* correction;
+  int ldx, ldw, N, K, E, top, groups, keep;  // E: outputs (experts and identities)
+  int32_t* idx;
+  float* wgt;
+  int32_t* offs;   // sort: the workgroup that finishes last sorts the pairs of all tokens (E <= 64, at most 1024 pairs)
+  int32_t* pair_of;
+  int32_t* pos_of;
+  int* counter;
+  int sort;
+};
+
+constexpr int RT = 16;  // tokens of a workgroup
+
+// The products of 16 tokens with all router rows, 64 rows at a time with K split over the four waves; then four tokens per wave,
+// lane l looking at outputs l, l + 64, ...
+template <typename T, int MAXPL>
+__global__ __launch_bounds__(256) void moe_router_kernel(RouterArgs<T> a) {
+  extern __shared__ __align__(16) float zs[];  // [RT][E]
+  __shared__ float red[4][4][64][4];
+  __shared__ int wcnt[16][64];
+  __shared__ int is_last;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 15, g = lane >> 4;
+  const int t0 = blockIdx.x * RT, KS = (a.K + 31) >> 5;
+  const T* xr = a.x + (size_t)min(t0 + m, a.N - 1) * a.ldx + 8 * g;
+  for (int e0 = 0; e0 < a.E; e0 += 64) {
+    f32x4 acc[4];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) acc[s] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const T* wr[4];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) wr[s] = a.w + (size_t)min(e0 + 16 * s + m, a.E - 1) * a.ldw + 8 * g;
+    constexpr int CH = sizeof(T) == 2 ? 4 : 2;  // steps whose loads are issued together
+    for (int jb = wave; jb < KS; jb += 4 * CH) {
+      Frag<T> xf[CH], wf[CH][4];
+#pragma unroll
+      for (int c = 0; c < CH; ++c) {
+        const int j = jb + 4 * c;
+        const bool in = 32 * j + 8 * g < a.K;  // K is a multiple of 8
+        if (in) frag_load(xf[c], xr + 32 * j);
+        else frag_zero(xf[c]);
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+          if (in) frag_load(wf[c][s], wr[s] + 32 * j);
+          else frag_zero(wf[c][s]);
+        }
+      }
+#pragma unroll
+      for (int c = 0; c < CH; ++c)
+#pragma unroll
+        for (int s = 0; s < 4; ++s) acc[s] = mma(wf[c][s], xf[c], acc[s]);
+    }
+    if (e0) __syncthreads();
+#pragma unroll
+    for (int s = 0; s < 4; ++s)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) red[wave][s][lane][i] = acc[s][i];
+    __syncthreads();
+    // wave s finishes rows 16 s .. : lane (token m, rows 4 g ..)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int e = e0 + 16 * wave + 4 * g + i;
+      if (e < a.E)
+        zs[m * a.E + e] = ((red[0][wave][lane][i] + red[1][wave][lane][i]) + red[2][wave][lane][i]) + red[3][wave][lane][i];
+    }
+  }
+  __syncthreads();
+  const int per = a.E / a.groups;
+  for (int tt = 0; tt < RT / 4; ++tt) {
+    const int t = (RT / 4) * wave + tt, n = t0 + t;
+    float* z = zs + t * a.E;
+    float s[MAXPL], ch[MAXPL], mx = -INFINITY, sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < MAXPL; ++i) {
+      const int e = 64 * i + lane;
+      s[i] = e < a.E ? z[e] : -INFINITY;
+      mx = fmaxf(mx, s[i]);
+    }
+    mx = wave_max(mx);
+#pragma unroll
+    for (int i = 0; i < MAXPL; ++i) {
+      s[i] = 64 * i + lane < a.E ? expf(s[i] - mx) : 0.f;
+      sum += s[i];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < MAXPL; ++i) {
+      const int e = 64 * i + lane;
+      s[i] /= sum;
+      ch[i] = e < a.E ? s[i] + (a.correction ? a.correction[e] : 0.f) : -INFINITY;
+      if (!(ch[i] == ch[i])) ch[i] = -INFINITY;  // a padding row may hold anything: every row still picks distinct outputs
+    }
+    if (a.groups > 1) {  // the same for all waves
+#pragma unroll
+      for (int i = 0; i < MAXPL; ++i)
+        if (64 * i + lane < a.E) z[64 * i + lane] = ch[i];
+      __syncthreads();
+      float best = -INFINITY;  // of group `lane`
+      if (lane < a.groups)
+        for (int e = lane * per; e < (lane + 1) * per; ++e) best = fmaxf(best, z[e]);
+      int rank = 0;
+      for (int o = 0; o < a.groups; ++o) {
+        const float v = __uint_as_float((uint32_t)__builtin_amdgcn_readlane((int)__float_as_uint(best), o));
+        rank += v > best || (v == best && o < lane) ? 1 : 0;
+      }
+      const unsigned long long open = __ballot(lane < a.groups && rank < a.keep);
+#pragma unroll
+      for (int i = 0; i < MAXPL; ++i) {
+        const int e = 64 * i + lane;
+        if (e < a.E && !((open >> (e / per)) & 1ull)) ch[i] = -INFINITY;
+      }
+    }
+    // the best `top`, winner j kept by lane j
+    uint32_t taken = 0;
+    int my_id = 0;
+    float my_s = 0.f;
+    for (int j = 0; j < a.top; ++j) {
+      float bv = -INFINITY;
+      int bi = 0x7fffffff;
+#pragma unroll
+      for (int i = 0; i < MAXPL; ++i) {
+        const int e = 64 * i + lane;
+        if (e < a.E && !((taken >> i) & 1u) && (ch[i] > bv || bi == 0x7fffffff)) {
+          bv = ch[i];
+          bi = e;
+        }
+      }
+      lane_xor_argmax<32>(bv, bi);
+      lane_xor_argmax<16>(bv, bi);
+      lane_xor_argmax<8>(bv, bi);
+      lane_xor_argmax<4>(bv, bi);
+      lane_xor_argmax<2>(bv, bi);
+      lane_xor_argmax<1>(bv, bi);
+      float r = 0.f;
+#pragma unroll
+      for (int i = 0; i < MAXPL; ++i)
+        if (64 * i + lane == bi) {
+          r = s[i];
+          taken |= 1u << i;
+        }
+      r = __uint_as_float((uint32_t)__builtin_amdgcn_readlane((int)__float_as_uint(r), bi & 63));
+      if (lane == j) {
+        my_s = r;
+        my_id = bi;
+      }
+    }
+    float tot = 0.f;
+    for (int j = 0; j < a.top; ++j) tot += __uint_as_float((uint32_t)__builtin_amdgcn_readlane((int)__float_as_uint(my_s), j));
+    if (n < a.N && lane < a.top) {
+      st_coh4(a.idx + (size_t)n * a.top + lane, (uint32_t)my_id);  // (read by the workgroup that sorts)
+      a.wgt[(size_t)n * a.top + lane] = my_s / (tot + 1e-20f);
+    }
+  }
+  if (!a.sort) return;
+  wait_own_stores();
+  __syncthreads();
+  if (tid == 0) {
+    const int old = __hip_atomic_fetch_add(a.counter, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    is_last = old == (int)gridDim.x - 1;
+    if (is_last) __hip_atomic_store(a.counter, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // ready for the next call
+  }
+  __syncthreads();
+  if (is_last) sort_small_256(a.idx, a.N * a.top, a.E, a.offs, a.pair_of, a.pos_of, wcnt);
+}
+
+// The sort for many pairs on many workgroups: counts of every block of 1024 pairs, then every block places its own.
+__global__ __launch_bounds__(1024) void moe_count_kernel(const int32_t* idx, int NK, int E, int32_t* hist) {
+  __shared__ int cnt[1024];
+  const int tid = threadIdx.x, p = blockIdx.x * 1024 + tid;
+  cnt[tid] = 0;
+  __syncthreads();
+  if (p < NK) atomicAdd(&cnt[idx[p]], 1);
+  __syncthreads();
+  if (tid < E) hist[(size_t)blockIdx.x * E + tid] = cnt[tid];
+}
+__global__ __launch_bounds__(1024) void moe_place_kernel(const int32_t* idx, int NK, int E, const int32_t* hist, int32_t* offs,
+                                                         int32_t* pair_of, int32_t* pos_of) {
+  __shared__ int first[1024];  // sorted position of this block's first pair of every expert
+  __shared__ int wsum[16];
+  __shared__ __align__(16) int sidx[1024];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, blk = blockIdx.x, nb = gridDim.x;
+  int total = 0, before = 0;
+  if (tid < E)
+    for (int b = 0; b < nb; ++b) {
+      const int c = hist[(size_t)b * E + tid];
+      total += c;
+      before += b < blk ? c : 0;
+    }
+  const int incl = wave_incl_scan_i(total);
+  if (lane == 63) wsum[wave] = incl;
+  const int p = blk * 1024 + tid, e = p < NK ? idx[p] : -1;
+  sidx[tid] = e;
+  __syncthreads();
+  int run = incl - total;
+  for (int w = 0; w < wave; ++w) run += wsum[w];
+  if (tid < E) first[tid] = run + before;
+  if (blk == 0) {
+    if (tid < E) offs[tid] = run;
+    if (tid == E - 1) offs[E] = run + total;
+  }
+  __syncthreads();
+  // pairs before this one with the same expert: a wave scans the entries below its last lane
+  const int wave_first = tid & ~63;
+  const int n4 = blk * 1024 + wave_first < NK ? (min(wave_first + 64, NK - blk * 1024) + 3) >> 2 : 0;
+  int rank = 0;
+  const int4* s4 = reinterpret_cast<const int4*>(sidx);
+#pragma unroll 4
+  for (int t4 = 0; t4 < n4; ++t4) {
+    const int4 v = s4[t4];
+    const int t = 4 * t4;
+    rank += (t < tid && v.x == e) + (t + 1 < tid && v.y == e) + (t + 2 < tid && v.z == e) + (t + 3 < tid && v.w == e);
+  }
+  if (e >= 0) {
+    const int o = first[e] + rank;
+    pair_of[o] = p;
+    pos_of[p] = o;
+  }
+}
+
+// ---- many pairs: tiles of 128 pairs of one expert x 128 packed weight rows -----------------------------
+// The structure of gemm_tile_kernel: weights straight from the packed layout, the activation rows (gathered by pair, or by
+// sorted position) through LDS, double-buffered.
+struct ExpertTileArgs {
+  const uint4* wp;
+  size_t expert_stride;   // uint4 per expert
+  const bf16_t* x;
+  int ldx;
+  const int32_t* offs;
+  const int32_t* pair_of;
+  int top, E, N_out, K;
+  bf16_t* out;
+  int ldo;
+  OharaGlu glu;
+};
+
+template <int EPI>
+__global__ __launch_bounds__(256, 2) void moe_tile_kernel(ExpertTileArgs a, int NT, int nstrips) {
+  constexpr int TM = 128, TS = 8, KB = 64, LDX = KB + 8;
+  __shared__ __align__(16) bf16_t xs[2][TM][LDX];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 15, g = lane >> 4;
+  const int xcd = blockIdx.x & 7, q = blockIdx.x >> 3;
+  const int tn = q % NT;
+  int tile = (q / NT) * 8 + xcd, e = 0;  // the tile-th tile of pairs: which expert's
+  {
+    bool found = false;
+    for (int e0 = 0; e0 < a.E && !found; e0 += 64) {  // the same for all waves
+      const int c = e0 + lane < a.E ? (a.offs[e0 + lane + 1] - a.offs[e0 + lane] + TM - 1) / TM : 0;
+      const int incl = wave_incl_scan_i(c);
+      const unsigned long long past = __ballot(incl > tile);
+      if (past) {
+        const int l = __ffsll((long long)past) - 1;
+        tile -= __builtin_amdgcn_readlane(incl - c, l);
+        e = e0 + l;
+        found = true;
+      } else {
+        tile -= __builtin_amdgcn_readlane(incl, 63);
+      }
+    }
+    if (!found) return;
+  }
+  const int row0 = a.offs[e] + tile * TM, rows = min(TM, a.offs[e + 1] - row0);
+  const int strip0 = tn * TS + wave * 2, KS = (a.K + 31) >> 5, nsteps = (KS + 1) >> 1;
+  const int lr = tid >> 3, lc = (tid & 7) * 8;
+  const bf16_t* xp[4];
+#pragma unroll
+  for (int p = 0; p < 4; ++p) {
+    const int r = row0 + min(p * 32 + lr, rows - 1);
+    xp[p] = a.x + (size_t)(EPI == X_GLU ? a.pair_of[r] / a.top : r) * a.ldx;
+  }
+  auto load_x = [&](int step, uint4* xr) {
+    const int k = step * KB + lc;
+#pragma unroll
+    for (int p = 0; p < 4; ++p) xr[p] = k < a.K ? ldg16(xp[p] + k) : make_uint4(0, 0, 0, 0);
+  };
+  auto store_x = [&](int buf, const uint4* xr) {
+#pragma unroll
+    for (int p = 0; p < 4; ++p) *reinterpret_cast<uint4*>(&xs[buf][p * 32 + lr][lc]) = xr[p];
+  };
+  const uint4* w0 = a.wp + (size_t)e * a.expert_stride + (size_t)strip0 * KS * 64 + lane;
+  const uint4* w1 = w0 + (size_t)KS * 64;
+  const bool live0 = strip0 < nstrips, live1 = strip0 + 1 < nstrips;
+  auto load_w = [&](int step, uint4* wv) {
+    const int j = step * 2;
+    wv[0] = (live0 && j < KS) ? ldg16(w0 + (size_t)j * 64) : make_uint4(0, 0, 0, 0);
+    wv[1] = (live0 && j + 1 < KS) ? ldg16(w0 + (size_t)(j + 1) * 64) : make_uint4(0, 0, 0, 0);
+    wv[2] = (live1 && j < KS) ? ldg16(w1 + (size_t)j * 64) : make_uint4(0, 0, 0, 0);
+    wv[3] = (live1 && j + 1 < KS) ? ldg16(w1 + (size_t)(j + 1) * 64) : make_uint4(0, 0, 0, 0);
+  };
+  f32x4 acc[2][8];
+#pragma unroll
+  for (int u = 0; u < 2; ++u)
+#pragma unroll
+    for (int t = 0; t < 8; ++t) acc[u][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  uint4 xr[4], wv[4], wn[4];
+  load_x(0, xr);
+  load_w(0, wv);
+  store_x(0, xr);
+  __syncthreads();
+  for (int s = 0; s < nsteps; ++s) {
+    const int buf = s & 1;
+    const bool more = s + 1 < nsteps;
+    if (more) {
+      load_x(s + 1, xr);
+      load_w(s + 1, wn);
+    }
+#pragma unroll
+    for (int jj = 0; jj < 2; ++jj) {
+      uint4 bv[8];
+#pragma unroll
+      for (int t = 0; t < 8; ++t) bv[t] = *reinterpret_cast<const uint4*>(&xs[buf][t * 16 + m][jj * 32 + 8 * g]);
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int t = 0; t < 8; ++t) {
+        acc[0][t] = mma_bf(wv[jj], bv[t], acc[0][t]);
+        acc[1][t] = mma_bf(wv[2 + jj], bv[t], acc[1][t]);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    if (more) {
+      store_x(buf ^ 1, xr);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) wv[i] = wn[i];
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    const int strip = strip0 + u;
+    if (strip >= nstrips) continue;
+#pragma unroll
+    for (int t = 0; t < 8; ++t) {
+      if (t * 16 + m >= rows) continue;
+      bf16_t* o = a.out + (size_t)(row0 + t * 16 + m) * a.ldo;
+      const f32x4 c = acc[u][t];
+      if (EPI == X_GLU) {  // N_out and ldo are multiples of 8
+        const int f = strip * 8 + 2 * g;
+        if (f < a.N_out)
+          *reinterpret_cast<uint32_t*>(o + f) = pack_bf(clamped_glu(c[0], c[2], a.glu.limit, a.glu.alpha, a.glu.offset),
+                                                        clamped_glu(c[1], c[3], a.glu.limit, a.glu.alpha, a.glu.offset));
+      } else {
+        const int f = strip * 16 + 4 * g;
+        if (f < a.N_out) *reinterpret_cast<uint2*>(o + f) = make_uint2(pack_bf(c[0], c[1]), pack_bf(c[2], c[3]));
+      }
+    }
+  }
+}
+
+constexpr int TILE_PAIRS = 64;  // pairs per expert, on average, from which tiles beat streaming the weights per 16 pairs
+
+template <typename T>
+int launch_router(RouterArgs<T> a, int32_t* hist, hipStream_t st) {
+  if (!a.x || !a.w || !a.idx || !a.wgt || !a.offs || !a.pair_of || !a.pos_of || !a.counter) return OHARA_EINVAL;
+  if (a.N < 1 || a.K < 8 || (a.K & 7) || a.ldx < a.K || a.ldw < a.K || ((a.ldx | a.ldw) & 7) || a.E < 1) return OHARA_EINVAL;
+  if (a.top < 1 || a.top > a.E || a.groups < 1 || a.E % a.groups || a.keep < 1 || a.keep > a.groups) return OHARA_EINVAL;
+  if (a.keep * (a.E / a.groups) < a.top) return OHARA_EINVAL;
+  if (a.E > 1024 || a.top > 64 || a.groups > 64 || (int64_t)a.N * a.top > (1 << 30)) return OHARA_ESIZE;
+  const int NK = a.N * a.top;
+  a.sort = a.E <= 64 && NK <= 1024;
+  if (!a.sort && !hist) return OHARA_EINVAL;
+  const dim3 grid((unsigned)((a.N + RT - 1) / RT)), block(256);
+  const size_t smem = (size_t)RT * a.E * sizeof(float);
+  auto go = [&](auto kernel) {
+    if (smem > 32 * 1024) (void)hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+    hipLaunchKernelGGL(kernel, grid, block, smem, st, a);
+  };
+  if (a.E <= 64) go(moe_router_kernel<T, 1>);
+  else if (a.E <= 256) go(moe_router_kernel<T, 4>);
+  else go(moe_router_kernel<T, 16>);
+  if (!a.sort) {
+    const dim3 blocks((unsigned)((NK + 1023) / 1024));
+    hipLaunchKernelGGL(moe_count_kernel, blocks, dim3(1024), 0, st, a.idx, NK, a.E, hist);
+    hipLaunchKernelGGL(moe_place_kernel, blocks, dim3(1024), 0, st, a.idx, NK, a.E, hist, a.offs, a.pair_of, a.pos_of);
+  }
+  return ohara_launch_status();
+}
+
+template <int EPI>
+int launch_experts(ExpertArgs a, int n_pairs, int n_sh, hipStream_t st) {
+  constexpr bool GATED = EPI == X_GLU;
+  auto strips_of = [](int n) { return GATED ? 2 * ((n + 7) / 8 * 8) / 16 : (n + 15) / 16; };
+  int strips = strips_of(a.N_out);
+  if (n_pairs >= TILE_PAIRS * a.E && !n_sh) {
+    const ExpertTileArgs t{a.wp, a.expert_stride, a.x, a.ldx, a.offs, a.pair_of, a.k, a.E, a.N_out, a.K, a.out, a.ldo, a.glu};
+    const int NT = (strips + 7) / 8;
+    const int64_t tiles = (n_pairs + 127) / 128 + a.E, blocks = (tiles + 7) / 8 * 8 * NT;
+    if (blocks > INT32_MAX) return OHARA_ESIZE;
+    hipLaunchKernelGGL((moe_tile_kernel<EPI>), dim3((unsigned)blocks), dim3(256), 0, st, t, NT, strips);
+    return ohara_launch_status();
+  }
+  int rows = a.E, ks = (a.K + 31) / 32;
+  if (n_sh) {
+    const int s2 = strips_of(a.N_out_sh), k2 = (a.K_sh + 31) / 32;
+    strips = strips > s2 ? strips : s2;
+    ks = ks > k2 ? ks : k2;
+    rows += (n_sh + 15) / 16;
+  }
+  if (rows > 65535) return OHARA_ESIZE;
+  const dim3 grid((unsigned)strips, (unsigned)rows);
+  if (ks <= 16) hipLaunchKernelGGL((moe_expert_kernel<EPI, 4>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((moe_expert_kernel<EPI, 8>), grid, dim3(256), 0, st, a);
+  return ohara_launch_status();
 }
 
 // ---- combine ---------------------------------------------------------------------------------------
@@ -683,6 +1102,59 @@ int ohara_moe_combine(const uint16_t* y, int ldy, const int32_t* expert_idx, con
   hipLaunchKernelGGL(moe_combine_kernel, dim3(n_tokens), dim3(256), 0, (hipStream_t)stream, y, ldy, expert_idx, pos_of, k,
                      shared, ld_shared, resid, ldr, out, ldo, d);
   return ohara_launch_status();
+}
+
+int ohara_moe_router_bf16(const uint16_t* x, int ldx, const uint16_t* w, int ldw, const float* correction, int rows, int k, int n_out,
+                          int top, int groups, int keep, int32_t* idx, float* wgt, int32_t* offs, int32_t* pair_of,
+                          int32_t* pos_of, int32_t* hist, int32_t* counter, void* stream) {
+  return launch_router<bf16_t>(RouterArgs<bf16_t>{x, w, correction, ldx, ldw, rows, k, n_out, top, groups, keep, idx, wgt, offs,
+                                                  pair_of, pos_of, counter, 0}, hist, (hipStream_t)stream);
+}
+int ohara_moe_router_f32(const float* x, int ldx, const float* w, int ldw, const float* correction, int rows, int k, int n_out,
+                         int top, int groups, int keep, int32_t* idx, float* wgt, int32_t* offs, int32_t* pair_of,
+                         int32_t* pos_of, int32_t* hist, int32_t* counter, void* stream) {
+  return launch_router<float>(RouterArgs<float>{x, w, correction, ldx, ldw, rows, k, n_out, top, groups, keep, idx, wgt, offs,
+                                                pair_of, pos_of, counter, 0}, hist, (hipStream_t)stream);
+}
+
+int ohara_moe_glu_bf16(const uint16_t* x, int ldx, const uint16_t* wp, int64_t expert_stride_bytes, int n_experts, int hidden, int d,
+                       int top, int n_pairs, const int32_t* offs, const int32_t* pair_of, const OharaGlu* glu, uint16_t* act,
+                       int ld_act, const uint16_t* wp_shared, int hidden_shared, int n_tokens, const OharaGlu* glu_shared,
+                       uint16_t* act_shared, int ld_act_shared, void* stream) {
+  if (!x || !wp || !offs || !pair_of || !glu || !act || n_experts < 1 || top < 1 || n_pairs < 1) return OHARA_EINVAL;
+  if (d < 8 || hidden < 8 || ((d | hidden | ldx | ld_act) & 7) || ldx < d || ld_act < hidden) return OHARA_EINVAL;
+  ExpertArgs a{};
+  a.wp = reinterpret_cast<const uint4*>(wp); a.expert_stride = (size_t)expert_stride_bytes / 16;
+  a.x = x; a.ldx = ldx; a.offs = offs; a.pair_of = pair_of; a.k = top; a.N_out = hidden; a.K = d;
+  a.out = act; a.ldo = ld_act; a.E = n_experts; a.glu = *glu;
+  int n_sh = 0;
+  if (wp_shared) {
+    if (!act_shared || !glu_shared || n_tokens < 1 || hidden_shared < 8 || (hidden_shared & 7) || ld_act_shared < hidden_shared)
+      return OHARA_EINVAL;
+    a.N_sh = n_sh = n_tokens; a.wp_sh = reinterpret_cast<const uint4*>(wp_shared); a.x_sh = x; a.ldx_sh = ldx;
+    a.N_out_sh = hidden_shared; a.K_sh = d; a.out_sh = act_shared; a.ldo_sh = ld_act_shared; a.glu_sh = *glu_shared;
+  }
+  return launch_experts<X_GLU>(a, n_pairs, n_sh, (hipStream_t)stream);
+}
+
+int ohara_moe_down_bf16(const uint16_t* act, int ld_act, const uint16_t* wp, int64_t expert_stride_bytes, int n_experts, int d,
+                        int hidden, int n_pairs, const int32_t* offs, uint16_t* y, int ldy, const uint16_t* wp_shared,
+                        int hidden_shared, int n_tokens, const uint16_t* act_shared, int ld_act_shared, uint16_t* y_shared,
+                        int ldy_shared, void* stream) {
+  if (!act || !wp || !offs || !y || n_experts < 1 || n_pairs < 1) return OHARA_EINVAL;
+  if (d < 8 || hidden < 8 || ((d | hidden | ld_act) & 7) || (ldy & 3) || ld_act < hidden || ldy < d) return OHARA_EINVAL;
+  ExpertArgs a{};
+  a.wp = reinterpret_cast<const uint4*>(wp); a.expert_stride = (size_t)expert_stride_bytes / 16;
+  a.x = act; a.ldx = ld_act; a.offs = offs; a.k = 1; a.N_out = d; a.K = hidden; a.out = y; a.ldo = ldy; a.E = n_experts;
+  int n_sh = 0;
+  if (wp_shared) {
+    if (!act_shared || !y_shared || n_tokens < 1 || hidden_shared < 8 || ((hidden_shared | ld_act_shared) & 7) ||
+        ld_act_shared < hidden_shared || ldy_shared < d)
+      return OHARA_EINVAL;
+    a.N_sh = n_sh = n_tokens; a.wp_sh = reinterpret_cast<const uint4*>(wp_shared); a.x_sh = act_shared; a.ldx_sh = ld_act_shared;
+    a.N_out_sh = d; a.K_sh = hidden_shared; a.out_sh = y_shared; a.ldo_sh = ldy_shared;
+  }
+  return launch_experts<X_RAW>(a, n_pairs, n_sh, (hipStream_t)stream);
 }
 
 }  // extern "C"

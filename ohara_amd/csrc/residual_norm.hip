@@ -21,9 +21,43 @@ struct ResidualArgs {
   float* ring;
   int d, vocab, ldy, groups, ldo, mode, taps;
   int center_y, center_out;  // norm of y / of the output: layer norm (the mean is taken off first) instead of RMS
-  float eps;
+  float eps, table_scale;
+  OharaMixture mix;          // top > 0: its rows instead of y's
   OharaSeq seq;
 };
+
+// V columns from i on of a mixture's row, four of its terms in flight
+template <typename T, int V>
+__device__ __forceinline__ void mixture(const OharaMixture& q, int row, int i, float* v) {
+  auto load = [](const T* p, float* o) {
+    if constexpr (V == 4) ld4(p, o);
+    else o[0] = ldv(p);
+  };
+#pragma unroll
+  for (int u = 0; u < V; ++u) v[u] = 0.f;
+  float sh[V];
+  if (q.shared) load((const T*)q.shared + (size_t)row * q.lds + i, sh);
+  for (int j0 = 0; j0 < q.top; j0 += 4) {
+    float t[4][V], w[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int n = row * q.top + min(j0 + j, q.top - 1);
+      const bool real = q.idx[n] < q.experts;
+      w[j] = j0 + j < q.top ? q.w[n] : 0.f;
+      load(real ? (const T*)q.y + (size_t)q.pos_of[n] * q.ldy + i : (const T*)q.h + (size_t)row * q.ldh + i, t[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j0 + j < q.top) {
+#pragma unroll
+        for (int u = 0; u < V; ++u) v[u] += w[j] * t[j][u];
+      }
+  }
+  if (q.shared) {
+#pragma unroll
+    for (int u = 0; u < V; ++u) v[u] += sh[u];
+  }
+}
 
 // Takes the row's mean off a row in LDS (layer norms: one group).  Ends with a barrier.
 __device__ __forceinline__ void center_row(float* row, int d, float* red) {
@@ -86,21 +120,25 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualArgs<T> a) {
     if (id < 0 || id >= a.vocab) id = 0;  // the host validates ids; never read out of bounds
     const T* src = a.table + (size_t)id * d;
     for (int i = tid; i < d; i += 256) {
-      const float v = ldv(src + i);
+      const float v = a.table_scale * ldv(src + i);
       ys[i] = v;
       xr[i] = v;
     }
     __syncthreads();
-  } else if (a.y) {
+  } else if (a.y || a.mix.top) {
     const T* yr = a.y + (size_t)row * a.ldy;
     if (VEC) {
       for (int i = tid * 4; i < d; i += 1024) {
         float v[4];
-        ld4(yr + i, v);
+        if (a.mix.top) mixture<T, 4>(a.mix, row, i, v);
+        else ld4(yr + i, v);
         *reinterpret_cast<float4*>(ys + i) = make_float4(v[0], v[1], v[2], v[3]);
       }
     } else {
-      for (int i = tid; i < d; i += 256) ys[i] = ldv(yr + i);
+      for (int i = tid; i < d; i += 256) {
+        if (a.mix.top) mixture<T, 1>(a.mix, row, i, ys + i);
+        else ys[i] = ldv(yr + i);
+      }
     }
     __syncthreads();
     if (a.center_y) center_row(ys, d, red);
@@ -163,14 +201,14 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualArgs<T> a) {
 // The same for rows of at most 1024 * NP columns (all sizes multiples of 4): a thread owns NP pieces of four columns and
 // keeps them in registers, and everything that does not depend on the norm - residual, weights, the convolution's past
 // inputs (MT: taps at most) - is requested before the sums.  One round trip instead of four.
-template <typename T, int NP, int MT>
+template <typename T, int NP, int MT, bool MIX = false>
 __global__ __launch_bounds__(256) void residual_norm_regs_kernel(ResidualArgs<T> a) {
   extern __shared__ __align__(16) float smem[];  // groups > 1: a partial sum per piece, then 1 / rms per group
   __shared__ float red[4][4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, row = blockIdx.x, d = a.d;
   const int gs4 = d / a.groups / 4;  // pieces per group
   float* xr = a.x + (size_t)row * d;
-  const bool add = !a.ids && a.y;
+  const bool add = !a.ids && (MIX || a.y);
   float x[NP][4], y[NP][4], w[NP][4], past[NP][MT][4], cw[NP][MT][4];
   int64_t id = 0;
   if (a.ids) {
@@ -191,10 +229,16 @@ __global__ __launch_bounds__(256) void residual_norm_regs_kernel(ResidualArgs<T>
 #pragma unroll
     for (int u = 0; u < 4; ++u) x[p][u] = y[p][u] = w[p][u] = zero[u];
     if (!in) continue;
-    if (a.ids) ld4(a.table + (size_t)id * d + i, x[p]);
-    else ld4(xr + i, x[p]);
+    if (a.ids) {
+      ld4(a.table + (size_t)id * d + i, x[p]);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) x[p][u] *= a.table_scale;
+    } else {
+      ld4(xr + i, x[p]);
+    }
     if (add) {
-      ld4(a.y + (size_t)row * a.ldy + i, y[p]);
+      if constexpr (MIX) mixture<T, 4>(a.mix, row, i, y[p]);
+      else ld4(a.y + (size_t)row * a.ldy + i, y[p]);
       ld4(a.norm_w + i, w[p]);
     }
     if (MT > 1) {
@@ -371,7 +415,15 @@ __global__ __launch_bounds__(256) void ring_store_kernel(const T* src, int ld, i
 }
 
 template <typename T>
-int launch_residual(ResidualArgs<T> a, const OharaSeq* seq, hipStream_t st) {
+int launch_residual(ResidualArgs<T> a, const OharaMixture* mix, const OharaSeq* seq, hipStream_t st) {
+  if (mix) {
+    a.mix = *mix;
+    if (a.ids || a.y || mix->top < 1 || !mix->w || !mix->idx || !mix->pos_of || !mix->y || !mix->h || mix->experts < 1) return OHARA_EINVAL;
+    if (mix->ldy < a.d || mix->ldh < a.d || (mix->shared && mix->lds < a.d)) return OHARA_EINVAL;
+    if ((mix->ldy | mix->ldh | mix->lds) & 3) return OHARA_EINVAL;
+    if (!a.norm_w) return OHARA_EINVAL;
+    a.ldy = 0;  // not read
+  }
   a.center_y = (a.mode & OHARA_CENTER_Y) != 0;
   a.center_out = (a.mode & OHARA_CENTER_OUT) != 0;
   a.mode &= ~(OHARA_CENTER_Y | OHARA_CENTER_OUT);
@@ -389,10 +441,16 @@ int launch_residual(ResidualArgs<T> a, const OharaSeq* seq, hipStream_t st) {
   const dim3 grid((unsigned)(seq->batch * seq->seq_len));
   const bool vec = (a.d & 3) == 0 && ((a.d / a.groups) & 3) == 0 && (a.ldy & 3) == 0 && (a.ldo & 3) == 0;
   const bool conv = a.mode == OHARA_OUT_CONV;
-  if (vec && a.d <= 4096 && (!conv || a.taps <= 4)) {
+  if (vec && a.d <= 4096 && (!conv || (a.taps <= 4 && !mix))) {
     auto regs = [&](auto kernel, int np) {
       hipLaunchKernelGGL(kernel, grid, dim3(256), a.groups > 1 ? (256 * np + a.groups) * sizeof(float) : 0, st, a);
     };
+    if (mix && !conv) {
+      if (a.d <= 1024) regs(residual_norm_regs_kernel<T, 1, 1, true>, 1);
+      else if (a.d <= 2048) regs(residual_norm_regs_kernel<T, 2, 1, true>, 2);
+      else regs(residual_norm_regs_kernel<T, 4, 1, true>, 4);
+      return ohara_launch_status();
+    }
     if (a.d <= 1024) conv ? regs(residual_norm_regs_kernel<T, 1, 4>, 1) : regs(residual_norm_regs_kernel<T, 1, 1>, 1);
     else if (a.d <= 2048) conv ? regs(residual_norm_regs_kernel<T, 2, 4>, 2) : regs(residual_norm_regs_kernel<T, 2, 1>, 2);
     else conv ? regs(residual_norm_regs_kernel<T, 4, 4>, 4) : regs(residual_norm_regs_kernel<T, 4, 1>, 4);
@@ -430,19 +488,19 @@ int launch_ring_store(const T* src, int ld, int channels, int taps, T* ring, con
 
 extern "C" {
 
-int ohara_residual_norm_bf16(float* x, int d, const int64_t* ids, const uint16_t* table, int vocab, const uint16_t* y,
+int ohara_residual_norm_bf16(float* x, int d, const int64_t* ids, const uint16_t* table, int vocab, float table_scale, const uint16_t* y,
                              int ldy, const float* norm_w, int groups, float eps, int out_mode, uint16_t* out, int ldo,
-                             const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
+                             const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaMixture* mix, const OharaSeq* seq,
                              void* stream) {
   return launch_residual<bf16_t>(ResidualArgs<bf16_t>{x, ids, table, y, norm_w, out, norm2_w, conv_w, ring, d, vocab, ldy,
-                                                      groups, ldo, out_mode, taps, 0, 0, eps, {}}, seq, (hipStream_t)stream);
+                                                      groups, ldo, out_mode, taps, 0, 0, eps, table_scale, {}, {}}, mix, seq, (hipStream_t)stream);
 }
-int ohara_residual_norm_f32(float* x, int d, const int64_t* ids, const float* table, int vocab, const float* y, int ldy,
+int ohara_residual_norm_f32(float* x, int d, const int64_t* ids, const float* table, int vocab, float table_scale, const float* y, int ldy,
                             const float* norm_w, int groups, float eps, int out_mode, float* out, int ldo,
-                            const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaSeq* seq,
+                            const float* norm2_w, const float* conv_w, int taps, float* ring, const OharaMixture* mix, const OharaSeq* seq,
                             void* stream) {
   return launch_residual<float>(ResidualArgs<float>{x, ids, table, y, norm_w, out, norm2_w, conv_w, ring, d, vocab, ldy, groups,
-                                                    ldo, out_mode, taps, 0, 0, eps, {}}, seq, (hipStream_t)stream);
+                                                    ldo, out_mode, taps, 0, 0, eps, table_scale, {}, {}}, mix, seq, (hipStream_t)stream);
 }
 
 int ohara_input_conv_bf16(const float* x, int d, const float* conv_w, int taps, const float* ring, uint16_t* out, int ldo,

@@ -3,17 +3,21 @@
 Every class is one mechanism with its sizes and constants as constructor arguments; none knows a model's
 config keys or tensor names.  A mixer offers ``state(rows, max_seq_length)`` (the tensors it keeps per sequence) and
 ``__call__(h, state, seq)`` with h the (rows, width rounded up to 8) activations of the call and ``seq`` an
-``ops.Seq``.  Activations, caches and matrices are bfloat16 or, for a model served in 32-bit, fp32; the residual
+``ops.Seq``.  Mixers that can stand side by side in a ``ParallelMixer`` also offer ``heads_of(p, state, seq, out)``, what they do
+between their input projections (rows of p) and their output projection.  Activations, caches and matrices are bfloat16 or, for a model served in 32-bit, fp32; the residual
 stream, norms, scores, decays and recurrent states are fp32 in both.
 """
 
 from __future__ import annotations
 
+import ctypes
+import math
+
 import torch
 import torch.nn.functional as F
 
 from . import ops
-from ._lib import DELTA_SILU_GATE, OharaDelta
+from ._lib import DELTA_SILU_GATE, RETENTION_CHUNK, OharaDelta, OharaGlu, OharaRetention, check, lib
 
 BF16, F32 = torch.bfloat16, torch.float32
 
@@ -78,18 +82,119 @@ class SwiGLU:
         yield from self.down.tensors()
 
 
-class GroupNorm:
-    """RMS norm in ``groups`` equal runs of the row, times w (applied inside ``ops.residual_norm``)."""
+class ClampedGLU:
+    """down(g sigmoid(alpha g) (u + offset)), g = gate x capped by ``limit`` from above, u = up x from both sides; gate and up are one
+    launch."""
 
-    def __init__(self, w, groups: int, eps: float, device="cuda"):
+    def __init__(self, gate, up, down, *, limit: float, alpha: float = 1.702, offset: float = 1.0, dtype=BF16, device="cuda"):
+        ff, k = gate.shape
+        ffp, kp = ops.round8(ff), ops.round8(k)
+        gate, up = (_pad(w.detach().to(device=device, dtype=dtype), ffp, kp).contiguous() for w in (gate, up))
+        self.dtype, self.ff = dtype, ffp
+        self.constants = (float(limit), float(alpha), float(offset))
+        self.gate_up = (gate, up) if dtype == F32 else ops.pack_gate_up(gate, up)
+        self.down = Linear(_pad(down.detach(), down.shape[0], ffp), dtype=dtype, device=device)
+
+    def __call__(self, x: torch.Tensor) -> torch.Tensor:
+        return self.down(ops.gemm_glu(x, self.gate_up, *self.constants))
+
+    def tensors(self):
+        yield from (self.gate_up if self.dtype == F32 else (self.gate_up.data,))
+        yield from self.down.tensors()
+
+
+class RoutedExperts:
+    """Mixture of ``ClampedGLU`` experts: fp32 softmax router over experts and ``identity`` outputs that return the input itself; the
+    ``top`` best by score + correction inside the ``keep`` best of ``groups`` groups of neighbours, weighted by their scores without
+    it; a shared expert for every token.  experts: (gate, up, down) each; shared: the same and its limit, or None.
+
+    A call returns an ``ops.Mixture``: the residual update sums it."""
+
+    TILE_PAIRS = 64  # pairs per expert from which the experts run in tiles and the shared expert in launches of its own
+
+    def __init__(self, experts, router, correction, *, top: int, limit: float, groups: int = 1, keep: int = 1, identity: int = 0, shared=None,
+                 alpha: float = 1.702, offset: float = 1.0, dtype=BF16, device="cuda"):
+        n, k = len(experts), router.shape[1]
+        if router.shape[0] != n + identity or correction.numel() != n + identity:
+            raise ValueError(f"router and correction have {router.shape[0]} and {correction.numel()} entries, {n + identity} expected")
+        if n < 1 or not 1 <= top <= min(n + identity, 64) or n + identity > 1024:
+            raise ValueError("between 1 and 1024 outputs and a top of at most 64 of them are supported")
+        if groups < 1 or (n + identity) % groups or not 1 <= keep <= groups or groups > 64:
+            raise ValueError("groups (at most 64) must divide the router's outputs, and 1 to all of them be kept")
+        if keep * ((n + identity) // groups) < top:
+            raise ValueError("the kept groups hold fewer outputs than a token uses")
+        self.experts, self.top, self.groups, self.keep = n, top, groups, keep
+        self.width, self.k, self.ff = experts[0][2].shape[0], ops.round8(k), ops.round8(experts[0][0].shape[0])
+        self.dtype, self.device = dtype, device
+        dev = lambda w, rows, cols: _pad(w.detach().to(device=device, dtype=dtype), rows, cols).contiguous()  # noqa: E731
+        gates, ups, downs = ([dev(e[i], *size) for e in experts] for i, size in
+                             ((0, (self.ff, self.k)), (1, (self.ff, self.k)), (2, (ops.round8(self.width), self.ff))))
+        if dtype == F32:
+            self.gate_up, self.down = (torch.stack(gates), torch.stack(ups)), torch.stack(downs)
+        else:
+            self.gate_up = torch.stack([ops.pack_gate_up(g, u).data for g, u in zip(gates, ups)])
+            self.down = torch.stack([ops.pack_rows(d) for d in downs])
+        self.router = dev(router, n + identity, self.k)
+        self.correction = correction.detach().to(device=device, dtype=F32).contiguous()
+        self.glu = OharaGlu(limit, alpha, offset, 0)
+        self.shared = None if shared is None else ClampedGLU(*shared[:3], limit=shared[3], alpha=alpha, offset=offset, dtype=dtype,
+                                                             device=device)
+        self._counter = torch.zeros(1, dtype=torch.int32, device=device)
+        self.trace = None  # a list: a call appends (chosen outputs, weights)
+
+    def __call__(self, x: torch.Tensor) -> ops.Mixture:
+        rows, n8 = x.shape[0], ops.round8(self.width)
+        pairs = rows * self.top
+        idx, w, offs, pair_of, pos_of = ops.moe_router(x, self.router, self.correction, self.k, self.top, self.groups, self.keep,
+                                                       self._counter)
+        if self.trace is not None:
+            self.trace.append((idx, w))
+        empty = lambda *s: torch.empty(*s, dtype=self.dtype, device=x.device)  # noqa: E731
+        act, y = empty(pairs, self.ff), empty(pairs, n8)
+        p, glu, shared = ops._ptr, ctypes.byref(self.glu), None
+        if self.dtype == F32:
+            check(lib().ohara_moe_glu_f32(p(x), x.stride(0), p(self.gate_up[0]), p(self.gate_up[1]), self.experts, self.ff, self.k, self.top,
+                                          pairs, p(offs), p(pair_of), glu, p(act), self.ff, ops._stream()), "moe_glu")
+            check(lib().ohara_moe_down_f32(p(act), self.ff, p(self.down), self.experts, n8, self.ff, pairs, p(offs), p(y), n8,
+                                           ops._stream()), "moe_down")
+            if self.shared is not None:
+                shared = self.shared(x)
+        else:
+            up, down = (0, 0, 0, None, 0, 0), (0, 0, 0, 0, 0, 0, 0)  # the shared expert's part of the launches
+            if self.shared is not None and pairs >= self.TILE_PAIRS * self.experts:
+                shared = self.shared(x)
+            elif self.shared is not None:
+                s = self.shared
+                act_s, shared = empty(rows, s.ff), empty(rows, n8)
+                up = (p(s.gate_up.data), s.ff, rows, ctypes.byref(OharaGlu(*s.constants, 0)), p(act_s), s.ff)
+                down = (p(s.down.w.data), s.ff, rows, p(act_s), s.ff, p(shared), n8)
+            check(lib().ohara_moe_glu_bf16(p(x), x.stride(0), p(self.gate_up), self.gate_up.stride(0) * 2, self.experts, self.ff, self.k,
+                                           self.top, pairs, p(offs), p(pair_of), glu, p(act), self.ff, *up, ops._stream()), "moe_glu")
+            check(lib().ohara_moe_down_bf16(p(act), self.ff, p(self.down), self.down.stride(0) * 2, self.experts, n8, self.ff, pairs, p(offs),
+                                            p(y), n8, *down, ops._stream()), "moe_down")
+        return ops.Mixture(idx, w, pos_of, y, x, shared, self.experts)
+
+    def tensors(self):
+        yield from (self.gate_up if self.dtype == F32 else (self.gate_up,))
+        yield from (self.down, self.router, self.correction)
+        if self.shared is not None:
+            yield from self.shared.tensors()
+
+
+class GroupNorm:
+    """RMS norm in ``groups`` equal runs of the row, times w and, if given, ``scale`` (applied inside ``ops.residual_norm``)."""
+
+    def __init__(self, w, groups: int, eps: float, device="cuda", scale=None):
         if w.numel() % groups:
             raise ValueError("norm groups must divide the width")
         self.w = w.detach().to(device=device, dtype=F32).contiguous()
+        if scale is not None:
+            self.w = self.w * scale.detach().to(device=device, dtype=F32)
         self.groups, self.eps = groups, float(eps)
 
     def of(self, y) -> dict:
-        """What ``ops.residual_norm`` needs to add the norm of y."""
-        return dict(y=y, norm_w=self.w, groups=self.groups, eps=self.eps)
+        """What ``ops.residual_norm`` needs to add the norm of y (a tensor or an ``ops.Mixture``)."""
+        return dict({"mix" if isinstance(y, ops.Mixture) else "y": y}, norm_w=self.w, groups=self.groups, eps=self.eps)
 
     def out(self) -> dict:
         """What ``ops.residual_norm`` needs to return the norm of the residual."""
@@ -211,52 +316,88 @@ class BiasedAttention(CachedAttention):
 _ROTARY: dict = {}
 
 
-def rotary_tables(base: float, dims: int, positions: int, device):
+def scaled_frequencies(f: torch.Tensor, factor: float, low: float, high: float, original: float) -> torch.Tensor:
+    """Rotary frequencies stretched to longer contexts as in Llama 3.1: those that turn at least ``high`` times in ``original``
+    positions stay, those that turn at most ``low`` times are divided by ``factor``, in between the two are mixed linearly."""
+    turns = original * f / (2 * math.pi)
+    if high <= low:
+        return torch.where(turns < low, f / factor, f)
+    s = ((turns - low) / (high - low)).clamp(0, 1)
+    return (1 - s) * f / factor + s * f
+
+
+def rotary_tables(base: float, dims: int, positions: int, device, scaling: tuple | None = None):
     """(cos, sin) of position * base^(-2i / dims), i < dims / 2, as (positions, dims / 2) fp32; one pair for all layers that share
-    the constants."""
+    the constants.  ``scaling``: (factor, low, high, original) of ``scaled_frequencies``."""
     device = torch.device(device)
-    key = (float(base), dims, positions, device.type, device.index)
+    key = (float(base), dims, positions, device.type, device.index, scaling)
     if key not in _ROTARY:
         f = float(base) ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / max(dims, 1))
+        if scaling is not None:
+            f = scaled_frequencies(f, *scaling)
         a = torch.arange(positions, dtype=torch.float64).unsqueeze(1) * f
         _ROTARY[key] = (a.cos().to(device, F32).contiguous(), a.sin().to(device, F32).contiguous())
     return _ROTARY[key]
 
 
 class RotaryAttention(CachedAttention):
-    """Causal attention with the first ``rot_dims`` dimensions of q and k rotated in neighbouring pairs, soft-capped scores (``cap``,
-    0: none) and, with ``chunk`` > 0, keys of the query's own chunk of that many positions only."""
+    """Causal attention with the first ``rot_dims`` dimensions of q and k rotated in neighbouring pairs (``rot_scaling``: of
+    ``rotary_tables``), soft-capped scores (``cap``, 0: none), with ``chunk`` > 0 keys of the query's own chunk of that many positions
+    only, with ``window`` > 0 only that many keys up to the query's own.  q_norm, k_norm: every q / k head over its own root mean
+    square times these first.  sinks: per head a score that joins the softmax without a value.  ``bare``: the projections are a
+    ``ParallelMixer``'s, which scales the heads' outputs by ``out_scale``."""
 
     def __init__(self, q, k, v, out, *, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, rot_base: float, rot_dims: int,
-                 cap: float = 0.0, chunk: int = 0, dtype=BF16, device="cuda"):
+                 cap: float = 0.0, chunk: int = 0, window: int = 0, q_norm=None, k_norm=None, eps: float = 0.0, sinks=None,
+                 rot_scaling: tuple | None = None, bare: bool = False, dtype=BF16, device="cuda"):
         self._sizes(heads, kv_heads, dim, vdim, (("q", q, heads * dim), ("k", k, kv_heads * dim), ("v", v, kv_heads * vdim)), dtype, device)
         if rot_dims < 0 or rot_dims % 2 or rot_dims > dim:
             raise ValueError("rotated dimensions must be an even number up to the head size")
-        if cap < 0 or chunk < 0:
-            raise ValueError("soft cap and chunk size cannot be negative")
+        if cap < 0 or chunk < 0 or window < 0:
+            raise ValueError("soft cap, chunk and window sizes cannot be negative")
+        if (q_norm is None) != (k_norm is None) or any(t is not None and t.numel() != dim for t in (q_norm, k_norm)):
+            raise ValueError("head norms come for q and k, with one weight per dimension of a head")
         self.scale, self.cap, self.chunk, self.rot_base, self.rot_dims = float(scale), float(cap), chunk, float(rot_base), rot_dims
-        self.proj = Linear(torch.cat([q, k, v]), dtype=dtype, device=device)
-        self.out = Linear(out, dtype=dtype, device=device)
+        self.window, self.eps, self.out_scale = window, float(eps), 1.0
+        self.rot_scaling = None if rot_scaling is None else tuple(float(v) for v in rot_scaling)
+        dev = lambda t: None if t is None else t.detach().to(device=device, dtype=F32).contiguous()  # noqa: E731
+        self.q_norm, self.k_norm, self.sinks = dev(q_norm), dev(k_norm), dev(sinks)
+        self.in_weight, self.out_weight = torch.cat([q, k, v]), out
+        if not bare:
+            self.proj, self.out = (Linear(w, dtype=dtype, device=device) for w in (self.in_weight, out))
+            del self.in_weight, self.out_weight
 
     def _visible(self, max_seq_length: int) -> int:
-        return min(max_seq_length, self.chunk) if self.chunk else max_seq_length
+        return min([max_seq_length] + [n for n in (self.chunk, self.window) if n])
+
+    def _tables(self, positions: int):
+        return rotary_tables(self.rot_base, self.rot_dims, positions, self.device, self.rot_scaling)
 
     def state(self, rows: int, max_seq_length: int) -> dict:
-        rotary_tables(self.rot_base, self.rot_dims, max_seq_length, self.device)
+        self._tables(max_seq_length)
         return super().state(rows, max_seq_length)
 
-    def __call__(self, h, state, seq: ops.Seq):
-        p, t_max = self.proj(h), state.key.shape[1]
-        cos, sin = rotary_tables(self.rot_base, self.rot_dims, t_max, self.device)
-        q = ops.qkv_rotate_append(p, self.heads, self.kv_heads, self.dim, self.vdim, cos, sin, self.rot_dims, state.key, state.value, seq)
+    def heads_of(self, p, state, seq: ops.Seq, out=None):
+        t_max = state.key.shape[1]
+        cos, sin = self._tables(t_max)
+        sizes = (self.heads, self.kv_heads, self.dim, self.vdim)
+        if self.q_norm is not None:
+            q = ops.qkv_headnorm_rotate_append(p, *sizes, self.q_norm, self.k_norm, self.eps, cos, sin, self.rot_dims, state.key, state.value,
+                                               seq)
+        else:
+            q = ops.qkv_rotate_append(p, *sizes, cos, sin, self.rot_dims, state.key, state.value, seq)
         ns, ws = self._split(seq.batch, t_max) if seq.seq_len == 1 else (1, None)
-        att = ops.attn_scored(q, state.key, state.value, self.heads, self.kv_heads, self.dim, self.vdim, t_max, self.scale, seq,
-                              cap=self.cap, chunk=self.chunk, n_split=ns, workspace=ws)
-        return self.out(att)
+        return ops.attn_scored(q, state.key, state.value, *sizes, t_max, self.scale, seq, cap=self.cap, chunk=self.chunk, window=self.window,
+                               sinks=self.sinks, n_split=ns, workspace=ws, out_scale=self.out_scale, out=out)
+
+    def __call__(self, h, state, seq: ops.Seq):
+        return self.out(self.heads_of(self.proj(h), state, seq))
 
     def tensors(self):
-        yield from self.proj.tensors()
-        yield from self.out.tensors()
+        if hasattr(self, "proj"):
+            yield from self.proj.tensors()
+            yield from self.out.tensors()
+        yield from (t for t in (self.q_norm, self.k_norm, self.sinks) if t is not None)
 
 
 class LatentAttention:
@@ -494,3 +635,112 @@ class HeadDelta(DeltaRule):
         d, n = self._c, heads * vdim
         d.off_g, d.off_a, d.off_b = self.off_a, self.off_a + n, self.off_a + n + heads
         d.flags = DELTA_SILU_GATE
+
+
+class Retention:
+    """Linear attention with one fixed decay per head (see csrc/retention.hip): S <- decay S + k_scale k v^T, o = S^T q, every head's o
+    over its own root mean square, times silu of the gate.  q, k: (heads * dim, width); v, gate: (heads * vdim, width); out: (width,
+    heads * vdim).  ``bare``: as ``RotaryAttention``."""
+
+    WORKSPACE = 1 << 30  # bytes of chunk states at most; longer prompts are worked on in segments
+    _workspaces: dict = {}  # device -> the workspace every layer on that device shares (prompts run on one stream)
+
+    def __init__(self, q, k, v, gate, out, *, heads: int, dim: int, vdim: int, decay, k_scale: float, eps: float, bare: bool = False,
+                 dtype=BF16, device="cuda"):
+        for name, w, n in (("q", q, heads * dim), ("k", k, heads * dim), ("v", v, heads * vdim), ("gate", gate, heads * vdim)):
+            if w.shape[0] != n:
+                raise ValueError(f"retention {name} projection has {w.shape[0]} rows, {n} expected")
+        if out.shape[1] != heads * vdim:
+            raise ValueError(f"retention output projection has {out.shape[1]} columns, {heads * vdim} expected")
+        if max(dim, vdim) > 256:
+            raise ValueError("retention head sizes up to 256 are supported")
+        decay = torch.as_tensor(decay, dtype=torch.float64).reshape(-1)
+        if decay.numel() != heads or not bool(((decay >= 0) & (decay <= 1)).all()):
+            raise ValueError("one decay between 0 and 1 per head is required")
+        self.heads, self.dim, self.vdim = heads, ops.round8(dim), ops.round8(vdim)
+        self.dtype, self.device = dtype, torch.device(device)
+
+        def per_head(w, n):  # (heads * n, width) -> heads of round8(n) rows
+            return F.pad(w.detach().view(heads, n, -1), (0, 0, 0, ops.round8(n) - n)).flatten(0, 1)
+
+        self.in_weight = torch.cat([per_head(w, n) for w, n in ((q, dim), (k, dim), (v, vdim), (gate, vdim))])
+        self.out_weight = F.pad(out.detach().view(-1, heads, vdim), (0, self.vdim - vdim)).flatten(1)
+        self.powers = (decay.unsqueeze(1) ** torch.arange(RETENTION_CHUNK + 1, dtype=torch.float64)).to(self.device, F32).contiguous()
+        nk, nv = heads * self.dim, heads * self.vdim
+        self._c = OharaRetention(heads, self.dim, self.vdim, vdim, 0, nk, 2 * nk, 2 * nk + nv, eps, k_scale, 1.0, 0, self.powers.data_ptr())
+        if not bare:
+            self.proj, self.out = (Linear(w, dtype=dtype, device=device) for w in (self.in_weight, self.out_weight))
+            del self.in_weight, self.out_weight
+
+    @property
+    def out_scale(self) -> float:
+        return self._c.out_scale
+
+    @out_scale.setter
+    def out_scale(self, value: float) -> None:
+        self._c.out_scale = value
+
+    def state(self, rows: int, max_seq_length: int) -> dict:
+        return {"retention": torch.zeros(rows, self.heads, self.dim, self.vdim, dtype=F32, device=self.device)}
+
+    def _workspace(self, batch: int, tokens: int) -> torch.Tensor:
+        size = lambda n: ops.retention_workspace_bytes(self.heads, self.dim, self.vdim, batch, n)  # noqa: E731
+        need = max(min(size(tokens), self.WORKSPACE), size(1))
+        ws = Retention._workspaces.get(self.device)
+        if ws is None or ws.numel() < need:
+            ws = Retention._workspaces[self.device] = torch.empty(need, dtype=torch.uint8, device=self.device)
+        return ws
+
+    def heads_of(self, p, state, seq: ops.Seq, out=None):
+        ws = None if seq.seq_len == 1 else self._workspace(seq.batch, seq.seq_len)
+        return ops.retention(self._c, p, state.retention, ws, seq, out)
+
+    def __call__(self, h, state, seq: ops.Seq):
+        return self.out(self.heads_of(self.proj(h), state, seq))
+
+    def tensors(self):
+        if hasattr(self, "proj"):
+            yield from self.proj.tensors()
+            yield from self.out.tensors()
+        yield self.powers
+
+
+class _Part:
+    """The tensors of a layer's state whose names start with a prefix, under the rest of their names."""
+
+    def __init__(self, state, prefix: str):
+        self._state, self._prefix = state, prefix
+
+    def __getattr__(self, name):
+        return getattr(self._state, self._prefix + name)
+
+
+class ParallelMixer:
+    """left_scale * left(h) + right_scale * right(h) for two mixers built ``bare``: their input projections are one product, and so are
+    their output projections (the scales are applied to the heads, before those are rounded)."""
+
+    def __init__(self, left, right, left_scale: float, right_scale: float, *, dtype=BF16, device="cuda"):
+        self.parts = (("left_", left), ("right_", right))
+        left.out_scale, right.out_scale = float(left_scale), float(right_scale)
+        r8 = ops.round8
+        self.n_in, self.n_out = r8(left.in_weight.shape[0]), r8(left.out_weight.shape[1])
+        self.width_out = self.n_out + r8(right.out_weight.shape[1])
+        pad_cols = lambda w: _pad(w, w.shape[0], r8(w.shape[1]))  # noqa: E731
+        self.proj = Linear(torch.cat([_pad(left.in_weight, self.n_in), right.in_weight]), dtype=dtype, device=device)
+        self.out = Linear(torch.cat([pad_cols(left.out_weight), pad_cols(right.out_weight)], 1), dtype=dtype, device=device)
+        for _, part in self.parts:
+            del part.in_weight, part.out_weight
+
+    def state(self, rows: int, max_seq_length: int) -> dict:
+        return {prefix + name: t for prefix, part in self.parts for name, t in part.state(rows, max_seq_length).items()}
+
+    def __call__(self, h, state, seq: ops.Seq):
+        p = self.proj(h)
+        o = torch.empty(p.shape[0], self.width_out, dtype=p.dtype, device=p.device)
+        for (prefix, part), src, dst in zip(self.parts, (p[:, :self.n_in], p[:, self.n_in:]), (o[:, :self.n_out], o[:, self.n_out:])):
+            part.heads_of(src, _Part(state, prefix), seq, dst)
+        return self.out(o)
+
+    def tensors(self):
+        for part in (self.proj, self.out, *(part for _, part in self.parts)):
+            yield from part.tensors()

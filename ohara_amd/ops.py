@@ -635,10 +635,26 @@ class Seq:
         return C.byref(self.c)
 
 
-def residual_norm(x, seq: Seq, dtype, *, ids=None, table=None, y=None, norm_w=None, groups=1, eps=0.0, mode="none",
-                  norm2_w=None, conv_w=None, ring=None, center_y=False, center_out=False):
-    """x (rows, d) fp32 <- table[ids], or x + norm_w * group_rms(y), in place; returns what ``mode`` asks for as
-    (rows, d rounded up to 8) in ``dtype``: "copy" of x, "conv" (x + causal depthwise convolution over time, one token per
+class Mixture:
+    """What routed experts leave to be summed (OharaMixture): row n of the layer's output is sum_j w[n, j] * (y[pos_of[n, j]], or h[n]
+    where idx[n, j] names an identity output) + shared[n]."""
+
+    __slots__ = ("c", "_keep")
+
+    def __init__(self, idx, w, pos_of, y, h, shared, experts: int):
+        self._keep = (idx, w, pos_of, y, h, shared)
+        self.c = _lib.OharaMixture(idx.shape[1], experts, y.stride(0), h.stride(0), 0 if shared is None else shared.stride(0), 0, _ptr(w),
+                                   _ptr(idx), _ptr(pos_of), _ptr(y), _ptr(h), _ptr(shared))
+
+    @property
+    def dtype(self):
+        return self._keep[3].dtype
+
+
+def residual_norm(x, seq: Seq, dtype, *, ids=None, table=None, table_scale=1.0, y=None, mix: Mixture | None = None, norm_w=None, groups=1,
+                  eps=0.0, mode="none", norm2_w=None, conv_w=None, ring=None, center_y=False, center_out=False):
+    """x (rows, d) fp32 <- table_scale * table[ids], or x + norm_w * group_rms(y) (``mix``: of a mixture of experts), in place; returns
+    what ``mode`` asks for as (rows, d rounded up to 8) in ``dtype``: "copy" of x, "conv" (x + causal depthwise convolution over time, one token per
     sequence, ring updated), "norm" (group RMS norm of x times norm2_w), or None.  ``center_y`` / ``center_out``: the norm
     of y / of the output is a layer norm without bias."""
     _need(x, F32, "x")
@@ -650,11 +666,13 @@ def residual_norm(x, seq: Seq, dtype, *, ids=None, table=None, y=None, norm_w=No
     for t, name in ((y, "y"), (table, "table")):
         if t is not None:
             _need(t, dtype, name)
+    if mix is not None and mix.dtype != dtype:
+        raise ValueError("the mixture is of another dtype")
     out = torch.empty(rows, round8(d), dtype=dtype, device=x.device) if mode != "none" else None
     check(_typed("residual_norm", dtype)(
-        _ptr(x), d, _ptr(ids), _ptr(table), 0 if table is None else table.shape[0], _ptr(y), 0 if y is None else y.stride(0),
-        _ptr(norm_w), groups, eps, m, _ptr(out), 0 if out is None else out.stride(0), _ptr(norm2_w), _ptr(conv_w),
-        0 if conv_w is None else conv_w.shape[0], _ptr(ring), seq.ref, _stream()), "residual_norm")
+        _ptr(x), d, _ptr(ids), _ptr(table), 0 if table is None else table.shape[0], table_scale, _ptr(y),
+        0 if y is None else y.stride(0), _ptr(norm_w), groups, eps, m, _ptr(out), 0 if out is None else out.stride(0), _ptr(norm2_w), _ptr(conv_w),
+        0 if conv_w is None else conv_w.shape[0], _ptr(ring), None if mix is None else C.byref(mix.c), seq.ref, _stream()), "residual_norm")
     return out
 
 
@@ -759,6 +777,19 @@ def qkv_rotate_append(p, h, h_kv, dh, dv, cos, sin, rot, kcache, vcache, seq: Se
     return q
 
 
+def qkv_headnorm_rotate_append(p, h, h_kv, dh, dv, qn, kn, eps, cos, sin, rot, kcache, vcache, seq: Seq):
+    """``qkv_rotate_append`` with every q and k head first over its own root mean square times qn / kn (dh entries, fp32)."""
+    if rot and (cos.shape != (cos.shape[0], rot // 2) or cos.shape[0] < kcache.shape[1] or cos.shape != sin.shape):
+        raise ValueError("rotary tables must cover the cache's positions with rot / 2 angles each")
+    if qn.numel() != dh or kn.numel() != dh:
+        raise ValueError("head norms have one weight per dimension of a head")
+    q = torch.empty(p.shape[0], h * round8(dh), dtype=p.dtype, device=p.device)
+    check(_typed("qkv_headnorm_rotate_append", p.dtype)(
+        _ptr(p), p.stride(0), h, h_kv, dh, dv, _ptr(qn), _ptr(kn), eps, _ptr(cos), _ptr(sin), rot, _ptr(q), _ptr(kcache), _ptr(vcache),
+        kcache.shape[1], seq.ref, _stream()), "qkv_headnorm_rotate_append")
+    return q
+
+
 def qkv_norm_append(p, h, h_kv, dh, dv, qn, kn, eps, kcache, vcache, seq: Seq):
     """p rows [q; k; v; ...] -> normalised q (rows, h * round8(dh)); keys and values into the caches."""
     q = torch.empty(p.shape[0], h * round8(dh), dtype=p.dtype, device=p.device)
@@ -785,14 +816,18 @@ def attn_bias(q, kcache, vcache, h, h_kv, dh, dv, scale, slopes, gate, seq: Seq,
     return out
 
 
-def attn_scored(q, keys, values, h, h_kv, dh, dv, t_max, scale, seq: Seq, *, cap=0.0, chunk=0, slopes=None, gate=None,
-                gate_elements=False, ld_k=0, ld_v=0, n_split=1, workspace=None):
+def attn_scored(q, keys, values, h, h_kv, dh, dv, t_max, scale, seq: Seq, *, cap=0.0, chunk=0, window=0, sinks=None, slopes=None,
+                gate=None, gate_elements=False, ld_k=0, ld_v=0, n_split=1, workspace=None, out_scale=1.0, out=None):
     """Causal attention over positions of ``keys`` / ``values`` (cache rows of t_max positions, ``ld_k`` / ``ld_v`` elements apart if
     not densely packed) -> (rows, round8(h * dv)).  Scores: scale q . k, soft-capped by ``cap``, minus slopes[head] * distance;
     ``chunk``: inside chunks of that many positions.  gate: a (rows, h) or, ``gate_elements``, (rows, h * dv) column slice,
-    through the sigmoid."""
-    out = torch.empty(q.shape[0], round8(h * dv), dtype=q.dtype, device=q.device)
-    sc = _lib.OharaScores(scale, cap, chunk, int(gate_elements), ld_k, ld_v, _ptr(slopes))
+    through the sigmoid.  ``window``: only that many keys up to the query's own; ``sinks`` (h,) fp32: scores that join the softmax
+    without a value.  ``out``: a column slice of a wider buffer."""
+    if out is None:
+        out = torch.empty(q.shape[0], round8(h * dv), dtype=q.dtype, device=q.device)
+    elif out.shape != (q.shape[0], round8(h * dv)) or out.dtype != q.dtype or out.stride(1) != 1:
+        raise ValueError("out must be (rows, round8(h * dv)) with unit column stride")
+    sc = _lib.OharaScores(scale, cap, chunk, int(gate_elements), ld_k, ld_v, _ptr(slopes), _ptr(sinks), window, out_scale)
     check(_typed("attn_scored", q.dtype)(
         _ptr(q), _ptr(keys), _ptr(values), h, h_kv, dh, dv, t_max, C.byref(sc), _ptr(gate), 0 if gate is None else gate.stride(0),
         n_split, _ptr(workspace), _ptr(out), out.stride(0), seq.ref, _stream()), "attn_scored")
@@ -862,4 +897,55 @@ def delta_prefill(d: "_lib.OharaDelta", p, za, zg, state, ring, workspace, seq: 
         C.byref(d), _ptr(p), p.stride(0), _ptr(za), 0 if za is None else za.stride(0), _ptr(zg), 0 if zg is None else zg.stride(0),
         _ptr(state), _ptr(ring), _ptr(workspace), workspace.numel(), _ptr(o_tmp), _ptr(out), out.stride(0), seq.ref, _stream()), "delta_prefill")
     conv_ring_store(p, 2 * d.kv_heads * d.dim + d.heads * d.vdim, ring, seq)
+    return out
+
+
+def gemm_glu(x, w, limit: float, alpha: float, offset: float, out=None):
+    """g sigmoid(alpha g) (u + offset), g = min(x Wg^T, limit), u = clamp(x Wu^T, +-limit); w: packed (bf16) or a pair of (n, k) fp32."""
+    f32 = x.dtype == F32
+    n, k = w[0].shape if f32 else (w.n, w.k)
+    if not x.is_cuda or x.stride(1) != 1 or x.shape[1] != k:
+        raise ValueError("x must be a device matrix with unit column stride and W's columns")
+    if out is None:
+        out = torch.empty(x.shape[0], n, dtype=x.dtype, device=x.device)
+    ptrs = (_ptr(w[0]), _ptr(w[1])) if f32 else (_ptr(w.data),)
+    check(_typed("gemm_glu", x.dtype)(_ptr(x), x.stride(0), *ptrs, n, k, limit, alpha, offset, x.shape[0], _ptr(out), out.stride(0),
+                                      _stream()), "gemm_glu")
+    return out
+
+
+def moe_router(x, w, correction, k: int, top: int, groups: int, keep: int, counter):
+    """x (rows, k), w (outputs, k) -> (idx (rows, top) int32, weights (rows, top) fp32, offs, pair_of, pos_of): see
+    ohara_moe_router_*.  counter: one int32, zero between calls."""
+    rows, n = x.shape[0], w.shape[0]
+    i32 = lambda *s: torch.empty(*s, dtype=torch.int32, device=x.device)  # noqa: E731
+    idx, wgt = i32(rows, top), torch.empty(rows, top, dtype=F32, device=x.device)
+    offs, pair_of, pos_of, hist = i32(n + 1), i32(rows * top), i32(rows * top), i32((rows * top + 1023) // 1024 * n)
+    check(_typed("moe_router", x.dtype)(
+        _ptr(x), x.stride(0), _ptr(w), w.stride(0), _ptr(correction), rows, k, n, top, groups, keep, _ptr(idx), _ptr(wgt), _ptr(offs),
+        _ptr(pair_of), _ptr(pos_of), _ptr(hist), _ptr(counter), _stream()), "moe_router")
+    return idx, wgt, offs, pair_of, pos_of
+
+
+def retention_workspace_bytes(heads, dim, vdim, batch, tokens) -> int:
+    n = lib().ohara_retention_workspace_bytes(heads, dim, vdim, batch, tokens)
+    if n < 0:
+        raise ValueError("bad retention shape")
+    return n
+
+
+def retention(r: "_lib.OharaRetention", p, state, workspace, seq: Seq, out=None):
+    """Normed and gated heads (rows, heads * vdim) of the tokens in p; the state moves on.  One token per sequence needs no
+    workspace.  ``out``: a column slice of a wider buffer."""
+    n = r.heads * r.vdim
+    if out is None:
+        out = torch.empty(p.shape[0], n, dtype=p.dtype, device=p.device)
+    elif out.shape != (p.shape[0], n) or out.dtype != p.dtype or out.stride(1) != 1:
+        raise ValueError("out must be (rows, heads * vdim) with unit column stride")
+    if seq.seq_len == 1:
+        check(_typed("retention_step", p.dtype)(C.byref(r), _ptr(p), p.stride(0), _ptr(state), _ptr(out), out.stride(0), seq.ref, _stream()),
+              "retention_step")
+    else:
+        check(_typed("retention_prefill", p.dtype)(C.byref(r), _ptr(p), p.stride(0), _ptr(state), _ptr(workspace), workspace.numel(),
+                                                   _ptr(out), out.stride(0), seq.ref, _stream()), "retention_prefill")
     return out

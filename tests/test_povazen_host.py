@@ -74,10 +74,10 @@ def test_entry_points_check_their_arguments():
     r = ctypes.byref
     buf = ctypes.create_string_buffer(4096)
     p = ctypes.addressof(buf)
-    assert L.ohara_residual_norm_bf16(0, 8, 0, 0, 0, 0, 0, 0, 1, 1e-5, 0, 0, 0, 0, 0, 0, 0, r(seq), 0) == _lib.EINVAL
+    assert L.ohara_residual_norm_bf16(0, 8, 0, 0, 0, 1.0, 0, 0, 0, 1, 1e-5, 0, 0, 0, 0, 0, 0, 0, None, r(seq), 0) == _lib.EINVAL
     # groups do not divide the width; the fused convolution takes one token per sequence
-    assert L.ohara_residual_norm_bf16(p, 8, 0, 0, 0, p, 8, p, 3, 1e-5, 0, 0, 0, 0, 0, 0, 0, r(seq), 0) == _lib.EINVAL
-    assert L.ohara_residual_norm_f32(p, 8, 0, 0, 0, p, 8, p, 1, 1e-5, 2, p, 8, 0, p, 2, p, r(two), 0) == _lib.EINVAL
+    assert L.ohara_residual_norm_bf16(p, 8, 0, 0, 0, 1.0, p, 8, p, 3, 1e-5, 0, 0, 0, 0, 0, 0, 0, None, r(seq), 0) == _lib.EINVAL
+    assert L.ohara_residual_norm_f32(p, 8, 0, 0, 0, 1.0, p, 8, p, 1, 1e-5, 2, p, 8, 0, p, 2, p, None, r(two), 0) == _lib.EINVAL
     assert L.ohara_attn_bias_bf16(p, p, p, 2, 1, 300, 8, 16, 1.0, p, 0, 0, 1, 0, p, 16, r(seq), 0) == _lib.ESIZE
     assert L.ohara_attn_bias_bf16(p, p, p, 3, 2, 8, 8, 16, 1.0, p, 0, 0, 1, 0, p, 24, r(seq), 0) == _lib.EINVAL
     assert L.ohara_attn_bias_bf16(p, p, p, 2, 1, 8, 8, 16, 1.0, p, 0, 0, 2, 0, p, 16, r(seq), 0) == _lib.EINVAL  # no workspace

@@ -74,7 +74,7 @@ def test_entry_points_check_their_arguments():
     assert attn(scores(gate_elements=1), gate=p, ldg=2) == E  # a gate per element has h * dv columns
     assert attn(scores(), ns=2) == E and attn(scores(), seq=late) == E
     # layer norms have one group
-    assert L.ohara_residual_norm_bf16(p, 8, 0, 0, 0, p, 8, p, 2, 1e-5, 16, 0, 0, 0, 0, 0, 0, r(seq), 0) == E
+    assert L.ohara_residual_norm_bf16(p, 8, 0, 0, 0, 1.0, p, 8, p, 2, 1e-5, 16, 0, 0, 0, 0, 0, 0, None, r(seq), 0) == E
     assert L.ohara_gemm_gelu_lookup_bf16(p, 8, p, 8, 8, p, 4, p, 3, 1, p, 8, 0) == E  # table rows shorter than n
     assert L.ohara_gemm_gelu_lookup_f32(p, 8, p, 4, 6, p, 4, p, 3, 1, p, 4, 0) == E   # k % 4
     side = lambda d=8, ldy=8, n=8, R=1, ldo=8: L.ohara_token_side_bf16(  # noqa: E731
