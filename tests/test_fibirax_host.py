@@ -1,0 +1,123 @@
+"""Fibirax's host side without a GPU: configuration and registry, rotary tables, powers of the decays, argument checks of the entry
+points."""
+
+import copy
+import ctypes
+import json
+
+import pytest
+import torch
+
+from _fibirax import CONFIGS, experts
+from ohara_amd import _lib
+from ohara_amd.checkpoint import _architecture, architecture_of, load_checkpoint
+from ohara_amd.fibirax import Fibirax, FibiraxConfig
+from ohara_amd.hybrid import rotary_tables, scaled_frequencies
+from oracle import fibirax_ref as R
+
+
+def test_config_from_json_and_registry(tmp_path):
+    from safetensors.torch import save_file
+
+    save_file({"embed": torch.zeros(2, 2, dtype=torch.bfloat16)}, str(tmp_path / "model.safetensors"))
+    (tmp_path / "config.json").write_text(json.dumps(CONFIGS["odd"]))
+    assert architecture_of(tmp_path) == "Fibirax"
+    cfg, state = load_checkpoint(tmp_path, max_sequence_length=77)
+    assert isinstance(cfg, FibiraxConfig) and list(state) == ["embed"]
+    assert (cfg.vocab_size, cfg.hidden_size, cfg.embedding_scale, cfg.norm_eps, cfg.max_sequence_length) == (97, 60, 0.37, 2e-3, 77)
+    assert cfg.num_hidden_layers == 3 and cfg.num_attention_heads == 6
+    one = cfg.layers[0]
+    a, r, m = one.left, one.right, one.mlp
+    assert (a.heads, a.kv_heads, a.dim, a.vdim, a.scale, a.rot_base, a.rot_dims, a.softcap, a.window) == (6, 2, 20, 12, 0.3, 300.0, 12, 8.0, 45)
+    assert a.rot_scaling == (4.0, 1.0, 4.0, 64.0) and cfg.layers[1].left.rot_scaling is None
+    assert (r.heads, r.dim, r.vdim, r.decay) == (3, 12, 20, (0.9, 0.99, 0.5))
+    assert (one.left_scale, one.right_scale) == (1.3, 0.8)
+    assert (m.experts, m.top, m.ff, m.limit, m.identity, m.groups, m.keep, m.shared_ff, m.shared_limit) == (10, 3, 36, 0.9, 2, 4, 2, 20, 1.7)
+    assert cfg.layers[1].mlp is None and cfg.layers[2].mlp.shared_ff == 0 and cfg.layers[2].mlp.groups == 1
+    assert load_checkpoint(tmp_path)[0].max_sequence_length == FibiraxConfig.max_sequence_length
+    assert _architecture("Fibirax") == (FibiraxConfig, Fibirax)
+
+
+@pytest.mark.parametrize("change, message", [
+    (dict(type="attention"), "unknown mixer"),
+    (dict(mlp={"kind": "dense", "ff": 8}), "unknown feed-forward"),
+])
+def test_config_rejects_what_it_does_not_know(change, message):
+    with pytest.raises(ValueError, match=message):
+        FibiraxConfig.from_dict({**CONFIGS["odd"], "layers": [{**CONFIGS["odd"]["layers"][0], **change}]})
+
+
+def test_optional_entries_may_be_missing_or_null():
+    for null in (False, True):
+        cfg = copy.deepcopy(CONFIGS["odd"])
+        left, mlp = cfg["layers"][0]["mixer"]["left"], cfg["layers"][0]["mlp"]
+        for holder, key in ((left, "softcap"), (left, "mask"), (left, "rot"), (mlp["router"], "groups"), (mlp["router"], "identity"),
+                            (mlp, "shared")):
+            if null:
+                holder[key] = None
+            else:
+                del holder[key]
+        one = FibiraxConfig.from_dict(cfg).layers[0]
+        assert (one.left.softcap, one.left.window, one.left.rot_dims, one.left.rot_scaling) == (0.0, 0, 0, None)
+        assert (one.mlp.groups, one.mlp.keep, one.mlp.identity, one.mlp.shared_ff) == (1, 1, 0, 0)
+
+
+@pytest.mark.parametrize("base, dims, scaling", [(1e4, 64, (8.0, 1.0, 4.0, 2048)), (300.0, 12, (4.0, 1.0, 4.0, 64)), (5e5, 10, (2.5, 0.5, 9.0, 77)),
+                                                 (50.0, 6, (3.0, 2.0, 2.0, 40))])
+def test_scaled_rotary_tables(base, dims, scaling):
+    f = base ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims)
+    want = R.rotary_frequencies(base, dims, dict(zip(("factor", "low", "high", "original"), scaling))) if scaling[1] < scaling[2] else [
+        a / scaling[0] if scaling[3] * a / (2 * torch.pi) < scaling[1] else a for a in f.tolist()]
+    want = torch.tensor(want, dtype=torch.float64)
+    assert torch.allclose(scaled_frequencies(f, *scaling), want, rtol=1e-13)
+    cos, sin = rotary_tables(base, dims, 3000, "cpu", scaling)
+    assert (cos[2999] - (2999 * want).cos()).abs().max() < 1e-7 and (sin[2999] - (2999 * want).sin()).abs().max() < 1e-7
+    assert rotary_tables(base, dims, 3000, "cpu")[0] is not cos and rotary_tables(base, dims, 3000, "cpu", scaling)[0] is cos
+
+
+def test_random_weights_cover_the_config():
+    w = R.random_weights(CONFIGS["odd"])
+    assert w["l0.mlp.router"].shape == (12, 60) and w["l0.mlp.e9.down"].shape == (60, 36) and "l1.mlp.router" not in w
+    assert "l2.mlp.shared.gate" not in w and w["l0.mix.left.q.norm"].shape == (20,) and experts(2, 1, 8, 1.0)["kind"] == "moe"
+
+
+def test_entry_points_check_their_arguments():
+    L, r = _lib.lib(), ctypes.byref
+    seq, two = _lib.OharaSeq(1, 1, 0, 0, None, None, None), _lib.OharaSeq(1, 2, 0, 0, None, None, None)
+    buf = ctypes.create_string_buffer(4096)
+    p = ctypes.addressof(buf)
+    E, S = _lib.EINVAL, _lib.ESIZE
+    ret = lambda **kw: _lib.OharaRetention(*({**dict(heads=2, dim=8, vdim=8, used=8, q=0, k=16, v=32, g=48, eps=1e-5, ks=1.0, os=1.0, res=0,  # noqa: E731
+                                                     pw=p), **kw}.values()))
+    step = lambda d, ldp=64, ldo=16, seq=seq: L.ohara_retention_step_bf16(r(d), p, ldp, p, p, ldo, r(seq), 0)  # noqa: E731
+    assert step(ret(dim=12)) == E and step(ret(used=9)) == E and step(ret(used=0)) == E and step(ret(q=4)) == E and step(ret(g=56)) == E
+    assert step(ret(pw=None)) == E and step(ret(), ldo=8) == E and step(ret(), seq=two) == E and step(ret(heads=1, dim=264)) == S
+    pre = lambda d, ws=p, n=4096: L.ohara_retention_prefill_f32(r(d), p, 64, p, ws, n, p, 16, r(two), 0)  # noqa: E731
+    assert pre(ret(), ws=None) == E and pre(ret(), n=64) == E
+    assert L.ohara_retention_workspace_bytes(2, 8, 8, 1, 129) == 2 * 2 * 32 * 16 * 4 and L.ohara_retention_workspace_bytes(2, 0, 8, 1, 1) == E
+    router = lambda n=8, top=2, groups=1, keep=1, k=8, ldx=8, w=p: L.ohara_moe_router_bf16(  # noqa: E731
+        p, ldx, w, 8, p, 1, k, n, top, groups, keep, p, p, p, p, p, p, p, 0)
+    assert router(top=9) == E and router(groups=3) == E and router(groups=4, keep=5) == E and router(groups=4, keep=0) == E
+    assert router(groups=4, keep=1, top=3) == E and router(k=12) == E and router(ldx=4) == E and router(w=0) == E
+    assert router(n=2048) == S and router(n=128, top=65) == S
+    glu = r(_lib.OharaGlu(1.0, 1.7, 1.0, 0))
+    assert L.ohara_moe_glu_bf16(p, 8, p, 1024, 2, 12, 8, 1, 4, p, p, glu, p, 16, 0, 0, 0, None, 0, 0, 0) == E   # hidden % 8
+    assert L.ohara_moe_glu_bf16(p, 8, p, 1024, 2, 8, 8, 1, 4, p, p, glu, p, 8, p, 8, 0, glu, p, 8, 0) == E      # no rows of the shared expert
+    assert L.ohara_moe_down_bf16(p, 8, p, 1024, 2, 8, 8, 4, p, p, 4, 0, 0, 0, 0, 0, 0, 0, 0) == E               # ldy < d
+    assert L.ohara_moe_glu_f32(p, 8, p, p, 2, 8, 6, 1, 4, p, p, glu, p, 8, 0) == E                              # d % 4
+    assert L.ohara_moe_down_f32(p, 8, p, 2, 8, 8, 4, p, p, 4, 0) == E
+    assert L.ohara_gemm_glu_bf16(p, 8, p, 8, 8, 1.0, 1.7, 1.0, 1, p, 6, 0) == E and L.ohara_gemm_glu_f32(p, 8, p, p, 4, 6, 1.0, 1.7, 1.0, 1, p, 4, 0) == E
+    norm = lambda dh=8, dv=8, qn=p, ldp=32: L.ohara_qkv_headnorm_rotate_append_bf16(  # noqa: E731
+        p, ldp, 2, 1, dh, dv, qn, p, 1e-5, p, p, 2, p, p, p, 4, r(seq), 0)
+    assert norm(qn=0) == E and norm(ldp=24) == E and norm(dh=300, ldp=2048) == S
+    mix = _lib.OharaMixture(2, 3, 8, 8, 0, 0, p, p, p, p, p, None)
+    res = lambda m, y=0, ids=0, w=p: L.ohara_residual_norm_bf16(  # noqa: E731
+        p, 8, ids, p, 4, 1.0, y, 8, w, 1, 1e-5, 0, 0, 0, 0, 0, 0, 0, r(m), r(seq), 0)
+    assert res(mix, y=p) == E and res(mix, ids=p) == E and res(mix, w=0) == E
+    for bad in (dict(top=0), dict(experts=0), dict(ldy=4), dict(ldh=10), dict(y=None)):
+        m = _lib.OharaMixture.from_buffer_copy(mix)
+        for k, v in bad.items():
+            setattr(m, k, v)
+        assert res(m) == E, bad
+    scores = _lib.OharaScores(1.0, 0.0, 0, 0, 0, 0, None, None, -1, 1.0)
+    assert L.ohara_attn_scored_bf16(p, p, p, 2, 1, 8, 8, 16, r(scores), 0, 0, 1, 0, p, 16, r(seq), 0) == E
