@@ -77,4 +77,4 @@ def agrees(got, want, dtype):
         return rows.max() < 1e-4 and (len(rows) < 8 or rows.median() < 6e-6)
     if len(rows) < 8:
         return rows.max() < 1.0
-    return rows.median() < 0.04 and rows.quantile(0.85) < 0.2
+    return rows.median() < 0.08 and rows.quantile(0.8) < 0.25

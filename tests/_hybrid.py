@@ -1,6 +1,7 @@
 """Helpers of the hybrid decoders' tests: random inputs, comparisons with float64, caches full of an earlier owner's leftovers."""
 
 import torch
+import torch.nn.functional as F
 
 BF, F32 = torch.bfloat16, torch.float32
 
@@ -55,6 +56,26 @@ def poisoned(model, rows):
         for t in c.tensors.values():
             t.fill_(float("nan"))
     return cache
+
+
+def i32(values):
+    return torch.tensor(values, dtype=torch.int32, device="cuda")
+
+
+def in_portions(mixer, h, cuts, dtype, start=0):
+    """The rows of h through a mixer in portions, in row 1 of a state full of an earlier owner's leftovers."""
+    from ohara_amd import ops
+    from ohara_amd.state_cache import LayerState
+
+    st = LayerState(512, {k: torch.full_like(t, float("nan")) for k, t in mixer.state(3, 512).items()})
+    at, got, slots = 0, [], i32([1])
+    for n in cuts:
+        seq = ops.Seq(1, n, at, slots=slots, host=([at], [n], [1]))
+        x = F.pad(h[at:at + n], (0, ops.round8(h.shape[1]) - h.shape[1]))
+        got.append(mixer(dev(x, dtype), st, seq)[:, :h.shape[1]])
+        at += n
+    assert at == len(h) and all(torch.isnan(t[[0, 2]]).all() for t in st.tensors.values())
+    return torch.cat(got)
 
 
 class Tok:

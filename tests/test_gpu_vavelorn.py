@@ -10,7 +10,7 @@ import pytest
 import torch
 import torch.nn.functional as F
 
-from _hybrid import Tok, close, dev, poisoned, rnd, tokens
+from _hybrid import Tok, close, dev, i32, in_portions, poisoned, rnd, tokens
 from _vavelorn import CONFIGS, agrees, attention, build, config, delta, latent, reference
 from oracle import vavelorn_ref as R
 
@@ -18,30 +18,10 @@ pytestmark = pytest.mark.gpu
 BF, F32, D = torch.bfloat16, torch.float32, torch.float64
 
 
-def i32(values):
-    return torch.tensor(values, dtype=torch.int32, device="cuda")
-
-
 def mixer_weights(layer, width, seed=0):
     """The tensors of one layer's mixer by their names inside the mixer."""
     w = R.random_weights({"width": width, "vocab": 4, "token_side": {"dim": 1}, "layers": [layer]}, seed)
     return {k[len("l0.mix."):]: t for k, t in w.items() if k.startswith("l0.mix.")}
-
-
-def in_portions(mixer, h, cuts, dtype, start=0):
-    """The rows of h through a mixer in portions, in row 1 of a state full of an earlier owner's leftovers."""
-    from ohara_amd import ops
-    from ohara_amd.state_cache import LayerState
-
-    st = LayerState(512, {k: torch.full_like(t, float("nan")) for k, t in mixer.state(3, 512).items()})
-    at, got, slots = 0, [], i32([1])
-    for n in cuts:
-        seq = ops.Seq(1, n, at, slots=slots, host=([at], [n], [1]))
-        x = F.pad(h[at:at + n], (0, ops.round8(h.shape[1]) - h.shape[1]))
-        got.append(mixer(dev(x, dtype), st, seq)[:, :h.shape[1]])
-        at += n
-    assert at == len(h) and all(torch.isnan(t[[0, 2]]).all() for t in st.tensors.values())
-    return torch.cat(got)
 
 
 # ---- mechanisms -------------------------------------------------------------------------------
