@@ -1110,6 +1110,196 @@ def bench_vavelorn(dev, sizes=("d1024", "d2048")):
     return out
 
 
+FIBIRAX_EXPERTS = (28, 4, 4, 4, 2)  # experts, identity outputs, used per token, groups, groups kept
+
+
+def fibirax_size(name):
+    """The config dict: attention in a window of 1024 beside retention in every layer, four of 28 experts (and four identity
+    outputs) of an eighth of the feed-forward and a shared one of half of it."""
+    d, n, H, G, dh, ff = HYBRID_SIZES[name]
+    experts, identity, top, groups, keep = FIBIRAX_EXPERTS
+    left = {"heads": H, "kv_heads": G, "dim": dh, "vdim": dh, "scale": dh ** -0.5, "softcap": 30.0, "mask": {"size": 1024},
+            "rot": {"base": 5e5, "dims": dh, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    right = {"heads": H, "dim": dh, "vdim": dh, "decay": [1 - 2.0 ** (-5 - 7 * h / H) for h in range(H)]}
+    mlp = {"kind": "moe", "router": {"experts": experts, "identity": identity, "top": top, "groups": {"count": groups, "keep": keep}},
+           "expert": {"ff": ff // 8, "limit": 7.0}, "shared": {"ff": ff // 2, "limit": 7.0}}
+    one = {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 1.0, "right_scale": 1.0}, "mlp": mlp}
+    return {"width": d, "vocab": 32000, "embedding": {"scale": d ** 0.5}, "norm": {"eps": 1e-6}, "layers": [one] * n}
+
+
+def fibirax_state(cfg, dev, seed=5):
+    """Random weights: matrices N(0, 1/columns), unit norms, corrections of a tenth of a score."""
+    g = torch.Generator(device=dev).manual_seed(seed)
+    n = lambda *shape, s=1.0: (torch.randn(*shape, generator=g, device=dev) * s).to(torch.bfloat16)  # noqa: E731
+    lin = lambda o, i: n(o, i, s=i ** -0.5)  # noqa: E731
+    one = lambda k: torch.ones(k, device=dev, dtype=torch.bfloat16)  # noqa: E731
+    d = cfg["width"]
+    st = {"embed": n(cfg["vocab"], d), "head": lin(cfg["vocab"], d), "final.norm": one(d)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, a, r, mlp = f"l{i}.", layer["mixer"]["left"], layer["mixer"]["right"], layer["mlp"]
+        st.update({p + k: one(d) for k in ("norm1", "norm2", "ls1", "ls2")})
+        q = p + "mix.left."
+        st.update({q + "q": lin(a["heads"] * a["dim"], d), q + "k": lin(a["kv_heads"] * a["dim"], d), q + "v": lin(a["kv_heads"] * a["vdim"], d),
+                   q + "o": lin(d, a["heads"] * a["vdim"]), q + "q.norm": one(a["dim"]), q + "k.norm": one(a["dim"])})
+        q = p + "mix.right."
+        nk, nv = r["heads"] * r["dim"], r["heads"] * r["vdim"]
+        st.update({q + "q": lin(nk, d), q + "k": lin(nk, d), q + "v": lin(nv, d), q + "g": lin(nv, d), q + "o": lin(d, nv)})
+        q, total = p + "mlp.", mlp["router"]["experts"] + mlp["router"]["identity"]
+        st.update({q + "router": lin(total, d), q + "correction": n(total, s=0.1 / total)})
+        for name, ff in [(f"e{e}", mlp["expert"]["ff"]) for e in range(mlp["router"]["experts"])] + [("shared", mlp["shared"]["ff"])]:
+            st.update({f"{q}{name}.gate": lin(ff, d), f"{q}{name}.up": lin(ff, d), f"{q}{name}.down": lin(d, ff)})
+    return st
+
+
+def _like_grouped_moe(name, dev):
+    """A Llama's grouped mixture of experts of the same sizes (every output an expert, four of them per token, one shared expert)."""
+    from ohara_amd.moe import GroupedMoE
+
+    d, _, _, _, _, ff = HYBRID_SIZES[name]
+    E, f, fs = sum(FIBIRAX_EXPERTS[:2]), ff // 8, ff // 2
+    g = torch.Generator(device=dev).manual_seed(6)
+    n = lambda *shape: (torch.randn(*shape, generator=g, device=dev) * d ** -0.5).to(torch.bfloat16)  # noqa: E731
+    return GroupedMoE(n(E, d, f), n(E, d, f), n(E, f, d), n(E, d), torch.zeros(E, device=dev), FIBIRAX_EXPERTS[2],
+                      shared=(n(fs, d), n(fs, d), n(d, fs)), device=dev)
+
+
+def bench_fibirax_kernels(name, dev):
+    """The design's own kernels at one layer's sizes, each beside the like kernel of Vavelorn or of Llama's experts."""
+    from ohara_amd import ops
+    from ohara_amd.fibirax import Fibirax, FibiraxConfig
+    from ohara_amd.vavelorn import Vavelorn, VavelornConfig
+
+    bf, cfg, vcfg = torch.bfloat16, fibirax_size(name), vavelorn_size(name)
+    cfg = {**cfg, "layers": cfg["layers"][:1]}
+    model = Fibirax(FibiraxConfig.from_dict(cfg, 4096), fibirax_state(cfg, dev), device=dev)
+    vav = _sole_layers(Vavelorn, VavelornConfig.from_dict, vavelorn_state(vcfg, dev), vcfg, ("delta",), dev)
+    like = _like_grouped_moe(name, dev)
+    block, delta = model.layers[0], vav.layers[0]["mixer"]
+    mixer, experts, norm = block["mixer"], block["mlp"], block["norm2"]
+    att, ret = (part for _, part in mixer.parts)
+    H, G, D, V, d, W = att.heads, att.kv_heads, att.dim, att.vdim, cfg["width"], att.window
+    top, ff, ffs, E = experts.top, experts.ff, experts.shared.ff, experts.experts
+    rnd = lambda *shape, dt=bf: torch.randn(*shape, device=dev).to(dt)  # noqa: E731
+    rows = []
+
+    def timed(fn, n=8):  # n calls per graph: what a single-launch graph costs to start would swamp the small kernels
+        return graph_time(lambda: [fn() for _ in range(n)], iters=20) / n
+
+    for B, L in ((1, 4096), (8, 4096), (32, 2048)):
+        seq = ops.Seq(B, 1, L - 1)
+        q, k, v = rnd(B, H * D), rnd(B, L, G, D), rnd(B, L, G, V)
+        ns, ws = att._split(B, L)
+        by = 2.0 * G * (D + V) * B * W
+        big, buf, cos, sin = rnd(B, mixer.proj.n), rnd(B, 2 * H * D), *(torch.ones(L, D // 2, device=dev) for _ in range(2))
+        small = 4.0 * B * (H * D + G * (D + V))
+        rows.append({
+            "kernel": "decode attention", "batch": B, "context": L, "window": W,
+            "attn_bias_kernel (window, cap, sink)": _hbm(timed(lambda: ops.attn_scored(
+                q, k, v, H, G, D, V, L, 0.1, seq, cap=30.0, window=W, sinks=att.sinks, n_split=ns, workspace=ws)), by),
+            "vavelorn attn_bias_kernel (chunk, cap)": _hbm(timed(lambda: ops.attn_scored(
+                q, k, v, H, G, D, V, L, 0.1, seq, cap=30.0, chunk=W, n_split=ns, workspace=ws)), by),
+            "qkv_headnorm_rotate_append_kernel": _hbm(timed(lambda: ops.qkv_headnorm_rotate_append(
+                big, H, G, D, V, att.q_norm, att.k_norm, 1e-6, cos, sin, D, k, v, seq)), small),
+            "vavelorn qkv_rotate_append_kernel": _hbm(timed(lambda: ops.qkv_rotate_append(big, H, G, D, V, cos, sin, D, k, v, seq)), small)})
+        row, st, rst = {"kernel": "recurrence, one token", "batch": B}, delta.state(B, 4096), ret.state(B, 4096)["retention"]
+        p, dst = big[:, mixer.n_in:], buf[:, mixer.n_out:mixer.n_out + H * V]
+        row["retention_step_kernel"] = _hbm(timed(lambda: ops.retention(ret._c, p, rst, None, seq, dst)), 8.0 * B * H * D * V + 10.0 * B * H * V)
+        pv = rnd(B, delta.proj.n)
+        row["vavelorn delta_step_kernel"] = _hbm(timed(lambda: ops.delta_step(delta._c, pv, st["delta"], st["ring"], seq)),
+                                                 8.0 * B * H * D * V + 10.0 * B * H * V)
+        rows.append(row)
+        x, h = rnd(B, d, dt=torch.float32), rnd(B, d)
+        experts.trace = []
+        mix = experts(h)
+        used = len({e for e in experts.trace[0][0].flatten().tolist() if e < E})
+        experts.trace = None
+        like.trace = []
+        like.forward_block(h, norm.w.to(bf), 1e-6)
+        used_l = len(set(like.trace[0][1].flatten().tolist()))
+        like.trace = None
+        one = torch.ones(d, device=dev, dtype=bf)
+        by = lambda n: 2.0 * (3 * d * (n * ff + ffs) + (E + 4) * d)  # noqa: E731
+        rows.append({
+            "kernel": "experts, one token per sequence", "batch": B, "experts used": (used, used_l),
+            "router + units + down + residual with their sum (4 launches)": _hbm(timed(lambda: ops.residual_norm(
+                x, seq, bf, **{**norm.of(experts(h)), "mode": "copy"})), by(used)),
+            "llama norm + router + SwiGLU + down + combine (4 launches)": _hbm(timed(lambda: like.forward_block(h, one, 1e-6)), by(used_l)),
+            "router alone": round(timed(lambda: ops.moe_router(h, experts.router, experts.correction, experts.k, top, experts.groups,
+                                                              experts.keep, experts._counter)) * 1e6, 1),
+            "residual_norm_kernel with mixture": _hbm(timed(lambda: ops.residual_norm(x, seq, bf, **{**norm.of(mix), "mode": "copy"})),
+                                                      B * d * (10.0 + 2 * top + 2 + 2)),
+            "residual_norm_kernel": _hbm(timed(lambda: ops.residual_norm(x, seq, bf, **{**norm.of(h), "mode": "copy"})), B * d * 12.0)})
+    for B, S in ((1, 4096), (8, 1024)):
+        seq, n = ops.Seq(B, S, 0), B * S
+        q, k, v = rnd(n, H * D), rnd(B, S, G, D), rnd(B, S, G, V)
+        fl = 2.0 * B * H * (D + V) * sum(min(i + 1, W) for i in range(S))
+        flc = 2.0 * B * H * (D + V) * sum(i % W + 1 for i in range(S))
+        row = {"kernel": "prompt", "batch": B, "tokens": S,
+               "attn_bias_prefill_kernel (window, cap, sink)": _flops(timed(lambda: ops.attn_scored(
+                   q, k, v, H, G, D, V, S, 0.1, seq, cap=30.0, window=W, sinks=att.sinks)), fl, MFMA_BF16_PEAK_TFLOPS),
+               "vavelorn attn_bias_prefill_kernel (chunk, cap)": _flops(timed(lambda: ops.attn_scored(
+                   q, k, v, H, G, D, V, S, 0.1, seq, cap=30.0, chunk=W)), flc, MFMA_BF16_PEAK_TFLOPS)}
+        big, buf, cos, sin = rnd(n, mixer.proj.n), rnd(n, mixer.width_out), *(torch.ones(S, D // 2, device=dev) for _ in range(2))
+        by = 4.0 * n * (H * D + G * (D + V))
+        row["qkv_headnorm_rotate_append_kernel"] = _hbm(timed(lambda: ops.qkv_headnorm_rotate_append(
+            big, H, G, D, V, att.q_norm, att.k_norm, 1e-6, cos, sin, D, k, v, seq)), by)
+        row["vavelorn qkv_rotate_append_kernel"] = _hbm(timed(lambda: ops.qkv_rotate_append(big, H, G, D, V, cos, sin, D, k, v, seq)), by)
+        rst, ws, p, dst = ret.state(B, 4096)["retention"], ret._workspace(B, S), big[:, mixer.n_in:], buf[:, mixer.n_out:]
+        fl = 5.0 * n * H * D * V  # the recurrence's own work: decay, the write, the product with q
+        t = timed(lambda: ops.retention(ret._c, p, rst, ws, seq, dst))
+        row["retention_prefill (3 kernels)"] = {**_flops(t, fl, FP32_MFMA_PEAK_TFLOPS),
+                                                "frac_of_hbm_peak (q, k, v, gate, output)": _hbm(t, 2.0 * n * H * (2 * D + 3 * V))["frac_of_hbm_peak"]}
+        st, pv, wd = delta.state(B, 4096), rnd(n, delta.proj.n), delta._workspace(B, S)
+        row["vavelorn delta_prefill (3 kernels)"] = _flops(timed(lambda: ops.delta_prefill(
+            delta._c, pv, None, None, st["delta"], st["ring"], wd, seq)), 7.0 * n * H * D * V, FP32_MFMA_PEAK_TFLOPS)
+        x, h = rnd(n, d, dt=torch.float32), rnd(n, d)
+        experts.trace = []
+        mix = experts(h)
+        pairs = int((experts.trace[0][0] < E).sum())
+        experts.trace = None
+        row["experts' share of the chosen outputs"] = round(pairs / (n * top), 3)
+        row["router + sort (3 kernels)"] = _hbm(timed(lambda: ops.moe_router(
+            h, experts.router, experts.correction, experts.k, top, experts.groups, experts.keep, experts._counter)), 2.0 * n * d)
+        row["llama router + choice + sort (3 kernels)"] = _hbm(timed(lambda: _like_route(like, h)), 2.0 * n * d)
+        row["experts (router to down)"] = _flops(timed(lambda: experts(h)), 6.0 * d * (pairs * ff + n * ffs), MFMA_BF16_PEAK_TFLOPS)
+        row["llama experts (router to combine)"] = _flops(timed(lambda: like.forward_rows(h, residual=h)), 6.0 * d * n * (top * ff + ffs),
+                                                          MFMA_BF16_PEAK_TFLOPS)
+        row["residual_norm_kernel with mixture"] = _hbm(timed(lambda: ops.residual_norm(x, seq, bf, **{**norm.of(mix), "mode": "copy"})),
+                                                        n * d * (10.0 + 2 * top + 2))
+        row["residual_norm_kernel"] = _hbm(timed(lambda: ops.residual_norm(x, seq, bf, **{**norm.of(h), "mode": "copy"})), n * d * 12.0)
+        rows.append(row)
+    return rows
+
+
+def _like_route(like, h):
+    from ohara_amd import ops
+    from ohara_amd._lib import check, lib
+
+    idx, _ = like.route(h)
+    n = idx.numel()
+    i32 = lambda k: torch.empty(k, dtype=torch.int32, device=h.device)  # noqa: E731
+    offs, pair_of, pos_of = i32(like.E + 1), i32(n), i32(n)
+    check(lib().ohara_moe_sort_pairs(idx.data_ptr(), n, like.E, offs.data_ptr(), pair_of.data_ptr(), pos_of.data_ptr(), ops._stream()), "moe_sort")
+
+
+def bench_fibirax(dev, sizes=("d1024", "d2048")):
+    """Prefill and decode of Fibirax with random weights beside Vavelorn and Llama at the same width, depth, heads and active
+    feed-forward."""
+    from ohara_amd.fibirax import Fibirax, FibiraxConfig
+    from ohara_amd.vavelorn import Vavelorn, VavelornConfig
+
+    out = {}
+    for name in sizes:
+        cfg, vcfg = fibirax_size(name), vavelorn_size(name)
+        out[name] = {"layers": len(cfg["layers"]), "width": cfg["width"], **bench_models(name, (
+            ("fibirax", lambda: Fibirax(FibiraxConfig.from_dict(cfg, 4608), fibirax_state(cfg, dev), device=dev)),
+            ("vavelorn", lambda: Vavelorn(VavelornConfig.from_dict(vcfg, 4608), vavelorn_state(vcfg, dev), device=dev)),
+            ("llama", lambda: hybrid_llama(name, dev))), dev)}
+        out[name]["kernels"] = bench_fibirax_kernels(name, dev)
+        print(f"fibirax {name}: done", file=sys.stderr, flush=True)
+    return out
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1143,6 +1333,8 @@ def main():
                     help="run the Povazen prefill, decode and kernel figures beside Llama at equal sizes alone and exit")
     ap.add_argument("--vavelorn-only", type=str, nargs="?", const="d1024,d2048", default="", metavar="SIZES",
                     help="run the Vavelorn prefill, decode and kernel figures beside Povazen and Llama at equal sizes alone and exit")
+    ap.add_argument("--fibirax-only", type=str, nargs="?", const="d1024,d2048", default="", metavar="SIZES",
+                    help="run the Fibirax prefill, decode and kernel figures beside Vavelorn and Llama at equal sizes alone and exit")
     ap.add_argument("--phi-decode-only", type=int, default=0, metavar="B",
                     help="run 12 eager Phi-2 decode steps of B sequences at context 1024 and exit (profiling workload)")
     args = ap.parse_args()
@@ -1169,6 +1361,9 @@ def main():
         return
     if args.vavelorn_only:
         print(json.dumps(bench_vavelorn(dev, tuple(args.vavelorn_only.split(","))), indent=1))
+        return
+    if args.fibirax_only:
+        print(json.dumps(bench_fibirax(dev, tuple(args.fibirax_only.split(","))), indent=1))
         return
     if args.phi_decode_only:
         print(json.dumps(phi_decode_only(dev, args.phi_decode_only)))
