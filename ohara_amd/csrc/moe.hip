@@ -164,12 +164,14 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int32_t* idx, int 
 // The same sort for at most 64 experts and 1024 pairs (decode): a pair's rank among the earlier pairs of
 // its expert is a ballot match inside its wave (six ballots for the six bits of an expert id) plus the
 // counts of the waves before it, instead of a scan over all earlier pairs; the offsets are one wave's scan.
-__global__ __launch_bounds__(1024) void moe_sort_small_kernel(const int32_t* idx, int NK, int E, int32_t* offs,
-                                                              int32_t* pair_of, int32_t* pos_of) {
-  __shared__ int wcnt[16][64];   // pairs of expert e in wave w, then the first sorted position of that wave's pairs of e
+// COH: idx is read past the caches (other workgroups wrote it in this launch).  wcnt: pairs of expert e in wave w, then the first
+// sorted position of that wave's pairs of e.
+template <bool COH>
+__device__ __forceinline__ void sort_small_1024(const int32_t* idx, int NK, int E, int32_t* offs, int32_t* pair_of, int32_t* pos_of,
+                                                int (*wcnt)[64]) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   wcnt[wave][lane] = 0;
-  const int e = tid < NK ? idx[tid] : -1;
+  const int e = tid < NK ? (COH ? (int)ld_coh4(idx + tid) : idx[tid]) : -1;
   unsigned long long same = __ballot(e >= 0);
 #pragma unroll
   for (int bit = 0; bit < 6; ++bit) {
@@ -203,6 +205,11 @@ __global__ __launch_bounds__(1024) void moe_sort_small_kernel(const int32_t* idx
     pair_of[o] = tid;
     pos_of[tid] = o;
   }
+}
+__global__ __launch_bounds__(1024) void moe_sort_small_kernel(const int32_t* idx, int NK, int E, int32_t* offs,
+                                                              int32_t* pair_of, int32_t* pos_of) {
+  __shared__ int wcnt[16][64];
+  sort_small_1024<false>(idx, NK, E, offs, pair_of, pos_of, wcnt);
 }
 
 // ---- norm + router + selection + sort in one launch (decode: at most 64 experts and 1024 pairs) -------
@@ -524,37 +531,38 @@ struct RouterArgs {
   int sort;
 };
 
-constexpr int RT = 16;  // tokens of a workgroup
+constexpr int RT = 16;  // tokens of a workgroup, waves of a workgroup
+constexpr int RED_LD = 260;  // floats of one wave's share of a strip (256), apart in LDS banks
 
-// The products of 16 tokens with all router rows, 64 rows at a time with K split over the four waves; then four tokens per wave,
-// lane l looking at outputs l, l + 64, ...
-template <typename T, int MAXPL>
-__global__ __launch_bounds__(256) void moe_router_kernel(RouterArgs<T> a) {
-  extern __shared__ __align__(16) float zs[];  // [RT][E]
-  __shared__ float red[4][4][64][4];
+// The products of 16 tokens with up to NS strips of 16 router rows at a time, K split over the sixteen waves (a single token's launch
+// is one round of loads); then a token per wave, lane l looking at outputs l, l + 64, ...
+template <typename T, int MAXPL, int NS>
+__global__ __launch_bounds__(1024) void moe_router_kernel(RouterArgs<T> a) {
+  extern __shared__ __align__(16) float zs[];  // [RT][E], then every wave's sums [RT][NS][RED_LD]
   __shared__ int wcnt[16][64];
   __shared__ int is_last;
+  float* red = zs + RT * a.E;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 15, g = lane >> 4;
   const int t0 = blockIdx.x * RT, KS = (a.K + 31) >> 5;
   const T* xr = a.x + (size_t)min(t0 + m, a.N - 1) * a.ldx + 8 * g;
-  for (int e0 = 0; e0 < a.E; e0 += 64) {
-    f32x4 acc[4];
+  for (int e0 = 0; e0 < a.E; e0 += 16 * NS) {
+    f32x4 acc[NS];
 #pragma unroll
-    for (int s = 0; s < 4; ++s) acc[s] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    const T* wr[4];
+    for (int s = 0; s < NS; ++s) acc[s] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const T* wr[NS];
 #pragma unroll
-    for (int s = 0; s < 4; ++s) wr[s] = a.w + (size_t)min(e0 + 16 * s + m, a.E - 1) * a.ldw + 8 * g;
-    constexpr int CH = sizeof(T) == 2 ? 4 : 2;  // steps whose loads are issued together
-    for (int jb = wave; jb < KS; jb += 4 * CH) {
-      Frag<T> xf[CH], wf[CH][4];
+    for (int s = 0; s < NS; ++s) wr[s] = a.w + (size_t)min(e0 + 16 * s + m, a.E - 1) * a.ldw + 8 * g;
+    constexpr int CH = (sizeof(T) == 2 ? 4 : 2) / (NS == 4 ? 2 : 1);  // steps whose loads are issued together
+    for (int jb = wave; jb < KS; jb += RT * CH) {
+      Frag<T> xf[CH], wf[CH][NS];
 #pragma unroll
       for (int c = 0; c < CH; ++c) {
-        const int j = jb + 4 * c;
+        const int j = jb + RT * c;
         const bool in = 32 * j + 8 * g < a.K;  // K is a multiple of 8
         if (in) frag_load(xf[c], xr + 32 * j);
         else frag_zero(xf[c]);
 #pragma unroll
-        for (int s = 0; s < 4; ++s) {
+        for (int s = 0; s < NS; ++s) {
           if (in) frag_load(wf[c][s], wr[s] + 32 * j);
           else frag_zero(wf[c][s]);
         }
@@ -562,27 +570,25 @@ __global__ __launch_bounds__(256) void moe_router_kernel(RouterArgs<T> a) {
 #pragma unroll
       for (int c = 0; c < CH; ++c)
 #pragma unroll
-        for (int s = 0; s < 4; ++s) acc[s] = mma(wf[c][s], xf[c], acc[s]);
+        for (int s = 0; s < NS; ++s) acc[s] = mma(wf[c][s], xf[c], acc[s]);
     }
     if (e0) __syncthreads();
 #pragma unroll
-    for (int s = 0; s < 4; ++s)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) red[wave][s][lane][i] = acc[s][i];
+    for (int s = 0; s < NS; ++s) *reinterpret_cast<f32x4*>(red + (wave * NS + s) * RED_LD + 4 * lane) = acc[s];
     __syncthreads();
-    // wave s finishes rows 16 s .. : lane (token m, rows 4 g ..)
+    for (int i = tid; i < NS * 256; i += 1024) {  // strip i / 256, row and token i % 256
+      const int s = i >> 8, r = (i >> 4) & 15, t = i & 15, e = e0 + 16 * s + r;
+      float z = 0.f;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int e = e0 + 16 * wave + 4 * g + i;
-      if (e < a.E)
-        zs[m * a.E + e] = ((red[0][wave][lane][i] + red[1][wave][lane][i]) + red[2][wave][lane][i]) + red[3][wave][lane][i];
+      for (int w = 0; w < RT; ++w) z += red[(w * NS + s) * RED_LD + 4 * (16 * (r >> 2) + t) + (r & 3)];
+      if (e < a.E) zs[t * a.E + e] = z;
     }
   }
   __syncthreads();
   const int per = a.E / a.groups;
-  for (int tt = 0; tt < RT / 4; ++tt) {
-    const int t = (RT / 4) * wave + tt, n = t0 + t;
-    float* z = zs + t * a.E;
+  const int n = t0 + wave;
+  if (n < a.N) {  // the same for the whole wave, whose row of zs is its own from here on
+    float* z = zs + wave * a.E;
     float s[MAXPL], ch[MAXPL], mx = -INFINITY, sum = 0.f;
 #pragma unroll
     for (int i = 0; i < MAXPL; ++i) {
@@ -604,11 +610,12 @@ __global__ __launch_bounds__(256) void moe_router_kernel(RouterArgs<T> a) {
       ch[i] = e < a.E ? s[i] + (a.correction ? a.correction[e] : 0.f) : -INFINITY;
       if (!(ch[i] == ch[i])) ch[i] = -INFINITY;  // a padding row may hold anything: every row still picks distinct outputs
     }
-    if (a.groups > 1) {  // the same for all waves
+    if (a.groups > 1) {
 #pragma unroll
       for (int i = 0; i < MAXPL; ++i)
         if (64 * i + lane < a.E) z[64 * i + lane] = ch[i];
-      __syncthreads();
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
       float best = -INFINITY;  // of group `lane`
       if (lane < a.groups)
         for (int e = lane * per; e < (lane + 1) * per; ++e) best = fmaxf(best, z[e]);
@@ -660,7 +667,7 @@ __global__ __launch_bounds__(256) void moe_router_kernel(RouterArgs<T> a) {
     }
     float tot = 0.f;
     for (int j = 0; j < a.top; ++j) tot += __uint_as_float((uint32_t)__builtin_amdgcn_readlane((int)__float_as_uint(my_s), j));
-    if (n < a.N && lane < a.top) {
+    if (lane < a.top) {
       st_coh4(a.idx + (size_t)n * a.top + lane, (uint32_t)my_id);  // (read by the workgroup that sorts)
       a.wgt[(size_t)n * a.top + lane] = my_s / (tot + 1e-20f);
     }
@@ -674,7 +681,7 @@ __global__ __launch_bounds__(256) void moe_router_kernel(RouterArgs<T> a) {
     if (is_last) __hip_atomic_store(a.counter, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // ready for the next call
   }
   __syncthreads();
-  if (is_last) sort_small_256(a.idx, a.N * a.top, a.E, a.offs, a.pair_of, a.pos_of, wcnt);
+  if (is_last) sort_small_1024<true>(a.idx, a.N * a.top, a.E, a.offs, a.pair_of, a.pos_of, wcnt);
 }
 
 // The sort for many pairs on many workgroups: counts of every block of 1024 pairs, then every block places its own.
@@ -871,15 +878,17 @@ int launch_router(RouterArgs<T> a, int32_t* hist, hipStream_t st) {
   const int NK = a.N * a.top;
   a.sort = a.E <= 64 && NK <= 1024;
   if (!a.sort && !hist) return OHARA_EINVAL;
-  const dim3 grid((unsigned)((a.N + RT - 1) / RT)), block(256);
-  const size_t smem = (size_t)RT * a.E * sizeof(float);
-  auto go = [&](auto kernel) {
+  const dim3 grid((unsigned)((a.N + RT - 1) / RT)), block(64 * RT);
+  auto go = [&](auto kernel, int ns) {
+    const size_t smem = (size_t)RT * (a.E + ns * RED_LD) * sizeof(float);
     if (smem > 32 * 1024) (void)hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
     hipLaunchKernelGGL(kernel, grid, block, smem, st, a);
   };
-  if (a.E <= 64) go(moe_router_kernel<T, 1>);
-  else if (a.E <= 256) go(moe_router_kernel<T, 4>);
-  else go(moe_router_kernel<T, 16>);
+  if (a.E <= 16) go(moe_router_kernel<T, 1, 1>, 1);
+  else if (a.E <= 32) go(moe_router_kernel<T, 1, 2>, 2);
+  else if (a.E <= 64) go(moe_router_kernel<T, 1, 4>, 4);
+  else if (a.E <= 256) go(moe_router_kernel<T, 4, 4>, 4);
+  else go(moe_router_kernel<T, 16, 4>, 4);
   if (!a.sort) {
     const dim3 blocks((unsigned)((NK + 1023) / 1024));
     hipLaunchKernelGGL(moe_count_kernel, blocks, dim3(1024), 0, st, a.idx, NK, a.E, hist);
