@@ -694,45 +694,56 @@ __global__ __launch_bounds__(1024) void moe_count_kernel(const int32_t* idx, int
   __syncthreads();
   if (tid < E) hist[(size_t)blockIdx.x * E + tid] = cnt[tid];
 }
+// A pair's rank among the earlier pairs of its expert: a ballot match inside its wave, and the counts of the waves before it.
 __global__ __launch_bounds__(1024) void moe_place_kernel(const int32_t* idx, int NK, int E, const int32_t* hist, int32_t* offs,
                                                          int32_t* pair_of, int32_t* pos_of) {
-  __shared__ int first[1024];  // sorted position of this block's first pair of every expert
+  extern __shared__ int wcnt[];  // [16][E]: pairs of an expert in a wave, then the sorted position of that wave's first
   __shared__ int wsum[16];
-  __shared__ __align__(16) int sidx[1024];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, blk = blockIdx.x, nb = gridDim.x;
+  const int p = blk * 1024 + tid, e = p < NK ? idx[p] : -1;
+  for (int i = tid; i < 16 * E; i += 1024) wcnt[i] = 0;
   int total = 0, before = 0;
-  if (tid < E)
-    for (int b = 0; b < nb; ++b) {
-      const int c = hist[(size_t)b * E + tid];
-      total += c;
-      before += b < blk ? c : 0;
+  if (tid < E) {
+    for (int b0 = 0; b0 < nb; b0 += 8) {  // eight blocks' counts in flight
+      int c[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) c[u] = hist[(size_t)min(b0 + u, nb - 1) * E + tid];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        total += b0 + u < nb ? c[u] : 0;
+        before += b0 + u < blk ? c[u] : 0;
+      }
     }
+  }
   const int incl = wave_incl_scan_i(total);
   if (lane == 63) wsum[wave] = incl;
-  const int p = blk * 1024 + tid, e = p < NK ? idx[p] : -1;
-  sidx[tid] = e;
+  unsigned long long same = __ballot(e >= 0);
+  for (int bit = 0; (E - 1) >> bit; ++bit) {
+    const unsigned long long b = __ballot((e >> bit) & 1);
+    same &= ((e >> bit) & 1) ? b : ~b;
+  }
+  const int rank = __popcll(same & ((1ull << lane) - 1ull));
+  __syncthreads();
+  if (e >= 0 && (same >> lane) == 1ull) wcnt[wave * E + e] = __popcll(same);  // the last lane of the wave with this expert
   __syncthreads();
   int run = incl - total;
   for (int w = 0; w < wave; ++w) run += wsum[w];
-  if (tid < E) first[tid] = run + before;
-  if (blk == 0) {
-    if (tid < E) offs[tid] = run;
-    if (tid == E - 1) offs[E] = run + total;
+  if (tid < E) {
+    if (blk == 0) {
+      offs[tid] = run;
+      if (tid == E - 1) offs[E] = run + total;
+    }
+    run += before;
+#pragma unroll
+    for (int w = 0; w < 16; ++w) {
+      const int c = wcnt[w * E + tid];
+      wcnt[w * E + tid] = run;
+      run += c;
+    }
   }
   __syncthreads();
-  // pairs before this one with the same expert: a wave scans the entries below its last lane
-  const int wave_first = tid & ~63;
-  const int n4 = blk * 1024 + wave_first < NK ? (min(wave_first + 64, NK - blk * 1024) + 3) >> 2 : 0;
-  int rank = 0;
-  const int4* s4 = reinterpret_cast<const int4*>(sidx);
-#pragma unroll 4
-  for (int t4 = 0; t4 < n4; ++t4) {
-    const int4 v = s4[t4];
-    const int t = 4 * t4;
-    rank += (t < tid && v.x == e) + (t + 1 < tid && v.y == e) + (t + 2 < tid && v.z == e) + (t + 3 < tid && v.w == e);
-  }
   if (e >= 0) {
-    const int o = first[e] + rank;
+    const int o = wcnt[wave * E + e] + rank;
     pair_of[o] = p;
     pos_of[p] = o;
   }
@@ -892,7 +903,9 @@ int launch_router(RouterArgs<T> a, int32_t* hist, hipStream_t st) {
   if (!a.sort) {
     const dim3 blocks((unsigned)((NK + 1023) / 1024));
     hipLaunchKernelGGL(moe_count_kernel, blocks, dim3(1024), 0, st, a.idx, NK, a.E, hist);
-    hipLaunchKernelGGL(moe_place_kernel, blocks, dim3(1024), 0, st, a.idx, NK, a.E, hist, a.offs, a.pair_of, a.pos_of);
+    const size_t lds = (size_t)16 * a.E * sizeof(int);
+    if (lds > 60 * 1024) (void)hipFuncSetAttribute((const void*)moe_place_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL(moe_place_kernel, blocks, dim3(1024), lds, st, a.idx, NK, a.E, hist, a.offs, a.pair_of, a.pos_of);
   }
   return ohara_launch_status();
 }

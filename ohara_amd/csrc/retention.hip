@@ -121,6 +121,11 @@ __device__ __forceinline__ void stage4x8(const T* rows, int ldp, int t, int n, b
 
 template <typename T> constexpr int ld_tokens() { return KB + 16 / (int)sizeof(T); }  // a staged column of KB tokens, 16 bytes apart mod 128
 
+__device__ __forceinline__ void ld_row8(const float* p, float* o) {  // eight floats from LDS
+  const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+  o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w; o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w;
+}
+
 constexpr int VS = 64;  // value columns of a workgroup of retention_local_kernel
 
 // sum_j g^(n-1-j) k_scale k_j v_j^T of a chunk, for VS of the value columns: a wave takes every fourth 16-row tile of the key channels.
@@ -366,23 +371,39 @@ __global__ __launch_bounds__(256, 1) void retention_out_kernel(RetentionArgs<T> 
       ss = lanes_sum<8, 1>(ss);
       if (m == 0) red[wave][16 * q + 4 * g + u] = ss;
     }
-  __syncthreads();
+  // half of the rows at a time through LDS, so that gates and outputs move eight columns per thread
+  const int ldy = Vp + 4, v8 = V / 8;
+  float* Y = reinterpret_cast<float*>(smem);  // [C / 2][ldy]
 #pragma unroll
-  for (int q = 0; q < QT; ++q)
+  for (int half = 0; half < 2; ++half) {
+    __syncthreads();
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int t = 16 * q + 4 * g + u;
-      if (t >= n) continue;
-      const float tot = ((red[0][t] + red[1][t]) + red[2][t]) + red[3][t];
-      const float inv = r.out_scale / sqrtf(tot / (float)r.vdim_used + r.eps);
-      const T* gp = rows + (size_t)t * a.ldp + r.off_g + h * V;
-      T* op = a.out + ((size_t)b * a.seq.seq_len + s0 + t) * a.ldo + h * V;
+    for (int q = 0; q < QT / 2; ++q)
 #pragma unroll
-      for (int i = 0; i < NT; ++i) {
-        const int c = 16 * (wave + 4 * i) + m;
-        if (c < V) stv(op + c, acc[i][q][u] * inv * silu_x(ldv(gp + c)));
+      for (int u = 0; u < 4; ++u) {
+        const int t = 16 * q + 4 * g + u, tt = t + half * (C / 2);
+        const float tot = ((red[0][tt] + red[1][tt]) + red[2][tt]) + red[3][tt];
+        const float inv = r.out_scale / sqrtf(tot / (float)r.vdim_used + r.eps);
+#pragma unroll
+        for (int i = 0; i < NT; ++i)
+          if (wave + 4 * i < vt) Y[t * ldy + 16 * (wave + 4 * i) + m] = acc[i][half * (QT / 2) + q][u] * inv;
       }
+    __syncthreads();
+    const int left = min(C / 2, n - half * (C / 2));
+    for (int i = tid; i < left * v8; i += 256) {
+      const int t = i / v8, c = 8 * (i - t * v8), tt = t + half * (C / 2);
+      Raw8<T> gr;
+      gr.load(rows + (size_t)tt * a.ldp + r.off_g + h * V + c);
+      float z[8], y[8];
+      gr.get(z);
+      ld_row8(Y + t * ldy + c, y);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) y[u] *= silu_x(z[u]);
+      T* op = a.out + ((size_t)b * a.seq.seq_len + s0 + tt) * a.ldo + h * V + c;
+      st4(op, y);
+      st4(op + 4, y + 4);
     }
+  }
 }
 
 template <typename T>
@@ -392,7 +413,7 @@ int retention_ok(const OharaRetention* r, const T* p, int ldp, const float* stat
   if (r->vdim_used < 1 || r->vdim_used > r->vdim) return OHARA_EINVAL;
   if (r->dim > 256 || r->vdim > 256 || r->heads > 65535 || seq->batch > 65535) return OHARA_ESIZE;
   const int nk = r->heads * r->dim, nv = r->heads * r->vdim;
-  if ((ldp & 7) || ((r->off_q | r->off_k | r->off_v | r->off_g) & 7) || ldo < nv) return OHARA_EINVAL;
+  if ((ldp & 7) || ((r->off_q | r->off_k | r->off_v | r->off_g) & 7) || (ldo & 3) || ldo < nv) return OHARA_EINVAL;
   for (int o : {r->off_q, r->off_k})
     if (o < 0 || o + nk > ldp) return OHARA_EINVAL;
   for (int o : {r->off_v, r->off_g})
@@ -439,7 +460,9 @@ int retention_prefill(const OharaRetention* r, const T* p, int ldp, float* state
   const int fit = (int)(ws_bytes / per_chunk < all ? ws_bytes / per_chunk : all);
   if (fit < 1) return OHARA_EINVAL;
   constexpr int LD = ld_tokens<T>(), PL = WideLds<T>::PLANES;
-  const size_t local_lds = ((size_t)Dp + PL * VS) * LD * sizeof(T), out_lds = ((size_t)PL * C + Vp) * LD * sizeof(T);
+  const size_t local_lds = ((size_t)Dp + PL * VS) * LD * sizeof(T);
+  size_t out_lds = ((size_t)PL * C + Vp) * LD * sizeof(T);
+  if (out_lds < (size_t)(C / 2) * (Vp + 4) * sizeof(float)) out_lds = (size_t)(C / 2) * (Vp + 4) * sizeof(float);
   const dim3 block(256);
   for (int c0 = 0; c0 < all; c0 += fit) {
     a.chunk0 = c0;
