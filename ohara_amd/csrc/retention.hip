@@ -267,9 +267,10 @@ __global__ __launch_bounds__(256, 1) void retention_out_kernel(RetentionArgs<T> 
   for (int i = 0; i < NT; ++i)
 #pragma unroll
     for (int q = 0; q < QT; ++q) acc[i][q] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  auto load_row = [&](Frag<T>& f, const T* base, int t, int d) {  // row t, columns d .. d+7
-    if (t < n && d < D) frag_load(f, base + (size_t)t * a.ldp + d);
-    else frag_zero(f);
+  // Row t, columns d .. d+7, loaded whatever t and d: rows past the chunk give scores nobody reads, columns past the head are zeroed.
+  auto load_row = [&](Frag<T>& f, const T* base, int t, int d) {
+    frag_load(f, base + (size_t)min(t, n - 1) * a.ldp + (d < D ? d : 0));
+    if (d >= D) frag_zero(f);
   };
   __syncthreads();
   // the state's part
